@@ -35,7 +35,7 @@ typedef enum {
 } lv_status;
 
 /* GGML element types the layer understands (types.h:28-43 of the reference) */
-enum { LV_F32 = 0, LV_F16 = 1, LV_Q4_0 = 2, LV_Q8_0 = 8 };
+enum { LV_F32 = 0, LV_F16 = 1, LV_Q4_0 = 2, LV_Q8_0 = 8, LV_BF16 = 30 /* block models, below */ };
 
 typedef struct lv_ctx lv_ctx;
 typedef struct lv_model lv_model;
@@ -76,6 +76,54 @@ int lv_model_hparams(const lv_model *model, lv_hparams *out);
 /* bytes of HBM the weight arena holds */
 int lv_model_arena_bytes(const lv_model *model, uint64_t *bytes);
 
+/* ---- block models: designs whose layers are put together from described mechanisms (no counterpart in the reference,
+ *      which knows one design).  A layer is  x += post1(mixer(pre1(x)));  x += post2(ff(pre2(x)))  with RMS norms on both
+ *      sides of each sublayer; the mixer is one or two branches reading the same input, summed with a scale each:
+ *        attention  grouped-query softmax attention (csrc/lv_gqa.h)
+ *        delta      gated delta rule with a decay per key channel (csrc/lv_delta.h)
+ *      and the feed-forward a mixture of experts whose weights multiply the experts' inputs, or none.
+ *      Weights are bfloat16, [out][in].  Every lv_session_* / lv_step_* / lv_logits_* / lv_argmax call works on sessions of
+ *      such a model; what differs is said at the call. ------------------------------------------------------------- */
+enum {
+    LV_ATTN_NORM_FULL = 1,       /* RMS norm with weights over the whole query projection and the whole key projection, before rotation */
+    LV_ATTN_KEYS_AS_VALUES = 2,  /* no value projection: the values are the projected keys (vdim == dim) */
+    LV_ATTN_SINK = 4             /* one learned logit per head joins the softmax denominator */
+};
+typedef struct {
+    uint32_t heads, kv_heads, dim, vdim;   /* heads 0: the layer has no attention branch */
+    float scale;
+    uint32_t chunk;                        /* a position sees its own chunk of this many positions, up to itself; 0: everything up to itself */
+    uint32_t rot_dims;                     /* rotated dimensions of a head (even), adjacent pairs, angle p * rot_base^(-2i / rot_dims) */
+    double rot_base;
+    uint32_t flags;
+} lv_attn_spec;
+typedef struct {
+    uint32_t heads, kv_heads, dim, vdim;   /* heads 0: no such branch */
+    uint32_t conv;                         /* taps of the causal convolutions on q, k and v (the current token included) */
+} lv_delta_spec;
+typedef struct {
+    uint32_t experts, top, ff;             /* experts 0: the layer has no feed-forward */
+} lv_moe_spec;
+typedef struct {
+    float attn_scale, delta_scale;         /* factors of the two branches */
+    lv_attn_spec attn;
+    lv_delta_spec delta;
+    lv_moe_spec moe;
+} lv_block_spec;
+typedef struct {
+    uint32_t vocab, dim, layers;
+    float eps;                             /* of every RMS norm */
+} lv_block_hparams;
+
+/* Uploads such a model.  Tensors are looked up by name in `table` (bf16; vectors may be f32): embed, final.norm, head, and
+ * per layer i, prefix "l<i>.": norm1, norm1b, norm2, norm2b, mix.left.{q,k,v,o,q.norm,k.norm,sink} (attention),
+ * mix.right.{q,k,v,b,a1,a2,g1,g2,o,q.conv,k.conv,v.conv,A_log,dt_bias,norm} (delta), mlp.router, mlp.e<j>.{gate,up,down}.
+ * The ranks of a1 / a2 and g1 / g2 are taken from the tensors.  compute: LV_BF16 = matrix products of batches on bf16
+ * activations with 32-bit accumulation and bf16 cache rows; LV_F32 = every operand in 32-bit.  Norms, scores, softmax,
+ * router, the recurrence and the residual stream are fp32 in both. */
+int lv_block_model_upload(lv_ctx *ctx, const void *base, uint64_t base_size, const lv_block_hparams *hp, const lv_block_spec *blocks,
+                          const lv_tensor_desc *table, uint32_t n_tensors, int compute, lv_model **out);
+
 /* ---- session: replaces llava_session::recreate_buffers (llava_session.cpp:49-79), set_backlog_size
  *      (:303-327) and llava_layer_session_data::flush_buffers_on_gpu (llava_layer_session_data.cpp:52-163) */
 int lv_session_create(lv_model *model, lv_session **out);
@@ -89,6 +137,8 @@ int lv_session_backlog(const lv_session *s, uint32_t *backlog);
  *      llava_command_buffer::record_execution / run (llava_command_buffer.cpp:29-55) and the whole shader chain
  *      of llava_layer::execute (llava_layer.cpp:39-75).
  *      Asynchronous.  Evaluates n tokens whose cache rows are pos .. pos+n-1 (pos = tokens already cached).
+ *      A block model's state moves on with every token: pos has to be where the last step ended (lv_session_position), or 0,
+ *      which starts a new sequence in the same session.
  *      Row z attends to cache rows 0 .. pos+z, like the batched shaders.  n == 1 replays a captured hipGraph. */
 int lv_step_begin(lv_session *s, const uint32_t *token_ids, uint32_t n, uint32_t pos);
 /* replaces llava_command_buffer::wait_idle (llava_command_buffer.cpp:25-27): the only sync point */
@@ -140,12 +190,22 @@ int lv_session_xcd_handover(lv_session *s, int *used);
  *      (llava_layer_session_data.cpp:165-181).  which: 0 = K, 1 = V.  n_tokens rows of `dim` fp16 values. */
 int lv_kv_read(lv_session *s, uint32_t layer, int which, uint32_t n_tokens, void *dst);
 int lv_kv_write(lv_session *s, uint32_t layer, int which, uint32_t n_tokens, const void *src);
+/* One layer's whole share of a sequence of n_tokens, whatever the model keeps per layer: K rows then V rows (lv_kv_read twice),
+ * or a block model's cache ring, convolution inputs and recurrent state (n_tokens has to be lv_session_position then, and a
+ * session is restored by writing every layer). */
+int lv_state_bytes(lv_session *s, uint32_t layer, uint32_t n_tokens, uint64_t *bytes);
+int lv_state_read(lv_session *s, uint32_t layer, uint32_t n_tokens, void *dst);
+int lv_state_write(lv_session *s, uint32_t layer, uint32_t n_tokens, const void *src);
+/* tokens the session's state stands at: where the next step of a block model may start (0 for other models, whose steps may
+ * start at any cached position) */
+int lv_session_position(const lv_session *s, uint32_t *pos);
 
 /* ---- record mode: replaces the per-layer trace buffers of llava_layer_session_data.cpp:79-86 and their
  *      routing in llava_layer.cpp:43-51.  When enabled, every step keeps, per layer and for every row of the step (the
  *      reference's buffers are batch_size rows long, llava_layer_session_data.cpp:80-85), the LV_TRACE_* below; the
  *      next step replaces them.  Memory: layers x rows x (5 x max(dim, ff) + backlog x heads) floats, grown to the
- *      longest step recorded so far. */
+ *      longest step recorded so far.  A block model records LV_TRACE_POST_ATTN (the residual stream behind the mixer) and
+ *      LV_TRACE_OUT (behind the layer). */
 enum {
     LV_TRACE_NORM_IN = 0,        /* normalized_input_logit  [dim] */
     LV_TRACE_POST_ATTN = 1,      /* post_attn_logit         [dim] */

@@ -19,7 +19,8 @@ import numpy as np
 PKG_DIR = os.path.dirname(os.path.abspath(__file__))
 ROOT_DIR = os.path.dirname(PKG_DIR)
 
-LV_F32, LV_F16, LV_Q4_0, LV_Q8_0 = 0, 1, 2, 8
+LV_F32, LV_F16, LV_Q4_0, LV_Q8_0, LV_BF16 = 0, 1, 2, 8, 30
+ATTN_NORM_FULL, ATTN_KEYS_AS_VALUES, ATTN_SINK = 1, 2, 4
 PATH_AUTO, PATH_KERNELS, PATH_GRAPH, PATH_PERSISTENT = range(4)
 TRACE_NORM_IN, TRACE_POST_ATTN, TRACE_POST_ATTN_NORM, TRACE_FF, TRACE_OUT, TRACE_ATTN = range(6)
 
@@ -38,6 +39,27 @@ class TensorDesc(C.Structure):
 class HParams(C.Structure):
     _fields_ = [("file_version", C.c_uint32), ("vocab", C.c_uint32), ("dim", C.c_uint32), ("heads", C.c_uint32),
                 ("layers", C.c_uint32), ("rot", C.c_uint32), ("ff", C.c_uint32)]
+
+
+class AttnSpec(C.Structure):
+    _fields_ = [("heads", C.c_uint32), ("kv_heads", C.c_uint32), ("dim", C.c_uint32), ("vdim", C.c_uint32), ("scale", C.c_float),
+                ("chunk", C.c_uint32), ("rot_dims", C.c_uint32), ("rot_base", C.c_double), ("flags", C.c_uint32)]
+
+
+class DeltaSpec(C.Structure):
+    _fields_ = [("heads", C.c_uint32), ("kv_heads", C.c_uint32), ("dim", C.c_uint32), ("vdim", C.c_uint32), ("conv", C.c_uint32)]
+
+
+class MoeSpec(C.Structure):
+    _fields_ = [("experts", C.c_uint32), ("top", C.c_uint32), ("ff", C.c_uint32)]
+
+
+class BlockSpec(C.Structure):
+    _fields_ = [("attn_scale", C.c_float), ("delta_scale", C.c_float), ("attn", AttnSpec), ("delta", DeltaSpec), ("moe", MoeSpec)]
+
+
+class BlockHParams(C.Structure):
+    _fields_ = [("vocab", C.c_uint32), ("dim", C.c_uint32), ("layers", C.c_uint32), ("eps", C.c_float)]
 
 
 class MkgConfig(C.Structure):
@@ -82,6 +104,11 @@ _HIP_SIGS = {
     "lv_session_timer_start": [_VP],
     "lv_session_timer_stop": [_VP, C.POINTER(C.c_float)],
     "lv_model_upload": [_VP, _VP, _U64, C.POINTER(HParams), C.POINTER(TensorDesc), _U32, C.POINTER(_VP)],
+    "lv_block_model_upload": [_VP, _VP, _U64, C.POINTER(BlockHParams), C.POINTER(BlockSpec), C.POINTER(TensorDesc), _U32, _I, C.POINTER(_VP)],
+    "lv_state_bytes": [_VP, _U32, _U32, C.POINTER(_U64)],
+    "lv_state_read": [_VP, _U32, _U32, _VP],
+    "lv_state_write": [_VP, _U32, _U32, _VP],
+    "lv_session_position": [_VP, C.POINTER(_U32)],
     "lv_model_destroy": [_VP],
     "lv_model_hparams": [_VP, C.POINTER(HParams)],
     "lv_model_arena_bytes": [_VP, C.POINTER(_U64)],
@@ -340,6 +367,29 @@ class Model:
             self.h = C.c_void_p()
 
 
+class BlockModel:
+    """A block model uploaded through lv_block_model_upload.  blocks: list of BlockSpec; table: (name, type, offset, rows, cols,
+    size) per tensor with offsets into `base` (a uint8 array; tensors may share bytes)."""
+
+    def __init__(self, ctx, base, table, blocks, vocab, dim, eps, compute=LV_BF16):
+        self.ctx = ctx
+        self.lib = ctx.lib
+        self.header = dict(vocab=vocab, dim=dim, layers=len(blocks), ff=0, heads=0)
+        descs = (TensorDesc * len(table))()
+        names = [t[0].encode() for t in table]
+        for d, t, nm in zip(descs, table, names):
+            d.name, d.ftype, d.offset, d.rows, d.cols, d.size = nm, t[1], t[2], t[3], t[4], t[5]
+        hp = BlockHParams(vocab, dim, len(blocks), eps)
+        self.h = C.c_void_p()
+        check(self.lib.lv_block_model_upload(ctx.h, C.c_void_p(base.ctypes.data), base.nbytes, C.byref(hp), (BlockSpec * len(blocks))(*blocks), descs,
+                                             len(table), compute, C.byref(self.h)))
+
+    def close(self):
+        if self.h:
+            self.lib.lv_model_destroy(self.h)
+            self.h = C.c_void_p()
+
+
 class Session:
     """lv_session: one stream, one K/V cache, one captured decode graph."""
 
@@ -423,6 +473,21 @@ class Session:
     def kv_write(self, layer, which, rows):
         rows = np.ascontiguousarray(rows, dtype=np.uint16)
         check(self.lib.lv_kv_write(self.h, layer, which, rows.shape[0], _ptr(rows)))
+
+    def position(self):
+        p = C.c_uint32()
+        check(self.lib.lv_session_position(self.h, C.byref(p)))
+        return p.value
+
+    def state(self, layer, n_tokens):
+        size = C.c_uint64()
+        check(self.lib.lv_state_bytes(self.h, layer, n_tokens, C.byref(size)))
+        out = np.empty(size.value, dtype=np.uint8)
+        check(self.lib.lv_state_read(self.h, layer, n_tokens, _ptr(out)))
+        return out
+
+    def state_write(self, layer, n_tokens, data):
+        check(self.lib.lv_state_write(self.h, layer, n_tokens, _ptr(np.ascontiguousarray(data))))
 
     def trace_enable(self, on=True):
         check(self.lib.lv_trace_enable(self.h, int(on)))

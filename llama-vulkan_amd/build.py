@@ -17,11 +17,12 @@ HOST_LIB = os.path.join(PKG, "libllava_host.so")
 MKGGML_LIB = os.path.join(PKG, "libmkggml.so")
 MKGGML_BIN = os.path.join(PKG, "bin", "mkggml")
 LLAVA_BIN = os.path.join(PKG, "bin", "llava")
+TRACE_BIN = os.path.join(PKG, "bin", "trace_run")
 ORACLE_LIB = os.path.join(ROOT, "oracle", "liboracle.so")
 
 # packed fp32 VALU ops are switched off for all device code
 HIPCC_FLAGS = [
-    "--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-shared", "-Wall", "-Wno-unused-function",
+    "--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-Wall", "-Wno-unused-function",
     "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
 ]
 
@@ -38,9 +39,23 @@ def hipcc():
     raise RuntimeError("hipcc not found: the HIP library cannot be built on this machine")
 
 
+HIP_UNITS = ("lv_api", "lv_block")    # translation units of libllava_hip.so, compiled side by side
+
+
 def build_hip():
-    src = os.path.join(PKG, "csrc", "lv_api.hip")
-    _run([hipcc(), *HIPCC_FLAGS, src, "-o", HIP_LIB])
+    objdir = os.path.join(PKG, "build")
+    os.makedirs(objdir, exist_ok=True)
+    objs, running = [], []
+    for unit in HIP_UNITS:
+        obj = os.path.join(objdir, unit + ".o")
+        cmd = [hipcc(), *HIPCC_FLAGS, "-c", os.path.join(PKG, "csrc", unit + ".hip"), "-o", obj]
+        print("+", " ".join(cmd), flush=True)
+        running.append((cmd, subprocess.Popen(cmd)))
+        objs.append(obj)
+    failed = [cmd for cmd, p in running if p.wait() != 0]
+    if failed:
+        raise subprocess.CalledProcessError(1, failed[0])
+    _run([hipcc(), "--offload-arch=gfx950", "-shared", "-fPIC", *objs, "-o", HIP_LIB])
     return HIP_LIB
 
 
@@ -54,7 +69,7 @@ def build_mkggml():
 
 def build_host():
     host = os.path.join(PKG, "host")
-    srcs = [os.path.join(host, f) for f in sorted(os.listdir(host)) if f.endswith(".cpp") and f != "main.cpp"]
+    srcs = [os.path.join(host, f) for f in sorted(os.listdir(host)) if f.endswith(".cpp") and f not in ("main.cpp", "trace_main.cpp")]
     server = os.path.join(host, "server")
     srcs += [os.path.join(server, f) for f in sorted(os.listdir(server)) if f.endswith(".cpp")]
     if not srcs:
@@ -62,10 +77,9 @@ def build_host():
     common = ["g++", "-std=c++17", "-O2", "-fPIC", "-Wall", "-Wextra", "-pthread", "-I", os.path.join(ROOT, "include")]
     link = ["-L", PKG, "-lllava_hip", "-Wl,-rpath,$ORIGIN", "-Wl,-rpath," + PKG]
     _run([*common, "-shared", *srcs, "-o", HOST_LIB, *link])
-    main = os.path.join(host, "main.cpp")
-    if os.path.exists(main):
-        os.makedirs(os.path.dirname(LLAVA_BIN), exist_ok=True)
-        _run([*common, main, "-o", LLAVA_BIN, "-L", PKG, "-lllava_host", "-lllava_hip",
+    os.makedirs(os.path.dirname(LLAVA_BIN), exist_ok=True)
+    for main, exe in (("main.cpp", LLAVA_BIN), ("trace_main.cpp", TRACE_BIN)):
+        _run([*common, os.path.join(host, main), "-o", exe, "-L", PKG, "-lllava_host", "-lllava_hip",
               "-Wl,-rpath,$ORIGIN/..", "-Wl,-rpath," + PKG])
     return HOST_LIB
 

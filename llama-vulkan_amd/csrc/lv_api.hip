@@ -18,6 +18,7 @@
 #include <string>
 #include <vector>
 
+#include "lv_block.h"
 #include "lv_kernels.h"
 #include "lv_mega.h"
 #include "lv_gemm.h"
@@ -31,7 +32,7 @@ using namespace lv;
 // -----------------------------------------------------------------------------------------------------------
 static thread_local char g_err[512] = "";
 
-static int fail(int code, const char *fmt, ...)
+int lv::fail(int code, const char *fmt, ...)
 {
     va_list ap;
     va_start(ap, fmt);
@@ -39,19 +40,6 @@ static int fail(int code, const char *fmt, ...)
     va_end(ap);
     return code;
 }
-
-#define HIP_TRY(expr)                                                                                         \
-    do {                                                                                                      \
-        hipError_t e_ = (expr);                                                                               \
-        if (e_ != hipSuccess) return fail(LV_ERR_HIP, "%s failed: %s (%s:%d)", #expr, hipGetErrorString(e_), \
-                                          __FILE__, __LINE__);                                                \
-    } while (0)
-
-#define LV_TRY(expr)              \
-    do {                          \
-        int rc_ = (expr);         \
-        if (rc_ != LV_OK) return rc_; \
-    } while (0)
 
 extern "C" const char *lv_last_error(void) { return g_err; }
 
@@ -170,6 +158,7 @@ struct lv_model {
     std::mutex prompt_mutex;
     int prompt_state = 0;           // 0 not made yet, 1 ready, -1 could not be made (batches then go token by token)
     uint16_t *prompt_arena = nullptr;
+    BlockModel *block = nullptr;    // a block model (lv_block.h): then nothing above but ctx and hp's vocab, dim and layers is set
     int output_state = 0;           // the same for the prompt copy of the output matrix, which only steps that keep every row's logits need
     uint16_t *output_copy = nullptr;
 };
@@ -260,6 +249,8 @@ struct lv_session {
     uint32_t trace_cap = 0;      // rows the two buffers have room for
     uint32_t trace_n = 0;        // rows the last recorded step wrote
     hipEvent_t ev_start = nullptr, ev_stop = nullptr;
+    BlockSession *block = nullptr;        // state and buffers of a block model's session, in place of everything LLaMA-specific above
+    uint32_t cfg_cap = 0;                 // token ids cfg and cfg_host have room for
 };
 
 static uint16_t *kv_ptr(const lv_session *s, uint32_t layer, int which)
@@ -423,7 +414,7 @@ __global__ void fill_zero_kernel(uint32_t *p, uint64_t words)
         p[i] = 0u;
 }
 
-static int zero_async(void *p, uint64_t bytes, hipStream_t st)
+int lv::zero_async(void *p, uint64_t bytes, hipStream_t st)
 {
     if (bytes == 0) return LV_OK;
     if (bytes % 4) return fail(LV_ERR_ARG, "zero fill: size not a multiple of 4");
@@ -1458,10 +1449,33 @@ extern "C" int lv_model_upload(lv_ctx *c, const void *base, uint64_t base_size, 
     return LV_OK;
 }
 
+extern "C" int lv_block_model_upload(lv_ctx *c, const void *base, uint64_t base_size, const lv_block_hparams *hp, const lv_block_spec *blocks,
+                                     const lv_tensor_desc *table, uint32_t n_tensors, int compute, lv_model **out)
+{
+    if (!c || !base || !hp || !blocks || !table || !out) return fail(LV_ERR_ARG, "lv_block_model_upload: null argument");
+    *out = nullptr;
+    HIP_TRY(hipSetDevice(c->device));
+    lv_model *m = new (std::nothrow) lv_model;
+    if (!m) return fail(LV_ERR_OOM, "lv_block_model_upload: host allocation");
+    m->ctx = c;
+    m->hp.vocab = hp->vocab;
+    m->hp.dim = hp->dim;
+    m->hp.layers = hp->layers;
+    const int rc = block_model_create(c->stream, base, base_size, hp, blocks, table, n_tensors, compute, &m->block);
+    if (rc != LV_OK) {
+        delete m;
+        return rc;
+    }
+    m->arena_bytes = block_model_bytes(m->block);
+    *out = m;
+    return LV_OK;
+}
+
 extern "C" int lv_model_destroy(lv_model *m)
 {
     if (!m) return LV_OK;
     (void)hipSetDevice(m->ctx->device);
+    block_model_destroy(m->block);
     (void)hipFree(m->prompt_arena);
     (void)hipFree(m->output_copy);
     (void)hipFree(m->mega_stream);
@@ -1507,6 +1521,7 @@ extern "C" int lv_session_destroy(lv_session *s)
         if (s->model->ctx->mega_last == s) s->model->ctx->mega_last = nullptr;   // its last launch has finished (stream synchronised)
     }
     drop_graph(s);
+    block_session_destroy(s->block);
     void *dev[] = {s->kv, s->trig, s->trig_abs, s->x, s->xn, s->q, s->k, s->v, s->vo, s->ff, s->logits, s->attn_part, s->attn_counters,
                    s->cfg, s->argmax_dev, s->trace_buf, s->trace_attn, s->pf_x, s->pf_xn, s->pf_q, s->pf_k, s->pf_v, s->pf_vo, s->pf_g1, s->pf_g2,
                    s->pf_xh, s->pf_xl, s->pf_xs, s->pf_planes, s->pf_fh, s->pf_fl, s->logits_all};
@@ -1525,11 +1540,32 @@ extern "C" int lv_session_destroy(lv_session *s)
     return LV_OK;
 }
 
+// position and token ids of a step, on the device and in pinned memory.  Growing drops the captured graph, which holds the address.
+static int cfg_reserve(lv_session *s, uint32_t tokens)
+{
+    if (tokens <= s->cfg_cap) return LV_OK;
+    HIP_TRY(hipStreamSynchronize(s->stream));
+    drop_graph(s);
+    (void)hipFree(s->cfg);
+    if (s->cfg_host) (void)hipHostFree(s->cfg_host);
+    s->cfg = s->cfg_host = nullptr;
+    s->cfg_cap = 0;
+    HIP_TRY(hipMalloc(reinterpret_cast<void **>(&s->cfg), (1 + (size_t)tokens) * 4));
+    HIP_TRY(hipHostMalloc(reinterpret_cast<void **>(&s->cfg_host), (1 + (size_t)tokens) * 4, hipHostMallocDefault));
+    s->cfg_cap = tokens;
+    return LV_OK;
+}
+
 static int session_alloc(lv_session *s)
 {
     const lv_hparams &hp = s->model->hp;
     const size_t D = hp.dim, F = hp.ff, V = hp.vocab;
     HIP_TRY(hipStreamCreateWithFlags(&s->stream, hipStreamNonBlocking));
+    HIP_TRY(hipMalloc(reinterpret_cast<void **>(&s->logits), V * 4));
+    HIP_TRY(hipMalloc(reinterpret_cast<void **>(&s->argmax_dev), 4));
+    HIP_TRY(hipHostMalloc(reinterpret_cast<void **>(&s->argmax_host), 4, hipHostMallocDefault));
+    LV_TRY(cfg_reserve(s, kMaxStepTokens));
+    if (s->model->block) return block_session_create(s->model->block, s->stream, &s->block);
     HIP_TRY(hipMalloc(reinterpret_cast<void **>(&s->x), D * 4));
     HIP_TRY(hipMalloc(reinterpret_cast<void **>(&s->xn), D * 4));
     HIP_TRY(hipMalloc(reinterpret_cast<void **>(&s->q), D * 4));
@@ -1537,11 +1573,6 @@ static int session_alloc(lv_session *s)
     HIP_TRY(hipMalloc(reinterpret_cast<void **>(&s->v), D * 4));
     HIP_TRY(hipMalloc(reinterpret_cast<void **>(&s->vo), D * 4));
     HIP_TRY(hipMalloc(reinterpret_cast<void **>(&s->ff), F * 4));
-    HIP_TRY(hipMalloc(reinterpret_cast<void **>(&s->logits), V * 4));
-    HIP_TRY(hipMalloc(reinterpret_cast<void **>(&s->cfg), (1 + kMaxStepTokens) * 4));
-    HIP_TRY(hipMalloc(reinterpret_cast<void **>(&s->argmax_dev), 4));
-    HIP_TRY(hipHostMalloc(reinterpret_cast<void **>(&s->cfg_host), (1 + kMaxStepTokens) * 4, hipHostMallocDefault));
-    HIP_TRY(hipHostMalloc(reinterpret_cast<void **>(&s->argmax_host), 4, hipHostMallocDefault));
     if (s->model->mega_kind) {
         size_t bytes = 0, local_bytes = 0;
         LV_TRY(mega_dispatch(s->model->mega_kind, [&](auto shape) -> int {
@@ -1632,6 +1663,11 @@ extern "C" int lv_session_reserve(lv_session *s, uint32_t backlog)
     HIP_TRY(hipSetDevice(s->model->ctx->device));
     HIP_TRY(hipStreamSynchronize(s->stream));
     drop_graph(s);
+    if (s->block) {
+        LV_TRY(block_session_reserve(s->block, backlog));
+        s->backlog = backlog;
+        return LV_OK;
+    }
 
     const size_t D = hp.dim, plane_new = (size_t)backlog * D, plane_old = (size_t)s->backlog * D;
     uint16_t *kv_new = nullptr;
@@ -1801,10 +1837,26 @@ static int trace_copy(lv_session *s, uint32_t layer, int which, uint32_t row, co
     return LV_OK;
 }
 
+// the trace buffers as a block model's step fills them
+static BlockTrace block_trace(const lv_session *s)
+{
+    const lv_hparams &hp = s->model->hp;
+    BlockTrace t;
+    t.base = s->trace_buf;
+    t.rows = s->trace_cap;
+    t.stride = hp.dim > hp.ff ? hp.dim : hp.ff;
+    t.kinds = LV_TRACE_ATTN;
+    return t;
+}
+
 // One token through every layer (llava_layer.cpp:53-73 + llava_command_buffer.cpp:38-39).  The token id is
 // cfg[1 + idx], its cache row cfg[0] + idx.  With_head = also compute the logits.
 static int record_token(lv_session *s, uint32_t idx, bool with_head)
 {
+    if (s->block) {
+        const BlockTrace t = block_trace(s);
+        return block_step_token(s->block, s->cfg, idx, with_head ? s->logits : nullptr, s->trace ? &t : nullptr);
+    }
     const lv_model *m = s->model;
     const lv_hparams &hp = m->hp;
     const uint32_t D = hp.dim, F = hp.ff;
@@ -1879,6 +1931,7 @@ static int record_token(lv_session *s, uint32_t idx, bool with_head)
 // 7B model; decode never reads it).  False when the device has no room for it: batches then go token by token.
 static bool ensure_prompt_copy(lv_model *m)
 {
+    if (m->block) return true;      // one copy of the weights serves both forms of a step
     std::lock_guard<std::mutex> lock(m->prompt_mutex);
     if (m->prompt_state) return m->prompt_state > 0;
     uint64_t halfs = 0;
@@ -1998,6 +2051,11 @@ static int launch_prefill_norm(hipStream_t st, lv_session *s, const float *w, ui
 // 0..pos+z: all K/V rows of the chunk are appended before any row attends, rows above its own are masked.
 static int record_prefill(lv_session *s, uint32_t idx0, uint32_t n, bool with_head, uint32_t row_base)
 {
+    if (s->block) {
+        const BlockTrace t = block_trace(s);
+        return block_step_batch(s->block, s->cfg, s->cfg_host[0] + idx0, idx0, n, with_head ? s->logits : nullptr,
+                                s->all_logits ? s->logits_all + (size_t)(row_base + idx0) * s->model->hp.vocab : nullptr, s->trace ? &t : nullptr);
+    }
     const lv_model *m = s->model;
     const lv_hparams &hp = m->hp;
     const uint32_t D = hp.dim, F = hp.ff;
@@ -2102,12 +2160,14 @@ extern "C" int lv_step_begin(lv_session *s, const uint32_t *tokens, uint32_t n, 
     if (!s || !tokens) return fail(LV_ERR_ARG, "lv_step_begin: null argument");
     if (s->in_flight) return fail(LV_ERR_STATE, "lv_step_begin: the previous step has not been waited for");
     if (n == 0) return fail(LV_ERR_ARG, "lv_step_begin: no tokens");
-    if (n > kMaxStepTokens) return fail(LV_ERR_RANGE, "lv_step_begin: %u tokens in one step (limit %u)", n, kMaxStepTokens);
+    if (n > kMaxStepTokens && !s->block) return fail(LV_ERR_RANGE, "lv_step_begin: %u tokens in one step (limit %u)", n, kMaxStepTokens);
     if (s->backlog == 0) return fail(LV_ERR_STATE, "lv_step_begin: lv_session_reserve has not been called");
     if ((uint64_t)pos + n > s->backlog)
         return fail(LV_ERR_RANGE, "lv_step_begin: rows %u..%u exceed the backlog of %u", pos, pos + n - 1, s->backlog);
     for (uint32_t i = 0; i < n; i++)
         if (tokens[i] >= s->model->hp.vocab) return fail(LV_ERR_RANGE, "lv_step_begin: token id %u of a vocabulary of %u", tokens[i], s->model->hp.vocab);
+    if (s->block && pos != 0 && pos != block_session_position(s->block))
+        return fail(LV_ERR_STATE, "lv_step_begin: the session's state stands at position %u, a step can start there or at 0, not at %u", block_session_position(s->block), pos);
     HIP_TRY(hipSetDevice(s->model->ctx->device));
 
     s->have_logits = false;
@@ -2164,6 +2224,10 @@ extern "C" int lv_step_begin(lv_session *s, const uint32_t *tokens, uint32_t n, 
                 HIP_TRY(hipMemcpyAsync(s->logits, s->logits_all + (size_t)(n - 1) * V, (size_t)V * 4, hipMemcpyDeviceToDevice, s->stream));
         }
     }
+    if (s->block) {
+        LV_TRY(cfg_reserve(s, n));
+        block_session_invalidate(s->block);      // until all of the step is on the stream
+    }
     if (!persistent) {             // the persistent kernel takes position and token id as launch arguments
         s->cfg_host[0] = pos;
         memcpy(s->cfg_host + 1, tokens, (size_t)n * 4);
@@ -2190,9 +2254,10 @@ extern "C" int lv_step_begin(lv_session *s, const uint32_t *tokens, uint32_t n, 
     } else {
         // rows are evaluated one after the other: row z sees cache rows 0..pos+z, which is what the batched
         // shaders compute (every row's K/V is appended before any row attends, and rows above are masked)
-        if (n >= kPrefillMin && !s->trace && ensure_prompt_copy(s->model)) {
-            for (uint32_t i = 0; i < n; i += kPrefillChunk) {
-                const uint32_t m = n - i < kPrefillChunk ? n - i : kPrefillChunk;
+        const uint32_t batch_min = s->block ? kBlockBatchMin : (uint32_t)kPrefillMin, batch_max = s->block ? kBlockBatch : kPrefillChunk;
+        if (n >= batch_min && (!s->trace || s->block) && ensure_prompt_copy(s->model)) {
+            for (uint32_t i = 0; i < n; i += batch_max) {
+                const uint32_t m = n - i < batch_max ? n - i : batch_max;
                 LV_TRY(record_prefill(s, i, m, i + m == n, row_base));
             }
         } else {
@@ -2203,6 +2268,7 @@ extern "C" int lv_step_begin(lv_session *s, const uint32_t *tokens, uint32_t n, 
             }
         }
     }
+    if (s->block) block_session_advance(s->block, pos + n);
     s->in_flight = true;
     s->have_logits = true;
     if (s->all_logits) s->logits_rows = n_rows;
@@ -2212,7 +2278,9 @@ extern "C" int lv_step_begin(lv_session *s, const uint32_t *tokens, uint32_t n, 
 extern "C" int lv_step_wait(lv_session *s)
 {
     if (!s) return fail(LV_ERR_ARG, "lv_step_wait: session is null");
-    HIP_TRY(hipStreamSynchronize(s->stream));
+    const hipError_t done = hipStreamSynchronize(s->stream);
+    if (done != hipSuccess && s->block) block_session_invalidate(s->block);
+    HIP_TRY(done);
     s->in_flight = false;
     const bool mega_step = s->mega_step;
     s->mega_step = false;
@@ -2315,9 +2383,10 @@ extern "C" int lv_session_timer_stop(lv_session *s, float *ms)
 // -----------------------------------------------------------------------------------------------------------
 // cache dump / restore, trace
 // -----------------------------------------------------------------------------------------------------------
-static int kv_args(const char *who, lv_session *s, uint32_t layer, uint32_t n_tokens, const void *p)
+static int kv_args(const char *who, lv_session *s, uint32_t layer, uint32_t n_tokens, const void *p, bool any_model = false)
 {
     if (!s || (n_tokens && !p)) return fail(LV_ERR_ARG, "%s: null argument", who);
+    if (s->block && !any_model) return fail(LV_ERR_ARG, "%s: this model keeps more than K and V rows (lv_state_read, lv_state_write)", who);
     if (layer >= s->model->hp.layers) return fail(LV_ERR_RANGE, "%s: layer %u of %u", who, layer, s->model->hp.layers);
     if (n_tokens > s->backlog) return fail(LV_ERR_RANGE, "%s: %u rows of a backlog of %u", who, n_tokens, s->backlog);
     if (s->in_flight) return fail(LV_ERR_STATE, "%s: a step is in flight", who);
@@ -2339,6 +2408,47 @@ extern "C" int lv_kv_write(lv_session *s, uint32_t layer, int which, uint32_t n_
     if (n_tokens == 0) return LV_OK;
     HIP_TRY(hipMemcpyAsync(kv_ptr(s, layer, which), src, (size_t)n_tokens * s->model->hp.dim * 2, hipMemcpyHostToDevice, s->stream));
     HIP_TRY(hipStreamSynchronize(s->stream));
+    return LV_OK;
+}
+
+extern "C" int lv_state_bytes(lv_session *s, uint32_t layer, uint32_t n_tokens, uint64_t *bytes)
+{
+    if (!s || !bytes) return fail(LV_ERR_ARG, "lv_state_bytes: null argument");
+    if (layer >= s->model->hp.layers) return fail(LV_ERR_RANGE, "lv_state_bytes: layer %u of %u", layer, s->model->hp.layers);
+    *bytes = s->block ? block_state_bytes(s->block, layer, n_tokens) : (uint64_t)n_tokens * s->model->hp.dim * 4;
+    return LV_OK;
+}
+
+extern "C" int lv_state_read(lv_session *s, uint32_t layer, uint32_t n_tokens, void *dst)
+{
+    LV_TRY(kv_args("lv_state_read", s, layer, n_tokens, dst, true));
+    if (n_tokens == 0) return LV_OK;
+    if (s->block) {
+        if (n_tokens != block_session_position(s->block))
+            return fail(LV_ERR_STATE, "lv_state_read: the session's state stands at position %u, not %u", block_session_position(s->block), n_tokens);
+        return block_state_copy(s->block, layer, n_tokens, dst, false);
+    }
+    LV_TRY(lv_kv_read(s, layer, 0, n_tokens, dst));
+    return lv_kv_read(s, layer, 1, n_tokens, static_cast<uint8_t *>(dst) + (size_t)n_tokens * s->model->hp.dim * 2);
+}
+
+extern "C" int lv_state_write(lv_session *s, uint32_t layer, uint32_t n_tokens, const void *src)
+{
+    LV_TRY(kv_args("lv_state_write", s, layer, n_tokens, src, true));
+    if (s->block) {
+        LV_TRY(block_state_copy(s->block, layer, n_tokens, const_cast<void *>(src), true));
+        block_session_advance(s->block, n_tokens);
+        return LV_OK;
+    }
+    if (n_tokens == 0) return LV_OK;
+    LV_TRY(lv_kv_write(s, layer, 0, n_tokens, src));
+    return lv_kv_write(s, layer, 1, n_tokens, static_cast<const uint8_t *>(src) + (size_t)n_tokens * s->model->hp.dim * 2);
+}
+
+extern "C" int lv_session_position(const lv_session *s, uint32_t *pos)
+{
+    if (!s || !pos) return fail(LV_ERR_ARG, "lv_session_position: null argument");
+    *pos = s->block ? block_session_position(s->block) : 0;
     return LV_OK;
 }
 
@@ -2369,6 +2479,8 @@ extern "C" int lv_trace_read_rows(lv_session *s, uint32_t layer, int which, uint
     if (!s->trace || !s->trace_buf) return fail(LV_ERR_STATE, "lv_trace_read_rows: record mode is off");
     const lv_hparams &hp = s->model->hp;
     if (layer >= hp.layers || which < 0 || which >= LV_TRACE_COUNT) return fail(LV_ERR_RANGE, "lv_trace_read_rows: layer %u / buffer %d", layer, which);
+    if (s->block && which != LV_TRACE_POST_ATTN && which != LV_TRACE_OUT)
+        return fail(LV_ERR_RANGE, "lv_trace_read_rows: this model records the residual stream only, not buffer %d", which);
     if (row0 > s->trace_n || n_rows > s->trace_n - row0)
         return fail(LV_ERR_RANGE, "lv_trace_read_rows: rows %u..%u of a step of %u", row0, row0 + n_rows, s->trace_n);
     if (n_rows == 0) return LV_OK;

@@ -1,0 +1,301 @@
+// lv_bf16_gemm.h — matrix products of models whose weights are bfloat16: out[token][row] = sum_k x[token][k] * W[row][k].
+//
+// Two kernels with one set of epilogues:
+//   gemm_bf16_kernel  bf16 activations, v_mfma_f32_16x16x32_bf16 (32-bit accumulation): the serving precision
+//   gemm_f32_kernel   fp32 activations, v_mfma_f32_16x16x4_f32 on weights widened to fp32: true 32-bit products
+// Both can be grouped (mixture of experts): a table of token tiles says which expert's rows a tile takes and which
+// positions of the expert-sorted token list it covers.
+//
+// Weights are row-major [rows][kp], kp a multiple of 64 (zero columns), rows padded with zero rows to a multiple of 128.
+// In the MFMA a weight tile is operand A (M = weight row) and the tokens are operand B (N = token): lane l of the result
+// holds token l % 16 and four consecutive weight rows 4 * (l / 16) .. + 3, i.e. one 16-byte store into the token's row.
+//
+// gemm_bf16_kernel: workgroup = 4 waves, tile 128 weight rows x 128 tokens, K step 64, each wave 64 x 64.  Both operand
+// tiles go to LDS by direct loads, two stages.  A row of a tile is 128 bytes; its eight 16-byte chunks are stored in the
+// order chunk ^ (row % 8), so that the 16 rows an MFMA operand reads at one k spread over all banks.
+#pragma once
+
+#include "lv_device.h"
+
+namespace lv {
+
+typedef __bf16 lv_bf8 __attribute__((ext_vector_type(8)));
+typedef float lv_f4 __attribute__((ext_vector_type(4)));
+typedef __attribute__((address_space(3))) void lv_lds_any;
+typedef const __attribute__((address_space(1))) void lv_glb_any;
+
+__device__ __forceinline__ float bf16_to_float(uint16_t h) { return __uint_as_float((uint32_t)h << 16); }
+__device__ __forceinline__ uint16_t float_to_bf16(float f) { return __builtin_bit_cast(uint16_t, (__bf16)f); }   // round to nearest even
+// activations and cache rows come in two element types: uint16_t (bf16 bits) and float
+__device__ __forceinline__ float elem_to_float(uint16_t v) { return bf16_to_float(v); }
+__device__ __forceinline__ float elem_to_float(float v) { return v; }
+template <class T> __device__ __forceinline__ T float_to_elem(float f)
+{
+    if constexpr (sizeof(T) == 2) return float_to_bf16(f);
+    else return f;
+}
+// eight consecutive elements (16-byte aligned) as floats
+__device__ __forceinline__ void load8(float (&f)[8], const uint16_t *p)
+{
+    const uint4 v = *reinterpret_cast<const uint4 *>(p);
+    const uint32_t w[4] = {v.x, v.y, v.z, v.w};
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+        f[2 * i] = __uint_as_float(w[i] << 16);
+        f[2 * i + 1] = __uint_as_float(w[i] & 0xffff0000u);
+    }
+}
+__device__ __forceinline__ void load8(float (&f)[8], const float *p)
+{
+    const float4 a = reinterpret_cast<const float4 *>(p)[0], b = reinterpret_cast<const float4 *>(p)[1];
+    f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w; f[4] = b.x; f[5] = b.y; f[6] = b.z; f[7] = b.w;
+}
+
+__device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + __expf(-z)); }
+__device__ __forceinline__ float silu_f(float z) { return z / (1.f + __expf(-z)); }
+__device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z : log1pf(expf(z)); }
+
+enum BfEpilogue {
+    kEpStore = 0,    // out[token][row]
+    kEpDecay = 1,    // out[token][head][lane-padded channel] = exp(-exp(A_log[head]) * softplus(v + bias[row]))
+    kEpSigmoid = 2,  // out[token][row] = sigmoid(v)
+    kEpGlu = 3,      // rows alternate 16 gate, 16 up: act[position][f] = silu(w g) * (w u), w = the expert's weight for the token
+    kEpScatter = 4,  // grouped: out[slots[position]][row]
+};
+
+struct BfGemmArgs {
+    const void *x;           // activations (bf16 or fp32), rows readable up to the next multiple of the token tile
+    const uint16_t *w;
+    uint32_t ldx, kp;        // row stride of x in elements; padded K
+    uint32_t rows;           // weight rows that exist
+    uint32_t n;              // tokens (ungrouped)
+    uint32_t row_tiles, token_tiles;
+    float *out;
+    uint32_t ldo;
+    // decay epilogue
+    const float *a_log, *bias;
+    uint32_t head_dim, head_stride;
+    // grouped
+    const uint32_t *tiles;   // [0] = number of tiles, then {expert, first position, positions} each
+    const uint32_t *slots;   // position in expert order -> token * top + choice
+    const float *weights;    // [token * top + choice]
+    uint32_t top, expert_rows;   // weight rows from one expert to the next
+    bool gather;             // x rows are tokens (slots[position] / top), otherwise positions
+    void *act;               // kEpGlu output [position][lda]
+    uint32_t lda;
+};
+
+// four results of one token: weight rows row .. row + 3
+template <int EP>
+__device__ __forceinline__ void bf_store4(const BfGemmArgs &a, uint32_t orow, uint32_t row, const lv_f4 v)
+{
+    if (row >= a.rows) return;
+    float r[4] = {v[0], v[1], v[2], v[3]};
+    if constexpr (EP == kEpDecay) {
+#pragma unroll
+        for (int i = 0; i < 4; i++)
+            if (row + i < a.rows) {
+                const uint32_t h = (row + i) / a.head_dim, d = (row + i) % a.head_dim;
+                a.out[(size_t)orow * a.ldo + h * a.head_stride + d] = expf(-expf(a.a_log[h]) * softplus_f(r[i] + a.bias[row + i]));
+            }
+        return;
+    }
+    if constexpr (EP == kEpSigmoid) {
+#pragma unroll
+        for (int i = 0; i < 4; i++) r[i] = sigmoid_f(r[i]);
+    }
+    float *o = a.out + (size_t)orow * a.ldo + row;
+    if (row + 3 < a.rows && (a.ldo & 3) == 0) {
+        *reinterpret_cast<float4 *>(o) = make_float4(r[0], r[1], r[2], r[3]);
+    } else {
+#pragma unroll
+        for (int i = 0; i < 4; i++)
+            if (row + i < a.rows) o[i] = r[i];
+    }
+}
+
+template <class T>
+__device__ __forceinline__ void bf_store_glu(const BfGemmArgs &a, uint32_t position, uint32_t f, float wt, const lv_f4 g, const lv_f4 u)
+{
+    T *o = static_cast<T *>(a.act) + (size_t)position * a.lda + f;
+#pragma unroll
+    for (int i = 0; i < 4; i++) o[i] = float_to_elem<T>(silu_f(wt * g[i]) * (wt * u[i]));
+}
+
+// Tile of this workgroup: workgroups are dealt to the 8 XCDs in turn; an XCD takes every eighth row tile and walks the token
+// tiles of one row tile before the next, so that the weight tile is read into its L2 once.
+template <bool GROUPED>
+__device__ __forceinline__ bool bf_tile(const BfGemmArgs &a, uint32_t tile_tokens, uint32_t &rt, uint32_t &expert, uint32_t &first, uint32_t &count)
+{
+    const uint32_t pid = blockIdx.x, q = pid >> 3;
+    rt = q / a.token_tiles * 8 + (pid & 7);
+    const uint32_t tt = q % a.token_tiles;
+    if (rt >= a.row_tiles) return false;
+    if constexpr (GROUPED) {
+        if (tt >= a.tiles[0]) return false;
+        expert = a.tiles[1 + 3 * tt];
+        first = a.tiles[2 + 3 * tt];
+        count = a.tiles[3 + 3 * tt];
+    } else {
+        expert = 0;
+        first = tt * tile_tokens;
+        count = min(tile_tokens, a.n - first);
+    }
+    return true;
+}
+inline uint32_t bf_grid(const BfGemmArgs &a) { return (a.row_tiles + 7) / 8 * 8 * a.token_tiles; }
+
+constexpr int kBfTile = 128;       // weight rows and tokens per workgroup, bf16
+constexpr int kBfStep = 64;
+constexpr int kBfStageBytes = 2 * kBfTile * kBfStep * 2;
+
+template <int EP, bool GROUPED>
+__global__ __launch_bounds__(256, 2) void gemm_bf16_kernel(BfGemmArgs a)
+{
+    __shared__ __attribute__((aligned(128))) uint8_t lds[2 * kBfStageBytes];
+    uint32_t rt, expert, first, count;
+    if (!bf_tile<GROUPED>(a, kBfTile, rt, expert, first, count)) return;
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int l16 = lane & 15, g4 = lane >> 4;
+    const uint32_t kp = a.kp;
+
+    // direct loads: a wave brings 32 rows of each tile, 8 rows (1 KB) per instruction
+    const uint16_t *gw[4], *gx[4];
+    {
+        const int r8 = lane >> 3, c = (lane & 7) ^ r8;
+        const uint16_t *wt = a.w + ((size_t)expert * a.expert_rows + (size_t)rt * kBfTile) * kp;
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            const int row = wave * 32 + i * 8 + r8;
+            gw[i] = wt + (size_t)row * kp + c * 8;
+            size_t xr = (size_t)first + row;
+            if constexpr (GROUPED) {
+                const uint32_t p = first + min((uint32_t)row, count - 1);
+                xr = a.gather ? a.slots[p] / a.top : p;
+            }
+            gx[i] = static_cast<const uint16_t *>(a.x) + xr * a.ldx + c * 8;
+        }
+    }
+    auto issue = [&](int s, uint32_t k0) {
+        uint8_t *buf = lds + s * kBfStageBytes + wave * 32 * 128;
+#pragma unroll
+        for (int i = 0; i < 4; i++) __builtin_amdgcn_global_load_lds((lv_glb_any *)(gw[i] + k0), (lv_lds_any *)(buf + i * 1024), 16, 0, 0);
+#pragma unroll
+        for (int i = 0; i < 4; i++) __builtin_amdgcn_global_load_lds((lv_glb_any *)(gx[i] + k0), (lv_lds_any *)(buf + kBfStageBytes / 2 + i * 1024), 16, 0, 0);
+    };
+
+    const int wm = wave & 1, wn = wave >> 1;
+    lv_f4 acc[4][4];
+#pragma unroll
+    for (int i = 0; i < 4; i++)
+#pragma unroll
+        for (int j = 0; j < 4; j++) acc[i][j] = lv_f4{0.f, 0.f, 0.f, 0.f};
+
+    const uint32_t steps = kp / kBfStep;
+    issue(0, 0);
+    for (uint32_t st = 0; st < steps; st++) {
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        __syncthreads();      // the stage is in LDS for everyone, and everyone is done with the other one
+        if (st + 1 < steps) issue((st + 1) & 1, (st + 1) * kBfStep);
+        const uint8_t *bw = lds + (st & 1) * kBfStageBytes, *bx = bw + kBfStageBytes / 2;
+#pragma unroll
+        for (int kk = 0; kk < 2; kk++) {
+            lv_bf8 fa[4], fb[4];
+            const int ch = ((kk * 4 + g4) ^ (l16 & 7)) * 16;
+#pragma unroll
+            for (int i = 0; i < 4; i++) fa[i] = *reinterpret_cast<const lv_bf8 *>(bw + (wm * 64 + i * 16 + l16) * 128 + ch);
+#pragma unroll
+            for (int i = 0; i < 4; i++) fb[i] = *reinterpret_cast<const lv_bf8 *>(bx + (wn * 64 + i * 16 + l16) * 128 + ch);
+#pragma unroll
+            for (int i = 0; i < 4; i++)
+#pragma unroll
+                for (int j = 0; j < 4; j++) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa[i], fb[j], acc[i][j], 0, 0, 0);
+        }
+    }
+#pragma unroll
+    for (int j = 0; j < 4; j++) {
+        const uint32_t t = wn * 64 + j * 16 + l16;
+        if (t >= count) continue;
+        const uint32_t p = first + t;
+        if constexpr (EP == kEpGlu) {
+            const float wt = a.weights[a.slots[p]];
+#pragma unroll
+            for (int i = 0; i < 4; i += 2) {
+                const uint32_t row = rt * kBfTile + wm * 64 + i * 16;        // the pair's gate block
+                bf_store_glu<uint16_t>(a, p, row / 2 + g4 * 4, wt, acc[i][j], acc[i + 1][j]);
+            }
+        } else {
+            const uint32_t orow = EP == kEpScatter ? a.slots[p] : p;
+#pragma unroll
+            for (int i = 0; i < 4; i++) bf_store4<EP>(a, orow, rt * kBfTile + wm * 64 + i * 16 + g4 * 4, acc[i][j]);
+        }
+    }
+}
+
+constexpr int kF32Tile = 64;
+constexpr int kF32Step = 32;
+constexpr int kF32Ld = kF32Step + 4;
+
+template <int EP, bool GROUPED>
+__global__ __launch_bounds__(256) void gemm_f32_kernel(BfGemmArgs a)
+{
+    __shared__ __attribute__((aligned(16))) float ws[kF32Tile * kF32Ld], xs[kF32Tile * kF32Ld];
+    uint32_t rt, expert, first, count;
+    if (!bf_tile<GROUPED>(a, kF32Tile, rt, expert, first, count)) return;
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, g4 = lane >> 4;
+    const int wm = wave & 1, wn = wave >> 1;
+    const uint32_t kp = a.kp;
+    const int lr = threadIdx.x >> 2, lc = (threadIdx.x & 3) * 8;     // this thread's row and 8 columns of the tiles it loads
+    const uint16_t *gw = a.w + ((size_t)expert * a.expert_rows + (size_t)rt * kF32Tile + lr) * kp + lc;
+    size_t xr = (size_t)first + lr;
+    if constexpr (GROUPED) {
+        const uint32_t p = first + min((uint32_t)lr, count - 1);
+        xr = a.gather ? a.slots[p] / a.top : p;
+    }
+    const float *gx = static_cast<const float *>(a.x) + xr * a.ldx + lc;
+    lv_f4 acc[2][2];
+#pragma unroll
+    for (int i = 0; i < 2; i++)
+#pragma unroll
+        for (int j = 0; j < 2; j++) acc[i][j] = lv_f4{0.f, 0.f, 0.f, 0.f};
+    for (uint32_t k0 = 0; k0 < kp; k0 += kF32Step) {
+        float fw[8], fx[8];
+        load8(fw, gw + k0);
+        load8(fx, gx + k0);
+        __syncthreads();
+#pragma unroll
+        for (int i = 0; i < 8; i += 4) {
+            *reinterpret_cast<float4 *>(ws + lr * kF32Ld + lc + i) = make_float4(fw[i], fw[i + 1], fw[i + 2], fw[i + 3]);
+            *reinterpret_cast<float4 *>(xs + lr * kF32Ld + lc + i) = make_float4(fx[i], fx[i + 1], fx[i + 2], fx[i + 3]);
+        }
+        __syncthreads();
+#pragma unroll
+        for (int kk = 0; kk < kF32Step / 4; kk++) {
+            float fa[2], fb[2];
+#pragma unroll
+            for (int i = 0; i < 2; i++) {
+                fa[i] = ws[(wm * 32 + i * 16 + l16) * kF32Ld + kk * 4 + g4];
+                fb[i] = xs[(wn * 32 + i * 16 + l16) * kF32Ld + kk * 4 + g4];
+            }
+#pragma unroll
+            for (int i = 0; i < 2; i++)
+#pragma unroll
+                for (int j = 0; j < 2; j++) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x4f32(fa[i], fb[j], acc[i][j], 0, 0, 0);
+        }
+    }
+#pragma unroll
+    for (int j = 0; j < 2; j++) {
+        const uint32_t t = wn * 32 + j * 16 + l16;
+        if (t >= count) continue;
+        const uint32_t p = first + t;
+        if constexpr (EP == kEpGlu) {
+            bf_store_glu<float>(a, p, (rt * kF32Tile + wm * 32) / 2 + g4 * 4, a.weights[a.slots[p]], acc[0][j], acc[1][j]);
+        } else {
+            const uint32_t orow = EP == kEpScatter ? a.slots[p] : p;
+#pragma unroll
+            for (int i = 0; i < 2; i++) bf_store4<EP>(a, orow, rt * kF32Tile + wm * 32 + i * 16 + g4 * 4, acc[i][j]);
+        }
+    }
+}
+
+}  // namespace lv

@@ -1,0 +1,1018 @@
+// lv_block.hip — block models: upload, per-sequence state, and the step as launches of the kernels in lv_bf16_gemm.h,
+// lv_bf16_gemv.h, lv_gqa.h, lv_delta.h and lv_block_kernels.h.
+//
+// Device layout.  Matrices bf16 row-major, columns padded with zeros to a multiple of 64, rows to a multiple of 128.  All
+// projections that read a layer's normed input are one matrix (sections padded to 16 rows), the two branches' output
+// projections are one matrix over the concatenated branch outputs, and an expert's gate and up rows alternate in blocks of
+// 16, so that both products and the SwiGLU between them are one launch.  Vectors are fp32.
+#include "lv_block.h"
+
+#include <algorithm>
+#include <cmath>
+#include <cstring>
+#include <functional>
+#include <new>
+#include <string>
+#include <unordered_map>
+#include <vector>
+
+#include "lv_block_kernels.h"
+#include "lv_gqa_tile.h"
+
+namespace lv {
+
+static uint32_t up(uint32_t v, uint32_t a) { return (v + a - 1) / a * a; }
+
+struct BfMatrix {
+    const uint16_t *w = nullptr;
+    uint32_t rows = 0, kp = 0;
+};
+
+struct BlockLayer {
+    lv_block_spec spec{};
+    bool attn = false, delta = false, moe = false;
+    BfMatrix in, out, a2, g2, router, gate_up, down;
+    uint32_t q_off = 0, k_off = 0, v_off = 0, dq_off = 0, dk_off = 0, dv_off = 0, b_off = 0, a_off = 0, g_off = 0;   // rows of `in`
+    uint32_t a_rank = 0, g_rank = 0;
+    uint32_t left_kp = 0;              // where the recurrent part starts in the joint output projection's input
+    uint32_t gu_rows = 0, down_rows = 0;   // rows from one expert to the next
+    uint32_t dp = 64, r = 1, groups = 1;   // attention: padded head size, heads per group, groups per kv head
+    const float *norm1 = nullptr, *norm1b = nullptr, *norm2 = nullptr, *norm2b = nullptr;
+    const float *q_norm = nullptr, *k_norm = nullptr, *sink = nullptr;
+    const double *freq = nullptr;
+    const float *conv = nullptr, *a_log = nullptr, *dt_bias = nullptr, *onorm = nullptr;
+    uint32_t dstride() const { return up(spec.delta.dim, 64); }
+    uint32_t channels() const { return 2 * spec.delta.kv_heads * spec.delta.dim + spec.delta.heads * spec.delta.vdim; }
+};
+
+struct BlockModel {
+    lv_block_hparams hp{};
+    bool f32 = false;                  // activations of batches and cache rows are fp32
+    uint32_t dp = 0;                   // hp.dim rounded up to 64
+    uint8_t *arena = nullptr;
+    uint64_t arena_bytes = 0;
+    const uint16_t *embed = nullptr;   // [vocab][dim], not padded
+    const float *final_norm = nullptr;
+    BfMatrix head;
+    std::vector<BlockLayer> layers;
+    uint32_t elem() const { return f32 ? 4 : 2; }
+};
+
+// per layer and sequence
+struct LayerState {
+    uint32_t ring = 0;                 // cache rows
+    uint8_t *kc = nullptr, *vc = nullptr;
+    float *state = nullptr, *conv = nullptr;
+};
+
+struct Workspace {                     // of batches; sized for `cap` tokens
+    uint32_t cap = 0;
+    float *x = nullptr, *y1 = nullptr, *y = nullptr, *dq = nullptr, *dk = nullptr, *dv = nullptr, *dg = nullptr, *beta = nullptr, *qk = nullptr, *o = nullptr,
+          *gate = nullptr, *z = nullptr, *scores = nullptr;
+    void *act = nullptr, *q = nullptr, *k = nullptr, *v = nullptr, *vt = nullptr, *a1 = nullptr, *g1 = nullptr, *cat = nullptr, *ff = nullptr;
+    uint32_t *ids = nullptr, *slots = nullptr, *tiles = nullptr;
+    uint32_t vt_keys = 0;
+};
+
+struct BlockSession {
+    const BlockModel *m = nullptr;
+    hipStream_t st = nullptr;
+    uint32_t positions = 0, position = 0;
+    bool valid = true;
+    std::vector<LayerState> layers;
+    // one token
+    float *xa = nullptr, *xb = nullptr, *y1 = nullptr, *left = nullptr, *o = nullptr, *gate = nullptr, *yo = nullptr, *h2 = nullptr, *z = nullptr, *act = nullptr,
+          *yd = nullptr, *scores = nullptr, *part = nullptr;
+    uint32_t *ids = nullptr, *counters = nullptr;
+    uint32_t part_splits = 0;
+    Workspace ws;
+};
+
+// ---------------------------------------------------------------------------------------------------------------------------
+// model
+// ---------------------------------------------------------------------------------------------------------------------------
+namespace {
+
+// one block of the arena: fill(dst) produces `bytes` bytes in host memory
+struct Fill {
+    uint64_t off, bytes;
+    std::function<void(uint8_t *)> fill;
+};
+
+class Loader {
+public:
+    Loader(const void *base, uint64_t size, const lv_tensor_desc *table, uint32_t n) : base_(static_cast<const uint8_t *>(base)), size_(size)
+    {
+        for (uint32_t i = 0; i < n; i++)
+            if (table[i].name) by_name_.emplace(table[i].name, &table[i]);
+    }
+    int error = LV_OK;
+    uint64_t bytes = 0;
+    std::vector<Fill> fills;
+
+    // tensor `name` of rows x cols; null and error set when it is absent or has another shape.  rows 0: any number of rows
+    const lv_tensor_desc *find(const std::string &name, uint32_t rows, uint32_t cols, bool vector)
+    {
+        if (error != LV_OK) return nullptr;
+        const auto it = by_name_.find(name);
+        if (it == by_name_.end()) {
+            error = fail(LV_ERR_MISSING, "lv_block_model_upload: tensor %s is not in the table", name.c_str());
+            return nullptr;
+        }
+        const lv_tensor_desc &d = *it->second;
+        if ((rows && d.rows != rows) || (cols && d.cols != cols) || !d.rows || !d.cols) {
+            error = fail(LV_ERR_ARG, "lv_block_model_upload: %s is %u x %u, expected %u x %u", d.name, d.rows, d.cols, rows, cols);
+            return nullptr;
+        }
+        const uint64_t e = d.ftype == LV_BF16 ? 2 : d.ftype == LV_F32 && vector ? 4 : 0, raw = e * d.rows * d.cols;
+        if (!e || d.size != raw || d.offset > size_ || raw > size_ - d.offset) {
+            error = fail(LV_ERR_ARG, "lv_block_model_upload: %s has type %u / %llu bytes at %llu (file holds %llu)", d.name, d.ftype, (unsigned long long)d.size,
+                         (unsigned long long)d.offset, (unsigned long long)size_);
+            return nullptr;
+        }
+        return &d;
+    }
+    const uint8_t *data(const lv_tensor_desc *d) const { return base_ + d->offset; }
+
+    uint64_t place(uint64_t n, std::function<void(uint8_t *)> fn)
+    {
+        const uint64_t off = bytes;
+        fills.push_back({off, n, std::move(fn)});
+        bytes += (n + 255) / 256 * 256;
+        return off;
+    }
+
+    // fp32 vector of `padded` floats from n tensor elements (rows x cols flattened), zeros behind
+    uint64_t vec(const std::string &name, uint32_t rows, uint32_t cols, uint32_t padded)
+    {
+        const lv_tensor_desc *d = find(name, rows, cols, true);
+        if (!d) return 0;
+        const uint8_t *src = data(d);
+        const uint32_t n = d->rows * d->cols, type = d->ftype;
+        return place((uint64_t)padded * 4, [=](uint8_t *dst) { widen(dst, src, n, type); });
+    }
+    static void widen(uint8_t *dst, const uint8_t *src, uint32_t n, uint32_t type)
+    {
+        if (type == LV_F32) {
+            std::memcpy(dst, src, (size_t)n * 4);
+            return;
+        }
+        for (uint32_t i = 0; i < n; i++) {
+            uint16_t h;
+            std::memcpy(&h, src + 2 * (size_t)i, 2);
+            const uint32_t w = (uint32_t)h << 16;
+            std::memcpy(dst + 4 * (size_t)i, &w, 4);
+        }
+    }
+
+    // sections of one matrix: tensor rows to matrix rows from `row`, tensor columns to matrix columns from `col`
+    struct Part {
+        const lv_tensor_desc *d;
+        uint32_t row, col;
+    };
+    uint64_t matrix(const std::vector<Part> &parts, uint32_t rows, uint32_t kp, BfMatrix *m)
+    {
+        if (error != LV_OK) return 0;
+        m->rows = rows;
+        m->kp = kp;
+        std::vector<std::pair<const uint8_t *, Part>> src;
+        for (const Part &p : parts) src.push_back({data(p.d), p});
+        return place((uint64_t)up(rows, 128) * kp * 2, [=](uint8_t *dst) {
+            for (const auto &s : src)
+                for (uint32_t r = 0; r < s.second.d->rows; r++)
+                    std::memcpy(dst + ((uint64_t)(s.second.row + r) * kp + s.second.col) * 2, s.first + (uint64_t)r * s.second.d->cols * 2, (size_t)s.second.d->cols * 2);
+        });
+    }
+
+private:
+    const uint8_t *base_;
+    uint64_t size_;
+    std::unordered_map<std::string, const lv_tensor_desc *> by_name_;
+};
+
+int check_spec(const lv_block_spec &b, uint32_t layer)
+{
+    const lv_attn_spec &a = b.attn;
+    if (a.heads) {
+        if (!a.kv_heads || a.heads % a.kv_heads || !a.dim || !a.vdim || std::max(a.dim, a.vdim) > 256)
+            return fail(LV_ERR_ARG, "lv_block_model_upload: layer %u: attention of %u / %u heads of %u and %u (head sizes to 256 are built)", layer, a.heads, a.kv_heads, a.dim, a.vdim);
+        if (a.rot_dims % 2 || a.rot_dims > a.dim || (a.rot_dims && !(a.rot_base > 0)))
+            return fail(LV_ERR_ARG, "lv_block_model_upload: layer %u: rotation of %u of %u dimensions, base %g", layer, a.rot_dims, a.dim, a.rot_base);
+        if ((a.flags & LV_ATTN_KEYS_AS_VALUES) && a.vdim != a.dim)
+            return fail(LV_ERR_ARG, "lv_block_model_upload: layer %u: values are keys but head sizes differ (%u, %u)", layer, a.dim, a.vdim);
+    }
+    const lv_delta_spec &d = b.delta;
+    if (d.heads && (!d.kv_heads || d.heads % d.kv_heads || !d.dim || d.dim > kDeltaMaxDim || !d.vdim || !d.conv))
+        return fail(LV_ERR_ARG, "lv_block_model_upload: layer %u: delta rule of %u / %u heads, %u x %u, %u taps (key sizes to %u are built)", layer, d.heads, d.kv_heads, d.dim, d.vdim, d.conv,
+                    kDeltaMaxDim);
+    if (!a.heads && !d.heads) return fail(LV_ERR_ARG, "lv_block_model_upload: layer %u has no mixer", layer);
+    const lv_moe_spec &e = b.moe;
+    if (e.experts && (!e.top || e.top > e.experts || e.top > kMaxTop || e.experts > kMaxExperts || !e.ff))
+        return fail(LV_ERR_ARG, "lv_block_model_upload: layer %u: %u of %u experts of %u", layer, e.top, e.experts, e.ff);
+    return LV_OK;
+}
+
+}  // namespace
+
+int block_model_create(hipStream_t st, const void *base, uint64_t base_size, const lv_block_hparams *hp, const lv_block_spec *blocks, const lv_tensor_desc *table,
+                       uint32_t n_tensors, int compute, BlockModel **out)
+{
+    *out = nullptr;
+    if (!hp->vocab || !hp->dim || !hp->layers || hp->dim > 32768) return fail(LV_ERR_ARG, "lv_block_model_upload: vocabulary %u, width %u, %u layers", hp->vocab, hp->dim, hp->layers);
+    if (compute != LV_BF16 && compute != LV_F32) return fail(LV_ERR_ARG, "lv_block_model_upload: compute type %d", compute);
+    for (uint32_t i = 0; i < hp->layers; i++) LV_TRY(check_spec(blocks[i], i));
+    BlockModel *m = new (std::nothrow) BlockModel;
+    if (!m) return fail(LV_ERR_OOM, "lv_block_model_upload: host allocation");
+    m->hp = *hp;
+    m->f32 = compute == LV_F32;
+    const uint32_t D = hp->dim, V = hp->vocab, Dp = m->dp = up(D, 64);
+    m->layers.resize(hp->layers);
+
+    // where everything goes; pointers are set once the arena exists
+    Loader ld(base, base_size, table, n_tensors);
+    struct Fix { void *at; uint64_t off; };       // a pointer member of the model and its place in the arena
+    std::vector<Fix> fixes;
+    auto at = [&](auto **p, uint64_t off) { fixes.push_back({static_cast<void *>(p), off}); };
+    using Part = Loader::Part;
+    auto matrix = [&](BfMatrix *dst, const std::vector<Part> &parts, uint32_t rows, uint32_t kp) {
+        const uint64_t off = ld.matrix(parts, rows, kp, dst);
+        at(&dst->w, off);
+    };
+    auto vec = [&](const float **dst, const std::string &name, uint32_t rows, uint32_t cols, uint32_t padded) { at(dst, ld.vec(name, rows, cols, padded)); };
+    auto tensor = [&](const std::string &name, uint32_t rows, uint32_t cols) { return ld.find(name, rows, cols, false); };
+
+    if (const lv_tensor_desc *d = tensor("embed", V, D)) {
+        const uint8_t *src = ld.data(d);
+        const uint64_t n = d->size;
+        at(&m->embed, ld.place(n, [=](uint8_t *dst) { std::memcpy(dst, src, n); }));
+    }
+    vec(&m->final_norm, "final.norm", D, 1, Dp);
+    if (const lv_tensor_desc *d = tensor("head", V, D)) matrix(&m->head, {{d, 0, 0}}, V, Dp);
+    for (uint32_t i = 0; i < hp->layers && ld.error == LV_OK; i++) {
+        BlockLayer &l = m->layers[i];
+        l.spec = blocks[i];
+        const lv_attn_spec &a = l.spec.attn;
+        const lv_delta_spec &dl = l.spec.delta;
+        const lv_moe_spec &e = l.spec.moe;
+        l.attn = a.heads != 0;
+        l.delta = dl.heads != 0;
+        l.moe = e.experts != 0;
+        const std::string p = "l" + std::to_string(i) + ".", pa = p + "mix.left.", pd = p + "mix.right.", pm = p + "mlp.";
+        vec(&l.norm1, p + "norm1", D, 1, Dp);
+        vec(&l.norm1b, p + "norm1b", D, 1, Dp);
+        std::vector<Part> in, outp;
+        uint32_t row = 0;
+        auto section = [&](const std::string &name, uint32_t rows, uint32_t *off) -> uint32_t {   // rows 0: the tensor's own
+            const lv_tensor_desc *d = tensor(name, rows, D);
+            if (!d) return 0;
+            *off = row;
+            in.push_back({d, row, 0});
+            row += up(d->rows, 16);
+            return d->rows;
+        };
+        if (l.attn) {
+            section(pa + "q", a.heads * a.dim, &l.q_off);
+            section(pa + "k", a.kv_heads * a.dim, &l.k_off);
+            if (a.flags & LV_ATTN_KEYS_AS_VALUES) l.v_off = l.k_off;
+            else section(pa + "v", a.kv_heads * a.vdim, &l.v_off);
+            if (a.flags & LV_ATTN_NORM_FULL) {
+                vec(&l.q_norm, pa + "q.norm", a.heads * a.dim, 1, a.heads * a.dim);
+                vec(&l.k_norm, pa + "k.norm", a.kv_heads * a.dim, 1, a.kv_heads * a.dim);
+            }
+            if (a.flags & LV_ATTN_SINK) vec(&l.sink, pa + "sink", a.heads, 1, a.heads);
+            if (a.rot_dims) {
+                const uint32_t half = a.rot_dims / 2, dims = a.rot_dims;
+                const double rb = a.rot_base;
+                at(&l.freq, ld.place((uint64_t)half * 8, [=](uint8_t *dst) {
+                    for (uint32_t k = 0; k < half; k++) {
+                        const double f = std::pow(rb, -2.0 * k / dims);
+                        std::memcpy(dst + 8 * (size_t)k, &f, 8);
+                    }
+                }));
+            }
+            l.left_kp = up(a.heads * a.vdim, 64);
+            if (const lv_tensor_desc *d = tensor(pa + "o", D, a.heads * a.vdim)) outp.push_back({d, 0, 0});
+            l.dp = 64;
+            while (l.dp < std::max(a.dim, a.vdim)) l.dp *= 2;
+            const uint32_t per = a.heads / a.kv_heads;
+            l.groups = (per + 7) / 8;
+            const uint32_t rr = (per + l.groups - 1) / l.groups;
+            l.r = rr == 1 ? 1 : rr <= 4 ? 4 : 8;
+            l.groups = (per + l.r - 1) / l.r;
+        }
+        if (l.delta) {
+            section(pd + "q", dl.kv_heads * dl.dim, &l.dq_off);
+            section(pd + "k", dl.kv_heads * dl.dim, &l.dk_off);
+            section(pd + "v", dl.heads * dl.vdim, &l.dv_off);
+            section(pd + "b", dl.heads, &l.b_off);
+            l.a_rank = section(pd + "a1", 0, &l.a_off);
+            l.g_rank = section(pd + "g1", 0, &l.g_off);
+            if (l.a_rank > kDeltaMaxRank || l.g_rank > kDeltaMaxRank) ld.error = fail(LV_ERR_ARG, "lv_block_model_upload: layer %u: ranks %u and %u", i, l.a_rank, l.g_rank);
+            if (const lv_tensor_desc *d = tensor(pd + "a2", dl.heads * dl.dim, l.a_rank)) matrix(&l.a2, {{d, 0, 0}}, d->rows, up(l.a_rank, 64));
+            if (const lv_tensor_desc *d = tensor(pd + "g2", dl.heads * dl.vdim, l.g_rank)) matrix(&l.g2, {{d, 0, 0}}, d->rows, up(l.g_rank, 64));
+            if (const lv_tensor_desc *d = tensor(pd + "o", D, dl.heads * dl.vdim)) outp.push_back({d, 0, l.left_kp});
+            const uint32_t nq = dl.kv_heads * dl.dim, nv = dl.heads * dl.vdim, taps = dl.conv;
+            const lv_tensor_desc *cq = ld.find(pd + "q.conv", nq, taps, true), *ck = ld.find(pd + "k.conv", nq, taps, true), *cv = ld.find(pd + "v.conv", nv, taps, true);
+            if (cq && ck && cv) {
+                const uint8_t *s0 = ld.data(cq), *s1 = ld.data(ck), *s2 = ld.data(cv);
+                const uint32_t t0 = cq->ftype, t1 = ck->ftype, t2 = cv->ftype;
+                at(&l.conv, ld.place((uint64_t)l.channels() * taps * 4, [=](uint8_t *dst) {
+                    Loader::widen(dst, s0, nq * taps, t0);
+                    Loader::widen(dst + (uint64_t)nq * taps * 4, s1, nq * taps, t1);
+                    Loader::widen(dst + (uint64_t)2 * nq * taps * 4, s2, nv * taps, t2);
+                }));
+            }
+            vec(&l.a_log, pd + "A_log", dl.heads, 1, dl.heads);
+            vec(&l.dt_bias, pd + "dt_bias", dl.heads * dl.dim, 1, dl.heads * dl.dim);
+            vec(&l.onorm, pd + "norm", dl.vdim, 1, dl.vdim);
+        }
+        matrix(&l.in, in, row, Dp);
+        matrix(&l.out, outp, D, up(l.left_kp + dl.heads * dl.vdim, 64));
+        if (l.moe) {
+            vec(&l.norm2, p + "norm2", D, 1, Dp);
+            vec(&l.norm2b, p + "norm2b", D, 1, Dp);
+            if (const lv_tensor_desc *d = tensor(pm + "router", e.experts, D)) matrix(&l.router, {{d, 0, 0}}, e.experts, Dp);
+            l.gu_rows = up(up(e.ff, 16) * 2, 128);
+            l.down_rows = up(D, 128);
+            const uint32_t ffp = l.gu_rows / 2;
+            l.gate_up.rows = l.gu_rows;
+            l.gate_up.kp = Dp;
+            l.down.rows = D;
+            l.down.kp = ffp;
+            for (uint32_t x = 0; x < e.experts && ld.error == LV_OK; x++) {
+                const std::string px = pm + "e" + std::to_string(x) + ".";
+                const lv_tensor_desc *g = tensor(px + "gate", e.ff, D), *u = tensor(px + "up", e.ff, D);
+                if (!g || !u) break;
+                const uint8_t *sg = ld.data(g), *su = ld.data(u);
+                const uint32_t ff = e.ff;
+                const uint64_t off = ld.place((uint64_t)l.gu_rows * Dp * 2, [=](uint8_t *dst) {
+                    for (uint32_t f = 0; f < ff; f++) {
+                        const uint64_t r = (uint64_t)(f / 16) * 32 + f % 16;
+                        std::memcpy(dst + r * Dp * 2, sg + (uint64_t)f * D * 2, (size_t)D * 2);
+                        std::memcpy(dst + (r + 16) * Dp * 2, su + (uint64_t)f * D * 2, (size_t)D * 2);
+                    }
+                });
+                if (x == 0) at(&l.gate_up.w, off);      // expert after expert: every block is a multiple of 256 bytes
+            }
+            for (uint32_t x = 0; x < e.experts && ld.error == LV_OK; x++) {
+                const lv_tensor_desc *d = tensor(pm + "e" + std::to_string(x) + ".down", D, e.ff);
+                if (!d) break;
+                BfMatrix tmp;
+                const uint64_t off = ld.matrix({{d, 0, 0}}, D, ffp, &tmp);
+                if (x == 0) at(&l.down.w, off);
+            }
+        }
+        const uint32_t widest = std::max(std::max(l.out.kp, Dp + (l.moe ? e.experts : 0)), l.moe ? e.top * l.down.kp : 0);
+        if (widest > 36864) ld.error = fail(LV_ERR_ARG, "lv_block_model_upload: layer %u: a product over %u columns (36864 are built)", i, widest);
+    }
+    if (ld.error != LV_OK) {
+        delete m;
+        return ld.error;
+    }
+    hipError_t er = hipMalloc(reinterpret_cast<void **>(&m->arena), ld.bytes);
+    if (er != hipSuccess) {
+        (void)hipGetLastError();
+        delete m;
+        return fail(er == hipErrorOutOfMemory ? LV_ERR_OOM : LV_ERR_HIP, "lv_block_model_upload: arena of %llu bytes: %s", (unsigned long long)ld.bytes, hipGetErrorString(er));
+    }
+    m->arena_bytes = ld.bytes;
+    std::vector<uint8_t> staging;
+    for (const Fill &f : ld.fills) {
+        staging.assign(f.bytes, 0);
+        f.fill(staging.data());
+        er = hipMemcpyAsync(m->arena + f.off, staging.data(), f.bytes, hipMemcpyHostToDevice, st);
+        if (er == hipSuccess) er = hipStreamSynchronize(st);
+        if (er != hipSuccess) {
+            (void)hipFree(m->arena);
+            delete m;
+            return fail(LV_ERR_HIP, "lv_block_model_upload: %s", hipGetErrorString(er));
+        }
+    }
+    for (const Fix &f : fixes) {
+        const uint8_t *p = m->arena + f.off;
+        std::memcpy(f.at, &p, sizeof p);
+    }
+    *out = m;
+    return LV_OK;
+}
+
+void block_model_destroy(BlockModel *m)
+{
+    if (!m) return;
+    (void)hipFree(m->arena);
+    delete m;
+}
+
+uint64_t block_model_bytes(const BlockModel *m) { return m->arena_bytes; }
+
+// ---------------------------------------------------------------------------------------------------------------------------
+// session
+// ---------------------------------------------------------------------------------------------------------------------------
+template <class T> static int dev_alloc(T **p, uint64_t bytes)
+{
+    const hipError_t e = hipMalloc(reinterpret_cast<void **>(p), std::max<uint64_t>(bytes, 256));
+    if (e == hipSuccess) return LV_OK;
+    (void)hipGetLastError();
+    *p = nullptr;
+    return fail(e == hipErrorOutOfMemory ? LV_ERR_OOM : LV_ERR_HIP, "session: %llu bytes: %s", (unsigned long long)bytes, hipGetErrorString(e));
+}
+// zeroed, so that padding columns that no kernel writes are finite
+template <class T> static int dev_zeroed(hipStream_t st, T **p, uint64_t bytes)
+{
+    bytes = (bytes + 255) / 256 * 256;
+    LV_TRY(dev_alloc(p, bytes));
+    return zero_async(*p, bytes, st);
+}
+template <class T> static void drop(T *&p)
+{
+    (void)hipFree((void *)p);
+    p = nullptr;
+}
+
+template <class F> static uint32_t layer_max(const BlockModel *m, F f)
+{
+    uint32_t v = 0;
+    for (const BlockLayer &l : m->layers) v = std::max<uint32_t>(v, f(l));
+    return v;
+}
+
+int block_session_create(const BlockModel *m, hipStream_t st, BlockSession **out)
+{
+    *out = nullptr;
+    BlockSession *s = new (std::nothrow) BlockSession;
+    if (!s) return fail(LV_ERR_OOM, "session: host allocation");
+    s->m = m;
+    s->st = st;
+    s->layers.resize(m->layers.size());
+    auto make = [&]() -> int {
+        const uint32_t Dp = m->dp;
+        LV_TRY(dev_zeroed(st, &s->xa, Dp * 4ull));
+        LV_TRY(dev_zeroed(st, &s->xb, Dp * 4ull));
+        LV_TRY(dev_zeroed(st, &s->yo, Dp * 4ull));
+        LV_TRY(dev_zeroed(st, &s->yd, Dp * 4ull));
+        LV_TRY(dev_zeroed(st, &s->h2, Dp * 4ull));
+        LV_TRY(dev_zeroed(st, &s->y1, 4ull * layer_max(m, [](const BlockLayer &l) { return l.in.rows; })));
+        LV_TRY(dev_zeroed(st, &s->left, 4ull * layer_max(m, [](const BlockLayer &l) { return l.spec.attn.heads * l.spec.attn.vdim; })));
+        const uint64_t hv = 4ull * layer_max(m, [](const BlockLayer &l) { return l.spec.delta.heads * l.spec.delta.vdim; });
+        LV_TRY(dev_zeroed(st, &s->o, hv));
+        LV_TRY(dev_zeroed(st, &s->gate, hv));
+        LV_TRY(dev_zeroed(st, &s->z, 4ull * layer_max(m, [](const BlockLayer &l) { return l.spec.moe.experts; })));
+        LV_TRY(dev_zeroed(st, &s->act, 4ull * layer_max(m, [](const BlockLayer &l) { return l.spec.moe.top * l.down.kp; })));
+        LV_TRY(dev_zeroed(st, &s->scores, 4ull * kMaxTop));
+        LV_TRY(dev_zeroed(st, &s->ids, 4ull * kMaxTop));
+        LV_TRY(dev_zeroed(st, &s->counters, 4ull * layer_max(m, [](const BlockLayer &l) { return l.spec.attn.kv_heads * l.groups; })));
+        for (size_t i = 0; i < m->layers.size(); i++) {
+            const BlockLayer &l = m->layers[i];
+            if (!l.delta) continue;
+            LV_TRY(dev_zeroed(st, &s->layers[i].state, 4ull * l.spec.delta.heads * l.spec.delta.vdim * l.dstride()));
+            LV_TRY(dev_zeroed(st, &s->layers[i].conv, 4ull * l.spec.delta.conv * l.channels()));
+        }
+        HIP_TRY(hipStreamSynchronize(st));
+        return LV_OK;
+    };
+    const int rc = make();
+    if (rc != LV_OK) {
+        block_session_destroy(s);
+        return rc;
+    }
+    *out = s;
+    return LV_OK;
+}
+
+static void workspace_free(Workspace &w)
+{
+    for (float **p : {&w.x, &w.y1, &w.y, &w.dq, &w.dk, &w.dv, &w.dg, &w.beta, &w.qk, &w.o, &w.gate, &w.z, &w.scores}) drop(*p);
+    for (void **p : {&w.act, &w.q, &w.k, &w.v, &w.vt, &w.a1, &w.g1, &w.cat, &w.ff}) drop(*p);
+    for (uint32_t **p : {&w.ids, &w.slots, &w.tiles}) drop(*p);
+    w.cap = 0;
+    w.vt_keys = 0;
+}
+
+void block_session_destroy(BlockSession *s)
+{
+    if (!s) return;
+    for (LayerState &l : s->layers) {
+        drop(l.kc);
+        drop(l.vc);
+        drop(l.state);
+        drop(l.conv);
+    }
+    for (float **p : {&s->xa, &s->xb, &s->y1, &s->left, &s->o, &s->gate, &s->yo, &s->h2, &s->z, &s->act, &s->yd, &s->scores, &s->part}) drop(*p);
+    drop(s->ids);
+    drop(s->counters);
+    workspace_free(s->ws);
+    delete s;
+}
+
+uint32_t block_session_position(const BlockSession *s) { return s->valid ? s->position : 0; }
+void block_session_invalidate(BlockSession *s)
+{
+    s->valid = false;
+    s->position = 0;
+}
+void block_session_advance(BlockSession *s, uint32_t pos)
+{
+    s->valid = true;
+    s->position = pos;
+}
+
+int block_session_reserve(BlockSession *s, uint32_t positions)
+{
+    const BlockModel *m = s->m;
+    uint64_t part = 0;
+    for (size_t i = 0; i < m->layers.size(); i++) {
+        const BlockLayer &l = m->layers[i];
+        if (!l.attn) continue;
+        LayerState &ls = s->layers[i];
+        const uint32_t ring = l.spec.attn.chunk ? std::min(l.spec.attn.chunk, positions) : positions;
+        const uint64_t splits = (ring + kGqaSplit - 1) / kGqaSplit;
+        part = std::max<uint64_t>(part, l.spec.attn.kv_heads * l.groups * splits * l.r * (l.dp + 2));
+        if (ring == ls.ring) continue;
+        // A ring that grows has not wrapped yet (it held every position so far), and one that shrinks keeps the rows that
+        // the smaller number of positions can have: row = position in both.
+        const uint64_t row = (uint64_t)l.spec.attn.kv_heads * l.dp * m->elem(), keep = std::min(ring, ls.ring);
+        uint8_t *fresh[2] = {nullptr, nullptr};
+        for (int w = 0; w < 2; w++) {
+            int rc = dev_zeroed(s->st, &fresh[w], ring * row);
+            if (rc == LV_OK && keep && hipMemcpyAsync(fresh[w], w ? ls.vc : ls.kc, keep * row, hipMemcpyDeviceToDevice, s->st) != hipSuccess)
+                rc = fail(LV_ERR_HIP, "session: cache copy");
+            if (rc != LV_OK) {
+                (void)hipStreamSynchronize(s->st);
+                drop(fresh[0]);
+                drop(fresh[1]);
+                return rc;
+            }
+        }
+        HIP_TRY(hipStreamSynchronize(s->st));
+        drop(ls.kc);
+        drop(ls.vc);
+        ls.kc = fresh[0];
+        ls.vc = fresh[1];
+        ls.ring = ring;
+    }
+    HIP_TRY(hipStreamSynchronize(s->st));
+    drop(s->part);
+    LV_TRY(dev_alloc(&s->part, part * 4));
+    s->positions = positions;
+    return LV_OK;
+}
+
+// ---------------------------------------------------------------------------------------------------------------------------
+// launches
+// ---------------------------------------------------------------------------------------------------------------------------
+template <class K> static int allow_lds(K kernel, size_t bytes)
+{
+    if (bytes > 65536) HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void *>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)bytes));
+    return LV_OK;
+}
+
+template <int MODE, int INPUT, int R, int DEPTH> static int launch_gemv(hipStream_t st, const BfGemvArgs &a, uint32_t units, size_t lds)
+{
+    const uint32_t per_wg = kBfGemvWaves * R, wgs = std::min((units + per_wg - 1) / per_wg, 512u);
+    auto *k = &bf16_gemv_kernel<MODE, INPUT, R, DEPTH>;
+    LV_TRY(allow_lds(k, lds));
+    k<<<dim3(wgs), dim3(kBfGemvThreads), lds, st>>>(a);
+    HIP_TRY(hipGetLastError());
+    return LV_OK;
+}
+
+// rows a wave walks together: as many as still give every wave of the chip work
+template <int MODE, int INPUT> static int gemv(hipStream_t st, const BfGemvArgs &a)
+{
+    const size_t lds = (size_t)a.kp * (MODE == kGemvDown ? a.top : 1) * 4 + (MODE == kGemvExperts ? a.experts * 4ull : 0);
+    if constexpr (MODE == kGemvExperts) {
+        const uint32_t units = a.top * (a.expert_rows / 2);
+        return units >= 8192 ? launch_gemv<MODE, INPUT, 2, 2>(st, a, units, lds) : launch_gemv<MODE, INPUT, 1, 4>(st, a, units, lds);
+    } else {
+        if (a.rows >= 16384) return launch_gemv<MODE, INPUT, 4, 2>(st, a, a.rows, lds);
+        if (a.rows >= 8192) return launch_gemv<MODE, INPUT, 2, 4>(st, a, a.rows, lds);
+        return launch_gemv<MODE, INPUT, 1, 8>(st, a, a.rows, lds);
+    }
+}
+
+template <int EP, bool GROUPED> static int gemm(hipStream_t st, bool f32, BfGemmArgs a, const BfMatrix &w, uint32_t n, uint32_t experts = 1)
+{
+    const uint32_t tile = f32 ? kF32Tile : kBfTile;
+    a.w = w.w;
+    a.kp = w.kp;
+    a.rows = w.rows;
+    a.n = n;
+    a.row_tiles = (w.rows + tile - 1) / tile;
+    a.token_tiles = (n + tile - 1) / tile;
+    if (GROUPED) a.token_tiles = std::min(a.token_tiles + experts, n);
+    if (f32) gemm_f32_kernel<EP, GROUPED><<<dim3(bf_grid(a)), dim3(256), 0, st>>>(a);
+    else gemm_bf16_kernel<EP, GROUPED><<<dim3(bf_grid(a)), dim3(256), 0, st>>>(a);
+    HIP_TRY(hipGetLastError());
+    return LV_OK;
+}
+
+// calls fn(element, integral constant DP, integral constant R) for a layer's attention
+template <class Fn> static int gqa_dispatch(bool f32, const BlockLayer &l, Fn &&fn)
+{
+    auto with_r = [&](auto elem, auto dp) -> int {
+        switch (l.r) {
+        case 1: return fn(elem, dp, std::integral_constant<int, 1>{});
+        case 4: return fn(elem, dp, std::integral_constant<int, 4>{});
+        default: return fn(elem, dp, std::integral_constant<int, 8>{});
+        }
+    };
+    auto with_dp = [&](auto elem) -> int {
+        switch (l.dp) {
+        case 64: return with_r(elem, std::integral_constant<int, 64>{});
+        case 128: return with_r(elem, std::integral_constant<int, 128>{});
+        default: return with_r(elem, std::integral_constant<int, 256>{});
+        }
+    };
+    return f32 ? with_dp(float{}) : with_dp(uint16_t{});
+}
+
+static GqaSpec gqa_spec(const BlockSession *s, size_t i)
+{
+    const BlockLayer &l = s->m->layers[i];
+    const lv_attn_spec &a = l.spec.attn;
+    GqaSpec g{};
+    if (!l.attn) return g;
+    g.heads = a.heads; g.kv_heads = a.kv_heads; g.dim = a.dim; g.vdim = a.vdim;
+    g.q_off = l.q_off; g.k_off = l.k_off; g.v_off = l.v_off;
+    g.q_norm = l.q_norm; g.k_norm = l.k_norm; g.sink = l.sink; g.freq = l.freq;
+    g.rot_dims = a.rot_dims; g.chunk = a.chunk; g.scale = a.scale; g.eps = s->m->hp.eps;
+    g.ring = s->layers[i].ring; g.kc = s->layers[i].kc; g.vc = s->layers[i].vc;
+    return g;
+}
+
+static DeltaSpec delta_spec(const BlockSession *s, size_t i)
+{
+    const BlockLayer &l = s->m->layers[i];
+    const lv_delta_spec &d = l.spec.delta;
+    DeltaSpec g{};
+    if (!l.delta) return g;
+    g.heads = d.heads; g.kv_heads = d.kv_heads; g.dim = d.dim; g.vdim = d.vdim; g.taps = d.conv;
+    g.q_off = l.dq_off; g.k_off = l.dk_off; g.v_off = l.dv_off; g.b_off = l.b_off; g.a_off = l.a_off; g.g_off = l.g_off;
+    g.a_rank = l.a_rank; g.g_rank = l.g_rank; g.a_kp = l.a2.kp; g.g_kp = l.g2.kp;
+    g.conv = l.conv; g.a_log = l.a_log; g.dt_bias = l.dt_bias; g.norm = l.onorm;
+    g.a2 = l.a2.w; g.g2 = l.g2.w; g.eps = s->m->hp.eps;
+    g.state = s->layers[i].state; g.ring = s->layers[i].conv; g.dstride = l.dstride();
+    return g;
+}
+
+static NormInput norm_in(const BlockModel *m, const float *x, const float *wpre)
+{
+    NormInput n{};
+    n.x = x; n.wpre = wpre; n.dim = m->hp.dim; n.dp = m->dp; n.parts = 1; n.part_stride = m->dp; n.eps = m->hp.eps;
+    return n;
+}
+
+int block_step_token(BlockSession *s, const uint32_t *cfg, uint32_t idx, float *logits, const BlockTrace *trace)
+{
+    const BlockModel *m = s->m;
+    hipStream_t st = s->st;
+    const uint32_t D = m->hp.dim, Dp = m->dp;
+    embed_bf16_kernel<<<dim3((Dp + 255) / 256, 1), dim3(256), 0, st>>>(s->xa, m->embed, cfg + 1 + idx, D, Dp);
+    HIP_TRY(hipGetLastError());
+    float *cur = s->xa, *other = s->xb;
+    const float *pend = nullptr, *wpost = nullptr;      // sublayer output not yet in the residual stream, and its norm
+    auto take = [&](NormInput &n) {                     // the launch that gets n leaves the new residual in `other`
+        if (!pend) return;
+        n.y = pend;
+        n.wpost = wpost;
+        n.x_out = other;
+        std::swap(cur, other);
+        pend = nullptr;
+    };
+    auto keep = [&](uint32_t layer, int which) -> int {
+        if (trace) HIP_TRY(hipMemcpyAsync(trace->slot(layer, which, idx), cur, D * 4ull, hipMemcpyDeviceToDevice, st));
+        return LV_OK;
+    };
+    for (size_t i = 0; i < m->layers.size(); i++) {
+        const BlockLayer &l = m->layers[i];
+        BfGemvArgs g{};
+        g.w = l.in.w; g.rows = l.in.rows; g.kp = Dp; g.out = s->y1;
+        g.norm = norm_in(m, cur, l.norm1);
+        take(g.norm);
+        LV_TRY((gemv<kGemvRows, kInNorm>(st, g)));
+        if (i) {
+            if (!m->layers[i - 1].moe) LV_TRY(keep(i - 1, LV_TRACE_POST_ATTN));
+            LV_TRY(keep(i - 1, LV_TRACE_OUT));
+        }
+
+        MixStepArgs mx{};
+        mx.delta.s = delta_spec(s, i);
+        mx.delta.y = s->y1; mx.delta.pos_ptr = cfg; mx.delta.pos_add = idx;
+        mx.delta.blocks = l.delta ? (l.spec.delta.vdim + kDeltaCols - 1) / kDeltaCols : 1;
+        mx.delta.o = s->o; mx.delta.gate = s->gate;
+        mx.delta_wgs = l.spec.delta.heads * mx.delta.blocks;
+        mx.attn.s = gqa_spec(s, i);
+        mx.attn.y = s->y1; mx.attn.pos_ptr = cfg; mx.attn.pos_add = idx;
+        mx.attn.groups = l.groups;
+        mx.attn.splits = l.attn ? (s->layers[i].ring + kGqaSplit - 1) / kGqaSplit : 1;
+        mx.attn.part = s->part; mx.attn.counters = s->counters; mx.attn.out = s->left;
+        const uint32_t wgs = mx.delta_wgs + (l.attn ? l.spec.attn.kv_heads * l.groups * mx.attn.splits : 0);
+        LV_TRY(gqa_dispatch(m->f32, l, [&](auto elem, auto dp, auto r) -> int {
+            constexpr int DP = decltype(dp)::value, R = decltype(r)::value;
+            const size_t lds = 4ull * std::max<uint32_t>(l.attn ? gqa_lds_floats<DP, R>() : 0, l.delta ? delta_step_lds_floats(l.a2.kp, l.g2.kp) : 0);
+            auto *k = &mix_step_kernel<decltype(elem), DP, R>;
+            LV_TRY(allow_lds(k, lds));
+            k<<<dim3(wgs), dim3(256), lds, st>>>(mx);
+            HIP_TRY(hipGetLastError());
+            return LV_OK;
+        }));
+
+        BfGemvArgs o{};
+        o.w = l.out.w; o.rows = D; o.kp = l.out.kp; o.out = s->yo;
+        o.branch = {s->left, s->o, s->gate, l.onorm, l.spec.attn.heads * l.spec.attn.vdim, l.left_kp, l.spec.delta.heads, l.spec.delta.vdim,
+                    l.spec.attn_scale, l.spec.delta_scale, m->hp.eps};
+        LV_TRY((gemv<kGemvRows, kInBranch>(st, o)));
+        pend = s->yo;
+        wpost = l.norm1b;
+        if (!l.moe) continue;
+
+        BfGemvArgs rt{};
+        rt.w = l.router.w; rt.rows = l.spec.moe.experts; rt.kp = Dp; rt.out = s->z;
+        rt.norm = norm_in(m, cur, l.norm2);
+        rt.norm.h_out = s->h2;
+        take(rt.norm);
+        LV_TRY((gemv<kGemvRows, kInNorm>(st, rt)));
+        LV_TRY(keep(i, LV_TRACE_POST_ATTN));
+        BfGemvArgs gu{};
+        gu.w = l.gate_up.w; gu.rows = l.gu_rows; gu.kp = Dp; gu.out = s->act; gu.x = s->h2;
+        gu.z = s->z; gu.experts = l.spec.moe.experts; gu.top = l.spec.moe.top; gu.expert_rows = l.gu_rows; gu.ids = s->ids; gu.scores = s->scores;
+        LV_TRY((gemv<kGemvExperts, kInPlain>(st, gu)));
+        BfGemvArgs dn{};
+        dn.w = l.down.w; dn.rows = D; dn.kp = l.down.kp; dn.out = s->yd; dn.x = s->act;
+        dn.top = l.spec.moe.top; dn.expert_rows = l.down_rows; dn.ids = s->ids;
+        LV_TRY((gemv<kGemvDown, kInPlain>(st, dn)));
+        pend = s->yd;
+        wpost = l.norm2b;
+    }
+    if (trace) {      // the residual behind the last layer, which otherwise only the head's input holds
+        NormRowsArgs n{};
+        n.in = norm_in(m, cur, m->final_norm);
+        take(n.in);
+        norm_rows_kernel<float><<<dim3(1), dim3(256), Dp * 4ull, st>>>(n);
+        HIP_TRY(hipGetLastError());
+        const uint32_t last = (uint32_t)m->layers.size() - 1;
+        if (!m->layers[last].moe) LV_TRY(keep(last, LV_TRACE_POST_ATTN));
+        LV_TRY(keep(last, LV_TRACE_OUT));
+    }
+    if (logits) {
+        BfGemvArgs h{};
+        h.w = m->head.w; h.rows = m->hp.vocab; h.kp = Dp; h.out = logits;
+        h.norm = norm_in(m, cur, m->final_norm);
+        if (pend) {
+            h.norm.y = pend;
+            h.norm.wpost = wpost;
+        }
+        LV_TRY((gemv<kGemvRows, kInNorm>(st, h)));
+    }
+    return LV_OK;
+}
+
+// ---- batches ---------------------------------------------------------------------------------------------------------------
+static int workspace_reserve(BlockSession *s, uint32_t n)
+{
+    const BlockModel *m = s->m;
+    Workspace &w = s->ws;
+    const uint32_t cap = up(n, 128);
+    if (cap <= w.cap) return LV_OK;
+    HIP_TRY(hipStreamSynchronize(s->st));
+    workspace_free(w);
+    const uint64_t T = cap, E = m->elem();
+    auto mx = [&](auto f) -> uint64_t { return layer_max(m, f); };
+    hipStream_t st = s->st;
+    LV_TRY(dev_zeroed(st, &w.x, T * m->dp * 4));
+    LV_TRY(dev_zeroed(st, &w.act, T * m->dp * E));
+    LV_TRY(dev_zeroed(st, &w.y1, T * mx([](const BlockLayer &l) { return l.in.rows; }) * 4));
+    LV_TRY(dev_zeroed(st, &w.y, T * m->dp * 4 * mx([](const BlockLayer &l) { return std::max(1u, l.spec.moe.top); })));
+    LV_TRY(dev_zeroed(st, &w.q, T * E * mx([](const BlockLayer &l) { return l.spec.attn.heads * l.dp; })));
+    const uint64_t kv = mx([](const BlockLayer &l) { return l.spec.attn.kv_heads * l.dp; });
+    LV_TRY(dev_zeroed(st, &w.k, T * E * kv));
+    LV_TRY(dev_zeroed(st, &w.v, T * E * kv));
+    const uint64_t dk = mx([](const BlockLayer &l) { return l.delta ? l.spec.delta.kv_heads * l.dstride() : 0u; });
+    LV_TRY(dev_zeroed(st, &w.dq, T * 4 * dk));
+    LV_TRY(dev_zeroed(st, &w.dk, T * 4 * dk));
+    LV_TRY(dev_zeroed(st, &w.dg, T * 4 * mx([](const BlockLayer &l) { return l.delta ? l.spec.delta.heads * l.dstride() : 0u; })));
+    const uint64_t hv = mx([](const BlockLayer &l) { return l.spec.delta.heads * l.spec.delta.vdim; });
+    LV_TRY(dev_zeroed(st, &w.dv, T * 4 * hv));
+    LV_TRY(dev_zeroed(st, &w.o, T * 4 * hv));
+    LV_TRY(dev_zeroed(st, &w.gate, T * 4 * hv));
+    const uint64_t heads = mx([](const BlockLayer &l) { return l.spec.delta.heads; });
+    LV_TRY(dev_zeroed(st, &w.beta, T * 4 * heads));
+    LV_TRY(dev_zeroed(st, &w.qk, T * 4 * heads));
+    LV_TRY(dev_zeroed(st, &w.a1, T * E * mx([](const BlockLayer &l) { return l.a2.kp; })));
+    LV_TRY(dev_zeroed(st, &w.g1, T * E * mx([](const BlockLayer &l) { return l.g2.kp; })));
+    LV_TRY(dev_zeroed(st, &w.cat, T * E * mx([](const BlockLayer &l) { return l.out.kp; })));
+    const uint64_t experts = mx([](const BlockLayer &l) { return l.spec.moe.experts; }), top = mx([](const BlockLayer &l) { return l.spec.moe.top; });
+    LV_TRY(dev_zeroed(st, &w.z, T * 4 * up((uint32_t)experts, 4)));
+    LV_TRY(dev_zeroed(st, &w.scores, T * 4 * top));
+    LV_TRY(dev_zeroed(st, &w.ids, T * 4 * top));
+    LV_TRY(dev_zeroed(st, &w.slots, T * 4 * top));
+    LV_TRY(dev_zeroed(st, &w.tiles, 4 * (1 + 3 * (T * top / kF32Tile + experts + 1))));
+    // a tile of 128 positions may start at any of the T * top
+    LV_TRY(dev_zeroed(st, &w.ff, E * mx([&](const BlockLayer &l) { return (cap * l.spec.moe.top + 128) * l.down.kp; })));
+    w.cap = cap;
+    return LV_OK;
+}
+
+template <class T> static int norm_rows(hipStream_t st, const NormRowsArgs &a, uint32_t n)
+{
+    const size_t lds = a.in.dp * 4ull;
+    LV_TRY(allow_lds(&norm_rows_kernel<T>, lds));
+    norm_rows_kernel<T><<<dim3(n), dim3(256), lds, st>>>(a);
+    HIP_TRY(hipGetLastError());
+    return LV_OK;
+}
+
+template <class T>
+static int step_batch(BlockSession *s, const uint32_t *tokens, uint32_t pos, uint32_t row0, uint32_t n, float *logits_last, float *logits_all, const BlockTrace *trace)
+{
+    constexpr bool f32 = sizeof(T) == 4;
+    const BlockModel *m = s->m;
+    hipStream_t st = s->st;
+    const uint32_t D = m->hp.dim, Dp = m->dp;
+    LV_TRY(workspace_reserve(s, n));
+    Workspace &w = s->ws;
+    embed_bf16_kernel<<<dim3((Dp + 255) / 256, n), dim3(256), 0, st>>>(w.x, m->embed, tokens, D, Dp);
+    HIP_TRY(hipGetLastError());
+    const float *wpost = nullptr;
+    uint32_t parts = 0;                // vectors per token in w.y that wait to be added to the residual stream
+    auto norm = [&](const float *wpre, bool act) -> int {
+        NormRowsArgs a{};
+        a.in = norm_in(m, w.x, wpre);
+        if (parts) {
+            a.in.y = w.y;
+            a.in.parts = parts;
+            a.in.wpost = wpost;
+            a.in.x_out = w.x;
+        }
+        a.act = act ? w.act : nullptr;
+        parts = 0;
+        return norm_rows<T>(st, a, n);
+    };
+    auto keep = [&](uint32_t layer, int which) -> int {
+        if (trace) HIP_TRY(hipMemcpy2DAsync(trace->slot(layer, which, row0), trace->stride * 4ull, w.x, Dp * 4ull, D * 4ull, n, hipMemcpyDeviceToDevice, st));
+        return LV_OK;
+    };
+    for (size_t i = 0; i < m->layers.size(); i++) {
+        const BlockLayer &l = m->layers[i];
+        LV_TRY(norm(l.norm1, true));
+        if (i) {
+            if (!m->layers[i - 1].moe) LV_TRY(keep(i - 1, LV_TRACE_POST_ATTN));
+            LV_TRY(keep(i - 1, LV_TRACE_OUT));
+        }
+        BfGemmArgs g{};
+        g.x = w.act; g.ldx = Dp; g.out = w.y1; g.ldo = l.in.rows;
+        LV_TRY((gemm<kEpStore, false>(st, f32, g, l.in, n)));
+
+        PrepareArgs p{};
+        p.y = w.y1; p.ldy = l.in.rows; p.pos0 = pos; p.dp = l.dp;
+        p.attn = gqa_spec(s, i); p.q = w.q; p.k = w.k; p.v = w.v;
+        p.delta = delta_spec(s, i); p.dq = w.dq; p.dk = w.dk; p.dv = w.dv; p.beta = w.beta; p.qk = w.qk; p.a1 = w.a1; p.g1 = w.g1;
+        prepare_kernel<T><<<dim3(n), dim3(256), 0, st>>>(p);
+        HIP_TRY(hipGetLastError());
+        if (l.attn) {
+            GqaBatchArgs a{};
+            a.s = p.attn; a.pos0 = pos; a.n = n; a.q = w.q; a.k = w.k; a.v = w.v; a.out = w.cat; a.ldo = l.out.kp; a.groups = l.groups;
+            a.out_scale = l.spec.attn_scale;
+            LV_TRY(gqa_dispatch(f32, l, [&](auto elem, auto dp, auto r) -> int {
+                constexpr int DP = decltype(dp)::value, R = decltype(r)::value;
+                if constexpr (std::is_same_v<decltype(elem), T>) {
+                    gqa_rows_kernel<T, DP, R><<<dim3(l.spec.attn.kv_heads * l.groups, n), dim3(256), 4 * gqa_lds_floats<DP, R>(), st>>>(a);
+                    HIP_TRY(hipGetLastError());
+                }
+                return LV_OK;
+            }));
+        }
+        if (l.delta) {
+            const lv_delta_spec &d = l.spec.delta;
+            BfGemmArgs dg{};
+            dg.x = w.a1; dg.ldx = l.a2.kp; dg.out = w.dg; dg.ldo = d.heads * l.dstride(); dg.a_log = l.a_log; dg.bias = l.dt_bias; dg.head_dim = d.dim; dg.head_stride = l.dstride();
+            LV_TRY((gemm<kEpDecay, false>(st, f32, dg, l.a2, n)));
+            BfGemmArgs gg{};
+            gg.x = w.g1; gg.ldx = l.g2.kp; gg.out = w.gate; gg.ldo = d.heads * d.vdim;
+            LV_TRY((gemm<kEpSigmoid, false>(st, f32, gg, l.g2, n)));
+            DeltaScanArgs sc{};
+            sc.s = p.delta; sc.n = n; sc.fresh = pos == 0; sc.q = w.dq; sc.k = w.dk; sc.v = w.dv; sc.g = w.dg; sc.beta = w.beta; sc.qk = w.qk; sc.o = w.o;
+            auto scan = [&](auto j) -> int {
+                constexpr int J = decltype(j)::value;
+                const size_t lds = 2 * 4ull * scan_stage_floats<J>();
+                LV_TRY(allow_lds(&delta_scan_kernel<J>, lds));
+                delta_scan_kernel<J><<<dim3(d.heads, (d.vdim + 15) / 16), dim3(256), lds, st>>>(sc);
+                HIP_TRY(hipGetLastError());
+                return LV_OK;
+            };
+            switch (l.dstride() / 64) {
+            case 1: LV_TRY(scan(std::integral_constant<int, 1>{})); break;
+            case 2: LV_TRY(scan(std::integral_constant<int, 2>{})); break;
+            case 3: LV_TRY(scan(std::integral_constant<int, 3>{})); break;
+            default: LV_TRY(scan(std::integral_constant<int, 4>{})); break;
+            }
+            gated_rows_kernel<T><<<dim3(n), dim3(256), 0, st>>>(static_cast<T *>(w.cat) + l.left_kp, l.out.kp, w.o, w.gate, l.onorm, d.heads, d.vdim, m->hp.eps, l.spec.delta_scale);
+            HIP_TRY(hipGetLastError());
+        }
+        const uint32_t tail = std::min(n, std::max(l.attn ? p.attn.ring : 0u, l.delta ? p.delta.taps : 0u));
+        append_kernel<T><<<dim3(tail), dim3(256), 0, st>>>(p, n);
+        HIP_TRY(hipGetLastError());
+
+        BfGemmArgs o{};
+        o.x = w.cat; o.ldx = l.out.kp; o.out = w.y; o.ldo = Dp;
+        LV_TRY((gemm<kEpStore, false>(st, f32, o, l.out, n)));
+        parts = 1;
+        wpost = l.norm1b;
+        if (!l.moe) continue;
+
+        const lv_moe_spec &e = l.spec.moe;
+        const uint32_t ldz = up(e.experts, 4), total = n * e.top;
+        LV_TRY(norm(l.norm2, true));
+        LV_TRY(keep(i, LV_TRACE_POST_ATTN));
+        BfGemmArgs rt{};
+        rt.x = w.act; rt.ldx = Dp; rt.out = w.z; rt.ldo = ldz;
+        LV_TRY((gemm<kEpStore, false>(st, f32, rt, l.router, n)));
+        route_rows_kernel<<<dim3(n), dim3(64), e.experts * 4ull, st>>>(w.z, ldz, e.experts, e.top, w.ids, w.scores);
+        HIP_TRY(hipGetLastError());
+        sort_experts_kernel<<<dim3(1), dim3(1024), e.experts * 8ull, st>>>(w.ids, total, e.experts, f32 ? kF32Tile : kBfTile, w.slots, w.tiles);
+        HIP_TRY(hipGetLastError());
+        BfGemmArgs gu{};
+        gu.x = w.act; gu.ldx = Dp; gu.tiles = w.tiles; gu.slots = w.slots; gu.weights = w.scores; gu.top = e.top; gu.expert_rows = l.gu_rows; gu.gather = true;
+        gu.act = w.ff; gu.lda = l.down.kp;
+        LV_TRY((gemm<kEpGlu, true>(st, f32, gu, l.gate_up, total, e.experts)));
+        BfGemmArgs dn{};
+        dn.x = w.ff; dn.ldx = l.down.kp; dn.tiles = w.tiles; dn.slots = w.slots; dn.top = e.top; dn.expert_rows = l.down_rows; dn.out = w.y; dn.ldo = Dp;
+        LV_TRY((gemm<kEpScatter, true>(st, f32, dn, l.down, total, e.experts)));
+        parts = e.top;
+        wpost = l.norm2b;
+    }
+    const uint32_t last = (uint32_t)m->layers.size() - 1;
+    if (trace || logits_all) {
+        LV_TRY(norm(m->final_norm, logits_all != nullptr));
+        if (!m->layers[last].moe) LV_TRY(keep(last, LV_TRACE_POST_ATTN));
+        LV_TRY(keep(last, LV_TRACE_OUT));
+    }
+    if (logits_all) {
+        BfGemmArgs h{};
+        h.x = w.act; h.ldx = Dp; h.out = logits_all; h.ldo = m->hp.vocab;
+        LV_TRY((gemm<kEpStore, false>(st, f32, h, m->head, n)));
+        if (logits_last) HIP_TRY(hipMemcpyAsync(logits_last, logits_all + (size_t)(n - 1) * m->hp.vocab, m->hp.vocab * 4ull, hipMemcpyDeviceToDevice, st));
+    } else if (logits_last) {
+        BfGemvArgs h{};
+        h.w = m->head.w; h.rows = m->hp.vocab; h.kp = Dp; h.out = logits_last;
+        h.norm = norm_in(m, w.x + (size_t)(n - 1) * Dp, m->final_norm);
+        if (parts) {
+            h.norm.y = w.y + (size_t)(n - 1) * parts * Dp;
+            h.norm.parts = parts;
+            h.norm.wpost = wpost;
+        }
+        LV_TRY((gemv<kGemvRows, kInNorm>(st, h)));
+    }
+    return LV_OK;
+}
+
+int block_step_batch(BlockSession *s, const uint32_t *cfg, uint32_t pos, uint32_t idx0, uint32_t n, float *logits_last, float *logits_all, const BlockTrace *trace)
+{
+    const uint32_t *tokens = cfg + 1 + idx0;
+    return s->m->f32 ? step_batch<float>(s, tokens, pos, idx0, n, logits_last, logits_all, trace)
+                     : step_batch<uint16_t>(s, tokens, pos, idx0, n, logits_last, logits_all, trace);
+}
+
+// ---------------------------------------------------------------------------------------------------------------------------
+// state as bytes: K ring rows, V ring rows, convolution ring, recurrent state
+// ---------------------------------------------------------------------------------------------------------------------------
+namespace {
+struct StatePiece {
+    void *p;
+    uint64_t bytes;
+};
+void state_pieces(const BlockSession *s, uint32_t layer, uint32_t n_tokens, StatePiece (&out)[4])
+{
+    const BlockLayer &l = s->m->layers[layer];
+    const LayerState &ls = s->layers[layer];
+    const uint64_t rows = l.attn ? std::min(n_tokens, l.spec.attn.chunk ? l.spec.attn.chunk : n_tokens) : 0;
+    const uint64_t kv = rows * l.spec.attn.kv_heads * l.dp * s->m->elem();
+    out[0] = {ls.kc, kv};
+    out[1] = {ls.vc, kv};
+    out[2] = {ls.conv, l.delta && n_tokens ? 4ull * l.spec.delta.conv * l.channels() : 0};
+    out[3] = {ls.state, l.delta && n_tokens ? 4ull * l.spec.delta.heads * l.spec.delta.vdim * l.dstride() : 0};
+}
+}  // namespace
+
+uint64_t block_state_bytes(const BlockSession *s, uint32_t layer, uint32_t n_tokens)
+{
+    StatePiece p[4];
+    state_pieces(s, layer, n_tokens, p);
+    return p[0].bytes + p[1].bytes + p[2].bytes + p[3].bytes;
+}
+
+int block_state_copy(BlockSession *s, uint32_t layer, uint32_t n_tokens, void *host, bool write)
+{
+    StatePiece p[4];
+    state_pieces(s, layer, n_tokens, p);
+    uint8_t *h = static_cast<uint8_t *>(host);
+    for (const StatePiece &q : p) {
+        if (!q.bytes) continue;
+        HIP_TRY(hipMemcpyAsync(write ? q.p : (void *)h, write ? (const void *)h : q.p, q.bytes, write ? hipMemcpyHostToDevice : hipMemcpyDeviceToHost, s->st));
+        h += q.bytes;
+    }
+    HIP_TRY(hipStreamSynchronize(s->st));
+    return LV_OK;
+}
+
+}  // namespace lv

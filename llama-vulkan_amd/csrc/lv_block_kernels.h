@@ -1,0 +1,237 @@
+// lv_block_kernels.h — what a layer of a block model (lv_block.h) needs besides its products and mixers: embedding rows, row
+// norms with a pending sublayer output, the step that turns the joint projection into mixer operands, cache appends, and the
+// routing of a batch to experts.
+#pragma once
+
+#include "lv_delta.h"
+#include "lv_gqa.h"
+
+namespace lv {
+
+// x[z][0 .. dp) = table[token[z]], fp32, zero beyond dim
+__global__ __launch_bounds__(256) void embed_bf16_kernel(float *__restrict__ x, const uint16_t *__restrict__ table, const uint32_t *tokens, uint32_t dim, uint32_t dp)
+{
+    const uint32_t i = blockIdx.x * 256 + threadIdx.x, z = blockIdx.y;
+    if (i < dp) x[(size_t)z * dp + i] = i < dim ? bf16_to_float(table[(size_t)tokens[z] * dim + i]) : 0.f;
+}
+
+// NormInput for a batch: one workgroup per row; x in place, h as activations
+struct NormRowsArgs {
+    NormInput in;            // x, y, x_out: first row; h_out unused
+    void *act;               // [row][dp], null: only the residual is wanted
+    float *h32;              // the same in fp32, null: not wanted
+};
+template <class T>
+__global__ __launch_bounds__(256) void norm_rows_kernel(NormRowsArgs a)
+{
+    extern __shared__ float xs[];
+    __shared__ float scratch[4];
+    NormInput in = a.in;
+    const uint32_t row = blockIdx.x, dp = in.dp;
+    in.x += (size_t)row * dp;
+    if (in.y) in.y += (size_t)row * in.parts * in.part_stride;
+    float *x_out = in.x_out ? in.x_out + (size_t)row * dp : nullptr;
+    float ypost = 1.f;
+    if (in.y) {
+        float s = 0.f;
+        for (uint32_t i = threadIdx.x * 4; i < dp; i += 1024) {
+            float4 v = *reinterpret_cast<const float4 *>(in.y + i);
+            for (uint32_t p = 1; p < in.parts; p++) {
+                const float4 u = *reinterpret_cast<const float4 *>(in.y + (size_t)p * in.part_stride + i);
+                v.x += u.x; v.y += u.y; v.z += u.z; v.w += u.w;
+            }
+            s = fmaf(v.x, v.x, s); s = fmaf(v.y, v.y, s); s = fmaf(v.z, v.z, s); s = fmaf(v.w, v.w, s);
+            *reinterpret_cast<float4 *>(xs + i) = v;
+        }
+        if (in.wpost) ypost = 1.f / sqrtf(block_sum_256(s, scratch) / (float)in.dim + in.eps);
+    }
+    float s = 0.f;
+    for (uint32_t i = threadIdx.x * 4; i < dp; i += 1024) {
+        float4 v = *reinterpret_cast<const float4 *>(in.x + i);
+        if (in.y) {
+            const float4 y = *reinterpret_cast<const float4 *>(xs + i);
+            const float4 w = in.wpost ? *reinterpret_cast<const float4 *>(in.wpost + i) : make_float4(1.f, 1.f, 1.f, 1.f);
+            v.x += y.x * ypost * w.x; v.y += y.y * ypost * w.y; v.z += y.z * ypost * w.z; v.w += y.w * ypost * w.w;
+            if (x_out) *reinterpret_cast<float4 *>(x_out + i) = v;
+        }
+        s = fmaf(v.x, v.x, s); s = fmaf(v.y, v.y, s); s = fmaf(v.z, v.z, s); s = fmaf(v.w, v.w, s);
+        *reinterpret_cast<float4 *>(xs + i) = v;
+    }
+    if (!a.act) return;
+    const float inv = 1.f / sqrtf(block_sum_256(s, scratch) / (float)in.dim + in.eps);
+    for (uint32_t i = threadIdx.x * 4; i < dp; i += 1024) {
+        const float4 v = *reinterpret_cast<const float4 *>(xs + i), w = *reinterpret_cast<const float4 *>(in.wpre + i);
+        const float h[4] = {v.x * inv * w.x, v.y * inv * w.y, v.z * inv * w.z, v.w * inv * w.w};
+        T *o = static_cast<T *>(a.act) + (size_t)row * dp + i;
+        if constexpr (sizeof(T) == 2)
+            *reinterpret_cast<uint2 *>(o) = make_uint2((uint32_t)float_to_bf16(h[0]) | ((uint32_t)float_to_bf16(h[1]) << 16),
+                                                       (uint32_t)float_to_bf16(h[2]) | ((uint32_t)float_to_bf16(h[3]) << 16));
+        else *reinterpret_cast<float4 *>(o) = make_float4(h[0], h[1], h[2], h[3]);
+        if (a.h32) *reinterpret_cast<float4 *>(a.h32 + (size_t)row * dp + i) = make_float4(h[0], h[1], h[2], h[3]);
+    }
+}
+
+// Both mixers of one token in one launch: recurrent head blocks first (they take longest), then the attention groups.
+struct MixStepArgs {
+    DeltaStepArgs delta;
+    GqaStepArgs attn;
+    uint32_t delta_wgs;
+};
+template <class CT, int DP, int R>
+__global__ __launch_bounds__(256) void mix_step_kernel(MixStepArgs a)
+{
+    extern __shared__ float lds[];
+    if (blockIdx.x < a.delta_wgs) delta_step(a.delta, blockIdx.x, lds);
+    else gqa_step<CT, DP, R>(a.attn, blockIdx.x - a.delta_wgs, lds);
+}
+
+// ---- batches: joint projection -> mixer operands, one workgroup per token --------------------------------------------------
+struct PrepareArgs {
+    const float *y;              // [n][ldy]
+    uint32_t ldy, pos0, dp;      // dp: padded head size of q, k, v
+    GqaSpec attn;                // heads 0: none
+    void *q, *k, *v;
+    DeltaSpec delta;             // heads 0: none
+    float *dq, *dk, *dv, *beta, *qk;
+    void *a1, *g1;               // low-rank activations [n][a_kp], [n][g_kp]
+};
+template <class T>
+__global__ __launch_bounds__(256) void prepare_kernel(PrepareArgs a)
+{
+    __shared__ float scratch[4];
+    const uint32_t t = blockIdx.x, pos = a.pos0 + t;
+    const float *y = a.y + (size_t)t * a.ldy;
+    if (a.attn.heads) {
+        const GqaSpec &s = a.attn;
+        const uint32_t half = a.dp / 2;
+        const float inv_q = projection_inv(y + s.q_off, s.heads * s.dim, s.eps, s.q_norm, scratch);
+        const float inv_k = projection_inv(y + s.k_off, s.kv_heads * s.dim, s.eps, s.k_norm, scratch);
+        for (uint32_t i = threadIdx.x; i < s.heads * half; i += 256) {
+            const uint32_t h = i / half, p = i % half;
+            float u, v;
+            head_pair(u, v, y + s.q_off, s.q_norm, h * s.dim, p, s.dim, inv_q, s, pos);
+            T *o = static_cast<T *>(a.q) + ((size_t)t * s.heads + h) * a.dp + 2 * p;
+            o[0] = float_to_elem<T>(u * s.scale);
+            o[1] = float_to_elem<T>(v * s.scale);
+        }
+        for (uint32_t i = threadIdx.x; i < s.kv_heads * half; i += 256) {
+            const uint32_t h = i / half, p = i % half;
+            float u, v;
+            head_pair(u, v, y + s.k_off, s.k_norm, h * s.dim, p, s.dim, inv_k, s, pos);
+            const size_t o = ((size_t)t * s.kv_heads + h) * a.dp + 2 * p;
+            static_cast<T *>(a.k)[o] = float_to_elem<T>(u);
+            static_cast<T *>(a.k)[o + 1] = float_to_elem<T>(v);
+            static_cast<T *>(a.v)[o] = float_to_elem<T>(2 * p < s.vdim ? y[s.v_off + h * s.vdim + 2 * p] : 0.f);
+            static_cast<T *>(a.v)[o + 1] = float_to_elem<T>(2 * p + 1 < s.vdim ? y[s.v_off + h * s.vdim + 2 * p + 1] : 0.f);
+        }
+    }
+    if (a.delta.heads) {
+        const DeltaSpec &s = a.delta;
+        const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nq = s.kv_heads * s.dim;
+        for (uint32_t h = wave; h < s.kv_heads; h += 4) {
+            float q[kDeltaMaxDim / 64], k[kDeltaMaxDim / 64], sq = 0.f, sk = 0.f, sqk = 0.f;
+#pragma unroll
+            for (int j = 0; j < (int)kDeltaMaxDim / 64; j++) {
+                const uint32_t d = j * 64 + lane;
+                q[j] = k[j] = 0.f;
+                if (d < s.dim) {
+                    q[j] = delta_conv(s, y, a.ldy, t, h * s.dim + d, pos);
+                    k[j] = delta_conv(s, y, a.ldy, t, nq + h * s.dim + d, pos);
+                }
+                sq = fmaf(q[j], q[j], sq);
+                sk = fmaf(k[j], k[j], sk);
+            }
+            const float fq = 1.f / sqrtf(wave_sum(sq) + 1e-6f) / sqrtf((float)s.dim), fk = 1.f / sqrtf(wave_sum(sk) + 1e-6f);
+#pragma unroll
+            for (int j = 0; j < (int)kDeltaMaxDim / 64; j++) {
+                const uint32_t d = j * 64 + lane;
+                q[j] *= fq;
+                k[j] *= fk;
+                sqk = fmaf(q[j], k[j], sqk);
+                if (d < s.dstride) {
+                    a.dq[((size_t)t * s.kv_heads + h) * s.dstride + d] = q[j];
+                    a.dk[((size_t)t * s.kv_heads + h) * s.dstride + d] = k[j];
+                }
+            }
+            sqk = wave_sum(sqk);
+            if (lane == 0) a.qk[(size_t)t * s.kv_heads + h] = sqk;
+        }
+        for (uint32_t c = threadIdx.x; c < s.heads * s.vdim; c += 256) a.dv[(size_t)t * s.heads * s.vdim + c] = delta_conv(s, y, a.ldy, t, 2 * nq + c, pos);
+        for (uint32_t h = threadIdx.x; h < s.heads; h += 256) a.beta[(size_t)t * s.heads + h] = sigmoid_f(y[s.b_off + h]);
+        for (uint32_t i = threadIdx.x; i < s.a_kp; i += 256) static_cast<T *>(a.a1)[(size_t)t * s.a_kp + i] = float_to_elem<T>(i < s.a_rank ? y[s.a_off + i] : 0.f);
+        for (uint32_t i = threadIdx.x; i < s.g_kp; i += 256) static_cast<T *>(a.g1)[(size_t)t * s.g_kp + i] = float_to_elem<T>(i < s.g_rank ? y[s.g_off + i] : 0.f);
+    }
+}
+
+// The batch's last rows into the rings, after everything that reads older rows has run.  blockIdx.x = token counted from the
+// end (0 = last).
+template <class T>
+__global__ __launch_bounds__(256) void append_kernel(PrepareArgs a, uint32_t n)
+{
+    const uint32_t t = n - 1 - blockIdx.x, pos = a.pos0 + t;
+    if (a.attn.heads && blockIdx.x < a.attn.ring) {
+        const uint32_t w = a.attn.kv_heads * a.dp;
+        const size_t dst = (size_t)(pos % a.attn.ring) * w, src = (size_t)t * w;
+        for (uint32_t i = threadIdx.x; i < w; i += 256) {
+            static_cast<T *>(a.attn.kc)[dst + i] = static_cast<const T *>(a.k)[src + i];
+            static_cast<T *>(a.attn.vc)[dst + i] = static_cast<const T *>(a.v)[src + i];
+        }
+    }
+    if (a.delta.heads && blockIdx.x < a.delta.taps) {
+        const uint32_t C = a.delta.channels();
+        for (uint32_t c = threadIdx.x; c < C; c += 256) a.delta.ring[(size_t)(pos % a.delta.taps) * C + c] = a.y[(size_t)t * a.ldy + delta_channel_at(a.delta, c)];
+    }
+}
+
+// recurrent read-outs of a batch -> the columns of the joint output projection's input behind the attention part
+template <class T>
+__global__ __launch_bounds__(256) void gated_rows_kernel(T *__restrict__ act, uint32_t ld, const float *__restrict__ o, const float *__restrict__ gate,
+                                                         const float *__restrict__ w, uint32_t heads, uint32_t vdim, float eps, float scale)
+{
+    const size_t row = blockIdx.x, base = row * heads * vdim;
+    for (uint32_t h = threadIdx.x >> 6; h < heads; h += 4)
+        gated_head(o + base + h * vdim, gate + base + h * vdim, w, vdim, eps, scale, [&](uint32_t c, float v) { act[row * ld + h * vdim + c] = float_to_elem<T>(v); });
+}
+
+// ---- routing of a batch ----------------------------------------------------------------------------------------------------
+// one wave per token
+__global__ __launch_bounds__(64) void route_rows_kernel(const float *__restrict__ z, uint32_t ldz, uint32_t experts, uint32_t top, uint32_t *__restrict__ ids,
+                                                        float *__restrict__ scores)
+{
+    extern __shared__ float zs[];
+    const size_t t = blockIdx.x;
+    for (uint32_t e = threadIdx.x; e < experts; e += 64) zs[e] = z[t * ldz + e];
+    __syncthreads();
+    top_experts(zs, experts, top, ids + t * top, scores + t * top);
+}
+
+// Positions in expert order and the table of token tiles (BfGemmArgs::tiles).  One workgroup; LDS: 2 * experts words.  Where
+// a token lands inside its expert's run does not matter to its result.
+__global__ __launch_bounds__(1024) void sort_experts_kernel(const uint32_t *__restrict__ ids, uint32_t total, uint32_t experts, uint32_t tile, uint32_t *__restrict__ slots,
+                                                            uint32_t *__restrict__ tiles)
+{
+    extern __shared__ uint32_t cnt[];
+    uint32_t *at = cnt + experts;
+    for (uint32_t e = threadIdx.x; e < experts; e += 1024) cnt[e] = 0;
+    __syncthreads();
+    for (uint32_t i = threadIdx.x; i < total; i += 1024) atomicAdd(&cnt[ids[i]], 1u);
+    __syncthreads();
+    if (threadIdx.x == 0) {
+        uint32_t pos = 0, nt = 0;
+        for (uint32_t e = 0; e < experts; e++) {
+            const uint32_t c = cnt[e];
+            at[e] = pos;
+            for (uint32_t f = 0; f < c; f += tile, nt++) {
+                tiles[1 + 3 * nt] = e;
+                tiles[2 + 3 * nt] = pos + f;
+                tiles[3 + 3 * nt] = min(tile, c - f);
+            }
+            pos += c;
+        }
+        tiles[0] = nt;
+    }
+    __syncthreads();
+    for (uint32_t i = threadIdx.x; i < total; i += 1024) slots[atomicAdd(&at[ids[i]], 1u)] = i;
+}
+
+}  // namespace lv

@@ -1,0 +1,277 @@
+// lv_delta.h — the gated delta rule with a decay per key channel: a recurrent mixer with one dim x vdim state per head.
+//
+//   q, k, v  projections, each through a causal convolution of `taps` steps per channel and silu; q and k (kv_heads of them,
+//            shared by consecutive heads) are then unit vectors, q times dim^-1/2
+//   beta     = sigmoid(b), one per head
+//   g        = exp(-exp(A_log) softplus(a + dt_bias)), one per head and key channel
+//   S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
+//   out      = o / rms(o) * norm * gate, gate = sigmoid of a low-rank projection, vdim values per head
+//
+// All of it is fp32.  With S' = g S the read-out is o = S'^T q + (k . q) u, so the two reductions of a step, S'^T k and S'^T q,
+// do not wait for each other.  Columns of S do not interact: 16 lanes share a column, each holding 4 J of its dim entries.
+//
+// State of a sequence and layer: S as [head][vdim][64 J] (a column contiguous, zero beyond dim) and a ring of the
+// convolution's last `taps` inputs, [position % taps][channel], channels in the order q, k, v.  Nothing has to be cleared for
+// a new sequence: positions before 0 and the state at position 0 are never read.
+#pragma once
+
+#include "lv_bf16_gemv.h"
+
+namespace lv {
+
+struct DeltaSpec {
+    uint32_t heads, kv_heads, dim, vdim, taps;
+    uint32_t q_off, k_off, v_off, b_off, a_off, g_off;   // offsets in a token's joint projection
+    uint32_t a_rank, g_rank, a_kp, g_kp;                 // low-rank widths of decay and gate, as stored (padded to 64)
+    const float *conv;             // [channels][taps], last column = the current token
+    const float *a_log, *dt_bias, *norm;
+    const uint16_t *a2, *g2;       // [heads * dim][a_kp], [heads * vdim][g_kp]
+    float eps;
+    float *state, *ring;
+    uint32_t dstride;              // 64 J
+    __host__ __device__ uint32_t channels() const { return 2 * kv_heads * dim + heads * vdim; }
+};
+
+struct DeltaStepArgs {
+    DeltaSpec s;
+    const float *y;
+    const uint32_t *pos_ptr;
+    uint32_t pos_add;
+    uint32_t blocks;               // column blocks per head
+    float *o, *gate;               // [heads * vdim]
+};
+
+constexpr int kDeltaCols = 32;     // columns per workgroup of the one-token step
+constexpr uint32_t kDeltaMaxDim = 256;
+constexpr uint32_t kDeltaMaxRank = 4096;
+
+// channel c (in q, k, v order) of the joint projection
+__device__ __forceinline__ uint32_t delta_channel_at(const DeltaSpec &s, uint32_t c)
+{
+    const uint32_t nq = s.kv_heads * s.dim;
+    return c < nq ? s.q_off + c : c < 2 * nq ? s.k_off + (c - nq) : s.v_off + (c - 2 * nq);
+}
+
+// convolution and silu of channel c at position pos.  y: the token's projection row; rows before it (in steps of ld floats)
+// belong to positions pos - 1, pos - 2, .. as far as `behind` of them, older inputs are in the ring.
+__device__ __forceinline__ float delta_conv(const DeltaSpec &s, const float *y, size_t ld, uint32_t behind, uint32_t c, uint32_t pos)
+{
+    const float *w = s.conv + (size_t)c * s.taps;
+    const uint32_t at = delta_channel_at(s, c), C = s.channels();
+    float v = w[s.taps - 1] * y[at];
+    for (uint32_t j = 1; j < s.taps && j <= pos; j++) {
+        const float x = j <= behind ? y[at - (ptrdiff_t)(j * ld)] : s.ring[(size_t)((pos - j) % s.taps) * C + c];
+        v = fmaf(w[s.taps - 1 - j], x, v);
+    }
+    return silu_f(v);
+}
+
+// dot of one low-rank row with a vector in LDS, by 8 consecutive lanes; every lane of the eight gets it
+__device__ __forceinline__ float low_rank_dot(const uint16_t *row, const float *x, uint32_t kp)
+{
+    float t = 0.f;
+    for (uint32_t k = (threadIdx.x & 7) * 8; k < kp; k += 64) {
+        float w[8], v[8];
+        load8(w, row + k);
+        load8(v, x + k);
+#pragma unroll
+        for (int e = 0; e < 8; e++) t = fmaf(w[e], v[e], t);
+    }
+    return group8_sum(t);
+}
+
+__host__ __device__ constexpr uint32_t delta_step_lds_floats(uint32_t a_kp, uint32_t g_kp) { return 3 * kDeltaMaxDim + kDeltaCols + 16 + a_kp + g_kp; }
+
+// one token, one head, one block of kDeltaCols columns: 256 threads
+__device__ __forceinline__ void delta_step(const DeltaStepArgs &a, uint32_t idx, float *lds)
+{
+    const DeltaSpec &s = a.s;
+    const uint32_t head = idx / a.blocks, cb = idx % a.blocks, c_lo = cb * kDeltaCols, nc = min((uint32_t)kDeltaCols, s.vdim - c_lo);
+    const uint32_t pos = *a.pos_ptr + a.pos_add, rep = s.heads / s.kv_heads, kvh = head / rep, nq = s.kv_heads * s.dim, C = s.channels();
+    float *q = lds, *k = q + kDeltaMaxDim, *g = k + kDeltaMaxDim, *v = g + kDeltaMaxDim, *scratch = v + kDeltaCols, *al = scratch + 16, *gl = al + s.a_kp;
+    for (uint32_t i = threadIdx.x; i < s.a_kp; i += 256) al[i] = i < s.a_rank ? a.y[s.a_off + i] : 0.f;
+    for (uint32_t i = threadIdx.x; i < s.g_kp; i += 256) gl[i] = i < s.g_rank ? a.y[s.g_off + i] : 0.f;
+
+    float qv = 0.f, kv = 0.f;
+    const uint32_t d = threadIdx.x, rslot = pos % s.taps;
+    if (d < s.dim) {
+        const uint32_t cq = kvh * s.dim + d, ck = nq + cq;
+        qv = delta_conv(s, a.y, 0, 0, cq, pos);
+        kv = delta_conv(s, a.y, 0, 0, ck, pos);
+        if (cb == 0 && head % rep == 0) {
+            s.ring[(size_t)rslot * C + cq] = a.y[s.q_off + cq];
+            s.ring[(size_t)rslot * C + ck] = a.y[s.k_off + cq];
+        }
+    }
+    if (threadIdx.x < nc) {
+        const uint32_t c = head * s.vdim + c_lo + threadIdx.x;
+        v[threadIdx.x] = delta_conv(s, a.y, 0, 0, 2 * nq + c, pos);
+        s.ring[(size_t)rslot * C + 2 * nq + c] = a.y[s.v_off + c];
+    }
+    const float nqs = block_sum_waves(qv * qv, scratch, 4), nks = block_sum_waves(kv * kv, scratch, 4);
+    qv = qv / sqrtf(nqs + 1e-6f) / sqrtf((float)s.dim);
+    kv = kv / sqrtf(nks + 1e-6f);
+    const float qk = block_sum_waves(qv * kv, scratch, 4);
+    q[threadIdx.x] = qv;
+    k[threadIdx.x] = kv;
+    const float ea = expf(s.a_log[head]);
+    for (uint32_t r0 = 0; r0 < s.dstride; r0 += 32) {
+        const uint32_t r = r0 + (threadIdx.x >> 3);
+        float gv = 0.f;
+        if (r < s.dim) {
+            const uint32_t row = head * s.dim + r;
+            gv = expf(-ea * softplus_f(low_rank_dot(s.a2 + (size_t)row * s.a_kp, al, s.a_kp) + s.dt_bias[row]));
+        }
+        if ((threadIdx.x & 7) == 0) g[r] = gv;
+    }
+    {
+        const uint32_t c = threadIdx.x >> 3;
+        if (c < nc) {
+            const uint32_t row = head * s.vdim + c_lo + c;
+            const float t = low_rank_dot(s.g2 + (size_t)row * s.g_kp, gl, s.g_kp);
+            if ((threadIdx.x & 7) == 0) a.gate[row] = sigmoid_f(t);
+        }
+    }
+    __syncthreads();
+    const float beta = sigmoid_f(a.y[s.b_off + head]);
+    const int l16 = threadIdx.x & 15;
+    const uint32_t J = s.dstride / 64;
+    for (uint32_t c = threadIdx.x >> 4; c < nc; c += 16) {
+        float4 *col = reinterpret_cast<float4 *>(s.state + ((size_t)head * s.vdim + c_lo + c) * s.dstride);
+        float4 st[4];
+        float pk = 0.f, pq = 0.f;
+#pragma unroll
+        for (int j = 0; j < 4; j++)
+            if (j < (int)J) {
+                const int at = j * 64 + l16 * 4;
+                float4 x = pos ? col[at / 4] : make_float4(0.f, 0.f, 0.f, 0.f);
+                const float4 gg = *reinterpret_cast<const float4 *>(g + at), kk = *reinterpret_cast<const float4 *>(k + at), qq = *reinterpret_cast<const float4 *>(q + at);
+                x.x *= gg.x; x.y *= gg.y; x.z *= gg.z; x.w *= gg.w;
+                pk = fmaf(x.x, kk.x, pk); pk = fmaf(x.y, kk.y, pk); pk = fmaf(x.z, kk.z, pk); pk = fmaf(x.w, kk.w, pk);
+                pq = fmaf(x.x, qq.x, pq); pq = fmaf(x.y, qq.y, pq); pq = fmaf(x.z, qq.z, pq); pq = fmaf(x.w, qq.w, pq);
+                st[j] = x;
+            }
+        pk = group16_sum(pk);
+        pq = group16_sum(pq);
+        const float u = beta * (v[c] - pk);
+#pragma unroll
+        for (int j = 0; j < 4; j++)
+            if (j < (int)J) {
+                const int at = j * 64 + l16 * 4;
+                const float4 kk = *reinterpret_cast<const float4 *>(k + at);
+                st[j].x = fmaf(kk.x, u, st[j].x); st[j].y = fmaf(kk.y, u, st[j].y); st[j].z = fmaf(kk.z, u, st[j].z); st[j].w = fmaf(kk.w, u, st[j].w);
+                col[at / 4] = st[j];
+            }
+        if (l16 == 0) a.o[head * s.vdim + c_lo + c] = fmaf(qk, u, pq);
+    }
+}
+
+// ---- batches -------------------------------------------------------------------------------------------------------------
+struct DeltaScanArgs {
+    DeltaSpec s;
+    uint32_t n;
+    bool fresh;               // the batch starts the sequence: the state is zero
+    const float *q, *k;       // [n][kv_heads][dstride], unit vectors (q scaled), zero beyond dim
+    const float *v;           // [n][heads * vdim]
+    const float *g;           // [n][heads][dstride], finite beyond dim
+    const float *beta, *qk;   // [n][heads], [n][kv_heads]
+    float *o;                 // [n][heads * vdim]
+};
+
+constexpr int kScanTokens = 16;   // tokens staged in LDS at a time
+template <int J> constexpr int scan_stage_floats() { return kScanTokens * (3 * 64 * J + 16 + 2); }
+
+// All tokens of a batch for 16 columns of one head: a workgroup of 4 waves, 4 columns a wave.  grid (heads, vdim / 16 up).
+template <int J>
+__global__ __launch_bounds__(256) void delta_scan_kernel(DeltaScanArgs a)
+{
+    constexpr int W = 64 * J, SF = scan_stage_floats<J>();
+    extern __shared__ float lds[];       // two stages
+    const DeltaSpec &s = a.s;
+    const uint32_t head = blockIdx.x, kvh = head / (s.heads / s.kv_heads), HV = s.heads * s.vdim;
+    const int l16 = threadIdx.x & 15, ci = threadIdx.x >> 4;
+    const uint32_t col = blockIdx.y * 16 + ci;
+    const bool live = col < s.vdim;
+    float4 *const colp = reinterpret_cast<float4 *>(s.state + ((size_t)head * s.vdim + (live ? col : 0)) * W);
+    float4 S[J];
+#pragma unroll
+    for (int j = 0; j < J; j++) S[j] = a.fresh || !live ? make_float4(0.f, 0.f, 0.f, 0.f) : colp[j * 16 + l16];
+
+    // one stage: per thread J float4 of each of k, q, g, one value of v, and beta / qk by the first threads
+    constexpr int PER = kScanTokens * W / 4 / 256;       // float4 per thread and array
+    float4 rk[PER], rq[PER], rg[PER];
+    float rv = 0.f, rb = 0.f;
+    auto fetch = [&](uint32_t t0) {
+#pragma unroll
+        for (int i = 0; i < PER; i++) {
+            const int e = i * 256 + threadIdx.x;
+            const uint32_t t = min(t0 + e / (W / 4), a.n - 1), d = e % (W / 4) * 4;
+            rk[i] = *reinterpret_cast<const float4 *>(a.k + ((size_t)t * s.kv_heads + kvh) * W + d);
+            rq[i] = *reinterpret_cast<const float4 *>(a.q + ((size_t)t * s.kv_heads + kvh) * W + d);
+            rg[i] = *reinterpret_cast<const float4 *>(a.g + ((size_t)t * s.heads + head) * W + d);
+        }
+        {
+            const uint32_t t = min(t0 + threadIdx.x / 16, a.n - 1), c = blockIdx.y * 16 + threadIdx.x % 16;
+            rv = c < s.vdim ? a.v[(size_t)t * HV + head * s.vdim + c] : 0.f;
+        }
+        if (threadIdx.x < 32) {
+            const uint32_t t = min(t0 + (threadIdx.x & 15), a.n - 1);
+            rb = threadIdx.x < 16 ? a.beta[(size_t)t * s.heads + head] : a.qk[(size_t)t * s.kv_heads + kvh];
+        }
+    };
+    auto stash = [&](float *b) {
+#pragma unroll
+        for (int i = 0; i < PER; i++) {
+            const int e = (i * 256 + threadIdx.x) * 4;
+            *reinterpret_cast<float4 *>(b + e) = rk[i];
+            *reinterpret_cast<float4 *>(b + kScanTokens * W + e) = rq[i];
+            *reinterpret_cast<float4 *>(b + 2 * kScanTokens * W + e) = rg[i];
+        }
+        b[3 * kScanTokens * W + threadIdx.x] = rv;
+        if (threadIdx.x < 32) b[3 * kScanTokens * W + 256 + threadIdx.x] = rb;
+    };
+    fetch(0);
+    stash(lds);
+    for (uint32_t t0 = 0, st = 0; t0 < a.n; t0 += kScanTokens, st ^= 1) {
+        __syncthreads();
+        if (t0 + kScanTokens < a.n) fetch(t0 + kScanTokens);
+        const float *b = lds + st * SF, *bk = b, *bq = b + kScanTokens * W, *bg = b + 2 * kScanTokens * W, *bv = b + 3 * kScanTokens * W;
+        float keep = 0.f;
+        const int nt = (int)min((uint32_t)kScanTokens, a.n - t0);
+        auto token = [&](int t) {
+            float pk = 0.f, pq = 0.f;
+            float4 kk[J];
+#pragma unroll
+            for (int j = 0; j < J; j++) {
+                const int at = t * W + j * 64 + l16 * 4;
+                const float4 gg = *reinterpret_cast<const float4 *>(bg + at), qq = *reinterpret_cast<const float4 *>(bq + at);
+                kk[j] = *reinterpret_cast<const float4 *>(bk + at);
+                S[j].x *= gg.x; S[j].y *= gg.y; S[j].z *= gg.z; S[j].w *= gg.w;
+                pk = fmaf(S[j].x, kk[j].x, pk); pk = fmaf(S[j].y, kk[j].y, pk); pk = fmaf(S[j].z, kk[j].z, pk); pk = fmaf(S[j].w, kk[j].w, pk);
+                pq = fmaf(S[j].x, qq.x, pq); pq = fmaf(S[j].y, qq.y, pq); pq = fmaf(S[j].z, qq.z, pq); pq = fmaf(S[j].w, qq.w, pq);
+            }
+            pk = group16_sum(pk);
+            pq = group16_sum(pq);
+            const float u = bv[256 + t] * (bv[t * 16 + ci] - pk);
+#pragma unroll
+            for (int j = 0; j < J; j++) {
+                S[j].x = fmaf(kk[j].x, u, S[j].x); S[j].y = fmaf(kk[j].y, u, S[j].y); S[j].z = fmaf(kk[j].z, u, S[j].z); S[j].w = fmaf(kk[j].w, u, S[j].w);
+            }
+            if (l16 == t) keep = fmaf(bv[272 + t], u, pq);
+        };
+        if (nt == kScanTokens) {
+#pragma unroll
+            for (int t = 0; t < kScanTokens; t++) token(t);
+        } else {
+            for (int t = 0; t < nt; t++) token(t);
+        }
+        if (live && l16 < nt) a.o[(size_t)(t0 + l16) * HV + head * s.vdim + col] = keep;
+        if (t0 + kScanTokens < a.n) stash(lds + (st ^ 1) * SF);
+    }
+    if (live) {
+#pragma unroll
+        for (int j = 0; j < J; j++) colp[j * 16 + l16] = S[j];
+    }
+}
+
+}  // namespace lv

@@ -95,6 +95,26 @@ __device__ __forceinline__ float group_sum(float v)
     else return wave_sum(v);
 }
 
+// ---- sums over a 256-thread workgroup -------------------------------------------------------------------
+__device__ __forceinline__ float block_sum_256(float v, float *lds /* >= 4 floats */)
+{
+    v = wave_sum(v);
+    __syncthreads();  // protect lds reuse between consecutive calls
+    if ((threadIdx.x & 63) == 0) lds[threadIdx.x >> 6] = v;
+    __syncthreads();
+    return (lds[0] + lds[1]) + (lds[2] + lds[3]);
+}
+
+__device__ __forceinline__ float block_max_256(float v, float *lds /* >= 4 floats */)
+{
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) v = fmaxf(v, __shfl_xor(v, off, 64));
+    __syncthreads();  // protect lds reuse between consecutive calls
+    if ((threadIdx.x & 63) == 0) lds[threadIdx.x >> 6] = v;
+    __syncthreads();
+    return fmaxf(fmaxf(lds[0], lds[1]), fmaxf(lds[2], lds[3]));
+}
+
 // ---- fp16 ------------------------------------------------------------------------------------------------
 __device__ __forceinline__ float half_bits_to_float(uint16_t h)
 {

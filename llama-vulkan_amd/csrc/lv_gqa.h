@@ -1,0 +1,366 @@
+// lv_gqa.h — grouped-query softmax attention over a ring of cache rows, with optional normalised projections, interleaved
+// rotary positions, chunked visibility, values taken from the keys' projection, and a sink.
+//
+//   q, k   projections; RMS norm over the whole projection (weights), then rotation of the first rot_dims dimensions of a
+//          head: pair (2i, 2i+1) by the angle p * f_i
+//   s      = (q . k) * scale, over the keys j <= i with j / chunk == i / chunk (chunk 0: every j <= i)
+//   out    = sum_j exp(s_j) v_j / (sum_j exp(s_j) + exp(sink))
+//
+// Cache: per layer two rings of `ring` rows, [row][kv head][DP] each, DP = head size rounded up to a power of two; position p
+// lives in row p % ring.  A chunked layer needs chunk rows whatever the length of the sequence.  A batch of tokens keeps its
+// own rows in scratch while it is evaluated (keys from the batch's first position on come from there, older ones from the
+// ring) and is appended to the ring afterwards, so that a batch may run over any number of chunk borders.
+//
+// Everything but the MFMA path (attention_tile_kernel: bf16 operands, weights as two bf16 pieces) is fp32 arithmetic on
+// cache rows of either element type.
+#pragma once
+
+#include "lv_bf16_gemv.h"
+
+namespace lv {
+
+struct GqaSpec {
+    uint32_t heads, kv_heads, dim, vdim;
+    uint32_t q_off, k_off, v_off;       // where a token's projections start in its row of the joint projection
+    const float *q_norm, *k_norm;       // null: not normalised
+    const float *sink;                  // null: none
+    const double *freq;                 // rot_dims / 2 angles per position
+    uint32_t rot_dims, chunk;
+    float scale, eps;
+    uint32_t ring;                      // cache rows
+    void *kc, *vc;
+};
+
+struct GqaStepArgs {
+    GqaSpec s;
+    const float *y;                     // the token's joint projection
+    const uint32_t *pos_ptr;
+    uint32_t pos_add;
+    uint32_t groups;                    // head groups per kv head (R heads each, the last may hold fewer)
+    uint32_t splits;                    // key splits the grid provides
+    float *part;                        // [kv head][group][split][R][DP + 2]
+    uint32_t *counters;                 // [kv head][group], zero before and after
+    float *out;                         // [heads * vdim]
+};
+
+constexpr int kGqaSplit = 128;          // keys per workgroup
+
+__device__ __forceinline__ void rotate_pair(float &u, float &v, double freq, uint32_t pos)
+{
+    // angle reduced in double: positions far out lose nothing to the range reduction
+    const double a = (double)pos * freq, turn = 6.283185307179586476925;
+    float sn, cs;
+    sincosf((float)(a - turn * rint(a / turn)), &sn, &cs);
+    const float r = u * cs - v * sn;
+    v = v * cs + u * sn;
+    u = r;
+}
+
+template <int LPK> __device__ __forceinline__ float lanes_sum(float v)
+{
+    if constexpr (LPK == 8) return group8_sum(v);
+    v = group16_sum(v);
+    if constexpr (LPK == 32) v += __shfl_xor(v, 16, 64);
+    return v;
+}
+
+// Scores of the keys k_begin + 0 .. n - 1 against R queries in LDS, then weights and the weighted value sum.
+// key(j, f) / value(j, f): the 8 elements of key / value j (an index from 0) this lane holds (sub * 8 ..).
+template <int DP, int R>
+struct GqaLanes {
+    static constexpr int LPK = DP / 8;            // lanes per key
+    static constexpr int KPR = 256 / LPK;         // keys per round of the workgroup
+};
+
+// LDS, in floats
+template <int DP, int R> constexpr int gqa_lds_floats() { return R * DP + 2 * DP + R * kGqaSplit + 4 * R * DP + 4 * R + 16; }
+
+// q [R][DP] and sc [R][kGqaSplit] in LDS
+template <int DP, int R, class Key>
+__device__ __forceinline__ void gqa_scores(const float *q, float *sc, uint32_t n, Key key)
+{
+    using L = GqaLanes<DP, R>;
+    const int sub = threadIdx.x % L::LPK, kg = threadIdx.x / L::LPK;
+    float qr[R][8];
+#pragma unroll
+    for (int r = 0; r < R; r++) load8(qr[r], q + r * DP + sub * 8);
+    for (uint32_t j0 = 0; j0 < n; j0 += L::KPR) {
+        const uint32_t j = j0 + kg;
+        float f[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+        if (j < n) key(j, sub * 8, f);
+#pragma unroll
+        for (int r = 0; r < R; r++) {
+            float s = 0.f;
+#pragma unroll
+            for (int e = 0; e < 8; e++) s = fmaf(qr[r][e], f[e], s);
+            s = lanes_sum<L::LPK>(s);
+            if (sub == 0 && j < n) sc[r * kGqaSplit + j] = s;
+        }
+    }
+}
+
+template <int DP, int R, class Value>
+__device__ __forceinline__ void gqa_values(float (&acc)[R][8], const float *sc, uint32_t n, Value value)
+{
+    using L = GqaLanes<DP, R>;
+    const int sub = threadIdx.x % L::LPK, kg = threadIdx.x / L::LPK;
+    for (uint32_t j = kg; j < n; j += L::KPR) {
+        float f[8];
+        value(j, sub * 8, f);
+#pragma unroll
+        for (int r = 0; r < R; r++) {
+            const float p = sc[r * kGqaSplit + j];
+#pragma unroll
+            for (int e = 0; e < 8; e++) acc[r][e] = fmaf(p, f[e], acc[r][e]);
+        }
+    }
+}
+
+// acc of all key groups -> red[0 .. R*DP) (summed over the workgroup)
+template <int DP, int R>
+__device__ __forceinline__ void gqa_reduce(float (&acc)[R][8], float *red)
+{
+    using L = GqaLanes<DP, R>;
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+#pragma unroll
+    for (int r = 0; r < R; r++)
+#pragma unroll
+        for (int e = 0; e < 8; e++) {
+#pragma unroll
+            for (int off = L::LPK; off < 64; off <<= 1) acc[r][e] += __shfl_xor(acc[r][e], off, 64);
+        }
+    if (lane < L::LPK) {
+#pragma unroll
+        for (int r = 0; r < R; r++)
+#pragma unroll
+            for (int e = 0; e < 8; e++) red[(wave * R + r) * DP + lane * 8 + e] = acc[r][e];
+    }
+    __syncthreads();
+    for (int i = threadIdx.x; i < R * DP; i += 256) red[i] = (red[i] + red[R * DP + i]) + (red[2 * R * DP + i] + red[3 * R * DP + i]);
+    __syncthreads();
+}
+
+// inverse root mean square of a projection (1 when it is not normalised)
+__device__ __forceinline__ float projection_inv(const float *y, uint32_t n, float eps, const float *w, float *scratch)
+{
+    if (!w) return 1.f;
+    float s = 0.f;
+    for (uint32_t i = threadIdx.x; i < n; i += blockDim.x) s = fmaf(y[i], y[i], s);
+    return 1.f / sqrtf(block_sum_waves(s, scratch, blockDim.x >> 6) / (float)n + eps);
+}
+
+// elements 2i, 2i+1 of one head, normalised and rotated
+__device__ __forceinline__ void head_pair(float &u, float &v, const float *y, const float *w, uint32_t base, uint32_t i, uint32_t dim, float inv, const GqaSpec &s,
+                                          uint32_t pos)
+{
+    const uint32_t d = 2 * i;
+    u = d < dim ? y[base + d] * inv * (w ? w[base + d] : 1.f) : 0.f;
+    v = d + 1 < dim ? y[base + d + 1] * inv * (w ? w[base + d + 1] : 1.f) : 0.f;
+    if (d < s.rot_dims) rotate_pair(u, v, s.freq[i], pos);
+}
+
+// One token, one group of R heads that share a kv head, one split of its keys: 256 threads.  The splits of a group meet in the
+// last of them to arrive (see attention_kernel for what the hand-over relies on).  The split that holds the token's own
+// position also appends its rows.
+template <class CT, int DP, int R>
+__device__ __forceinline__ void gqa_step(const GqaStepArgs &a, uint32_t idx, float *lds)
+{
+    const GqaSpec &s = a.s;
+    const uint32_t split = idx % a.splits, grp = idx / a.splits, hg = grp % a.groups, kvh = grp / a.groups;
+    const uint32_t pos = *a.pos_ptr + a.pos_add;
+    const uint32_t c0 = s.chunk ? pos / s.chunk * s.chunk : 0;
+    const uint32_t active = (pos - c0) / kGqaSplit + 1;
+    if (split >= active) return;
+    const uint32_t k_begin = c0 + split * kGqaSplit, n = min((uint32_t)kGqaSplit, pos + 1 - k_begin);
+    const bool own = split == active - 1;
+    const uint32_t per_kv = s.heads / s.kv_heads, h0 = kvh * per_kv + hg * R, nh = min((uint32_t)R, per_kv - hg * R);
+    float *q = lds, *krow = q + R * DP, *vrow = krow + DP, *sc = vrow + DP, *red = sc + R * kGqaSplit, *ml = red + 4 * R * DP, *scratch = ml + 4 * R;
+
+    const float *yq = a.y + s.q_off, *yk = a.y + s.k_off, *yv = a.y + s.v_off;
+    const float inv_q = projection_inv(yq, s.heads * s.dim, s.eps, s.q_norm, scratch);
+    const float inv_k = projection_inv(yk, s.kv_heads * s.dim, s.eps, s.k_norm, scratch);
+    for (uint32_t i = threadIdx.x; i < R * DP / 2; i += 256) {
+        const uint32_t r = i / (DP / 2), p = i % (DP / 2);
+        float u = 0.f, v = 0.f;
+        if (r < nh) head_pair(u, v, yq, s.q_norm, (h0 + r) * s.dim, p, s.dim, inv_q, s, pos);
+        q[r * DP + 2 * p] = u * s.scale;
+        q[r * DP + 2 * p + 1] = v * s.scale;
+    }
+    CT *const kc = static_cast<CT *>(s.kc), *const vc = static_cast<CT *>(s.vc);
+    if (own) {
+        const size_t row = ((size_t)(pos % s.ring) * s.kv_heads + kvh) * DP;
+        for (uint32_t p = threadIdx.x; p < DP / 2; p += 256) {
+            float u, v;
+            head_pair(u, v, yk, s.k_norm, kvh * s.dim, p, s.dim, inv_k, s, pos);
+            const CT cu = float_to_elem<CT>(u), cv = float_to_elem<CT>(v);
+            krow[2 * p] = elem_to_float(cu);
+            krow[2 * p + 1] = elem_to_float(cv);
+            const CT v0 = float_to_elem<CT>(2 * p < s.vdim ? yv[kvh * s.vdim + 2 * p] : 0.f), v1 = float_to_elem<CT>(2 * p + 1 < s.vdim ? yv[kvh * s.vdim + 2 * p + 1] : 0.f);
+            vrow[2 * p] = elem_to_float(v0);
+            vrow[2 * p + 1] = elem_to_float(v1);
+            if (hg == 0) {
+                kc[row + 2 * p] = cu; kc[row + 2 * p + 1] = cv;
+                vc[row + 2 * p] = v0; vc[row + 2 * p + 1] = v1;
+            }
+        }
+    }
+    __syncthreads();
+    auto from = [&](const CT *c, const float *mine, uint32_t j, int d, float (&f)[8]) {
+        const uint32_t p = k_begin + j;
+        if (p == pos) load8(f, mine + d);
+        else load8(f, c + ((size_t)(p % s.ring) * s.kv_heads + kvh) * DP + d);
+    };
+    gqa_scores<DP, R>(q, sc, n, [&](uint32_t j, int d, float (&f)[8]) { from(kc, krow, j, d, f); });
+    __syncthreads();
+    {
+        const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+        for (int r = wave; r < R; r += 4) {
+            float m = -INFINITY, l = 0.f;
+            for (uint32_t j = lane; j < n; j += 64) m = fmaxf(m, sc[r * kGqaSplit + j]);
+#pragma unroll
+            for (int off = 1; off < 64; off <<= 1) m = fmaxf(m, __shfl_xor(m, off, 64));
+            for (uint32_t j = lane; j < n; j += 64) {
+                const float p = __expf(sc[r * kGqaSplit + j] - m);
+                sc[r * kGqaSplit + j] = p;
+                l += p;
+            }
+            l = wave_sum(l);
+            if (lane == 0) { ml[2 * r] = m; ml[2 * r + 1] = l; }
+        }
+    }
+    __syncthreads();
+    float acc[R][8];
+#pragma unroll
+    for (int r = 0; r < R; r++)
+#pragma unroll
+        for (int e = 0; e < 8; e++) acc[r][e] = 0.f;
+    gqa_values<DP, R>(acc, sc, n, [&](uint32_t j, int d, float (&f)[8]) { from(vc, vrow, j, d, f); });
+    gqa_reduce<DP, R>(acc, red);
+
+    if (active == 1) {
+        for (uint32_t i = threadIdx.x; i < nh * s.vdim; i += 256) {
+            const uint32_t r = i / s.vdim, c = i % s.vdim;
+            const float m = ml[2 * r], sk = s.sink ? s.sink[h0 + r] : -INFINITY, M = fmaxf(m, sk);
+            a.out[(h0 + r) * s.vdim + c] = red[r * DP + c] * __expf(m - M) / (ml[2 * r + 1] * __expf(m - M) + __expf(sk - M));
+        }
+        return;
+    }
+    constexpr int PS = R * (DP + 2);
+    uint32_t *part = reinterpret_cast<uint32_t *>(a.part + (size_t)grp * a.splits * PS);
+    for (uint32_t i = threadIdx.x; i < PS; i += 256) {
+        const uint32_t r = i / (DP + 2), c = i % (DP + 2);
+        const float v = c < DP ? red[r * DP + c] : ml[2 * r + (c - DP)];
+        __hip_atomic_store(part + (size_t)split * PS + i, __float_as_uint(v), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    }
+    uint32_t *arrived = reinterpret_cast<uint32_t *>(scratch);
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    __syncthreads();
+    if (threadIdx.x == 0) *arrived = __hip_atomic_fetch_add(&a.counters[grp], 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    __syncthreads();
+    if (*arrived != active - 1) return;
+    auto get = [&](uint32_t sp, uint32_t i) { return __uint_as_float(__hip_atomic_load(part + (size_t)sp * PS + i, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT)); };
+    // per head: the largest score and the sum over the splits, sink included
+    if (threadIdx.x < R) {
+        const uint32_t r = threadIdx.x;
+        const float sk = s.sink && r < nh ? s.sink[h0 + r] : -INFINITY;
+        float M = sk;
+        for (uint32_t sp = 0; sp < active; sp++) M = fmaxf(M, get(sp, r * (DP + 2) + DP));
+        float l = __expf(sk - M);
+        for (uint32_t sp = 0; sp < active; sp++) l += get(sp, r * (DP + 2) + DP + 1) * __expf(get(sp, r * (DP + 2) + DP) - M);
+        ml[2 * r] = M;
+        ml[2 * r + 1] = l;
+    }
+    __syncthreads();
+    for (uint32_t i = threadIdx.x; i < nh * s.vdim; i += 256) {
+        const uint32_t r = i / s.vdim, c = i % s.vdim;
+        float t = 0.f;
+        for (uint32_t sp = 0; sp < active; sp++) t = fmaf(get(sp, r * (DP + 2) + c), __expf(get(sp, r * (DP + 2) + DP) - ml[2 * r]), t);
+        a.out[(h0 + r) * s.vdim + c] = t / ml[2 * r + 1];
+    }
+    if (threadIdx.x == 0) a.counters[grp] = 0u;
+}
+
+// ---- batches -------------------------------------------------------------------------------------------------------------
+struct GqaBatchArgs {
+    GqaSpec s;
+    uint32_t pos0, n;            // the batch's first position and its tokens
+    const void *q;               // [n][heads][DP], normalised, rotated, scaled
+    const void *k, *v;           // [n][kv head][DP]: the batch's own rows
+    void *out;                   // [n][ldo] activations, heads * vdim columns
+    uint32_t ldo, groups;
+    float out_scale;
+};
+
+// One token and head group per workgroup, fp32 arithmetic: the batch form for 32-bit models (and any head size).
+template <class CT, int DP, int R>
+__global__ __launch_bounds__(256) void gqa_rows_kernel(GqaBatchArgs a)
+{
+    extern __shared__ float lds[];
+    const GqaSpec &s = a.s;
+    const uint32_t t = blockIdx.y, hg = blockIdx.x % a.groups, kvh = blockIdx.x / a.groups, pos = a.pos0 + t;
+    const uint32_t per_kv = s.heads / s.kv_heads, h0 = kvh * per_kv + hg * R, nh = min((uint32_t)R, per_kv - hg * R);
+    float *q = lds, *sc = q + R * DP + 2 * DP, *red = sc + R * kGqaSplit, *ml = red + 4 * R * DP;
+    for (uint32_t i = threadIdx.x; i < R * DP; i += 256) {
+        const uint32_t r = i / DP;
+        q[i] = r < nh ? elem_to_float(static_cast<const CT *>(a.q)[((size_t)t * s.heads + h0 + r) * DP + i % DP]) : 0.f;
+    }
+    if (threadIdx.x < R) {     // running maximum, running sum, factor for the sums so far
+        const float sk = s.sink && threadIdx.x < nh ? s.sink[h0 + threadIdx.x] : -INFINITY;
+        ml[4 * threadIdx.x] = sk;
+        ml[4 * threadIdx.x + 1] = s.sink && threadIdx.x < nh ? 1.f : 0.f;
+    }
+    __syncthreads();
+    float acc[R][8];
+#pragma unroll
+    for (int r = 0; r < R; r++)
+#pragma unroll
+        for (int e = 0; e < 8; e++) acc[r][e] = 0.f;
+    const uint32_t c0 = s.chunk ? pos / s.chunk * s.chunk : 0;
+    for (uint32_t k_begin = c0; k_begin <= pos; k_begin += kGqaSplit) {
+        const uint32_t n = min((uint32_t)kGqaSplit, pos + 1 - k_begin);
+        auto from = [&](const void *ring, const void *mine, uint32_t j, int d, float (&f)[8]) {
+            const uint32_t p = k_begin + j;
+            if (p >= a.pos0) load8(f, static_cast<const CT *>(mine) + ((size_t)(p - a.pos0) * s.kv_heads + kvh) * DP + d);
+            else load8(f, static_cast<const CT *>(ring) + ((size_t)(p % s.ring) * s.kv_heads + kvh) * DP + d);
+        };
+        gqa_scores<DP, R>(q, sc, n, [&](uint32_t j, int d, float (&f)[8]) { from(s.kc, a.k, j, d, f); });
+        __syncthreads();
+        const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+        for (int r = wave; r < R; r += 4) {
+            float m = ml[4 * r];
+            const float old = m;
+            for (uint32_t j = lane; j < n; j += 64) m = fmaxf(m, sc[r * kGqaSplit + j]);
+#pragma unroll
+            for (int off = 1; off < 64; off <<= 1) m = fmaxf(m, __shfl_xor(m, off, 64));
+            float l = 0.f;
+            for (uint32_t j = lane; j < n; j += 64) {
+                const float p = __expf(sc[r * kGqaSplit + j] - m);
+                sc[r * kGqaSplit + j] = p;
+                l += p;
+            }
+            l = wave_sum(l);
+            if (lane == 0) {
+                const float f = __expf(old - m);
+                ml[4 * r] = m;
+                ml[4 * r + 1] = ml[4 * r + 1] * f + l;
+                ml[4 * r + 2] = f;
+            }
+        }
+        __syncthreads();
+#pragma unroll
+        for (int r = 0; r < R; r++) {
+            const float f = ml[4 * r + 2];
+#pragma unroll
+            for (int e = 0; e < 8; e++) acc[r][e] *= f;
+        }
+        gqa_values<DP, R>(acc, sc, n, [&](uint32_t j, int d, float (&f)[8]) { from(s.vc, a.v, j, d, f); });
+        __syncthreads();
+    }
+    gqa_reduce<DP, R>(acc, red);
+    for (uint32_t i = threadIdx.x; i < nh * s.vdim; i += 256) {
+        const uint32_t r = i / s.vdim, c = i % s.vdim;
+        static_cast<CT *>(a.out)[(size_t)t * a.ldo + (h0 + r) * s.vdim + c] = float_to_elem<CT>(red[r * DP + c] / ml[4 * r + 1] * a.out_scale);
+    }
+}
+
+}  // namespace lv

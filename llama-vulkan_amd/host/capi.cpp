@@ -86,10 +86,10 @@ unsigned llh_file_detokenize(void *f, const unsigned *ids, unsigned n, char *out
 void *llh_context_new() { return new llava_context; }
 void llh_context_free(void *c) { delete static_cast<llava_context *>(c); }
 // no C++ exception leaves this file: a load that throws (allocation failure) is a failed load
-int llh_context_load(void *c, const char *path, int device)
+int llh_context_load(void *c, const char *path, int device, int compute)
 {
     try {
-        return static_cast<llava_context *>(c)->load_model(path, device) ? 0 : -1;
+        return static_cast<llava_context *>(c)->load_model(path, device, compute) ? 0 : -1;
     } catch (const std::exception &) {
         return -1;
     }
@@ -138,6 +138,10 @@ int llh_session_good(void *s) { return static_cast<llava_session *>(s)->good(); 
 int llh_session_set_text(void *s, const char *t, unsigned n) { return static_cast<llava_session *>(s)->set_text(std::string(t, n)); }
 int llh_session_add_text(void *s, const char *t, unsigned n) { return static_cast<llava_session *>(s)->add_text(std::string(t, n)); }
 int llh_session_push_token(void *s, unsigned t) { return static_cast<llava_session *>(s)->push_token(t); }
+int llh_session_push_tokens(void *s, const unsigned *t, unsigned n) { return static_cast<llava_session *>(s)->push_tokens(t, n); }
+int llh_session_wait(void *s) { return static_cast<llava_session *>(s)->wait(); }
+void llh_session_keep_all_logits(void *s, int on) { static_cast<llava_session *>(s)->keep_all_logits(on != 0); }
+int llh_session_logits_row(void *s, unsigned row, float *dst) { return static_cast<llava_session *>(s)->read_logits_row(row, dst); }
 unsigned llh_session_token_count(void *s) { return static_cast<llava_session *>(s)->get_token_count(); }
 unsigned llh_session_tokens(void *s, unsigned *out, unsigned cap)
 {

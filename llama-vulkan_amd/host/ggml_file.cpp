@@ -17,6 +17,7 @@
 #include <unistd.h>
 #include <utility>
 
+#include "llava_hip.h"
 #include "utils.h"
 
 namespace {
@@ -262,9 +263,9 @@ std::size_t utf8_length(unsigned char first)
 
 }  // namespace
 
-void ggml_file::tokenize(std::vector<u32> &output, const std::string &text, bool bos) const
+bool ggml_file::tokenize(std::vector<u32> &output, const std::string &text, bool bos) const
 {
-    if (text.empty()) return;  // nothing at all, not even the BOS (ggml_file.cpp:251-253)
+    if (text.empty()) return true;  // nothing at all, not even the BOS (ggml_file.cpp:251-253)
     if (bos) output.push_back(1);
 
     // one piece per UTF-8 character (a truncated last character keeps what is there)
@@ -309,6 +310,7 @@ void ggml_file::tokenize(std::vector<u32> &output, const std::string &text, bool
             for (std::size_t j = 0; j < p.len; ++j) output.push_back(static_cast<unsigned char>(text[p.at + j]) + 3u);
         }
     }
+    return true;
 }
 
 std::string ggml_file::tokens_to_text(const u32 *ids, u32 count) const
@@ -317,4 +319,27 @@ std::string ggml_file::tokens_to_text(const u32 *ids, u32 count) const
     for (u32 j = 0; j < count; ++j)
         if (ids[j] < tokens.size()) out += tokens[ids[j]].text;
     return out;
+}
+
+// ---------------------------------------------------------------------------------------------------------------
+// device
+// ---------------------------------------------------------------------------------------------------------------
+u32 ggml_file::trace_floats(int which, u32 backlog) const
+{
+    switch (which) {
+    case LV_TRACE_ATTN: return backlog * header.n_heads;
+    case LV_TRACE_FF: return ff_size;
+    default: return header.dim;
+    }
+}
+
+int ggml_file::upload(lv_ctx *ctx, int, lv_model **out) const
+{
+    // one table entry per tensor record of the file, straight from the descriptors
+    std::vector<lv_tensor_desc> table;
+    table.reserve(tables.size());
+    for (const ggml_data_descriptor &d : tables)
+        table.push_back({d.name.c_str(), static_cast<uint32_t>(d.ftype), d.offset, d.shape1, d.shape2, d.size});
+    const lv_hparams hp = {header.file_version, header.vocab_size, header.dim, header.n_heads, header.n_layers, header.rot, ff_size};
+    return lv_model_upload(ctx, mapping, mapping_size, &hp, table.data(), static_cast<uint32_t>(table.size()), out);
 }

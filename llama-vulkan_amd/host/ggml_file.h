@@ -8,7 +8,7 @@
 #include <unordered_map>
 #include <vector>
 
-#include "types.h"
+#include "model_file.h"
 
 // the nine 32-bit words at the start of the file (ggml_file.h:12-22)
 struct ggml_header {
@@ -36,29 +36,42 @@ public:
     [[nodiscard]] std::size_t size_in_file() const;
 };
 
-class ggml_file {
+class ggml_file : public model_file {
 public:
     explicit ggml_file(const char *filepath);
-    ~ggml_file();
+    ~ggml_file() override;
     ggml_file(const ggml_file &) = delete;
     ggml_file &operator=(const ggml_file &) = delete;
 
-    void print_info() const;
-    void tokenize(std::vector<u32> &output, const std::string &text, bool bos) const;
-    [[nodiscard]] std::string tokens_to_text(const u32 *tokens, u32 count) const;
+    void print_info() const override;
+    bool tokenize(std::vector<u32> &output, const std::string &text, bool bos) const override;   // always true: any bytes have tokens
+    [[nodiscard]] std::string tokens_to_text(const u32 *tokens, u32 count) const override;
     // looks up `s`, then `s + ".weight"`; the name must exist (the reference asserts)
     [[nodiscard]] const ggml_data_descriptor &get_buffer_descriptor(const std::string &s) const;
     [[nodiscard]] const std::vector<ggml_token> &get_tokens() const { return tokens; }
 
     // ---- what the reference exposes to its friend classes -------------------------------------------------
-    [[nodiscard]] bool is_open() const { return mapping != nullptr; }
-    [[nodiscard]] const std::string &error() const { return problem; }   // why is_open() is false
+    [[nodiscard]] bool is_open() const override { return mapping != nullptr; }
+    [[nodiscard]] const std::string &error() const override { return problem; }   // why is_open() is false
     [[nodiscard]] const ggml_header &get_header() const { return header; }
     [[nodiscard]] u32 get_ff_size() const { return ff_size; }
     [[nodiscard]] const u8 *data() const { return mapping; }
     [[nodiscard]] std::size_t data_size() const { return mapping_size; }
     [[nodiscard]] const std::vector<ggml_data_descriptor> &get_tables() const { return tables; }
     [[nodiscard]] const ggml_data_descriptor *find_buffer_descriptor(const std::string &s) const;
+
+    // ---- what sessions ask of any model -------------------------------------------------------------------
+    [[nodiscard]] u32 vocab_size() const override { return header.vocab_size; }
+    [[nodiscard]] u32 layer_count() const override { return header.n_layers; }
+    [[nodiscard]] u32 width() const override { return header.dim; }
+    [[nodiscard]] u32 max_context() const override { return 2048; }    // llava_session.cpp:23-24
+    [[nodiscard]] u32 end_token() const override { return 2; }
+    [[nodiscard]] u32 newline_token() const override { return 13; }    // llava_session.cpp:157-167
+    [[nodiscard]] bool can_rewind() const override { return true; }
+    [[nodiscard]] u32 trace_floats(int which, u32 backlog) const override;
+    [[nodiscard]] std::string token_text(u32 token) const override { return tokens.at(token).text; }
+    int upload(lv_ctx *ctx, int compute, lv_model **out) const override;
+    [[nodiscard]] const ggml_file *as_ggml() const override { return this; }
 
 private:
     bool parse();

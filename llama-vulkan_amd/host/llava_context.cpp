@@ -19,7 +19,6 @@ llava_context::~llava_context()
 {
     if (device_model) lv_model_destroy(device_model);
     if (device_ctx) lv_ctx_destroy(device_ctx);
-    delete model;
 }
 
 bool llava_context::open_model_file(const std::string &path)
@@ -28,50 +27,32 @@ bool llava_context::open_model_file(const std::string &path)
         problem = "a model is already loaded";
         return false;
     }
-    ggml_file *file = new ggml_file(path.c_str());
+    std::unique_ptr<model_file> file = model_file::open(path);
     if (!file->is_open()) {
         problem = file->error();
-        delete file;
         return false;
     }
-    model = file;
+    model = std::move(file);
     return true;
 }
 
-bool llava_context::load_model(const std::string &path, int device)
+bool llava_context::load_model(const std::string &path, int device, int compute)
 {
-    if (model) {
-        problem = "a model is already loaded";
-        return false;
-    }
-    ggml_file *file = new ggml_file(path.c_str());
-    if (!file->is_open()) {
-        problem = file->error();
-        delete file;
-        return false;
-    }
+    if (!open_model_file(path)) return false;
     if (lv_ctx_create(device, &device_ctx) != LV_OK) {
         problem = lv_last_error();
         std::cerr << problem << std::endl;
-        delete file;
+        model.reset();
         return false;
     }
-    // one table entry per tensor record of the file, straight from the descriptors
-    std::vector<lv_tensor_desc> table;
-    table.reserve(file->get_tables().size());
-    for (const ggml_data_descriptor &d : file->get_tables())
-        table.push_back({d.name.c_str(), static_cast<uint32_t>(d.ftype), d.offset, d.shape1, d.shape2, d.size});
-    const ggml_header &h = file->get_header();
-    const lv_hparams hp = {h.file_version, h.vocab_size, h.dim, h.n_heads, h.n_layers, h.rot, file->get_ff_size()};
-    if (lv_model_upload(device_ctx, file->data(), file->data_size(), &hp, table.data(), static_cast<uint32_t>(table.size()), &device_model) != LV_OK) {
+    if (model->upload(device_ctx, compute < 0 ? LV_BF16 : compute, &device_model) != LV_OK) {
         problem = lv_last_error();
         std::cerr << problem << std::endl;
         lv_ctx_destroy(device_ctx);
         device_ctx = nullptr;
-        delete file;
+        model.reset();
         return false;
     }
-    model = file;
     return true;
 }
 
@@ -82,8 +63,10 @@ static void note_interrupt(int) { g_interrupted = 1; }
 
 static void print_usage(const char *argv0)
 {
-    std::cerr << "usage: " << argv0 << " [-m|--model FILE] [--print_header] [--greedy] [--seed N] [-n TOKENS] [-d DEVICE] [-v|--verbose] [-h] [PROMPT]\n"
+    std::cerr << "usage: " << argv0 << " [-m|--model FILE] [--print_header] [--greedy] [--seed N] [-n TOKENS] [-d DEVICE] [--dtype bfloat16|float32] [-v|--verbose] [-h] [PROMPT]\n"
               << "       " << argv0 << " [-m|--model FILE] -s|--server [--port N] [--bind ADDRESS]\n"
+              << "       FILE is a GGJT file or a folder with config.json and model.safetensors; a folder brings no vocabulary, and\n"
+              << "       PROMPT and the output are then token ids.  --dtype applies to folders\n"
               << "       the model path may also come from the LLAVA_MODEL environment variable\n";
 }
 
@@ -97,7 +80,7 @@ int llava_context::run(int argc, char **argv)
     bool print_header = false, greedy = false, have_seed = false, server_mode = false;
     u32 seed = 0, max_new = ~0u, port = 1337;
     std::string bind_address = "0.0.0.0";
-    int device = 0;
+    int device = 0, compute = -1;
     for (int i = 1; i < argc; ++i) {
         const std::string a = argv[i];
         auto value = [&](const char *flag) -> const char * {
@@ -119,6 +102,12 @@ int llava_context::run(int argc, char **argv)
         else if (a == "-m" || a == "--model") { const char *v = value("--model"); if (!v) return 1; path = v; }
         else if (a == "--seed") { const char *v = value("--seed"); if (!v) return 1; seed = static_cast<u32>(std::strtoul(v, nullptr, 0)); have_seed = true; }
         else if (a == "-n") { const char *v = value("-n"); if (!v) return 1; max_new = static_cast<u32>(std::strtoul(v, nullptr, 0)); }
+        else if (a == "--dtype") {
+            const char *v = value("--dtype");
+            if (!v) return 1;
+            compute = std::strcmp(v, "float32") == 0 ? static_cast<int>(LV_F32) : std::strcmp(v, "bfloat16") == 0 ? static_cast<int>(LV_BF16) : -1;
+            if (compute < 0) { std::cerr << "--dtype is bfloat16 or float32" << std::endl; return 1; }
+        }
         else if (a == "-d") { const char *v = value("-d"); if (!v) return 1; device = std::atoi(v); }
         else if (!a.empty() && a[0] == '-') { std::cerr << "Unknown argument " << a << std::endl; print_usage(argv[0]); return 1; }
         else prompt = a;
@@ -134,7 +123,7 @@ int llava_context::run(int argc, char **argv)
     // before the device runtime starts its threads: they inherit the mask (llava_context.cpp:284-287 sets up its
     // signalfd at the same point)
     if (server_mode) lsrv::llava_server::block_termination_signals();
-    if (!load_model(path, device)) return 1;
+    if (!load_model(path, device, compute)) return 1;
     if (print_header) model->print_info();
     if (verbosity) {
         char name[256];
@@ -154,11 +143,11 @@ int llava_context::run(int argc, char **argv)
     if (prompt.empty()) return 0;
 
     // the token loop of llava_context.cpp:336-373
-    const u32 eos_id = 2;
+    const u32 eos_id = model->end_token();
     llava_session session(this);
     if (have_seed) session.set_sampler_seed(seed);
     if (!session.good() || !session.set_text(prompt)) {
-        std::cerr << "[!] System prompt overflows backlog buffer !" << std::endl;
+        std::cerr << (model->as_ggml() ? "[!] System prompt overflows backlog buffer !" : "[!] The prompt is not a list of token ids this model has, or too long") << std::endl;
         return 1;
     }
     g_interrupted = 0;
@@ -178,11 +167,11 @@ int llava_context::run(int argc, char **argv)
             std::cerr << "Cannot start processing, unknown error" << std::endl;
             break;
         }
-        std::cout << model->get_tokens()[next].text << std::flush;  // printed while the device works
+        std::cout << model->token_text(next) << std::flush;  // printed while the device works
         ++produced;
         next = session.finish_next_token_prediction(greedy);
     }
-    if (~next != 0 && next != eos_id && produced < max_new) std::cout << model->get_tokens()[next].text;
+    if (~next != 0 && next != eos_id && produced < max_new) std::cout << model->token_text(next);
     std::cout << std::endl;
     std::signal(SIGINT, old_int);
     std::signal(SIGTERM, old_term);

@@ -3,10 +3,11 @@
 // objects (llava_context.h:15-86); what is left of that class is get_model() and run().
 #pragma once
 
+#include <memory>
 #include <mutex>
 #include <string>
 
-#include "ggml_file.h"
+#include "model_file.h"
 #include "types.h"
 
 struct lv_ctx;
@@ -23,12 +24,13 @@ public:
     int run(int argc, char **argv);
 
     // Opens and uploads a model without going through argv.  False + message on stderr when anything fails.
-    bool load_model(const std::string &path, int device = 0);
+    // compute: LV_BF16 or LV_F32, for models that leave the choice (block models; -1 = their serving precision, bfloat16).
+    bool load_model(const std::string &path, int device = 0, int compute = -1);
     // Opens and parses the file only: vocabulary and tensor table are available, sessions are not (for tools that
     // run without a device).
     bool open_model_file(const std::string &path);
 
-    [[nodiscard]] const ggml_file *get_model() const { return model; }
+    [[nodiscard]] const model_file *get_model() const { return model.get(); }
     [[nodiscard]] lv_ctx *get_device_context() const { return device_ctx; }
     [[nodiscard]] lv_model *get_device_model() const { return device_model; }
     [[nodiscard]] const std::string &last_error() const { return problem; }
@@ -39,7 +41,7 @@ public:
     int verbosity = 0;
 
 private:
-    ggml_file *model = nullptr;
+    std::unique_ptr<model_file> model;
     lv_ctx *device_ctx = nullptr;
     lv_model *device_model = nullptr;
     std::string problem;

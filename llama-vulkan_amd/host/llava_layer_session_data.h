@@ -11,7 +11,9 @@ class llava_layer_session_data {
 public:
     llava_layer_session_data(llava_session *session, u32 layer);
 
-    // K rows then V rows, token_count rows of `dim` fp16 values each (llava_layer_session_data.cpp:165-172)
+    // K rows then V rows, token_count rows of `dim` fp16 values each (llava_layer_session_data.cpp:165-172); of a block model
+    // whatever its layer keeps.  state_bytes: how much that is
+    [[nodiscard]] std::size_t state_bytes(u32 token_count) const;
     void dump_kv_cache(u8 *dst, u32 token_count);
     void restore_kv_cache(const u8 *src, u32 token_count);
     // appends this layer's record-mode buffers to out_fd in the frame format of llava_buffer.cpp:497-522

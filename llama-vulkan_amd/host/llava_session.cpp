@@ -13,27 +13,26 @@
 #include <sys/stat.h>
 #include <unistd.h>
 
+#include "ggml_file.h"
 #include "llava_context.h"
 #include "llava_hip.h"
 #include "utils.h"
 
 namespace {
 
-// llava_session.cpp:23-24: the context grows by doubling between these bounds
+// llava_session.cpp:23-24: the context grows by doubling, from here to the model's max_context()
 constexpr u32 kMinBacklog = 128;
-constexpr u32 kMaxBacklog = 2048;
 
 // record-mode buffers in the order they are dumped, with the names the reference gives them
 // (llava_layer_session_data.cpp:80-85)
-enum class TraceShape { dim, ff, attn };
-struct TraceSlot { int which; const char *name; TraceShape shape; };
+struct TraceSlot { int which; const char *name; };
 constexpr TraceSlot kTraceSlots[] = {
-    {LV_TRACE_ATTN, "attn_result", TraceShape::attn},
-    {LV_TRACE_FF, "ff_result", TraceShape::ff},
-    {LV_TRACE_NORM_IN, "normalized_input_logit", TraceShape::dim},
-    {LV_TRACE_POST_ATTN, "post_attn_logit", TraceShape::dim},
-    {LV_TRACE_POST_ATTN_NORM, "post_attn_norm_logit", TraceShape::dim},
-    {LV_TRACE_OUT, "output_logit", TraceShape::dim},
+    {LV_TRACE_ATTN, "attn_result"},
+    {LV_TRACE_FF, "ff_result"},
+    {LV_TRACE_NORM_IN, "normalized_input_logit"},
+    {LV_TRACE_POST_ATTN, "post_attn_logit"},
+    {LV_TRACE_POST_ATTN_NORM, "post_attn_norm_logit"},
+    {LV_TRACE_OUT, "output_logit"},
 };
 
 // RAII for a file descriptor
@@ -52,27 +51,27 @@ struct Fd {
 // ---------------------------------------------------------------------------------------------------------------
 llava_layer_session_data::llava_layer_session_data(llava_session *s, u32 l) : session(s), layer(l) {}
 
+std::size_t llava_layer_session_data::state_bytes(u32 token_count) const
+{
+    uint64_t bytes = 0;
+    if (lv_state_bytes(session->device_session, layer, token_count, &bytes) != LV_OK) std::cerr << "state_bytes: " << lv_last_error() << std::endl;
+    return bytes;
+}
+
 void llava_layer_session_data::dump_kv_cache(u8 *dst, u32 token_count)
 {
-    const std::size_t plane = static_cast<std::size_t>(token_count) * session->model->get_header().dim * 2;
-    if (lv_kv_read(session->device_session, layer, 0, token_count, dst) != LV_OK ||
-        lv_kv_read(session->device_session, layer, 1, token_count, dst + plane) != LV_OK)
-        std::cerr << "dump_kv_cache: " << lv_last_error() << std::endl;
+    if (lv_state_read(session->device_session, layer, token_count, dst) != LV_OK) std::cerr << "dump_kv_cache: " << lv_last_error() << std::endl;
 }
 
 void llava_layer_session_data::restore_kv_cache(const u8 *src, u32 token_count)
 {
-    const std::size_t plane = static_cast<std::size_t>(token_count) * session->model->get_header().dim * 2;
-    if (lv_kv_write(session->device_session, layer, 0, token_count, src) != LV_OK ||
-        lv_kv_write(session->device_session, layer, 1, token_count, src + plane) != LV_OK)
-        std::cerr << "restore_kv_cache: " << lv_last_error() << std::endl;
+    if (lv_state_write(session->device_session, layer, token_count, src) != LV_OK) std::cerr << "restore_kv_cache: " << lv_last_error() << std::endl;
 }
 
 // One buffer of a frame (llava_buffer.cpp:497-522): u32 shape0, u32 shape1, u32 type, name, zero padding up to a
 // multiple of 32 bytes, then the raw fp32 values.
 void llava_layer_session_data::dump_tracing_layers(int out_fd, const std::string &name)
 {
-    const u32 dim = session->model->get_header().dim, ff = session->model->get_ff_size(), heads = session->model->get_header().n_heads;
     // the rows of the last recorded step; before the first one the reference has no trace buffers at all
     // (llava_layer_session_data.cpp:79) and writes nothing
     u32 rows = 0;
@@ -84,8 +83,10 @@ void llava_layer_session_data::dump_tracing_layers(int out_fd, const std::string
     for (const TraceSlot &slot : kTraceSlots) {
         // shape as the reference's buffers have it: (values per row, rows); attn_result is (backlog, heads x rows).  In
         // memory both are one row of the step after the other.
-        const u32 shape0 = slot.shape == TraceShape::ff ? ff : slot.shape == TraceShape::attn ? session->backlog_size : dim;
-        const u32 shape1 = slot.shape == TraceShape::attn ? heads * rows : rows;
+        const u32 floats = session->model->trace_floats(slot.which, session->backlog_size);
+        if (floats == 0) continue;
+        const u32 shape0 = slot.which == LV_TRACE_ATTN ? session->backlog_size : floats;
+        const u32 shape1 = floats / shape0 * rows;
         const std::size_t count = static_cast<std::size_t>(shape0) * shape1;
         std::vector<float> values(count);
         if (lv_trace_read_rows(session->device_session, layer, slot.which, 0, rows, values.data()) != LV_OK) {
@@ -121,7 +122,7 @@ llava_session::llava_session(llava_context *_ctx)
         device_session = nullptr;
         return;
     }
-    for (u32 i = 0; i < model->get_header().n_layers; ++i) layer_data.push_back(new llava_layer_session_data(this, i));
+    for (u32 i = 0; i < model->layer_count(); ++i) layer_data.push_back(new llava_layer_session_data(this, i));
     recreate_spevars();
 }
 
@@ -146,7 +147,7 @@ void llava_session::set_sampler_seed(u32 seed)
 // llava_session.cpp:303-327
 bool llava_session::set_backlog_size(u32 new_size)
 {
-    if (new_size > kMaxBacklog) return false;
+    if (new_size > model->max_context()) return false;
     if (new_size == backlog_size) return true;
     if (new_size < kMinBacklog || new_size < current_tokens_in_gpu) return false;
     settle_step();
@@ -166,18 +167,25 @@ bool llava_session::set_text(const std::string &new_text)
 {
     if (!good()) return false;
     std::vector<u32> fresh;
-    model->tokenize(fresh, new_text, true);
+    if (!model->tokenize(fresh, new_text, true)) return false;
     u32 wanted = backlog_size;
     while (fresh.size() > wanted) wanted <<= 1;
-    if (wanted > kMaxBacklog || !set_backlog_size(wanted)) return false;
+    if (wanted > model->max_context() || !set_backlog_size(wanted)) return false;
     u32 keep = 0;
     while (keep < fresh.size() && keep < token_buffer.size() && keep < current_tokens_in_gpu && token_buffer[keep] == fresh[keep]) ++keep;
     // the last token of the new text is always evaluated again: the logits on the device then belong to this text, also
     // when it is a prefix of what was evaluated before (the reference re-evaluates in that case too)
     if (!fresh.empty() && keep == fresh.size()) --keep;
+    settle_step();
     token_buffer = std::move(fresh);
-    current_tokens_in_gpu = keep;
+    back_to(keep);
     return true;
+}
+
+// The evaluated prefix shrinks to `position` tokens.  A state that only moves forward has to be built again from the start.
+void llava_session::back_to(u32 position)
+{
+    if (position < current_tokens_in_gpu) current_tokens_in_gpu = model->can_rewind() ? position : 0;
 }
 
 // llava_session.cpp:279-282
@@ -189,11 +197,23 @@ bool llava_session::add_text(const std::string &s)
 // llava_session.cpp:284-297
 bool llava_session::push_token(u32 token)
 {
-    if (!good() || token >= model->get_tokens().size()) return false;
+    if (!good() || token >= model->vocab_size()) return false;
     if (token_buffer.size() == backlog_size) {
-        if (backlog_size == kMaxBacklog || !set_backlog_size(backlog_size * 2)) return false;
+        if (backlog_size == model->max_context() || !set_backlog_size(backlog_size * 2)) return false;
     }
     token_buffer.push_back(token);
+    return true;
+}
+
+bool llava_session::push_tokens(const u32 *tokens, std::size_t count)
+{
+    if (!good()) return false;
+    for (std::size_t i = 0; i < count; ++i)
+        if (tokens[i] >= model->vocab_size()) return false;
+    u64 wanted = backlog_size;
+    while (token_buffer.size() + count > wanted) wanted <<= 1;
+    if (wanted > model->max_context() || !set_backlog_size(static_cast<u32>(wanted))) return false;
+    token_buffer.insert(token_buffer.end(), tokens, tokens + count);
     return true;
 }
 
@@ -202,7 +222,7 @@ void llava_session::rewind(u32 n)
 {
     if (n < token_buffer.size()) {
         token_buffer.resize(n);
-        current_tokens_in_gpu = std::min(n, current_tokens_in_gpu);
+        back_to(n);
     }
 }
 
@@ -230,6 +250,8 @@ bool llava_session::start_next_token_prediction()
     }
     if (lv_step_begin(device_session, token_buffer.data() + current_tokens_in_gpu, to_process, current_tokens_in_gpu) != LV_OK) {
         std::cerr << "start_next_token_prediction: " << lv_last_error() << std::endl;
+        u32 at = current_tokens_in_gpu;
+        if (!model->can_rewind() && (lv_session_position(device_session, &at) != LV_OK || at != current_tokens_in_gpu)) back_to(0);
         return false;
     }
     step_in_flight = true;
@@ -243,7 +265,7 @@ bool llava_session::start_next_token_prediction()
 // start evaluates the same tokens into the same rows.
 void llava_session::step_failed()
 {
-    current_tokens_in_gpu = std::min(current_tokens_in_gpu, step_first_row);
+    back_to(step_first_row);
 }
 
 // waits for a step that was started and never finished; false when that step failed
@@ -256,6 +278,16 @@ bool llava_session::settle_step()
     step_failed();
     return false;
 }
+
+bool llava_session::wait() { return good() && settle_step(); }
+
+void llava_session::keep_all_logits(bool on)
+{
+    settle_step();
+    if (good() && lv_session_set_all_logits(device_session, on) != LV_OK) std::cerr << "keep_all_logits: " << lv_last_error() << std::endl;
+}
+
+bool llava_session::read_logits_row(u32 row, float *dst) { return wait() && lv_logits_read_rows(device_session, row, 1, dst) == LV_OK; }
 
 // llava_session.cpp:231-234; the reference always samples stochastically here
 u32 llava_session::finish_next_token_prediction(bool deterministic)
@@ -274,7 +306,7 @@ u32 llava_session::predict_next_token(bool deterministic)
 // llava_session.cpp:114-195
 u32 llava_session::get_last_predicted_token(bool deterministic)
 {
-    const u32 n_vocab = model->get_header().vocab_size;
+    const u32 n_vocab = model->vocab_size();
     last_logits.resize(n_vocab);
     const int rc = lv_logits_read(device_session, last_logits.data());  // waits for the step
     const bool was_in_flight = step_in_flight;
@@ -298,20 +330,20 @@ u32 llava_session::get_last_predicted_token(bool deterministic)
         return best;
     }
 
-    return sample_token(std::move(p), token_buffer.data(), token_buffer.size(), mirostat_mu, rng);
+    return sample_token(std::move(p), token_buffer.data(), token_buffer.size(), mirostat_mu, rng, nullptr, model->newline_token());
 }
 
 // llava_session.cpp:154-194
-u32 llava_session::sample_token(std::vector<float> p, const u32 *history, std::size_t history_size, float &mu, std::mt19937 &rng, sampler_probe *probe)
+u32 llava_session::sample_token(std::vector<float> p, const u32 *history, std::size_t history_size, float &mu, std::mt19937 &rng, sampler_probe *probe, u32 newline)
 {
     const u32 n_vocab = static_cast<u32>(p.size());
     // repetition / frequency penalty, applied to the newline token only (:157-167)
     std::map<u32, u32> recent;
     const std::size_t from = history_size > repeat_last_n ? history_size - repeat_last_n : 0;
     for (std::size_t i = from; i < history_size; ++i) recent[history[i]]++;
-    const auto nl = recent.find(13);
-    if (nl != recent.end() && 13 < n_vocab) {
-        float &l = p[13];
+    const auto nl = recent.find(newline);
+    if (nl != recent.end() && newline < n_vocab) {
+        float &l = p[newline];
         l = l <= 0 ? l * repeat_penalty : l / repeat_penalty;
         l -= alpha_frequency * static_cast<float>(nl->second) + alpha_presence;
     }
@@ -355,9 +387,11 @@ u32 llava_session::sample_token(std::vector<float> p, const u32 *history, std::s
 void llava_session::recreate_spevars()
 {
     specialization_variables_t &sv = specialization_variables;
-    const ggml_header &h = model->get_header();
-    const u32 wgs = ctx->workgroup_size, ff = model->get_ff_size();
     sv = {};
+    const ggml_file *const ggml = model->as_ggml();
+    if (!ggml) return;
+    const ggml_header &h = ggml->get_header();
+    const u32 wgs = ctx->workgroup_size, ff = ggml->get_ff_size();
     sv.head_count = h.n_heads;
     sv.rot = h.rot;
     sv.quarterrot = h.rot / 4;
@@ -411,16 +445,16 @@ ReturnCode llava_session::save_frame(const std::string &path)
 }
 
 // ---------------------------------------------------------------------------------------------------------------
-// snapshot / restore: u32 n, u32 tokens[n], then per layer K f16[n][dim] followed by V f16[n][dim]
+// snapshot / restore: u32 n, u32 tokens[n], then per layer K f16[n][dim] followed by V f16[n][dim] (block models: lv_state_read)
 // (llava_session.cpp:447-603, llava_layer_session_data.cpp:165-181)
 // ---------------------------------------------------------------------------------------------------------------
 ReturnCode llava_session::snapshot(const std::string &path)
 {
     if (!good()) return ReturnCode::nok;
     settle_step();
-    const u32 n = current_tokens_in_gpu, dim = model->get_header().dim;
-    const std::size_t per_layer = static_cast<std::size_t>(2) * n * dim * 2;
-    const std::size_t total = layer_data.size() * per_layer + 4 * static_cast<std::size_t>(n) + 4;
+    const u32 n = current_tokens_in_gpu;
+    std::size_t total = 4 * static_cast<std::size_t>(n) + 4;
+    for (const llava_layer_session_data *l : layer_data) total += l->state_bytes(n);
     Fd out(::open(path.c_str(), O_RDWR | O_CREAT | O_TRUNC, 0644));
     if (out.fd < 0) {
         std::perror("open");
@@ -441,7 +475,7 @@ ReturnCode llava_session::snapshot(const std::string &path)
     u8 *cursor = bytes + 4 + static_cast<std::size_t>(n) * 4;
     for (llava_layer_session_data *l : layer_data) {
         l->dump_kv_cache(cursor, n);
-        cursor += per_layer;
+        cursor += l->state_bytes(n);
     }
     if (msync(map, total, MS_SYNC) < 0) std::perror("msync");
     if (munmap(map, total) < 0) std::perror("munmap");
@@ -479,20 +513,20 @@ ReturnCode llava_session::restore(const std::string &path)
     const u8 *bytes = static_cast<const u8 *>(map);
     u32 n;
     std::memcpy(&n, bytes, 4);
-    if (n > kMaxBacklog) {
+    if (n > model->max_context()) {
         std::cerr << "Too many tokens" << std::endl;
         return ReturnCode::nok;
     }
-    const u32 dim = model->get_header().dim;
-    const std::size_t per_layer = static_cast<std::size_t>(2) * n * dim * 2;
-    if (layer_data.size() * per_layer + 4 * static_cast<std::size_t>(n) + 4 != size) {
+    std::size_t total = 4 * static_cast<std::size_t>(n) + 4;
+    for (const llava_layer_session_data *l : layer_data) total += l->state_bytes(n);
+    if (total != size) {
         std::cerr << "File size mismatch" << std::endl;
         return ReturnCode::nok;
     }
     std::vector<u32> toks(n);
     if (n) std::memcpy(toks.data(), bytes + 4, static_cast<std::size_t>(n) * 4);
     for (u32 t : toks)
-        if (t >= model->get_tokens().size()) {
+        if (t >= model->vocab_size()) {
             std::cerr << "Token id outside the vocabulary" << std::endl;
             return ReturnCode::nok;
         }
@@ -509,7 +543,7 @@ ReturnCode llava_session::restore(const std::string &path)
     const u8 *cursor = bytes + 4 + static_cast<std::size_t>(n) * 4;
     for (llava_layer_session_data *l : layer_data) {
         l->restore_kv_cache(cursor, n);
-        cursor += per_layer;
+        cursor += l->state_bytes(n);
     }
     return ReturnCode::ok;
 }

@@ -8,7 +8,7 @@
 #include <string>
 #include <vector>
 
-#include "ggml_file.h"
+#include "model_file.h"
 #include "llava_layer_session_data.h"
 #include "types.h"
 
@@ -37,6 +37,7 @@ public:
     [[nodiscard]] bool set_text(const std::string &new_text);
     [[nodiscard]] bool add_text(const std::string &s);
     [[nodiscard]] bool push_token(u32 token);
+    [[nodiscard]] bool push_tokens(const u32 *tokens, std::size_t count);   // all of them or none
     [[nodiscard]] u32 get_token_count() const { return static_cast<u32>(token_buffer.size()); }
     [[nodiscard]] const std::vector<u32> &get_token_buffer() const { return token_buffer; }
 
@@ -45,6 +46,11 @@ public:
     [[nodiscard]] bool start_next_token_prediction();
     [[nodiscard]] u32 finish_next_token_prediction(bool deterministic = false);
     [[nodiscard]] u32 predict_next_token(bool deterministic = false);
+    // ends a step without sampling: the wait alone, or the logits of chosen rows of it (row z = its z-th token), which
+    // keep_all_logits has to have been switched on for before the step started
+    [[nodiscard]] bool wait();
+    void keep_all_logits(bool on);
+    [[nodiscard]] bool read_logits_row(u32 row, float *dst);
 
     [[nodiscard]] const specialization_variables_t &get_spevar_struct() const { return specialization_variables; }
     [[nodiscard]] bool is_tracing_enabled() const { return options != 0; }
@@ -66,7 +72,8 @@ public:
     };
     // The stochastic branch of get_last_predicted_token (llava_session.cpp:154-194) as a function of its inputs: the logits
     // (taken by value, they are overwritten), the token history, the running mu and the generator.
-    static u32 sample_token(std::vector<float> p, const u32 *history, std::size_t history_size, float &mu, std::mt19937 &rng, sampler_probe *probe = nullptr);
+    static u32 sample_token(std::vector<float> p, const u32 *history, std::size_t history_size, float &mu, std::mt19937 &rng, sampler_probe *probe = nullptr,
+                            u32 newline = 13);
     void set_sampler_seed(u32 seed);                       // the reference seeds with time(nullptr)
     [[nodiscard]] u32 get_backlog_size() const { return backlog_size; }
     [[nodiscard]] u32 get_tokens_in_gpu() const { return current_tokens_in_gpu; }
@@ -75,11 +82,12 @@ public:
     [[nodiscard]] bool good() const { return device_session != nullptr; }
 
     llava_context *const ctx;
-    const ggml_file *const model;
+    const model_file *const model;
 
 private:
     [[nodiscard]] u32 get_last_predicted_token(bool deterministic);
     [[nodiscard]] bool set_backlog_size(u32 new_size);
+    void back_to(u32 position);
     void recreate_spevars();
     void step_failed();
     bool settle_step();

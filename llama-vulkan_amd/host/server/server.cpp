@@ -15,7 +15,7 @@
 #include <sys/socket.h>
 #include <unistd.h>
 
-#include "../ggml_file.h"
+#include "../model_file.h"
 #include "../llava_context.h"
 #include "session_wrapper.h"
 
@@ -36,10 +36,11 @@ llava_server::llava_server(llava_context *context, u16 _port, std::string _bind_
     : ctx(context), port(_port), bind_address(std::move(_bind_address))
 {
     // the vocabulary never changes: build the cmdGetTokenMap answer once (server/server.cpp:29-42)
-    if (const ggml_file *model = ctx->get_model())
-        for (const ggml_token &token : model->get_tokens()) {
-            put_u32(token_map_payload, static_cast<u32>(token.text.size()));
-            token_map_payload.insert(token_map_payload.end(), token.text.begin(), token.text.end());
+    if (const model_file *model = ctx->get_model())
+        for (u32 token = 0; token < model->vocab_size(); ++token) {
+            const std::string text = model->token_text(token);
+            put_u32(token_map_payload, static_cast<u32>(text.size()));
+            token_map_payload.insert(token_map_payload.end(), text.begin(), text.end());
         }
 }
 

@@ -22,6 +22,7 @@ enum class ReturnCode : u32 {
     not_tracing = 5, batched_tick = 6, bad_arguments = 7, unknown_command = 8,
 };
 
+class model_file;
 class ggml_file;
 class llava_context;
 class llava_session;

@@ -29,13 +29,14 @@ def lib():
             "llh_file_tensor": (C.c_int, [vp, cp, C.POINTER(u), C.POINTER(C.c_ulonglong), C.POINTER(u), C.POINTER(u), C.POINTER(C.c_ulonglong)]),
             "llh_file_token": (u, [vp, u, cp, u, C.POINTER(C.c_float)]),
             "llh_file_tokenize": (u, [vp, cp, u, C.c_int, C.POINTER(u), u]), "llh_file_detokenize": (u, [vp, C.POINTER(u), u, cp, u]),
-            "llh_context_new": (vp, []), "llh_context_free": (None, [vp]), "llh_context_load": (C.c_int, [vp, cp, C.c_int]),
+            "llh_context_new": (vp, []), "llh_context_free": (None, [vp]), "llh_context_load": (C.c_int, [vp, cp, C.c_int, C.c_int]),
             "llh_context_error": (u, [vp, cp, u]), "llh_context_run": (C.c_int, [vp, C.c_int, C.POINTER(cp)]),
             "llh_context_open_file": (C.c_int, [vp, cp]),
             "llh_server_start": (vp, [vp, C.c_ushort, cp]), "llh_server_port": (u, [vp]), "llh_server_stop": (None, [vp]),
             "llh_session_new": (vp, [vp]), "llh_session_free": (None, [vp]), "llh_session_good": (C.c_int, [vp]),
             "llh_session_set_text": (C.c_int, [vp, cp, u]), "llh_session_add_text": (C.c_int, [vp, cp, u]),
-            "llh_session_push_token": (C.c_int, [vp, u]), "llh_session_token_count": (u, [vp]), "llh_session_tokens": (u, [vp, C.POINTER(u), u]),
+            "llh_session_push_token": (C.c_int, [vp, u]), "llh_session_push_tokens": (C.c_int, [vp, C.POINTER(u), u]), "llh_session_wait": (C.c_int, [vp]),
+            "llh_session_keep_all_logits": (None, [vp, C.c_int]), "llh_session_logits_row": (C.c_int, [vp, u, C.c_void_p]), "llh_session_token_count": (u, [vp]), "llh_session_tokens": (u, [vp, C.POINTER(u), u]),
             "llh_session_start": (C.c_int, [vp]), "llh_session_finish": (u, [vp, C.c_int]), "llh_session_predict": (u, [vp, C.c_int]),
             "llh_session_rewind": (None, [vp, u]), "llh_session_set_options": (u, [vp, u]), "llh_session_is_tracing": (C.c_int, [vp]),
             "llh_session_save_frame": (u, [vp, cp]), "llh_session_snapshot": (u, [vp, cp]), "llh_session_restore": (u, [vp, cp]),
@@ -134,8 +135,9 @@ class LlavaContext:
     def __init__(self):
         self.h = lib().llh_context_new()
 
-    def load_model(self, path, device=0):
-        return lib().llh_context_load(self.h, os.fsencode(path), device) == 0
+    def load_model(self, path, device=0, compute=-1):
+        """compute: LV_BF16 or LV_F32 for block models (-1 = the serving precision)"""
+        return lib().llh_context_load(self.h, os.fsencode(path), device, compute) == 0
 
     def open_model_file(self, path):
         """parse only: vocabulary and tensor table, no device"""
@@ -189,6 +191,22 @@ class LlavaSession:
 
     def push_token(self, t):
         return bool(lib().llh_session_push_token(self.h, int(t)))
+
+    def push_tokens(self, tokens):
+        arr = (C.c_uint * max(len(tokens), 1))(*[int(t) for t in tokens])
+        return bool(lib().llh_session_push_tokens(self.h, arr, len(tokens)))
+
+    def wait(self):
+        return bool(lib().llh_session_wait(self.h))
+
+    def keep_all_logits(self, on=True):
+        lib().llh_session_keep_all_logits(self.h, int(on))
+
+    def logits_row(self, row, vocab):
+        out = np.empty(vocab, dtype=np.float32)
+        if not lib().llh_session_logits_row(self.h, row, out.ctypes.data_as(C.c_void_p)):
+            raise RuntimeError("logits row not readable")
+        return out
 
     def token_count(self):
         return lib().llh_session_token_count(self.h)

@@ -9,6 +9,7 @@ import subprocess
 import numpy as np
 import pytest
 
+import block_builder as bb
 import ggjt_builder as gb
 
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
@@ -21,8 +22,8 @@ def driver(tmp_path_factory):
         pytest.skip("no g++")
     exe = str(tmp_path_factory.mktemp("san") / "host_sanitize")
     cmd = ["g++", "-std=c++17", "-O1", "-g", "-fsanitize=address,undefined", "-fno-sanitize-recover=all", "-static-libasan",
-           "-static-libubsan", "-I", HOST, os.path.join(ROOT, "tests", "host_sanitize_main.cpp"), os.path.join(HOST, "ggml_file.cpp"),
-           os.path.join(HOST, "utils.cpp"), "-o", exe]
+           "-static-libubsan", "-I", HOST, "-I", os.path.join(ROOT, "include"), os.path.join(ROOT, "tests", "host_sanitize_main.cpp"),
+           *[os.path.join(HOST, f) for f in ("ggml_file.cpp", "utils.cpp", "json.cpp", "safetensors.cpp", "block_model_file.cpp", "block_designs.cpp")], "-o", exe]
     r = subprocess.run(cmd, capture_output=True, text=True)
     if r.returncode != 0:
         pytest.skip("sanitizer build unavailable here: " + r.stderr[-400:])
@@ -31,7 +32,7 @@ def driver(tmp_path_factory):
 
 def run(exe, paths):
     env = dict(os.environ, ASAN_OPTIONS="detect_leaks=1:abort_on_error=0", UBSAN_OPTIONS="halt_on_error=1:print_stacktrace=1")
-    return subprocess.run([exe, *paths], capture_output=True, text=True, env=env, timeout=300)
+    return subprocess.run([exe, *paths], capture_output=True, text=True, errors="replace", env=env, timeout=300)
 
 
 def test_parser_and_tokenizer_under_sanitizers(driver, tmp_path):
@@ -80,3 +81,33 @@ def test_parser_and_tokenizer_under_sanitizers(driver, tmp_path):
     assert "opened" in r.stdout
     opened = int(r.stdout.split()[1])
     assert 1 <= opened < len(paths)        # the valid file parses; the truncated ones cannot all parse
+
+
+def test_model_folder_under_sanitizers(driver, tmp_path):
+    """the same for a folder of config.json and model.safetensors: both files cut short, and bytes of either changed"""
+    cfg = bb.config(vocab=40, width=20, layers=[bb.layer(), bb.layer(experts=0)])
+    good = str(tmp_path / "good.folder")
+    bb.write_folder(good, cfg, seed=3)
+    parts = {n: np.fromfile(os.path.join(good, n), dtype=np.uint8) for n in ("config.json", "model.safetensors")}
+    head = int(parts["model.safetensors"][:8].view(np.uint64)[0]) + 8
+    rng = np.random.default_rng(11)
+    paths = [good]
+    for k in range(160):
+        name = "config.json" if k % 2 else "model.safetensors"
+        data = parts[name].copy()
+        zone = len(data) if k % 2 else head
+        if k < 40:
+            data = data[:int(rng.integers(0, zone + 1))]
+        elif k < 100:
+            data[int(rng.integers(0, zone))] = rng.integers(0, 256)
+        else:
+            data[int(rng.integers(0, zone))] = ord(rng.choice(list("[]{}\",:9-e0")))
+        p = str(tmp_path / f"m{k}.folder")
+        os.mkdir(p)
+        for n, d in parts.items():
+            (data if n == name else d).tofile(os.path.join(p, n))
+        paths.append(p)
+    r = run(driver, paths)
+    assert r.returncode == 0, (r.stdout[-500:], r.stderr[-3000:])
+    opened = int(r.stdout.split()[1])
+    assert 1 <= opened < len(paths)
