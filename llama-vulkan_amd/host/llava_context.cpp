@@ -153,7 +153,7 @@ int llava_context::run(int argc, char **argv)
     g_interrupted = 0;
     auto old_int = std::signal(SIGINT, note_interrupt);
     auto old_term = std::signal(SIGTERM, note_interrupt);
-    std::cout << prompt << std::flush;
+    std::cout << (model->as_ggml() ? prompt : model->tokens_to_text(session.get_token_buffer().data(), session.get_token_count())) << std::flush;
     u32 next = session.predict_next_token(greedy);
     u32 produced = 0;
     while (true) {

@@ -397,8 +397,6 @@ def test_greedy_generation_through_the_session_class(hostlib, folder):
     s.rewind(len(prompt) + 5)
     assert s.tokens_in_gpu() == 0 and s.predict(True) == want[5]
     # more text goes on from where the state stands; other text starts anew
-    s.rewind(len(prompt) + 5)
-    assert s.predict(True) == want[5]
     at = s.tokens_in_gpu()
     assert s.add_text(b"4, 5") and s.tokens_in_gpu() == at
     assert s.predict(True) == bo.greedy(prompt + want[:5] + [4, 5], 1, F, cfg)[0]
