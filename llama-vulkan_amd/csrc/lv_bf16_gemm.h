@@ -92,6 +92,14 @@ __device__ __forceinline__ void bf_store4(const BfGemmArgs &a, uint32_t orow, ui
     if (row >= a.rows) return;
     float r[4] = {v[0], v[1], v[2], v[3]};
     if constexpr (EP == kEpDecay) {
+        if (a.head_dim % 4 == 0) {      // the four rows belong to one head
+            const uint32_t h = row / a.head_dim, d = row - h * a.head_dim;
+            const float ea = expf(a.a_log[h]);
+            const float4 b = *reinterpret_cast<const float4 *>(a.bias + row);
+            *reinterpret_cast<float4 *>(a.out + (size_t)orow * a.ldo + h * a.head_stride + d) =
+                make_float4(expf(-ea * softplus_f(r[0] + b.x)), expf(-ea * softplus_f(r[1] + b.y)), expf(-ea * softplus_f(r[2] + b.z)), expf(-ea * softplus_f(r[3] + b.w)));
+            return;
+        }
 #pragma unroll
         for (int i = 0; i < 4; i++)
             if (row + i < a.rows) {
@@ -118,8 +126,13 @@ template <class T>
 __device__ __forceinline__ void bf_store_glu(const BfGemmArgs &a, uint32_t position, uint32_t f, float wt, const lv_f4 g, const lv_f4 u)
 {
     T *o = static_cast<T *>(a.act) + (size_t)position * a.lda + f;
+    float v[4];
 #pragma unroll
-    for (int i = 0; i < 4; i++) o[i] = float_to_elem<T>(silu_f(wt * g[i]) * (wt * u[i]));
+    for (int i = 0; i < 4; i++) v[i] = silu_f(wt * g[i]) * (wt * u[i]);
+    if constexpr (sizeof(T) == 2)
+        *reinterpret_cast<uint2 *>(o) = make_uint2((uint32_t)float_to_bf16(v[0]) | ((uint32_t)float_to_bf16(v[1]) << 16),
+                                                   (uint32_t)float_to_bf16(v[2]) | ((uint32_t)float_to_bf16(v[3]) << 16));
+    else *reinterpret_cast<float4 *>(o) = make_float4(v[0], v[1], v[2], v[3]);
 }
 
 // Tile of this workgroup: workgroups are dealt to the 8 XCDs in turn; an XCD takes every eighth row tile and walks the token

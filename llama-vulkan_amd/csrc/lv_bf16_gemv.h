@@ -68,6 +68,25 @@ __device__ __forceinline__ float block_sum_waves(float v, float *scratch, int nw
     return t;
 }
 
+// the same for N values at once; scratch holds N * nw floats
+template <int N>
+__device__ __forceinline__ void block_sums_waves(float (&v)[N], float *scratch, int nw)
+{
+#pragma unroll
+    for (int i = 0; i < N; i++) v[i] = wave_sum(v[i]);
+    __syncthreads();
+    if ((threadIdx.x & 63) == 0) {
+#pragma unroll
+        for (int i = 0; i < N; i++) scratch[i * nw + (threadIdx.x >> 6)] = v[i];
+    }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < N; i++) {
+        v[i] = 0.f;
+        for (int w = 0; w < nw; w++) v[i] += scratch[i * nw + w];
+    }
+}
+
 // NormInput into xs; every thread keeps to its own elements between the passes
 __device__ __forceinline__ void norm_input(const NormInput &a, float *xs, float *scratch)
 {

@@ -71,7 +71,7 @@ struct Workspace {                     // of batches; sized for `cap` tokens
           *gate = nullptr, *z = nullptr, *scores = nullptr;
     void *act = nullptr, *q = nullptr, *k = nullptr, *v = nullptr, *vt = nullptr, *a1 = nullptr, *g1 = nullptr, *cat = nullptr, *ff = nullptr;
     uint32_t *ids = nullptr, *slots = nullptr, *tiles = nullptr;
-    uint32_t vt_keys = 0;
+    uint64_t vt_elems = 0;
 };
 
 struct BlockSession {
@@ -485,7 +485,7 @@ static void workspace_free(Workspace &w)
     for (void **p : {&w.act, &w.q, &w.k, &w.v, &w.vt, &w.a1, &w.g1, &w.cat, &w.ff}) drop(*p);
     for (uint32_t **p : {&w.ids, &w.slots, &w.tiles}) drop(*p);
     w.cap = 0;
-    w.vt_keys = 0;
+    w.vt_elems = 0;
 }
 
 void block_session_destroy(BlockSession *s)
@@ -525,7 +525,7 @@ int block_session_reserve(BlockSession *s, uint32_t positions)
         if (!l.attn) continue;
         LayerState &ls = s->layers[i];
         const uint32_t ring = l.spec.attn.chunk ? std::min(l.spec.attn.chunk, positions) : positions;
-        const uint64_t splits = (ring + kGqaSplit - 1) / kGqaSplit;
+        const uint64_t splits = (ring + gqa_split(l.dp) - 1) / gqa_split(l.dp);
         part = std::max<uint64_t>(part, l.spec.attn.kv_heads * l.groups * splits * l.r * (l.dp + 2));
         if (ring == ls.ring) continue;
         // A ring that grows has not wrapped yet (it held every position so far), and one that shrinks keeps the rows that
@@ -704,7 +704,7 @@ int block_step_token(BlockSession *s, const uint32_t *cfg, uint32_t idx, float *
         mx.attn.s = gqa_spec(s, i);
         mx.attn.y = s->y1; mx.attn.pos_ptr = cfg; mx.attn.pos_add = idx;
         mx.attn.groups = l.groups;
-        mx.attn.splits = l.attn ? (s->layers[i].ring + kGqaSplit - 1) / kGqaSplit : 1;
+        mx.attn.splits = l.attn ? (s->layers[i].ring + gqa_split(l.dp) - 1) / gqa_split(l.dp) : 1;
         mx.attn.part = s->part; mx.attn.counters = s->counters; mx.attn.out = s->left;
         const uint32_t wgs = mx.delta_wgs + (l.attn ? l.spec.attn.kv_heads * l.groups * mx.attn.splits : 0);
         LV_TRY(gqa_dispatch(m->f32, l, [&](auto elem, auto dp, auto r) -> int {
@@ -822,6 +822,44 @@ template <class T> static int norm_rows(hipStream_t st, const NormRowsArgs &a, u
     return LV_OK;
 }
 
+// attention of a batch on the matrix cores: the transposed values, then the tiles
+static int gqa_tiles(BlockSession *s, const BlockLayer &l, const GqaBatchArgs &b)
+{
+    GqaTileArgs a{};
+    a.b = b;
+    a.base = b.s.chunk ? b.pos0 / b.s.chunk * b.s.chunk : 0;
+    a.keys = b.pos0 + b.n - a.base;
+    a.vt_ld = up(a.keys, kTileKeys);
+    Workspace &w = s->ws;
+    const uint64_t need = (uint64_t)b.s.kv_heads * l.dp * a.vt_ld;
+    if (need > w.vt_elems) {
+        HIP_TRY(hipStreamSynchronize(s->st));
+        drop(w.vt);
+        w.vt_elems = 0;
+        LV_TRY(dev_alloc(&w.vt, need * 2));
+        w.vt_elems = need;
+    }
+    a.vt = static_cast<uint16_t *>(w.vt);
+    auto run = [&](auto dp, auto qt) -> int {
+        constexpr int DP = decltype(dp)::value, QT = decltype(qt)::value;
+        gqa_values_kernel<DP><<<dim3(b.s.kv_heads, a.vt_ld / kTileKeys), dim3(256), 0, s->st>>>(a);
+        HIP_TRY(hipGetLastError());
+        auto *k = &gqa_tile_kernel<DP, QT>;
+        LV_TRY(allow_lds(k, gqa_tile_lds<DP>()));
+        k<<<dim3(b.s.heads, (b.n + 64 * QT - 1) / (64 * QT)), dim3(256), gqa_tile_lds<DP>(), s->st>>>(a);
+        HIP_TRY(hipGetLastError());
+        return LV_OK;
+    };
+    using std::integral_constant;
+    // two query tiles a wave halve the LDS reads per product; few queries are better spread over more workgroups
+    const bool wide = (uint64_t)b.n * b.s.heads >= 128 * 256;
+    switch (l.dp) {
+    case 64: return wide ? run(integral_constant<int, 64>{}, integral_constant<int, 2>{}) : run(integral_constant<int, 64>{}, integral_constant<int, 1>{});
+    case 128: return wide ? run(integral_constant<int, 128>{}, integral_constant<int, 2>{}) : run(integral_constant<int, 128>{}, integral_constant<int, 1>{});
+    default: return run(integral_constant<int, 256>{}, integral_constant<int, 1>{});
+    }
+}
+
 template <class T>
 static int step_batch(BlockSession *s, const uint32_t *tokens, uint32_t pos, uint32_t row0, uint32_t n, float *logits_last, float *logits_all, const BlockTrace *trace)
 {
@@ -873,14 +911,18 @@ static int step_batch(BlockSession *s, const uint32_t *tokens, uint32_t pos, uin
             GqaBatchArgs a{};
             a.s = p.attn; a.pos0 = pos; a.n = n; a.q = w.q; a.k = w.k; a.v = w.v; a.out = w.cat; a.ldo = l.out.kp; a.groups = l.groups;
             a.out_scale = l.spec.attn_scale;
-            LV_TRY(gqa_dispatch(f32, l, [&](auto elem, auto dp, auto r) -> int {
-                constexpr int DP = decltype(dp)::value, R = decltype(r)::value;
-                if constexpr (std::is_same_v<decltype(elem), T>) {
-                    gqa_rows_kernel<T, DP, R><<<dim3(l.spec.attn.kv_heads * l.groups, n), dim3(256), 4 * gqa_lds_floats<DP, R>(), st>>>(a);
-                    HIP_TRY(hipGetLastError());
-                }
-                return LV_OK;
-            }));
+            if constexpr (f32) {
+                LV_TRY(gqa_dispatch(f32, l, [&](auto elem, auto dp, auto r) -> int {
+                    constexpr int DP = decltype(dp)::value, R = decltype(r)::value;
+                    if constexpr (std::is_same_v<decltype(elem), float>) {
+                        gqa_rows_kernel<float, DP, R><<<dim3(l.spec.attn.kv_heads * l.groups, n), dim3(256), 4 * gqa_lds_floats<DP, R>(), st>>>(a);
+                        HIP_TRY(hipGetLastError());
+                    }
+                    return LV_OK;
+                }));
+            } else {
+                LV_TRY(gqa_tiles(s, l, a));
+            }
         }
         if (l.delta) {
             const lv_delta_spec &d = l.spec.delta;

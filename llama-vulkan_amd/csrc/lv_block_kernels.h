@@ -99,17 +99,20 @@ template <class T>
 __global__ __launch_bounds__(256) void prepare_kernel(PrepareArgs a)
 {
     __shared__ float scratch[4];
+    __shared__ float2 turn[kGqaMaxDim / 2];
     const uint32_t t = blockIdx.x, pos = a.pos0 + t;
     const float *y = a.y + (size_t)t * a.ldy;
     if (a.attn.heads) {
         const GqaSpec &s = a.attn;
         const uint32_t half = a.dp / 2;
+        rotation_table(turn, s, pos);
         const float inv_q = projection_inv(y + s.q_off, s.heads * s.dim, s.eps, s.q_norm, scratch);
         const float inv_k = projection_inv(y + s.k_off, s.kv_heads * s.dim, s.eps, s.k_norm, scratch);
+        __syncthreads();
         for (uint32_t i = threadIdx.x; i < s.heads * half; i += 256) {
             const uint32_t h = i / half, p = i % half;
             float u, v;
-            head_pair(u, v, y + s.q_off, s.q_norm, h * s.dim, p, s.dim, inv_q, s, pos);
+            head_pair(u, v, y + s.q_off, s.q_norm, h * s.dim, p, s.dim, inv_q, s, turn);
             T *o = static_cast<T *>(a.q) + ((size_t)t * s.heads + h) * a.dp + 2 * p;
             o[0] = float_to_elem<T>(u * s.scale);
             o[1] = float_to_elem<T>(v * s.scale);
@@ -117,7 +120,7 @@ __global__ __launch_bounds__(256) void prepare_kernel(PrepareArgs a)
         for (uint32_t i = threadIdx.x; i < s.kv_heads * half; i += 256) {
             const uint32_t h = i / half, p = i % half;
             float u, v;
-            head_pair(u, v, y + s.k_off, s.k_norm, h * s.dim, p, s.dim, inv_k, s, pos);
+            head_pair(u, v, y + s.k_off, s.k_norm, h * s.dim, p, s.dim, inv_k, s, turn);
             const size_t o = ((size_t)t * s.kv_heads + h) * a.dp + 2 * p;
             static_cast<T *>(a.k)[o] = float_to_elem<T>(u);
             static_cast<T *>(a.k)[o + 1] = float_to_elem<T>(v);

@@ -59,38 +59,94 @@ __device__ __forceinline__ float delta_conv(const DeltaSpec &s, const float *y, 
     const float *w = s.conv + (size_t)c * s.taps;
     const uint32_t at = delta_channel_at(s, c), C = s.channels();
     float v = w[s.taps - 1] * y[at];
-    for (uint32_t j = 1; j < s.taps && j <= pos; j++) {
-        const float x = j <= behind ? y[at - (ptrdiff_t)(j * ld)] : s.ring[(size_t)((pos - j) % s.taps) * C + c];
-        v = fmaf(w[s.taps - 1 - j], x, v);
+    for (uint32_t j0 = 1; j0 < s.taps && j0 <= pos; j0 += 3) {
+        float x[3], f[3];      // three inputs on their way at once
+#pragma unroll
+        for (uint32_t e = 0; e < 3; e++) {
+            const uint32_t j = j0 + e;
+            const bool ok = j < s.taps && j <= pos;
+            x[e] = !ok ? 0.f : j <= behind ? y[at - (ptrdiff_t)(j * ld)] : s.ring[(size_t)((pos - j) % s.taps) * C + c];
+            f[e] = ok ? w[s.taps - 1 - j] : 0.f;
+        }
+#pragma unroll
+        for (int e = 0; e < 3; e++) v = fmaf(f[e], x[e], v);
     }
     return silu_f(v);
 }
 
-// dot of one low-rank row with a vector in LDS, by 8 consecutive lanes; every lane of the eight gets it
-__device__ __forceinline__ float low_rank_dot(const uint16_t *row, const float *x, uint32_t kp)
-{
-    float t = 0.f;
-    for (uint32_t k = (threadIdx.x & 7) * 8; k < kp; k += 64) {
-        float w[8], v[8];
-        load8(w, row + k);
-        load8(v, x + k);
+// Rows row0 + 32 i (i < N) of a low-rank matrix against a vector in LDS, 8 consecutive lanes a row, every lane of the eight gets
+// the sum.  fetch() requests the first 128 columns of all N rows, which is usually all there is; dot() does the rest.
+template <int N>
+struct LowRankRows {
+    uint4 w[N][2];
+    const uint16_t *at;
+    uint32_t kp;
+    uint32_t rows;      // of the N that exist
+
+    __device__ __forceinline__ void fetch(const uint16_t *m, uint32_t row0, uint32_t end, uint32_t kp_)
+    {
+        kp = kp_;
+        rows = row0 < end ? min((uint32_t)N, (end - row0 + 31) / 32) : 0;
+        at = m + (size_t)row0 * kp + (threadIdx.x & 7) * 8;
 #pragma unroll
-        for (int e = 0; e < 8; e++) t = fmaf(w[e], v[e], t);
+        for (int i = 0; i < N; i++)
+#pragma unroll
+            for (int k = 0; k < 2; k++)
+                w[i][k] = i < (int)rows && k * 64 < (int)kp ? *reinterpret_cast<const uint4 *>(at + (size_t)i * 32 * kp + k * 64) : make_uint4(0, 0, 0, 0);
     }
-    return group8_sum(t);
-}
+    static __device__ __forceinline__ float dot8(const uint4 &v, const float *x)
+    {
+        const uint32_t u[4] = {v.x, v.y, v.z, v.w};
+        float t = 0.f;
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            t = fmaf(__uint_as_float(u[i] << 16), x[2 * i], t);
+            t = fmaf(__uint_as_float(u[i] & 0xffff0000u), x[2 * i + 1], t);
+        }
+        return t;
+    }
+    __device__ __forceinline__ void dot(float (&out)[N], const float *x)
+    {
+        x += (threadIdx.x & 7) * 8;
+#pragma unroll
+        for (int i = 0; i < N; i++) {
+            float t = dot8(w[i][0], x);
+            if (kp > 64) t += dot8(w[i][1], x + 64);
+            if (i < (int)rows)
+                for (uint32_t k = 128; k < kp; k += 64) t += dot8(*reinterpret_cast<const uint4 *>(at + (size_t)i * 32 * kp + k), x + k);
+            out[i] = group8_sum(t);
+        }
+    }
+};
 
 __host__ __device__ constexpr uint32_t delta_step_lds_floats(uint32_t a_kp, uint32_t g_kp) { return 3 * kDeltaMaxDim + kDeltaCols + 16 + a_kp + g_kp; }
 
-// one token, one head, one block of kDeltaCols columns: 256 threads
+// one token, one head, one block of kDeltaCols columns: 256 threads.  Everything the block reads is requested first.
 __device__ __forceinline__ void delta_step(const DeltaStepArgs &a, uint32_t idx, float *lds)
 {
     const DeltaSpec &s = a.s;
     const uint32_t head = idx / a.blocks, cb = idx % a.blocks, c_lo = cb * kDeltaCols, nc = min((uint32_t)kDeltaCols, s.vdim - c_lo);
     const uint32_t pos = *a.pos_ptr + a.pos_add, rep = s.heads / s.kv_heads, kvh = head / rep, nq = s.kv_heads * s.dim, C = s.channels();
     float *q = lds, *k = q + kDeltaMaxDim, *g = k + kDeltaMaxDim, *v = g + kDeltaMaxDim, *scratch = v + kDeltaCols, *al = scratch + 16, *gl = al + s.a_kp;
+    const int l16 = threadIdx.x & 15, c_own = threadIdx.x >> 4, r8 = threadIdx.x >> 3;
+    const int J = s.dstride / 64;
+
+    float4 st[2][4];      // this thread's parts of columns c_own and c_own + 16
+    float4 *col[2];
+#pragma unroll
+    for (int h = 0; h < 2; h++) {
+        const uint32_t c = min((uint32_t)(c_own + 16 * h), nc - 1);
+        col[h] = reinterpret_cast<float4 *>(s.state + ((size_t)head * s.vdim + c_lo + c) * s.dstride) + l16;
+#pragma unroll
+        for (int j = 0; j < 4; j++) st[h][j] = pos && j < J ? col[h][j * 16] : make_float4(0.f, 0.f, 0.f, 0.f);
+    }
+    LowRankRows<4> ra;
+    LowRankRows<1> rg;
+    ra.fetch(s.a2, head * s.dim + r8, (head + 1) * s.dim, s.a_kp);
+    rg.fetch(s.g2, head * s.vdim + c_lo + r8, head * s.vdim + c_lo + nc, s.g_kp);
     for (uint32_t i = threadIdx.x; i < s.a_kp; i += 256) al[i] = i < s.a_rank ? a.y[s.a_off + i] : 0.f;
     for (uint32_t i = threadIdx.x; i < s.g_kp; i += 256) gl[i] = i < s.g_rank ? a.y[s.g_off + i] : 0.f;
+    const float beta = sigmoid_f(a.y[s.b_off + head]), ea = expf(s.a_log[head]);
 
     float qv = 0.f, kv = 0.f;
     const uint32_t d = threadIdx.x, rslot = pos % s.taps;
@@ -108,59 +164,54 @@ __device__ __forceinline__ void delta_step(const DeltaStepArgs &a, uint32_t idx,
         v[threadIdx.x] = delta_conv(s, a.y, 0, 0, 2 * nq + c, pos);
         s.ring[(size_t)rslot * C + 2 * nq + c] = a.y[s.v_off + c];
     }
-    const float nqs = block_sum_waves(qv * qv, scratch, 4), nks = block_sum_waves(kv * kv, scratch, 4);
-    qv = qv / sqrtf(nqs + 1e-6f) / sqrtf((float)s.dim);
-    kv = kv / sqrtf(nks + 1e-6f);
-    const float qk = block_sum_waves(qv * kv, scratch, 4);
-    q[threadIdx.x] = qv;
-    k[threadIdx.x] = kv;
-    const float ea = expf(s.a_log[head]);
-    for (uint32_t r0 = 0; r0 < s.dstride; r0 += 32) {
-        const uint32_t r = r0 + (threadIdx.x >> 3);
-        float gv = 0.f;
-        if (r < s.dim) {
-            const uint32_t row = head * s.dim + r;
-            gv = expf(-ea * softplus_f(low_rank_dot(s.a2 + (size_t)row * s.a_kp, al, s.a_kp) + s.dt_bias[row]));
+    float sums[3] = {qv * qv, kv * kv, qv * kv};
+    block_sums_waves<3>(sums, scratch, 4);      // also publishes al, gl and v
+    const float fq = 1.f / sqrtf(sums[0] + 1e-6f) / sqrtf((float)s.dim), fk = 1.f / sqrtf(sums[1] + 1e-6f), qk = sums[2] * fq * fk;
+    q[threadIdx.x] = qv * fq;
+    k[threadIdx.x] = kv * fk;
+    for (uint32_t r0 = 0; r0 < s.dstride; r0 += 128) {
+        if (r0) ra.fetch(s.a2, head * s.dim + r0 + r8, (head + 1) * s.dim, s.a_kp);
+        float t[4];
+        ra.dot(t, al);
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            const uint32_t r = r0 + i * 32 + r8;
+            if ((threadIdx.x & 7) == i && r < s.dstride)      // four lanes of the eight share the exponentials
+                g[r] = r < s.dim ? expf(-ea * softplus_f(t[i] + s.dt_bias[head * s.dim + r])) : 0.f;
         }
-        if ((threadIdx.x & 7) == 0) g[r] = gv;
     }
     {
-        const uint32_t c = threadIdx.x >> 3;
-        if (c < nc) {
-            const uint32_t row = head * s.vdim + c_lo + c;
-            const float t = low_rank_dot(s.g2 + (size_t)row * s.g_kp, gl, s.g_kp);
-            if ((threadIdx.x & 7) == 0) a.gate[row] = sigmoid_f(t);
-        }
+        float t[1];
+        rg.dot(t, gl);
+        if (r8 < (int)nc && (threadIdx.x & 7) == 0) a.gate[head * s.vdim + c_lo + r8] = sigmoid_f(t[0]);
     }
     __syncthreads();
-    const float beta = sigmoid_f(a.y[s.b_off + head]);
-    const int l16 = threadIdx.x & 15;
-    const uint32_t J = s.dstride / 64;
-    for (uint32_t c = threadIdx.x >> 4; c < nc; c += 16) {
-        float4 *col = reinterpret_cast<float4 *>(s.state + ((size_t)head * s.vdim + c_lo + c) * s.dstride);
-        float4 st[4];
+#pragma unroll
+    for (int h = 0; h < 2; h++) {
+        const uint32_t c = c_own + 16 * h;
         float pk = 0.f, pq = 0.f;
 #pragma unroll
         for (int j = 0; j < 4; j++)
-            if (j < (int)J) {
+            if (j < J) {
                 const int at = j * 64 + l16 * 4;
-                float4 x = pos ? col[at / 4] : make_float4(0.f, 0.f, 0.f, 0.f);
+                float4 x = st[h][j];
                 const float4 gg = *reinterpret_cast<const float4 *>(g + at), kk = *reinterpret_cast<const float4 *>(k + at), qq = *reinterpret_cast<const float4 *>(q + at);
                 x.x *= gg.x; x.y *= gg.y; x.z *= gg.z; x.w *= gg.w;
                 pk = fmaf(x.x, kk.x, pk); pk = fmaf(x.y, kk.y, pk); pk = fmaf(x.z, kk.z, pk); pk = fmaf(x.w, kk.w, pk);
                 pq = fmaf(x.x, qq.x, pq); pq = fmaf(x.y, qq.y, pq); pq = fmaf(x.z, qq.z, pq); pq = fmaf(x.w, qq.w, pq);
-                st[j] = x;
+                st[h][j] = x;
             }
         pk = group16_sum(pk);
         pq = group16_sum(pq);
+        if (c >= nc) continue;
         const float u = beta * (v[c] - pk);
 #pragma unroll
         for (int j = 0; j < 4; j++)
-            if (j < (int)J) {
-                const int at = j * 64 + l16 * 4;
-                const float4 kk = *reinterpret_cast<const float4 *>(k + at);
-                st[j].x = fmaf(kk.x, u, st[j].x); st[j].y = fmaf(kk.y, u, st[j].y); st[j].z = fmaf(kk.z, u, st[j].z); st[j].w = fmaf(kk.w, u, st[j].w);
-                col[at / 4] = st[j];
+            if (j < J) {
+                const float4 kk = *reinterpret_cast<const float4 *>(k + j * 64 + l16 * 4);
+                float4 x = st[h][j];
+                x.x = fmaf(kk.x, u, x.x); x.y = fmaf(kk.y, u, x.y); x.z = fmaf(kk.z, u, x.z); x.w = fmaf(kk.w, u, x.w);
+                col[h][j * 16] = x;
             }
         if (l16 == 0) a.o[head * s.vdim + c_lo + c] = fmaf(qk, u, pq);
     }

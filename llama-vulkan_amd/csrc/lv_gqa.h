@@ -43,17 +43,22 @@ struct GqaStepArgs {
     float *out;                         // [heads * vdim]
 };
 
-constexpr int kGqaSplit = 128;          // keys per workgroup
+constexpr int kGqaSplit = 128;          // keys of a row kernel's block
+// keys per workgroup of the one-token step: what 8 rounds of loads bring
+__host__ __device__ constexpr uint32_t gqa_split(uint32_t dp) { return dp == 256 ? 64 : 128; }
 
-__device__ __forceinline__ void rotate_pair(float &u, float &v, double freq, uint32_t pos)
+constexpr uint32_t kGqaMaxDim = 256;
+
+// (cos, sin) of a position's angles, one per rotated pair; readable after the caller's next barrier.  Angles are reduced in
+// double: positions far out lose nothing to the range reduction.
+__device__ __forceinline__ void rotation_table(float2 *turn, const GqaSpec &s, uint32_t pos)
 {
-    // angle reduced in double: positions far out lose nothing to the range reduction
-    const double a = (double)pos * freq, turn = 6.283185307179586476925;
-    float sn, cs;
-    sincosf((float)(a - turn * rint(a / turn)), &sn, &cs);
-    const float r = u * cs - v * sn;
-    v = v * cs + u * sn;
-    u = r;
+    for (uint32_t i = threadIdx.x; i < s.rot_dims / 2; i += blockDim.x) {
+        const double a = (double)pos * s.freq[i], full = 6.283185307179586476925;
+        float sn, cs;
+        sincosf((float)(a - full * rint(a / full)), &sn, &cs);
+        turn[i] = make_float2(cs, sn);
+    }
 }
 
 template <int LPK> __device__ __forceinline__ float lanes_sum(float v)
@@ -73,7 +78,7 @@ struct GqaLanes {
 };
 
 // LDS, in floats
-template <int DP, int R> constexpr int gqa_lds_floats() { return R * DP + 2 * DP + R * kGqaSplit + 4 * R * DP + 4 * R + 16; }
+template <int DP, int R> constexpr int gqa_lds_floats() { return R * DP + 2 * DP + R * kGqaSplit + 4 * R * DP + 4 * R + 16 + DP; }
 
 // q [R][DP] and sc [R][kGqaSplit] in LDS
 template <int DP, int R, class Key>
@@ -151,47 +156,102 @@ __device__ __forceinline__ float projection_inv(const float *y, uint32_t n, floa
 
 // elements 2i, 2i+1 of one head, normalised and rotated
 __device__ __forceinline__ void head_pair(float &u, float &v, const float *y, const float *w, uint32_t base, uint32_t i, uint32_t dim, float inv, const GqaSpec &s,
-                                          uint32_t pos)
+                                          const float2 *turn)
 {
     const uint32_t d = 2 * i;
     u = d < dim ? y[base + d] * inv * (w ? w[base + d] : 1.f) : 0.f;
     v = d + 1 < dim ? y[base + d + 1] * inv * (w ? w[base + d + 1] : 1.f) : 0.f;
-    if (d < s.rot_dims) rotate_pair(u, v, s.freq[i], pos);
+    if (d < s.rot_dims) {
+        const float2 t = turn[i];
+        const float r = u * t.x - v * t.y;
+        v = v * t.x + u * t.y;
+        u = r;
+    }
 }
 
-// One token, one group of R heads that share a kv head, one split of its keys: 256 threads.  The splits of a group meet in the
-// last of them to arrive (see attention_kernel for what the hand-over relies on).  The split that holds the token's own
-// position also appends its rows.
+// eight elements as they lie in memory
+template <class CT> struct GqaRaw;
+template <> struct GqaRaw<uint16_t> {
+    uint4 v;
+    __device__ __forceinline__ void load(const uint16_t *p) { v = *reinterpret_cast<const uint4 *>(p); }
+    __device__ __forceinline__ void get(float (&f)[8]) const
+    {
+        const uint32_t w[4] = {v.x, v.y, v.z, v.w};
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            f[2 * i] = __uint_as_float(w[i] << 16);
+            f[2 * i + 1] = __uint_as_float(w[i] & 0xffff0000u);
+        }
+    }
+};
+template <> struct GqaRaw<float> {
+    float4 a, b;
+    __device__ __forceinline__ void load(const float *p)
+    {
+        a = reinterpret_cast<const float4 *>(p)[0];
+        b = reinterpret_cast<const float4 *>(p)[1];
+    }
+    __device__ __forceinline__ void get(float (&f)[8]) const { f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w; f[4] = b.x; f[5] = b.y; f[6] = b.z; f[7] = b.w; }
+};
+
+// One token, one group of R heads that share a kv head, one split of its keys: 256 threads.  All cache rows of the split are
+// requested before anything else.  The splits of a group meet in the last of them to arrive (see attention_kernel for what the
+// hand-over relies on).  The split that holds the token's own position also appends its rows.
 template <class CT, int DP, int R>
 __device__ __forceinline__ void gqa_step(const GqaStepArgs &a, uint32_t idx, float *lds)
 {
+    using L = GqaLanes<DP, R>;
+    constexpr int SPLIT = gqa_split(DP), ROUNDS = SPLIT / L::KPR;
     const GqaSpec &s = a.s;
     const uint32_t split = idx % a.splits, grp = idx / a.splits, hg = grp % a.groups, kvh = grp / a.groups;
     const uint32_t pos = *a.pos_ptr + a.pos_add;
     const uint32_t c0 = s.chunk ? pos / s.chunk * s.chunk : 0;
-    const uint32_t active = (pos - c0) / kGqaSplit + 1;
+    const uint32_t active = (pos - c0) / SPLIT + 1;
     if (split >= active) return;
-    const uint32_t k_begin = c0 + split * kGqaSplit, n = min((uint32_t)kGqaSplit, pos + 1 - k_begin);
+    const uint32_t k_begin = c0 + split * SPLIT, n = min((uint32_t)SPLIT, pos + 1 - k_begin);
     const bool own = split == active - 1;
     const uint32_t per_kv = s.heads / s.kv_heads, h0 = kvh * per_kv + hg * R, nh = min((uint32_t)R, per_kv - hg * R);
+    const int sub = threadIdx.x % L::LPK, kg = threadIdx.x / L::LPK, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    CT *const kc = static_cast<CT *>(s.kc), *const vc = static_cast<CT *>(s.vc);
+    GqaRaw<CT> kraw[ROUNDS], vraw[ROUNDS];
+#pragma unroll
+    for (int i = 0; i < ROUNDS; i++) {
+        const uint32_t p = k_begin + min((uint32_t)(i * L::KPR + kg), n - 1);
+        kraw[i].load(kc + ((size_t)(p % s.ring) * s.kv_heads + kvh) * DP + sub * 8);
+    }
+#pragma unroll
+    for (int i = 0; i < ROUNDS; i++) {
+        const uint32_t p = k_begin + min((uint32_t)(i * L::KPR + kg), n - 1);
+        vraw[i].load(vc + ((size_t)(p % s.ring) * s.kv_heads + kvh) * DP + sub * 8);
+    }
     float *q = lds, *krow = q + R * DP, *vrow = krow + DP, *sc = vrow + DP, *red = sc + R * kGqaSplit, *ml = red + 4 * R * DP, *scratch = ml + 4 * R;
+    float2 *turn = reinterpret_cast<float2 *>(scratch + 16);
 
     const float *yq = a.y + s.q_off, *yk = a.y + s.k_off, *yv = a.y + s.v_off;
-    const float inv_q = projection_inv(yq, s.heads * s.dim, s.eps, s.q_norm, scratch);
-    const float inv_k = projection_inv(yk, s.kv_heads * s.dim, s.eps, s.k_norm, scratch);
+    float sq[2] = {0.f, 0.f};
+    if (s.q_norm) {
+        const uint32_t nq = s.heads * s.dim, nk = s.kv_heads * s.dim;
+#pragma unroll 4
+        for (uint32_t i = threadIdx.x; i < nq; i += 256) sq[0] = fmaf(yq[i], yq[i], sq[0]);
+#pragma unroll 2
+        for (uint32_t i = threadIdx.x; i < nk; i += 256) sq[1] = fmaf(yk[i], yk[i], sq[1]);
+    }
+    rotation_table(turn, s, pos);
+    block_sums_waves<2>(sq, scratch, 4);      // also publishes the rotation table
+    const float inv_q = s.q_norm ? 1.f / sqrtf(sq[0] / (float)(s.heads * s.dim) + s.eps) : 1.f;
+    const float inv_k = s.q_norm ? 1.f / sqrtf(sq[1] / (float)(s.kv_heads * s.dim) + s.eps) : 1.f;
     for (uint32_t i = threadIdx.x; i < R * DP / 2; i += 256) {
         const uint32_t r = i / (DP / 2), p = i % (DP / 2);
         float u = 0.f, v = 0.f;
-        if (r < nh) head_pair(u, v, yq, s.q_norm, (h0 + r) * s.dim, p, s.dim, inv_q, s, pos);
+        if (r < nh) head_pair(u, v, yq, s.q_norm, (h0 + r) * s.dim, p, s.dim, inv_q, s, turn);
         q[r * DP + 2 * p] = u * s.scale;
         q[r * DP + 2 * p + 1] = v * s.scale;
     }
-    CT *const kc = static_cast<CT *>(s.kc), *const vc = static_cast<CT *>(s.vc);
     if (own) {
         const size_t row = ((size_t)(pos % s.ring) * s.kv_heads + kvh) * DP;
         for (uint32_t p = threadIdx.x; p < DP / 2; p += 256) {
             float u, v;
-            head_pair(u, v, yk, s.k_norm, kvh * s.dim, p, s.dim, inv_k, s, pos);
+            head_pair(u, v, yk, s.k_norm, kvh * s.dim, p, s.dim, inv_k, s, turn);
             const CT cu = float_to_elem<CT>(u), cv = float_to_elem<CT>(v);
             krow[2 * p] = elem_to_float(cu);
             krow[2 * p + 1] = elem_to_float(cv);
@@ -205,28 +265,39 @@ __device__ __forceinline__ void gqa_step(const GqaStepArgs &a, uint32_t idx, flo
         }
     }
     __syncthreads();
-    auto from = [&](const CT *c, const float *mine, uint32_t j, int d, float (&f)[8]) {
-        const uint32_t p = k_begin + j;
-        if (p == pos) load8(f, mine + d);
-        else load8(f, c + ((size_t)(p % s.ring) * s.kv_heads + kvh) * DP + d);
-    };
-    gqa_scores<DP, R>(q, sc, n, [&](uint32_t j, int d, float (&f)[8]) { from(kc, krow, j, d, f); });
-    __syncthreads();
     {
-        const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-        for (int r = wave; r < R; r += 4) {
-            float m = -INFINITY, l = 0.f;
-            for (uint32_t j = lane; j < n; j += 64) m = fmaxf(m, sc[r * kGqaSplit + j]);
+        float qr[R][8];
 #pragma unroll
-            for (int off = 1; off < 64; off <<= 1) m = fmaxf(m, __shfl_xor(m, off, 64));
-            for (uint32_t j = lane; j < n; j += 64) {
-                const float p = __expf(sc[r * kGqaSplit + j] - m);
-                sc[r * kGqaSplit + j] = p;
-                l += p;
+        for (int r = 0; r < R; r++) load8(qr[r], q + r * DP + sub * 8);
+#pragma unroll
+        for (int i = 0; i < ROUNDS; i++) {
+            const uint32_t j = i * L::KPR + kg;
+            float f[8];
+            kraw[i].get(f);
+            if (k_begin + j == pos) load8(f, krow + sub * 8);
+#pragma unroll
+            for (int r = 0; r < R; r++) {
+                float t = 0.f;
+#pragma unroll
+                for (int e = 0; e < 8; e++) t = fmaf(qr[r][e], f[e], t);
+                t = lanes_sum<L::LPK>(t);
+                if (sub == 0) sc[r * kGqaSplit + j] = j < n ? t : -INFINITY;
             }
-            l = wave_sum(l);
-            if (lane == 0) { ml[2 * r] = m; ml[2 * r + 1] = l; }
         }
+    }
+    __syncthreads();
+    for (int r = wave; r < R; r += 4) {
+        float m = -INFINITY, l = 0.f;
+        for (int j = lane; j < SPLIT; j += 64) m = fmaxf(m, sc[r * kGqaSplit + j]);
+#pragma unroll
+        for (int off = 1; off < 64; off <<= 1) m = fmaxf(m, __shfl_xor(m, off, 64));
+        for (int j = lane; j < SPLIT; j += 64) {
+            const float p = __expf(sc[r * kGqaSplit + j] - m);      // 0 beyond the split's keys
+            sc[r * kGqaSplit + j] = p;
+            l += p;
+        }
+        l = wave_sum(l);
+        if (lane == 0) { ml[2 * r] = m; ml[2 * r + 1] = l; }
     }
     __syncthreads();
     float acc[R][8];
@@ -234,7 +305,19 @@ __device__ __forceinline__ void gqa_step(const GqaStepArgs &a, uint32_t idx, flo
     for (int r = 0; r < R; r++)
 #pragma unroll
         for (int e = 0; e < 8; e++) acc[r][e] = 0.f;
-    gqa_values<DP, R>(acc, sc, n, [&](uint32_t j, int d, float (&f)[8]) { from(vc, vrow, j, d, f); });
+#pragma unroll
+    for (int i = 0; i < ROUNDS; i++) {
+        const uint32_t j = i * L::KPR + kg;
+        float f[8];
+        vraw[i].get(f);
+        if (k_begin + j == pos) load8(f, vrow + sub * 8);
+#pragma unroll
+        for (int r = 0; r < R; r++) {
+            const float p = sc[r * kGqaSplit + j];
+#pragma unroll
+            for (int e = 0; e < 8; e++) acc[r][e] = fmaf(p, f[e], acc[r][e]);
+        }
+    }
     gqa_reduce<DP, R>(acc, red);
 
     if (active == 1) {
@@ -259,22 +342,34 @@ __device__ __forceinline__ void gqa_step(const GqaStepArgs &a, uint32_t idx, flo
     __syncthreads();
     if (*arrived != active - 1) return;
     auto get = [&](uint32_t sp, uint32_t i) { return __uint_as_float(__hip_atomic_load(part + (size_t)sp * PS + i, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT)); };
-    // per head: the largest score and the sum over the splits, sink included
-    if (threadIdx.x < R) {
-        const uint32_t r = threadIdx.x;
-        const float sk = s.sink && r < nh ? s.sink[h0 + r] : -INFINITY;
+    // per head: the largest score and the sum over the splits, sink included; a wave per head, a lane per split
+    for (int r = wave; r < R; r += 4) {
+        const float sk = s.sink && r < (int)nh ? s.sink[h0 + r] : -INFINITY;
         float M = sk;
-        for (uint32_t sp = 0; sp < active; sp++) M = fmaxf(M, get(sp, r * (DP + 2) + DP));
-        float l = __expf(sk - M);
-        for (uint32_t sp = 0; sp < active; sp++) l += get(sp, r * (DP + 2) + DP + 1) * __expf(get(sp, r * (DP + 2) + DP) - M);
-        ml[2 * r] = M;
-        ml[2 * r + 1] = l;
+        for (uint32_t sp = lane; sp < active; sp += 64) M = fmaxf(M, get(sp, r * (DP + 2) + DP));
+#pragma unroll
+        for (int off = 1; off < 64; off <<= 1) M = fmaxf(M, __shfl_xor(M, off, 64));
+        float l = 0.f;
+        for (uint32_t sp = lane; sp < active; sp += 64) l += get(sp, r * (DP + 2) + DP + 1) * __expf(get(sp, r * (DP + 2) + DP) - M);
+        l = wave_sum(l) + __expf(sk - M);
+        if (lane == 0) { ml[2 * r] = M; ml[2 * r + 1] = l; }
     }
     __syncthreads();
     for (uint32_t i = threadIdx.x; i < nh * s.vdim; i += 256) {
         const uint32_t r = i / s.vdim, c = i % s.vdim;
         float t = 0.f;
-        for (uint32_t sp = 0; sp < active; sp++) t = fmaf(get(sp, r * (DP + 2) + c), __expf(get(sp, r * (DP + 2) + DP) - ml[2 * r]), t);
+        for (uint32_t s0 = 0; s0 < active; s0 += 8) {       // eight splits' loads in flight, summed in split order
+            float v[8], w[8];
+#pragma unroll
+            for (int e = 0; e < 8; e++) {
+                const uint32_t sp = min(s0 + e, active - 1);
+                v[e] = get(sp, r * (DP + 2) + c);
+                w[e] = get(sp, r * (DP + 2) + DP);
+            }
+#pragma unroll
+            for (int e = 0; e < 8; e++)
+                if (s0 + e < active) t = fmaf(v[e], __expf(w[e] - ml[2 * r]), t);
+        }
         a.out[(h0 + r) * s.vdim + c] = t / ml[2 * r + 1];
     }
     if (threadIdx.x == 0) a.counters[grp] = 0u;

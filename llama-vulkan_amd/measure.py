@@ -15,6 +15,8 @@
     python llama-vulkan_amd/measure.py gemm          isolated 512-token GEMMs at the 13B shapes, q8_0 (for kernel traces and counters)
     python llama-vulkan_amd/measure.py copy          1 GiB device-to-device copy: achievable bandwidth, counter calibration
     python llama-vulkan_amd/measure.py read-stream   4 GiB read by a kernel that only reads: the bandwidth a weight stream can reach
+    python llama-vulkan_amd/measure.py block [SIZE]  block models beside LLaMA layers of the same width (bench.py --block)
+    python llama-vulkan_amd/measure.py block-only SIZE   prompts and decode steps of a block model alone (for kernel traces)
     python llama-vulkan_amd/measure.py all
 
 Every figure is algorithmic bytes (weights as stored in the GGML file, 18 B / 34 B per 32 weights, plus vectors and the
@@ -302,6 +304,127 @@ def gemm_cases(ctx, report=emit):
     return out_cases
 
 
+# Block models of the Somesun design at the layer sizes of real models, next to LLaMA layers of the same width and a like number
+# of weights a token passes through
+BLOCK_SIZES = {
+    "4096": dict(vocab=32000, width=4096, layers=4, attn=(32, 8, 128, 8192), delta=(32, 16, 128, 128, 4), rank=128, moe=(64, 8, 1024),
+                 llama=dict(vocab=32000, dim=4096, heads=32, layers=4, ff=11008)),
+    "2048": dict(vocab=32000, width=2048, layers=6, attn=(16, 4, 128, 2048), delta=(16, 16, 128, 128, 4), rank=64, moe=(32, 4, 1024),
+                 llama=dict(vocab=32000, dim=2048, heads=16, layers=6, ff=5504)),
+}
+
+
+def block_model(ctx, size, compute=None):
+    """random weights: every matrix reads the same random bytes of host memory and gets its own place on the device, norm weights
+    are ones"""
+    import numpy as np
+    c = BLOCK_SIZES[size]
+    D, V, L, r = c["width"], c["vocab"], c["layers"], c["rank"]
+    H, G, d, chunk = c["attn"]
+    dh, dg, dk, dv, taps = c["delta"]
+    E, top, ff = c["moe"]
+    blob = max(V, H * d, dh * dv, ff) * max(D, H * d, dh * dv, ff)
+    rng = np.random.default_rng(7)
+    x = np.tile((rng.standard_normal(1 << 22) * 0.02).astype(np.float32), (blob + (1 << 22) - 1) >> 22)[:blob]
+    ones = max(D, H * d, dh * dk)
+    base = np.concatenate([(x.view(np.uint32) >> 16).astype(np.uint16), np.full(ones, 0x3F80, np.uint16)])
+    table = []
+
+    def t(name, rows, cols=1, one=False):
+        table.append((name, lva.LV_BF16, blob * 2 if one else 0, rows, cols, rows * cols * 2))
+    t("embed", V, D); t("head", V, D); t("final.norm", D, one=True)
+    for i in range(L):
+        p = f"l{i}."
+        for n in ("norm1", "norm1b", "norm2", "norm2b"):
+            t(p + n, D, one=True)
+        a = p + "mix.left."
+        t(a + "q", H * d, D); t(a + "k", G * d, D); t(a + "o", D, H * d); t(a + "sink", H)
+        t(a + "q.norm", H * d, one=True); t(a + "k.norm", G * d, one=True)
+        a = p + "mix.right."
+        for n, rows in (("q", dg * dk), ("k", dg * dk), ("v", dh * dv)):
+            t(a + n, rows, D); t(a + n + ".conv", rows, taps)
+        t(a + "b", dh, D); t(a + "a1", r, D); t(a + "a2", dh * dk, r); t(a + "g1", r, D); t(a + "g2", dh * dv, r)
+        t(a + "A_log", dh); t(a + "dt_bias", dh * dk); t(a + "norm", dv, one=True); t(a + "o", D, dh * dv)
+        t(p + "mlp.router", E, D)
+        for e in range(E):
+            t(f"{p}mlp.e{e}.gate", ff, D); t(f"{p}mlp.e{e}.up", ff, D); t(f"{p}mlp.e{e}.down", D, ff)
+    b = lva.BlockSpec()
+    b.attn_scale, b.delta_scale = 0.7, 0.7
+    b.attn = lva.AttnSpec(H, G, d, d, d ** -0.5, chunk, d, 500000.0, lva.ATTN_NORM_FULL | lva.ATTN_KEYS_AS_VALUES | lva.ATTN_SINK)
+    b.delta = lva.DeltaSpec(dh, dg, dk, dv, taps)
+    b.moe = lva.MoeSpec(E, top, ff)
+    return lva.BlockModel(ctx, base.view(np.uint8), table, [b] * L, V, D, 1e-5, lva.LV_BF16 if compute is None else compute)
+
+
+def block_step_cost(c, pos):
+    """bytes a decode step at position `pos` has to move (bf16 weights of what the token passes through, the chunk's cache rows, the
+    recurrent state in and out) and flops per token of a prompt (products with weights only)"""
+    D, V, L, r = c["width"], c["vocab"], c["layers"], c["rank"]
+    H, G, d, chunk = c["attn"]
+    dh, dg, dk, dv, _ = c["delta"]
+    E, top, ff = c["moe"]
+    w = D * (H * d + G * d + 2 * dg * dk + dh * dv + dh + 2 * r) + r * dh * (dk + dv) + D * (H * d + dh * dv) + E * D + top * 3 * ff * D
+    state = 2 * G * d * 2 * (pos % chunk + 1) + 2 * dh * dk * dv * 4
+    return L * (2 * w + state) + 2 * V * D, 2.0 * L * w
+
+
+def block_cases(ctx, report=emit, sizes=None, prompts=(512, 2048), steps=64):
+    """prefill and decode of a block model and of its LLaMA counterpart (q8_0, on the persistent kernel where it has one and on the
+    graph of single kernels), same machine, same clock"""
+    out_cases = []
+
+    def timed(s, vocab, label, cost, flops_per_token, **kw):
+        n_max = max(prompts)
+        for n in prompts:
+            toks = lva.synth_tokens(n, 3, vocab, seed=n)
+            for _ in range(2):
+                s.begin(toks, 0)
+                s.wait()
+            s.timer_start()
+            s.begin(toks, 0)
+            ms = s.timer_stop()
+            tf = flops_per_token * n / ms / 1e9
+            out_cases.append(report(case=label + " prompt", tokens=n, ms=round(ms, 3), tok_s=round(n / ms * 1e3, 1), TFLOPs=round(tf, 1),
+                                    frac_of_mfma_peak=round(tf / MFMA_PEAK_TFLOPS, 4), **kw))
+        s.begin(lva.synth_tokens(n_max, 3, vocab, seed=1), 0)
+        tok, pos, total = s.argmax(), n_max, 0
+        for i in range(8 + steps):
+            if i == 8:
+                t0 = time.perf_counter()
+            s.begin([tok], pos)
+            tok = s.argmax()
+            total += cost(pos) if i >= 8 else 0
+            pos += 1
+        dt = time.perf_counter() - t0
+        out_cases.append(report(case=label + " decode", positions=[n_max + 8, pos - 1], tok_s=round(steps / dt, 1), ms=round(dt / steps * 1e3, 4),
+                                GBps=round(total / dt / 1e9, 1), frac_of_hbm_peak=round(total / dt / 1e9 / HBM_PEAK_GBS, 4), **kw))
+
+    for size in sizes or BLOCK_SIZES:
+        c = BLOCK_SIZES[size]
+        m = block_model(ctx, size)
+        s = lva.Session(m, max(prompts) + steps + 16)
+        _, fl = block_step_cost(c, 0)
+        timed(s, c["vocab"], f"Somesun width {size}", lambda pos: block_step_cost(c, pos)[0], fl, layers=c["layers"])
+        s.close()
+        m.close()
+        L = c["llama"]
+        base = "/dev/shm" if os.access("/dev/shm", os.W_OK) else "/tmp"
+        path = os.path.join(base, f"llava_measure_block_{size}.ggml")
+        if not os.path.exists(path):
+            lva.write_model(path + ".tmp", wtype=lva.LV_Q8_0, seed=5, **L)
+            os.replace(path + ".tmp", path)
+        lm = lva.Model(ctx, path)
+        s = lva.Session(lm, max(prompts) + steps + 16)
+        kinds = [lva.PATH_PERSISTENT, lva.PATH_GRAPH] if s.path() == lva.PATH_PERSISTENT else [lva.PATH_GRAPH]
+        for k in kinds:
+            s.set_path(k)
+            timed(s, L["vocab"], f"LLaMA width {size} q8_0, {'persistent' if k == lva.PATH_PERSISTENT else 'graph'}", lambda pos: step_bytes(L, lva.LV_Q8_0, pos),
+                  2.0 * L["layers"] * (4 * L["dim"] ** 2 + 3 * L["dim"] * L["ff"]), layers=L["layers"])
+        s.close()
+        lm.close()
+    return out_cases
+
+
 def main():
     which = sys.argv[1] if len(sys.argv) > 1 else "all"
     ctx = lva.Context(0)
@@ -321,6 +444,21 @@ def main():
         attention_batch_cases(ctx)
     if which == "gemm":
         gemm_cases(ctx)
+    if which == "block":
+        block_cases(ctx, sizes=sys.argv[2:3] or None)
+    if which == "block-only":     # without the LLaMA side, for kernel traces: prompts of 2048, then decode
+        c = BLOCK_SIZES[sys.argv[2]]
+        m = block_model(ctx, sys.argv[2])
+        s = lva.Session(m, 2200)
+        toks = lva.synth_tokens(2048, 3, c["vocab"], seed=1)
+        for _ in range(3):
+            s.begin(toks, 0)
+            s.wait()
+        for pos in range(2048, 2080):
+            s.begin([5], pos)
+            s.wait()
+        s.close()
+        m.close()
     if which in ("decode-q8", "all"):
         decode_case(ctx, "decode-q8", "7b", lva.LV_Q8_0, 1, 2048, 1916, 128)
     if which in ("decode-q8-graph", "all"):
