@@ -51,9 +51,14 @@ __device__ __forceinline__ void load8(float (&f)[8], const float *p)
     f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w; f[4] = b.x; f[5] = b.y; f[6] = b.z; f[7] = b.w;
 }
 
-__device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + __expf(-z)); }
-__device__ __forceinline__ float silu_f(float z) { return z / (1.f + __expf(-z)); }
-__device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z : log1pf(expf(z)); }
+// fp32 to within a few units in the last place, in few instructions: decode kernels run once per launch, and every line of
+// their code is fetched on the way
+__device__ __forceinline__ float sigmoid_f(float z) { return __builtin_amdgcn_rcpf(1.f + __expf(-z)); }
+__device__ __forceinline__ float silu_f(float z) { return z * sigmoid_f(z); }
+// log(1 + e^z) with an absolute error of about 1e-7, which is what its use in an exponent asks for
+__device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z : __logf(1.f + __expf(z)); }
+// decay of one key channel: exp(-exp(A_log) softplus(z)), ea = exp(A_log)
+__device__ __forceinline__ float decay_f(float ea, float z) { return __expf(-ea * softplus_f(z)); }
 
 enum BfEpilogue {
     kEpStore = 0,    // out[token][row]
@@ -94,17 +99,17 @@ __device__ __forceinline__ void bf_store4(const BfGemmArgs &a, uint32_t orow, ui
     if constexpr (EP == kEpDecay) {
         if (a.head_dim % 4 == 0) {      // the four rows belong to one head
             const uint32_t h = row / a.head_dim, d = row - h * a.head_dim;
-            const float ea = expf(a.a_log[h]);
+            const float ea = __expf(a.a_log[h]);
             const float4 b = *reinterpret_cast<const float4 *>(a.bias + row);
             *reinterpret_cast<float4 *>(a.out + (size_t)orow * a.ldo + h * a.head_stride + d) =
-                make_float4(expf(-ea * softplus_f(r[0] + b.x)), expf(-ea * softplus_f(r[1] + b.y)), expf(-ea * softplus_f(r[2] + b.z)), expf(-ea * softplus_f(r[3] + b.w)));
+                make_float4(decay_f(ea, r[0] + b.x), decay_f(ea, r[1] + b.y), decay_f(ea, r[2] + b.z), decay_f(ea, r[3] + b.w));
             return;
         }
 #pragma unroll
         for (int i = 0; i < 4; i++)
             if (row + i < a.rows) {
                 const uint32_t h = (row + i) / a.head_dim, d = (row + i) % a.head_dim;
-                a.out[(size_t)orow * a.ldo + h * a.head_stride + d] = expf(-expf(a.a_log[h]) * softplus_f(r[i] + a.bias[row + i]));
+                a.out[(size_t)orow * a.ldo + h * a.head_stride + d] = decay_f(__expf(a.a_log[h]), r[i] + a.bias[row + i]);
             }
         return;
     }

@@ -105,7 +105,7 @@ __device__ __forceinline__ void norm_input(const NormInput &a, float *xs, float 
             s = fmaf(v.x, v.x, s); s = fmaf(v.y, v.y, s); s = fmaf(v.z, v.z, s); s = fmaf(v.w, v.w, s);
             *reinterpret_cast<float4 *>(xs + bf_xs(i, dp)) = v;
         }
-        if (a.wpost) ypost = 1.f / sqrtf(block_sum_waves(s, scratch, nw) / (float)a.dim + a.eps);
+        if (a.wpost) ypost = rsqrtf(block_sum_waves(s, scratch, nw) / (float)a.dim + a.eps);
     }
     float s = 0.f;
     for (uint32_t i = threadIdx.x * 4; i < dp; i += step) {
@@ -120,7 +120,7 @@ __device__ __forceinline__ void norm_input(const NormInput &a, float *xs, float 
         *slot = v;
         if (lead && a.x_out) *reinterpret_cast<float4 *>(a.x_out + i) = v;
     }
-    const float inv = 1.f / sqrtf(block_sum_waves(s, scratch, nw) / (float)a.dim + a.eps);
+    const float inv = rsqrtf(block_sum_waves(s, scratch, nw) / (float)a.dim + a.eps);
     for (uint32_t i = threadIdx.x * 4; i < dp; i += step) {
         float4 *slot = reinterpret_cast<float4 *>(xs + bf_xs(i, dp));
         const float4 w = *reinterpret_cast<const float4 *>(a.wpre + i);
@@ -138,7 +138,7 @@ __device__ __forceinline__ void gated_head(const float *o, const float *gate, co
     const uint32_t lane = threadIdx.x & 63;
     float s = 0.f;
     for (uint32_t c = lane; c < vdim; c += 64) s = fmaf(o[c], o[c], s);
-    const float inv = 1.f / sqrtf(wave_sum(s) / (float)vdim + eps);
+    const float inv = rsqrtf(wave_sum(s) / (float)vdim + eps);
     for (uint32_t c = lane; c < vdim; c += 64) put(c, o[c] * inv * w[c] * gate[c] * scale);
 }
 
@@ -173,7 +173,7 @@ __device__ __forceinline__ void top_experts(float *zs, uint32_t n, uint32_t top,
         if (at == 0xffffffffu) at = 0;      // nothing but NaN left
         if (lane == 0) {
             ids[k] = at;
-            scores[k] = 1.f / (1.f + expf(-best));
+            scores[k] = sigmoid_f(best);
             zs[at] = -INFINITY;
         }
         __builtin_amdgcn_wave_barrier();

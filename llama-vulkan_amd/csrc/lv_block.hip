@@ -285,7 +285,7 @@ int block_model_create(hipStream_t st, const void *base, uint64_t base_size, con
                 const double rb = a.rot_base;
                 at(&l.freq, ld.place((uint64_t)half * 8, [=](uint8_t *dst) {
                     for (uint32_t k = 0; k < half; k++) {
-                        const double f = std::pow(rb, -2.0 * k / dims);
+                        const double f = std::pow(rb, -2.0 * k / dims) / 6.283185307179586476925;      // in full turns
                         std::memcpy(dst + 8 * (size_t)k, &f, 8);
                     }
                 }));
@@ -317,9 +317,14 @@ int block_model_create(hipStream_t st, const void *base, uint64_t base_size, con
                 const uint8_t *s0 = ld.data(cq), *s1 = ld.data(ck), *s2 = ld.data(cv);
                 const uint32_t t0 = cq->ftype, t1 = ck->ftype, t2 = cv->ftype;
                 at(&l.conv, ld.place((uint64_t)l.channels() * taps * 4, [=](uint8_t *dst) {
-                    Loader::widen(dst, s0, nq * taps, t0);
-                    Loader::widen(dst + (uint64_t)nq * taps * 4, s1, nq * taps, t1);
-                    Loader::widen(dst + (uint64_t)2 * nq * taps * 4, s2, nv * taps, t2);
+                    std::vector<float> w((size_t)(2 * nq + nv) * taps);      // [channel][tap], as the file has it
+                    uint8_t *b = reinterpret_cast<uint8_t *>(w.data());
+                    Loader::widen(b, s0, nq * taps, t0);
+                    Loader::widen(b + (uint64_t)nq * taps * 4, s1, nq * taps, t1);
+                    Loader::widen(b + (uint64_t)2 * nq * taps * 4, s2, nv * taps, t2);
+                    const size_t C = 2 * nq + nv;
+                    for (size_t c = 0; c < C; c++)
+                        for (size_t j = 0; j < taps; j++) std::memcpy(dst + (j * C + c) * 4, &w[c * taps + j], 4);
                 }));
             }
             vec(&l.a_log, pd + "A_log", dl.heads, 1, dl.heads);
@@ -636,7 +641,7 @@ static GqaSpec gqa_spec(const BlockSession *s, size_t i)
     g.q_off = l.q_off; g.k_off = l.k_off; g.v_off = l.v_off;
     g.q_norm = l.q_norm; g.k_norm = l.k_norm; g.sink = l.sink; g.freq = l.freq;
     g.rot_dims = a.rot_dims; g.chunk = a.chunk; g.scale = a.scale; g.eps = s->m->hp.eps;
-    g.ring = s->layers[i].ring; g.kc = s->layers[i].kc; g.vc = s->layers[i].vc;
+    g.kc = s->layers[i].kc; g.vc = s->layers[i].vc;
     return g;
 }
 
@@ -905,7 +910,7 @@ static int step_batch(BlockSession *s, const uint32_t *tokens, uint32_t pos, uin
         p.y = w.y1; p.ldy = l.in.rows; p.pos0 = pos; p.dp = l.dp;
         p.attn = gqa_spec(s, i); p.q = w.q; p.k = w.k; p.v = w.v;
         p.delta = delta_spec(s, i); p.dq = w.dq; p.dk = w.dk; p.dv = w.dv; p.beta = w.beta; p.qk = w.qk; p.a1 = w.a1; p.g1 = w.g1;
-        prepare_kernel<T><<<dim3(n), dim3(256), 0, st>>>(p);
+        prepare_kernel<T><<<dim3(prepare_grid(p, n)), dim3(256), 0, st>>>(p, n);
         HIP_TRY(hipGetLastError());
         if (l.attn) {
             GqaBatchArgs a{};
@@ -951,7 +956,7 @@ static int step_batch(BlockSession *s, const uint32_t *tokens, uint32_t pos, uin
             gated_rows_kernel<T><<<dim3(n), dim3(256), 0, st>>>(static_cast<T *>(w.cat) + l.left_kp, l.out.kp, w.o, w.gate, l.onorm, d.heads, d.vdim, m->hp.eps, l.spec.delta_scale);
             HIP_TRY(hipGetLastError());
         }
-        const uint32_t tail = std::min(n, std::max(l.attn ? p.attn.ring : 0u, l.delta ? p.delta.taps : 0u));
+        const uint32_t tail = std::min(n, std::max(l.attn ? s->layers[i].ring : 0u, l.delta ? p.delta.taps : 0u));
         append_kernel<T><<<dim3(tail), dim3(256), 0, st>>>(p, n);
         HIP_TRY(hipGetLastError());
 

@@ -43,7 +43,7 @@ __global__ __launch_bounds__(256) void norm_rows_kernel(NormRowsArgs a)
             s = fmaf(v.x, v.x, s); s = fmaf(v.y, v.y, s); s = fmaf(v.z, v.z, s); s = fmaf(v.w, v.w, s);
             *reinterpret_cast<float4 *>(xs + i) = v;
         }
-        if (in.wpost) ypost = 1.f / sqrtf(block_sum_256(s, scratch) / (float)in.dim + in.eps);
+        if (in.wpost) ypost = rsqrtf(block_sum_256(s, scratch) / (float)in.dim + in.eps);
     }
     float s = 0.f;
     for (uint32_t i = threadIdx.x * 4; i < dp; i += 1024) {
@@ -58,7 +58,7 @@ __global__ __launch_bounds__(256) void norm_rows_kernel(NormRowsArgs a)
         *reinterpret_cast<float4 *>(xs + i) = v;
     }
     if (!a.act) return;
-    const float inv = 1.f / sqrtf(block_sum_256(s, scratch) / (float)in.dim + in.eps);
+    const float inv = rsqrtf(block_sum_256(s, scratch) / (float)in.dim + in.eps);
     for (uint32_t i = threadIdx.x * 4; i < dp; i += 1024) {
         const float4 v = *reinterpret_cast<const float4 *>(xs + i), w = *reinterpret_cast<const float4 *>(in.wpre + i);
         const float h[4] = {v.x * inv * w.x, v.y * inv * w.y, v.z * inv * w.z, v.w * inv * w.w};
@@ -85,84 +85,114 @@ __global__ __launch_bounds__(256) void mix_step_kernel(MixStepArgs a)
     else gqa_step<CT, DP, R>(a.attn, blockIdx.x - a.delta_wgs, lds);
 }
 
-// ---- batches: joint projection -> mixer operands, one workgroup per token --------------------------------------------------
+// ---- batches: joint projection -> mixer operands ---------------------------------------------------------------------------
 struct PrepareArgs {
     const float *y;              // [n][ldy]
-    uint32_t ldy, pos0, dp;      // dp: padded head size of q, k, v
+    uint32_t ldy, pos0, dp;      // dp: padded head size of q, k, v (a power of two)
     GqaSpec attn;                // heads 0: none
     void *q, *k, *v;
     DeltaSpec delta;             // heads 0: none
     float *dq, *dk, *dv, *beta, *qk;
     void *a1, *g1;               // low-rank activations [n][a_kp], [n][g_kp]
 };
-template <class T>
-__global__ __launch_bounds__(256) void prepare_kernel(PrepareArgs a)
+constexpr uint32_t kPrepareTokens = 8;     // per workgroup of the recurrent branch
+// workgroups: one per token (attention, and what is small), then per 8 tokens one for each key head and each 256 value channels
+inline uint32_t prepare_columns(const DeltaSpec &s) { return s.heads ? s.kv_heads + (s.heads * s.vdim + 255) / 256 : 0; }
+inline uint32_t prepare_grid(const PrepareArgs &a, uint32_t n) { return n + (n + kPrepareTokens - 1) / kPrepareTokens * prepare_columns(a.delta); }
+
+template <class T> __device__ __forceinline__ void store_pair(T *o, float u, float v)
 {
-    __shared__ float scratch[4];
-    __shared__ float2 turn[kGqaMaxDim / 2];
-    const uint32_t t = blockIdx.x, pos = a.pos0 + t;
+    if constexpr (sizeof(T) == 2) *reinterpret_cast<uint32_t *>(o) = (uint32_t)float_to_bf16(u) | ((uint32_t)float_to_bf16(v) << 16);
+    else *reinterpret_cast<float2 *>(o) = make_float2(u, v);
+}
+
+template <class T>
+__device__ __forceinline__ void prepare_token(const PrepareArgs &a, uint32_t t, float2 *turn, float *scratch)
+{
+    const uint32_t pos = a.pos0 + t;
     const float *y = a.y + (size_t)t * a.ldy;
     if (a.attn.heads) {
         const GqaSpec &s = a.attn;
-        const uint32_t half = a.dp / 2;
+        const uint32_t sh = 31 - __clz(a.dp / 2);
         rotation_table(turn, s, pos);
-        const float inv_q = projection_inv(y + s.q_off, s.heads * s.dim, s.eps, s.q_norm, scratch);
-        const float inv_k = projection_inv(y + s.k_off, s.kv_heads * s.dim, s.eps, s.k_norm, scratch);
-        __syncthreads();
-        for (uint32_t i = threadIdx.x; i < s.heads * half; i += 256) {
-            const uint32_t h = i / half, p = i % half;
+        float sq[2] = {0.f, 0.f};
+        if (s.q_norm) {
+            for (uint32_t i = threadIdx.x; i < s.heads * s.dim; i += 256) sq[0] = fmaf(y[s.q_off + i], y[s.q_off + i], sq[0]);
+            for (uint32_t i = threadIdx.x; i < s.kv_heads * s.dim; i += 256) sq[1] = fmaf(y[s.k_off + i], y[s.k_off + i], sq[1]);
+        }
+        block_sums_waves<2>(sq, scratch, 4);
+        const float inv_q = s.q_norm ? rsqrtf(sq[0] / (float)(s.heads * s.dim) + s.eps) : 1.f;
+        const float inv_k = s.q_norm ? rsqrtf(sq[1] / (float)(s.kv_heads * s.dim) + s.eps) : 1.f;
+        for (uint32_t i = threadIdx.x; i < s.heads << sh; i += 256) {
+            const uint32_t h = i >> sh, p = i & ((1u << sh) - 1);
             float u, v;
             head_pair(u, v, y + s.q_off, s.q_norm, h * s.dim, p, s.dim, inv_q, s, turn);
-            T *o = static_cast<T *>(a.q) + ((size_t)t * s.heads + h) * a.dp + 2 * p;
-            o[0] = float_to_elem<T>(u * s.scale);
-            o[1] = float_to_elem<T>(v * s.scale);
+            store_pair(static_cast<T *>(a.q) + ((size_t)t * s.heads + h) * a.dp + 2 * p, u * s.scale, v * s.scale);
         }
-        for (uint32_t i = threadIdx.x; i < s.kv_heads * half; i += 256) {
-            const uint32_t h = i / half, p = i % half;
+        for (uint32_t i = threadIdx.x; i < s.kv_heads << sh; i += 256) {
+            const uint32_t h = i >> sh, p = i & ((1u << sh) - 1);
             float u, v;
             head_pair(u, v, y + s.k_off, s.k_norm, h * s.dim, p, s.dim, inv_k, s, turn);
             const size_t o = ((size_t)t * s.kv_heads + h) * a.dp + 2 * p;
-            static_cast<T *>(a.k)[o] = float_to_elem<T>(u);
-            static_cast<T *>(a.k)[o + 1] = float_to_elem<T>(v);
-            static_cast<T *>(a.v)[o] = float_to_elem<T>(2 * p < s.vdim ? y[s.v_off + h * s.vdim + 2 * p] : 0.f);
-            static_cast<T *>(a.v)[o + 1] = float_to_elem<T>(2 * p + 1 < s.vdim ? y[s.v_off + h * s.vdim + 2 * p + 1] : 0.f);
+            store_pair(static_cast<T *>(a.k) + o, u, v);
+            const float *yv = y + s.v_off + h * s.vdim + 2 * p;
+            store_pair(static_cast<T *>(a.v) + o, 2 * p < s.vdim ? yv[0] : 0.f, 2 * p + 1 < s.vdim ? yv[1] : 0.f);
         }
     }
     if (a.delta.heads) {
         const DeltaSpec &s = a.delta;
-        const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nq = s.kv_heads * s.dim;
-        for (uint32_t h = wave; h < s.kv_heads; h += 4) {
-            float q[kDeltaMaxDim / 64], k[kDeltaMaxDim / 64], sq = 0.f, sk = 0.f, sqk = 0.f;
-#pragma unroll
-            for (int j = 0; j < (int)kDeltaMaxDim / 64; j++) {
-                const uint32_t d = j * 64 + lane;
-                q[j] = k[j] = 0.f;
-                if (d < s.dim) {
-                    q[j] = delta_conv(s, y, a.ldy, t, h * s.dim + d, pos);
-                    k[j] = delta_conv(s, y, a.ldy, t, nq + h * s.dim + d, pos);
-                }
-                sq = fmaf(q[j], q[j], sq);
-                sk = fmaf(k[j], k[j], sk);
-            }
-            const float fq = 1.f / sqrtf(wave_sum(sq) + 1e-6f) / sqrtf((float)s.dim), fk = 1.f / sqrtf(wave_sum(sk) + 1e-6f);
-#pragma unroll
-            for (int j = 0; j < (int)kDeltaMaxDim / 64; j++) {
-                const uint32_t d = j * 64 + lane;
-                q[j] *= fq;
-                k[j] *= fk;
-                sqk = fmaf(q[j], k[j], sqk);
-                if (d < s.dstride) {
-                    a.dq[((size_t)t * s.kv_heads + h) * s.dstride + d] = q[j];
-                    a.dk[((size_t)t * s.kv_heads + h) * s.dstride + d] = k[j];
-                }
-            }
-            sqk = wave_sum(sqk);
-            if (lane == 0) a.qk[(size_t)t * s.kv_heads + h] = sqk;
-        }
-        for (uint32_t c = threadIdx.x; c < s.heads * s.vdim; c += 256) a.dv[(size_t)t * s.heads * s.vdim + c] = delta_conv(s, y, a.ldy, t, 2 * nq + c, pos);
         for (uint32_t h = threadIdx.x; h < s.heads; h += 256) a.beta[(size_t)t * s.heads + h] = sigmoid_f(y[s.b_off + h]);
         for (uint32_t i = threadIdx.x; i < s.a_kp; i += 256) static_cast<T *>(a.a1)[(size_t)t * s.a_kp + i] = float_to_elem<T>(i < s.a_rank ? y[s.a_off + i] : 0.f);
         for (uint32_t i = threadIdx.x; i < s.g_kp; i += 256) static_cast<T *>(a.g1)[(size_t)t * s.g_kp + i] = float_to_elem<T>(i < s.g_rank ? y[s.g_off + i] : 0.f);
+    }
+}
+
+template <class T>
+__global__ __launch_bounds__(256) void prepare_kernel(PrepareArgs a, uint32_t n)
+{
+    __shared__ float scratch[8];
+    __shared__ float2 turn[kGqaMaxDim / 2];
+    if (blockIdx.x < n) return prepare_token<T>(a, blockIdx.x, turn, scratch);
+    const DeltaSpec &s = a.delta;
+    const uint32_t nq = s.kv_heads * s.dim, nv = s.heads * s.vdim, cols = s.kv_heads + (nv + 255) / 256;
+    const uint32_t idx = blockIdx.x - n, col = idx % cols, first = idx / cols * kPrepareTokens, last = min(first + kPrepareTokens, n);
+    if (col >= s.kv_heads) {
+        const uint32_t c = (col - s.kv_heads) * 256 + threadIdx.x;
+        if (c >= nv) return;
+        for (uint32_t t = first; t < last; t++)
+            a.dv[(size_t)t * nv + c] = delta_conv(s, a.y + (size_t)t * a.ldy, a.ldy, t, 2 * nq + c, a.pos0 + t, (a.pos0 + t) % s.taps);
+        return;
+    }
+    const uint32_t lane = threadIdx.x & 63, h = col;
+    for (uint32_t t = first + (threadIdx.x >> 6); t < last; t += 4) {
+        const uint32_t pos = a.pos0 + t, slot = pos % s.taps;
+        const float *y = a.y + (size_t)t * a.ldy;
+        float q[kDeltaMaxDim / 64], k[kDeltaMaxDim / 64], sq = 0.f, sk = 0.f, sqk = 0.f;
+#pragma unroll
+        for (int j = 0; j < (int)kDeltaMaxDim / 64; j++) {
+            const uint32_t d = j * 64 + lane;
+            q[j] = k[j] = 0.f;
+            if (d < s.dim) {
+                q[j] = delta_conv(s, y, a.ldy, t, h * s.dim + d, pos, slot);
+                k[j] = delta_conv(s, y, a.ldy, t, nq + h * s.dim + d, pos, slot);
+            }
+            sq = fmaf(q[j], q[j], sq);
+            sk = fmaf(k[j], k[j], sk);
+        }
+        const float fq = rsqrtf(wave_sum(sq) + 1e-6f) * rsqrtf((float)s.dim), fk = rsqrtf(wave_sum(sk) + 1e-6f);
+#pragma unroll
+        for (int j = 0; j < (int)kDeltaMaxDim / 64; j++) {
+            const uint32_t d = j * 64 + lane;
+            q[j] *= fq;
+            k[j] *= fk;
+            sqk = fmaf(q[j], k[j], sqk);
+            if (d < s.dstride) {
+                a.dq[((size_t)t * s.kv_heads + h) * s.dstride + d] = q[j];
+                a.dk[((size_t)t * s.kv_heads + h) * s.dstride + d] = k[j];
+            }
+        }
+        sqk = wave_sum(sqk);
+        if (lane == 0) a.qk[(size_t)t * s.kv_heads + h] = sqk;
     }
 }
 
@@ -172,12 +202,15 @@ template <class T>
 __global__ __launch_bounds__(256) void append_kernel(PrepareArgs a, uint32_t n)
 {
     const uint32_t t = n - 1 - blockIdx.x, pos = a.pos0 + t;
-    if (a.attn.heads && blockIdx.x < a.attn.ring) {
-        const uint32_t w = a.attn.kv_heads * a.dp;
-        const size_t dst = (size_t)(pos % a.attn.ring) * w, src = (size_t)t * w;
+    // cache rows: what the next position's chunk may still need of this batch
+    const uint32_t c0 = a.attn.heads ? gqa_chunk_start(a.attn, a.pos0 + n - 1) : 0;
+    if (a.attn.heads && pos >= c0) {
+        const uint32_t w = a.attn.kv_heads * a.dp / 8;      // 8 elements at a time
+        const size_t dst = (size_t)(pos - c0) * w, src = (size_t)t * w;
+        struct alignas(16) Eight { T e[8]; };
         for (uint32_t i = threadIdx.x; i < w; i += 256) {
-            static_cast<T *>(a.attn.kc)[dst + i] = static_cast<const T *>(a.k)[src + i];
-            static_cast<T *>(a.attn.vc)[dst + i] = static_cast<const T *>(a.v)[src + i];
+            static_cast<Eight *>(a.attn.kc)[dst + i] = static_cast<const Eight *>(a.k)[src + i];
+            static_cast<Eight *>(a.attn.vc)[dst + i] = static_cast<const Eight *>(a.v)[src + i];
         }
     }
     if (a.delta.heads && blockIdx.x < a.delta.taps) {

@@ -23,7 +23,7 @@ struct DeltaSpec {
     uint32_t heads, kv_heads, dim, vdim, taps;
     uint32_t q_off, k_off, v_off, b_off, a_off, g_off;   // offsets in a token's joint projection
     uint32_t a_rank, g_rank, a_kp, g_kp;                 // low-rank widths of decay and gate, as stored (padded to 64)
-    const float *conv;             // [channels][taps], last column = the current token
+    const float *conv;             // [taps][channels], last row = the current token
     const float *a_log, *dt_bias, *norm;
     const uint16_t *a2, *g2;       // [heads * dim][a_kp], [heads * vdim][g_kp]
     float eps;
@@ -52,21 +52,21 @@ __device__ __forceinline__ uint32_t delta_channel_at(const DeltaSpec &s, uint32_
     return c < nq ? s.q_off + c : c < 2 * nq ? s.k_off + (c - nq) : s.v_off + (c - 2 * nq);
 }
 
-// convolution and silu of channel c at position pos.  y: the token's projection row; rows before it (in steps of ld floats)
+// convolution and silu of channel c at position pos (slot = pos % taps).  y: the token's projection row; rows before it (in steps of ld floats)
 // belong to positions pos - 1, pos - 2, .. as far as `behind` of them, older inputs are in the ring.
-__device__ __forceinline__ float delta_conv(const DeltaSpec &s, const float *y, size_t ld, uint32_t behind, uint32_t c, uint32_t pos)
+__device__ __forceinline__ float delta_conv(const DeltaSpec &s, const float *y, size_t ld, uint32_t behind, uint32_t c, uint32_t pos, uint32_t slot)
 {
-    const float *w = s.conv + (size_t)c * s.taps;
     const uint32_t at = delta_channel_at(s, c), C = s.channels();
-    float v = w[s.taps - 1] * y[at];
+    const float *w = s.conv + (size_t)(s.taps - 1) * C + c;
+    float v = w[0] * y[at];
     for (uint32_t j0 = 1; j0 < s.taps && j0 <= pos; j0 += 3) {
         float x[3], f[3];      // three inputs on their way at once
 #pragma unroll
         for (uint32_t e = 0; e < 3; e++) {
             const uint32_t j = j0 + e;
             const bool ok = j < s.taps && j <= pos;
-            x[e] = !ok ? 0.f : j <= behind ? y[at - (ptrdiff_t)(j * ld)] : s.ring[(size_t)((pos - j) % s.taps) * C + c];
-            f[e] = ok ? w[s.taps - 1 - j] : 0.f;
+            x[e] = !ok ? 0.f : j <= behind ? y[at - (ptrdiff_t)(j * ld)] : s.ring[(size_t)(slot >= j ? slot - j : slot + s.taps - j) * C + c];
+            f[e] = ok ? w[-(ptrdiff_t)(j * (size_t)C)] : 0.f;
         }
 #pragma unroll
         for (int e = 0; e < 3; e++) v = fmaf(f[e], x[e], v);
@@ -146,14 +146,14 @@ __device__ __forceinline__ void delta_step(const DeltaStepArgs &a, uint32_t idx,
     rg.fetch(s.g2, head * s.vdim + c_lo + r8, head * s.vdim + c_lo + nc, s.g_kp);
     for (uint32_t i = threadIdx.x; i < s.a_kp; i += 256) al[i] = i < s.a_rank ? a.y[s.a_off + i] : 0.f;
     for (uint32_t i = threadIdx.x; i < s.g_kp; i += 256) gl[i] = i < s.g_rank ? a.y[s.g_off + i] : 0.f;
-    const float beta = sigmoid_f(a.y[s.b_off + head]), ea = expf(s.a_log[head]);
+    const float beta = sigmoid_f(a.y[s.b_off + head]), ea = __expf(s.a_log[head]);
 
     float qv = 0.f, kv = 0.f;
     const uint32_t d = threadIdx.x, rslot = pos % s.taps;
     if (d < s.dim) {
         const uint32_t cq = kvh * s.dim + d, ck = nq + cq;
-        qv = delta_conv(s, a.y, 0, 0, cq, pos);
-        kv = delta_conv(s, a.y, 0, 0, ck, pos);
+        qv = delta_conv(s, a.y, 0, 0, cq, pos, rslot);
+        kv = delta_conv(s, a.y, 0, 0, ck, pos, rslot);
         if (cb == 0 && head % rep == 0) {
             s.ring[(size_t)rslot * C + cq] = a.y[s.q_off + cq];
             s.ring[(size_t)rslot * C + ck] = a.y[s.k_off + cq];
@@ -161,12 +161,12 @@ __device__ __forceinline__ void delta_step(const DeltaStepArgs &a, uint32_t idx,
     }
     if (threadIdx.x < nc) {
         const uint32_t c = head * s.vdim + c_lo + threadIdx.x;
-        v[threadIdx.x] = delta_conv(s, a.y, 0, 0, 2 * nq + c, pos);
+        v[threadIdx.x] = delta_conv(s, a.y, 0, 0, 2 * nq + c, pos, rslot);
         s.ring[(size_t)rslot * C + 2 * nq + c] = a.y[s.v_off + c];
     }
     float sums[3] = {qv * qv, kv * kv, qv * kv};
     block_sums_waves<3>(sums, scratch, 4);      // also publishes al, gl and v
-    const float fq = 1.f / sqrtf(sums[0] + 1e-6f) / sqrtf((float)s.dim), fk = 1.f / sqrtf(sums[1] + 1e-6f), qk = sums[2] * fq * fk;
+    const float fq = rsqrtf(sums[0] + 1e-6f) * rsqrtf((float)s.dim), fk = rsqrtf(sums[1] + 1e-6f), qk = sums[2] * fq * fk;
     q[threadIdx.x] = qv * fq;
     k[threadIdx.x] = kv * fk;
     for (uint32_t r0 = 0; r0 < s.dstride; r0 += 128) {
@@ -177,7 +177,7 @@ __device__ __forceinline__ void delta_step(const DeltaStepArgs &a, uint32_t idx,
         for (int i = 0; i < 4; i++) {
             const uint32_t r = r0 + i * 32 + r8;
             if ((threadIdx.x & 7) == i && r < s.dstride)      // four lanes of the eight share the exponentials
-                g[r] = r < s.dim ? expf(-ea * softplus_f(t[i] + s.dt_bias[head * s.dim + r])) : 0.f;
+                g[r] = r < s.dim ? decay_f(ea, t[i] + s.dt_bias[head * s.dim + r]) : 0.f;
         }
     }
     {
@@ -230,7 +230,7 @@ struct DeltaScanArgs {
 };
 
 constexpr int kScanTokens = 16;   // tokens staged in LDS at a time
-template <int J> constexpr int scan_stage_floats() { return kScanTokens * (3 * 64 * J + 16 + 2); }
+template <int J> constexpr int scan_stage_floats() { return kScanTokens * (3 * 64 * J + 16) + 64; }
 
 // All tokens of a batch for 16 columns of one head: a workgroup of 4 waves, 4 columns a wave.  grid (heads, vdim / 16 up).
 template <int J>
@@ -248,48 +248,39 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaScanArgs a)
 #pragma unroll
     for (int j = 0; j < J; j++) S[j] = a.fresh || !live ? make_float4(0.f, 0.f, 0.f, 0.f) : colp[j * 16 + l16];
 
-    // one stage: per thread J float4 of each of k, q, g, one value of v, and beta / qk by the first threads
-    constexpr int PER = kScanTokens * W / 4 / 256;       // float4 per thread and array
-    float4 rk[PER], rq[PER], rg[PER];
-    float rv = 0.f, rb = 0.f;
-    auto fetch = [&](uint32_t t0) {
+    // One stage in LDS: k, q, g [16][W] each, v [16][16], beta [16], k.q [16].  Direct loads, lane after lane in LDS order; tokens
+    // past the end and columns past vdim bring some other value that nothing uses.
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    auto issue = [&](uint32_t t0, int st) {
+        float *b = lds + st * SF;
 #pragma unroll
-        for (int i = 0; i < PER; i++) {
-            const int e = i * 256 + threadIdx.x;
-            const uint32_t t = min(t0 + e / (W / 4), a.n - 1), d = e % (W / 4) * 4;
-            rk[i] = *reinterpret_cast<const float4 *>(a.k + ((size_t)t * s.kv_heads + kvh) * W + d);
-            rq[i] = *reinterpret_cast<const float4 *>(a.q + ((size_t)t * s.kv_heads + kvh) * W + d);
-            rg[i] = *reinterpret_cast<const float4 *>(a.g + ((size_t)t * s.heads + head) * W + d);
+        for (int i = 0; i < J; i++) {
+            const int e = i * 256 + wave * 64;                   // first float4 of the wave
+            const uint32_t t = min(t0 + (e + lane) / (W / 4), a.n - 1), d = (e + lane) % (W / 4) * 4;
+            const size_t kq = ((size_t)t * s.kv_heads + kvh) * W + d;
+            __builtin_amdgcn_global_load_lds((lv_glb_any *)(a.k + kq), (lv_lds_any *)(b + e * 4), 16, 0, 0);
+            __builtin_amdgcn_global_load_lds((lv_glb_any *)(a.q + kq), (lv_lds_any *)(b + kScanTokens * W + e * 4), 16, 0, 0);
+            __builtin_amdgcn_global_load_lds((lv_glb_any *)(a.g + ((size_t)t * s.heads + head) * W + d), (lv_lds_any *)(b + 2 * kScanTokens * W + e * 4), 16, 0, 0);
         }
         {
-            const uint32_t t = min(t0 + threadIdx.x / 16, a.n - 1), c = blockIdx.y * 16 + threadIdx.x % 16;
-            rv = c < s.vdim ? a.v[(size_t)t * HV + head * s.vdim + c] : 0.f;
+            const uint32_t t = min(t0 + wave * 4 + lane / 16, a.n - 1), c = min(blockIdx.y * 16 + lane % 16, s.vdim - 1);
+            __builtin_amdgcn_global_load_lds((lv_glb_any *)(a.v + (size_t)t * HV + head * s.vdim + c), (lv_lds_any *)(b + 3 * kScanTokens * W + wave * 64), 4, 0, 0);
         }
-        if (threadIdx.x < 32) {
-            const uint32_t t = min(t0 + (threadIdx.x & 15), a.n - 1);
-            rb = threadIdx.x < 16 ? a.beta[(size_t)t * s.heads + head] : a.qk[(size_t)t * s.kv_heads + kvh];
+        if (wave == 0) {
+            const uint32_t t = min(t0 + (lane & 15), a.n - 1);
+            const float *src = lane & 16 ? a.qk + (size_t)t * s.kv_heads + kvh : a.beta + (size_t)t * s.heads + head;
+            __builtin_amdgcn_global_load_lds((lv_glb_any *)src, (lv_lds_any *)(b + 3 * kScanTokens * W + 256), 4, 0, 0);
         }
     };
-    auto stash = [&](float *b) {
-#pragma unroll
-        for (int i = 0; i < PER; i++) {
-            const int e = (i * 256 + threadIdx.x) * 4;
-            *reinterpret_cast<float4 *>(b + e) = rk[i];
-            *reinterpret_cast<float4 *>(b + kScanTokens * W + e) = rq[i];
-            *reinterpret_cast<float4 *>(b + 2 * kScanTokens * W + e) = rg[i];
-        }
-        b[3 * kScanTokens * W + threadIdx.x] = rv;
-        if (threadIdx.x < 32) b[3 * kScanTokens * W + 256 + threadIdx.x] = rb;
-    };
-    fetch(0);
-    stash(lds);
+    issue(0, 0);
     for (uint32_t t0 = 0, st = 0; t0 < a.n; t0 += kScanTokens, st ^= 1) {
-        __syncthreads();
-        if (t0 + kScanTokens < a.n) fetch(t0 + kScanTokens);
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        __syncthreads();      // this stage is in LDS for everyone, and everyone is done with the other one
+        if (t0 + kScanTokens < a.n) issue(t0 + kScanTokens, st ^ 1);
         const float *b = lds + st * SF, *bk = b, *bq = b + kScanTokens * W, *bg = b + 2 * kScanTokens * W, *bv = b + 3 * kScanTokens * W;
-        float keep = 0.f;
+        uint32_t keep = 0;
         const int nt = (int)min((uint32_t)kScanTokens, a.n - t0);
-        auto token = [&](int t) {
+        auto token = [&](int t) __attribute__((always_inline)) {
             float pk = 0.f, pq = 0.f;
             float4 kk[J];
 #pragma unroll
@@ -308,7 +299,8 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaScanArgs a)
             for (int j = 0; j < J; j++) {
                 S[j].x = fmaf(kk[j].x, u, S[j].x); S[j].y = fmaf(kk[j].y, u, S[j].y); S[j].z = fmaf(kk[j].z, u, S[j].z); S[j].w = fmaf(kk[j].w, u, S[j].w);
             }
-            if (l16 == t) keep = fmaf(bv[272 + t], u, pq);
+            // lane t of the sixteen stores token t's read-out; picked by a mask, so that no branch parts the tokens
+            keep |= __float_as_uint(fmaf(bv[272 + t], u, pq)) & (uint32_t)((int)((l16 ^ t) - 1) >> 31);
         };
         if (nt == kScanTokens) {
 #pragma unroll
@@ -316,8 +308,7 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaScanArgs a)
         } else {
             for (int t = 0; t < nt; t++) token(t);
         }
-        if (live && l16 < nt) a.o[(size_t)(t0 + l16) * HV + head * s.vdim + col] = keep;
-        if (t0 + kScanTokens < a.n) stash(lds + (st ^ 1) * SF);
+        if (live && l16 < nt) a.o[(size_t)(t0 + l16) * HV + head * s.vdim + col] = __uint_as_float(keep);
     }
     if (live) {
 #pragma unroll

@@ -6,10 +6,11 @@
 //   s      = (q . k) * scale, over the keys j <= i with j / chunk == i / chunk (chunk 0: every j <= i)
 //   out    = sum_j exp(s_j) v_j / (sum_j exp(s_j) + exp(sink))
 //
-// Cache: per layer two rings of `ring` rows, [row][kv head][DP] each, DP = head size rounded up to a power of two; position p
-// lives in row p % ring.  A chunked layer needs chunk rows whatever the length of the sequence.  A batch of tokens keeps its
-// own rows in scratch while it is evaluated (keys from the batch's first position on come from there, older ones from the
-// ring) and is appended to the ring afterwards, so that a batch may run over any number of chunk borders.
+// Cache: per layer two rings of rows, [row][kv head][DP] each, DP = head size rounded up to a power of two; a position lives in
+// the row that counts it from its chunk's start, so a chunked layer needs chunk rows whatever the length of the sequence, and
+// a new chunk overwrites the one before.  A batch of tokens keeps its own rows in scratch while it is evaluated (keys from the
+// batch's first position on come from there, older ones from the ring); those of its last chunk are appended afterwards, so
+// that a batch may run over any number of chunk borders.
 //
 // Everything but the MFMA path (attention_tile_kernel: bf16 operands, weights as two bf16 pieces) is fp32 arithmetic on
 // cache rows of either element type.
@@ -24,12 +25,13 @@ struct GqaSpec {
     uint32_t q_off, k_off, v_off;       // where a token's projections start in its row of the joint projection
     const float *q_norm, *k_norm;       // null: not normalised
     const float *sink;                  // null: none
-    const double *freq;                 // rot_dims / 2 angles per position
+    const double *freq;                 // rot_dims / 2 angles per position, in full turns
     uint32_t rot_dims, chunk;
     float scale, eps;
-    uint32_t ring;                      // cache rows
     void *kc, *vc;
 };
+
+__device__ __forceinline__ uint32_t gqa_chunk_start(const GqaSpec &s, uint32_t pos) { return s.chunk ? pos - pos % s.chunk : 0; }
 
 struct GqaStepArgs {
     GqaSpec s;
@@ -54,9 +56,9 @@ constexpr uint32_t kGqaMaxDim = 256;
 __device__ __forceinline__ void rotation_table(float2 *turn, const GqaSpec &s, uint32_t pos)
 {
     for (uint32_t i = threadIdx.x; i < s.rot_dims / 2; i += blockDim.x) {
-        const double a = (double)pos * s.freq[i], full = 6.283185307179586476925;
+        const double a = (double)pos * s.freq[i];      // in turns
         float sn, cs;
-        sincosf((float)(a - full * rint(a / full)), &sn, &cs);
+        sincospif(2.f * (float)(a - rint(a)), &sn, &cs);
         turn[i] = make_float2(cs, sn);
     }
 }
@@ -151,7 +153,7 @@ __device__ __forceinline__ float projection_inv(const float *y, uint32_t n, floa
     if (!w) return 1.f;
     float s = 0.f;
     for (uint32_t i = threadIdx.x; i < n; i += blockDim.x) s = fmaf(y[i], y[i], s);
-    return 1.f / sqrtf(block_sum_waves(s, scratch, blockDim.x >> 6) / (float)n + eps);
+    return rsqrtf(block_sum_waves(s, scratch, blockDim.x >> 6) / (float)n + eps);
 }
 
 // elements 2i, 2i+1 of one head, normalised and rotated
@@ -205,7 +207,7 @@ __device__ __forceinline__ void gqa_step(const GqaStepArgs &a, uint32_t idx, flo
     const GqaSpec &s = a.s;
     const uint32_t split = idx % a.splits, grp = idx / a.splits, hg = grp % a.groups, kvh = grp / a.groups;
     const uint32_t pos = *a.pos_ptr + a.pos_add;
-    const uint32_t c0 = s.chunk ? pos / s.chunk * s.chunk : 0;
+    const uint32_t c0 = gqa_chunk_start(s, pos);
     const uint32_t active = (pos - c0) / SPLIT + 1;
     if (split >= active) return;
     const uint32_t k_begin = c0 + split * SPLIT, n = min((uint32_t)SPLIT, pos + 1 - k_begin);
@@ -216,13 +218,13 @@ __device__ __forceinline__ void gqa_step(const GqaStepArgs &a, uint32_t idx, flo
     GqaRaw<CT> kraw[ROUNDS], vraw[ROUNDS];
 #pragma unroll
     for (int i = 0; i < ROUNDS; i++) {
-        const uint32_t p = k_begin + min((uint32_t)(i * L::KPR + kg), n - 1);
-        kraw[i].load(kc + ((size_t)(p % s.ring) * s.kv_heads + kvh) * DP + sub * 8);
+        const uint32_t row = split * SPLIT + min((uint32_t)(i * L::KPR + kg), n - 1);
+        kraw[i].load(kc + ((size_t)row * s.kv_heads + kvh) * DP + sub * 8);
     }
 #pragma unroll
     for (int i = 0; i < ROUNDS; i++) {
-        const uint32_t p = k_begin + min((uint32_t)(i * L::KPR + kg), n - 1);
-        vraw[i].load(vc + ((size_t)(p % s.ring) * s.kv_heads + kvh) * DP + sub * 8);
+        const uint32_t row = split * SPLIT + min((uint32_t)(i * L::KPR + kg), n - 1);
+        vraw[i].load(vc + ((size_t)row * s.kv_heads + kvh) * DP + sub * 8);
     }
     float *q = lds, *krow = q + R * DP, *vrow = krow + DP, *sc = vrow + DP, *red = sc + R * kGqaSplit, *ml = red + 4 * R * DP, *scratch = ml + 4 * R;
     float2 *turn = reinterpret_cast<float2 *>(scratch + 16);
@@ -238,8 +240,8 @@ __device__ __forceinline__ void gqa_step(const GqaStepArgs &a, uint32_t idx, flo
     }
     rotation_table(turn, s, pos);
     block_sums_waves<2>(sq, scratch, 4);      // also publishes the rotation table
-    const float inv_q = s.q_norm ? 1.f / sqrtf(sq[0] / (float)(s.heads * s.dim) + s.eps) : 1.f;
-    const float inv_k = s.q_norm ? 1.f / sqrtf(sq[1] / (float)(s.kv_heads * s.dim) + s.eps) : 1.f;
+    const float inv_q = s.q_norm ? rsqrtf(sq[0] / (float)(s.heads * s.dim) + s.eps) : 1.f;
+    const float inv_k = s.q_norm ? rsqrtf(sq[1] / (float)(s.kv_heads * s.dim) + s.eps) : 1.f;
     for (uint32_t i = threadIdx.x; i < R * DP / 2; i += 256) {
         const uint32_t r = i / (DP / 2), p = i % (DP / 2);
         float u = 0.f, v = 0.f;
@@ -248,7 +250,7 @@ __device__ __forceinline__ void gqa_step(const GqaStepArgs &a, uint32_t idx, flo
         q[r * DP + 2 * p + 1] = v * s.scale;
     }
     if (own) {
-        const size_t row = ((size_t)(pos % s.ring) * s.kv_heads + kvh) * DP;
+        const size_t row = ((size_t)(pos - c0) * s.kv_heads + kvh) * DP;
         for (uint32_t p = threadIdx.x; p < DP / 2; p += 256) {
             float u, v;
             head_pair(u, v, yk, s.k_norm, kvh * s.dim, p, s.dim, inv_k, s, turn);
@@ -342,35 +344,34 @@ __device__ __forceinline__ void gqa_step(const GqaStepArgs &a, uint32_t idx, flo
     __syncthreads();
     if (*arrived != active - 1) return;
     auto get = [&](uint32_t sp, uint32_t i) { return __uint_as_float(__hip_atomic_load(part + (size_t)sp * PS + i, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT)); };
-    // per head: the largest score and the sum over the splits, sink included; a wave per head, a lane per split
-    for (int r = wave; r < R; r += 4) {
-        const float sk = s.sink && r < (int)nh ? s.sink[h0 + r] : -INFINITY;
-        float M = sk;
-        for (uint32_t sp = lane; sp < active; sp += 64) M = fmaxf(M, get(sp, r * (DP + 2) + DP));
-#pragma unroll
-        for (int off = 1; off < 64; off <<= 1) M = fmaxf(M, __shfl_xor(M, off, 64));
-        float l = 0.f;
-        for (uint32_t sp = lane; sp < active; sp += 64) l += get(sp, r * (DP + 2) + DP + 1) * __expf(get(sp, r * (DP + 2) + DP) - M);
-        l = wave_sum(l) + __expf(sk - M);
-        if (lane == 0) { ml[2 * r] = M; ml[2 * r + 1] = l; }
-    }
-    __syncthreads();
+    // every thread sums its element over the splits, in split order, with a running maximum of its own: one pass of loads
     for (uint32_t i = threadIdx.x; i < nh * s.vdim; i += 256) {
         const uint32_t r = i / s.vdim, c = i % s.vdim;
-        float t = 0.f;
-        for (uint32_t s0 = 0; s0 < active; s0 += 8) {       // eight splits' loads in flight, summed in split order
-            float v[8], w[8];
+        float M = s.sink ? s.sink[h0 + r] : -INFINITY, l = s.sink ? 1.f : 0.f, t = 0.f;
+        for (uint32_t s0 = 0; s0 < active; s0 += 8) {
+            float v[8], w[8], z[8];
 #pragma unroll
             for (int e = 0; e < 8; e++) {
                 const uint32_t sp = min(s0 + e, active - 1);
                 v[e] = get(sp, r * (DP + 2) + c);
                 w[e] = get(sp, r * (DP + 2) + DP);
+                z[e] = get(sp, r * (DP + 2) + DP + 1);
             }
+            float top = M;
 #pragma unroll
-            for (int e = 0; e < 8; e++)
-                if (s0 + e < active) t = fmaf(v[e], __expf(w[e] - ml[2 * r]), t);
+            for (int e = 0; e < 8; e++) top = fmaxf(top, w[e]);
+            const float f = __expf(M - top);
+            M = top;
+            t *= f;
+            l *= f;
+#pragma unroll
+            for (int e = 0; e < 8; e++) {
+                const float p = s0 + e < active ? __expf(w[e] - top) : 0.f;
+                t = fmaf(v[e], p, t);
+                l = fmaf(z[e], p, l);
+            }
         }
-        a.out[(h0 + r) * s.vdim + c] = t / ml[2 * r + 1];
+        a.out[(h0 + r) * s.vdim + c] = t / l;
     }
     if (threadIdx.x == 0) a.counters[grp] = 0u;
 }
@@ -410,13 +411,13 @@ __global__ __launch_bounds__(256) void gqa_rows_kernel(GqaBatchArgs a)
     for (int r = 0; r < R; r++)
 #pragma unroll
         for (int e = 0; e < 8; e++) acc[r][e] = 0.f;
-    const uint32_t c0 = s.chunk ? pos / s.chunk * s.chunk : 0;
+    const uint32_t c0 = gqa_chunk_start(s, pos);
     for (uint32_t k_begin = c0; k_begin <= pos; k_begin += kGqaSplit) {
         const uint32_t n = min((uint32_t)kGqaSplit, pos + 1 - k_begin);
         auto from = [&](const void *ring, const void *mine, uint32_t j, int d, float (&f)[8]) {
             const uint32_t p = k_begin + j;
             if (p >= a.pos0) load8(f, static_cast<const CT *>(mine) + ((size_t)(p - a.pos0) * s.kv_heads + kvh) * DP + d);
-            else load8(f, static_cast<const CT *>(ring) + ((size_t)(p % s.ring) * s.kv_heads + kvh) * DP + d);
+            else load8(f, static_cast<const CT *>(ring) + ((size_t)(p - c0) * s.kv_heads + kvh) * DP + d);
         };
         gqa_scores<DP, R>(q, sc, n, [&](uint32_t j, int d, float (&f)[8]) { from(s.kc, a.k, j, d, f); });
         __syncthreads();

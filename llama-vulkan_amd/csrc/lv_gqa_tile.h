@@ -14,7 +14,7 @@ namespace lv {
 
 struct GqaTileArgs {
     GqaBatchArgs b;
-    uint32_t base;       // position of the first key any query of the batch can see
+    uint32_t base;       // position of the first key any query of the batch can see: the start of its first token's chunk
     uint32_t keys;       // keys from there to the batch's last position
     uint32_t vt_ld;      // keys rounded up to 64
     uint16_t *vt;        // [kv head][DP][vt_ld]
@@ -27,7 +27,7 @@ __device__ __forceinline__ const uint16_t *gqa_row(const GqaTileArgs &a, const v
 {
     const GqaSpec &s = a.b.s;
     return p >= a.b.pos0 ? static_cast<const uint16_t *>(mine) + ((size_t)(p - a.b.pos0) * s.kv_heads + kvh) * dp
-                         : static_cast<const uint16_t *>(ring) + ((size_t)(p % s.ring) * s.kv_heads + kvh) * dp;
+                         : static_cast<const uint16_t *>(ring) + ((size_t)(p - a.base) * s.kv_heads + kvh) * dp;
 }
 
 // grid (kv heads, vt_ld / 64): transposes 64 keys' values
@@ -74,7 +74,7 @@ __global__ __launch_bounds__(256) void gqa_tile_kernel(GqaTileArgs a)
     const uint32_t head = blockIdx.x, kvh = head / (s.heads / s.kv_heads);
     const uint32_t t0 = (gridDim.y - 1 - blockIdx.y) * 64 * QT;      // the tiles with the most keys start first
     const uint32_t last = min(t0 + 64 * QT, a.b.n) - 1;
-    auto chunk_start = [&](uint32_t p) { return s.chunk ? p / s.chunk * s.chunk : 0u; };
+    auto chunk_start = [&](uint32_t p) { return gqa_chunk_start(s, p); };
 
     // this lane's queries: one per 16-query tile
     lv_bf8 q[QT][KS];
