@@ -631,6 +631,17 @@ template <class Fn> static int gqa_dispatch(bool f32, const BlockLayer &l, Fn &&
     return f32 ? with_dp(float{}) : with_dp(uint16_t{});
 }
 
+// calls fn(integral constant J) for a delta rule's key channels in units of 64
+template <class Fn> static int with_j(uint32_t j, Fn &&fn)
+{
+    switch (j) {
+    case 1: return fn(std::integral_constant<int, 1>{});
+    case 2: return fn(std::integral_constant<int, 2>{});
+    case 3: return fn(std::integral_constant<int, 3>{});
+    default: return fn(std::integral_constant<int, 4>{});
+    }
+}
+
 static GqaSpec gqa_spec(const BlockSession *s, size_t i)
 {
     const BlockLayer &l = s->m->layers[i];
@@ -714,10 +725,10 @@ int block_step_token(BlockSession *s, const uint32_t *cfg, uint32_t idx, float *
         const uint32_t wgs = mx.delta_wgs + (l.attn ? l.spec.attn.kv_heads * l.groups * mx.attn.splits : 0);
         LV_TRY(gqa_dispatch(m->f32, l, [&](auto elem, auto dp, auto r) -> int {
             constexpr int DP = decltype(dp)::value, R = decltype(r)::value;
-            const size_t lds = 4ull * std::max<uint32_t>(l.attn ? gqa_lds_floats<DP, R>() : 0, l.delta ? delta_step_lds_floats(l.a2.kp, l.g2.kp) : 0);
+            const size_t lds = 4ull * std::max<uint32_t>(l.attn ? gqa_lds_floats<DP, R, kGqaStepThreads>() : 0, l.delta ? delta_step_lds_floats(l.a2.kp, l.g2.kp) : 0);
             auto *k = &mix_step_kernel<decltype(elem), DP, R>;
             LV_TRY(allow_lds(k, lds));
-            k<<<dim3(wgs), dim3(256), lds, st>>>(mx);
+            k<<<dim3(wgs), dim3(kGqaStepThreads), lds, st>>>(mx);
             HIP_TRY(hipGetLastError());
             return LV_OK;
         }));
@@ -910,8 +921,11 @@ static int step_batch(BlockSession *s, const uint32_t *tokens, uint32_t pos, uin
         p.y = w.y1; p.ldy = l.in.rows; p.pos0 = pos; p.dp = l.dp;
         p.attn = gqa_spec(s, i); p.q = w.q; p.k = w.k; p.v = w.v;
         p.delta = delta_spec(s, i); p.dq = w.dq; p.dk = w.dk; p.dv = w.dv; p.beta = w.beta; p.qk = w.qk; p.a1 = w.a1; p.g1 = w.g1;
-        prepare_kernel<T><<<dim3(prepare_grid(p, n)), dim3(256), 0, st>>>(p, n);
-        HIP_TRY(hipGetLastError());
+        LV_TRY(with_j(l.delta ? l.dstride() / 64 : 1, [&](auto j) -> int {
+            prepare_kernel<T, decltype(j)::value><<<dim3(prepare_grid(p, n)), dim3(256), 0, st>>>(p, n);
+            HIP_TRY(hipGetLastError());
+            return LV_OK;
+        }));
         if (l.attn) {
             GqaBatchArgs a{};
             a.s = p.attn; a.pos0 = pos; a.n = n; a.q = w.q; a.k = w.k; a.v = w.v; a.out = w.cat; a.ldo = l.out.kp; a.groups = l.groups;
@@ -920,7 +934,10 @@ static int step_batch(BlockSession *s, const uint32_t *tokens, uint32_t pos, uin
                 LV_TRY(gqa_dispatch(f32, l, [&](auto elem, auto dp, auto r) -> int {
                     constexpr int DP = decltype(dp)::value, R = decltype(r)::value;
                     if constexpr (std::is_same_v<decltype(elem), float>) {
-                        gqa_rows_kernel<float, DP, R><<<dim3(l.spec.attn.kv_heads * l.groups, n), dim3(256), 4 * gqa_lds_floats<DP, R>(), st>>>(a);
+                        auto *k = &gqa_rows_kernel<float, DP, R>;
+                        const size_t lds = 4 * gqa_lds_floats<DP, R, kGqaRowThreads>();
+                        LV_TRY(allow_lds(k, lds));
+                        k<<<dim3(l.spec.attn.kv_heads * l.groups, n), dim3(kGqaRowThreads), lds, st>>>(a);
                         HIP_TRY(hipGetLastError());
                     }
                     return LV_OK;
@@ -939,20 +956,14 @@ static int step_batch(BlockSession *s, const uint32_t *tokens, uint32_t pos, uin
             LV_TRY((gemm<kEpSigmoid, false>(st, f32, gg, l.g2, n)));
             DeltaScanArgs sc{};
             sc.s = p.delta; sc.n = n; sc.fresh = pos == 0; sc.q = w.dq; sc.k = w.dk; sc.v = w.dv; sc.g = w.dg; sc.beta = w.beta; sc.qk = w.qk; sc.o = w.o;
-            auto scan = [&](auto j) -> int {
+            LV_TRY(with_j(l.dstride() / 64, [&](auto j) -> int {
                 constexpr int J = decltype(j)::value;
                 const size_t lds = 2 * 4ull * scan_stage_floats<J>();
                 LV_TRY(allow_lds(&delta_scan_kernel<J>, lds));
                 delta_scan_kernel<J><<<dim3(d.heads, (d.vdim + 15) / 16), dim3(256), lds, st>>>(sc);
                 HIP_TRY(hipGetLastError());
                 return LV_OK;
-            };
-            switch (l.dstride() / 64) {
-            case 1: LV_TRY(scan(std::integral_constant<int, 1>{})); break;
-            case 2: LV_TRY(scan(std::integral_constant<int, 2>{})); break;
-            case 3: LV_TRY(scan(std::integral_constant<int, 3>{})); break;
-            default: LV_TRY(scan(std::integral_constant<int, 4>{})); break;
-            }
+            }));
             gated_rows_kernel<T><<<dim3(n), dim3(256), 0, st>>>(static_cast<T *>(w.cat) + l.left_kp, l.out.kp, w.o, w.gate, l.onorm, d.heads, d.vdim, m->hp.eps, l.spec.delta_scale);
             HIP_TRY(hipGetLastError());
         }

@@ -71,6 +71,8 @@ __global__ __launch_bounds__(256) void norm_rows_kernel(NormRowsArgs a)
     }
 }
 
+static_assert(kDeltaStepThreads == kGqaStepThreads, "one launch for both");
+
 // Both mixers of one token in one launch: recurrent head blocks first (they take longest), then the attention groups.
 struct MixStepArgs {
     DeltaStepArgs delta;
@@ -78,7 +80,7 @@ struct MixStepArgs {
     uint32_t delta_wgs;
 };
 template <class CT, int DP, int R>
-__global__ __launch_bounds__(256) void mix_step_kernel(MixStepArgs a)
+__global__ __launch_bounds__(kGqaStepThreads) void mix_step_kernel(MixStepArgs a)
 {
     extern __shared__ float lds[];
     if (blockIdx.x < a.delta_wgs) delta_step(a.delta, blockIdx.x, lds);
@@ -114,7 +116,7 @@ __device__ __forceinline__ void prepare_token(const PrepareArgs &a, uint32_t t, 
     if (a.attn.heads) {
         const GqaSpec &s = a.attn;
         const uint32_t sh = 31 - __clz(a.dp / 2);
-        rotation_table(turn, s, pos);
+        for (uint32_t i = threadIdx.x; i < s.rot_dims / 2; i += 256) turn[i] = rotation(s.freq[i], pos);
         float sq[2] = {0.f, 0.f};
         if (s.q_norm) {
             for (uint32_t i = threadIdx.x; i < s.heads * s.dim; i += 256) sq[0] = fmaf(y[s.q_off + i], y[s.q_off + i], sq[0]);
@@ -147,7 +149,8 @@ __device__ __forceinline__ void prepare_token(const PrepareArgs &a, uint32_t t, 
     }
 }
 
-template <class T>
+// J = delta.dstride / 64
+template <class T, int J>
 __global__ __launch_bounds__(256) void prepare_kernel(PrepareArgs a, uint32_t n)
 {
     __shared__ float scratch[8];
@@ -167,9 +170,9 @@ __global__ __launch_bounds__(256) void prepare_kernel(PrepareArgs a, uint32_t n)
     for (uint32_t t = first + (threadIdx.x >> 6); t < last; t += 4) {
         const uint32_t pos = a.pos0 + t, slot = pos % s.taps;
         const float *y = a.y + (size_t)t * a.ldy;
-        float q[kDeltaMaxDim / 64], k[kDeltaMaxDim / 64], sq = 0.f, sk = 0.f, sqk = 0.f;
+        float q[J], k[J], sq = 0.f, sk = 0.f, sqk = 0.f;
 #pragma unroll
-        for (int j = 0; j < (int)kDeltaMaxDim / 64; j++) {
+        for (int j = 0; j < J; j++) {
             const uint32_t d = j * 64 + lane;
             q[j] = k[j] = 0.f;
             if (d < s.dim) {
@@ -181,15 +184,13 @@ __global__ __launch_bounds__(256) void prepare_kernel(PrepareArgs a, uint32_t n)
         }
         const float fq = rsqrtf(wave_sum(sq) + 1e-6f) * rsqrtf((float)s.dim), fk = rsqrtf(wave_sum(sk) + 1e-6f);
 #pragma unroll
-        for (int j = 0; j < (int)kDeltaMaxDim / 64; j++) {
+        for (int j = 0; j < J; j++) {
             const uint32_t d = j * 64 + lane;
             q[j] *= fq;
             k[j] *= fk;
             sqk = fmaf(q[j], k[j], sqk);
-            if (d < s.dstride) {
-                a.dq[((size_t)t * s.kv_heads + h) * s.dstride + d] = q[j];
-                a.dk[((size_t)t * s.kv_heads + h) * s.dstride + d] = k[j];
-            }
+            a.dq[((size_t)t * s.kv_heads + h) * s.dstride + d] = q[j];
+            a.dk[((size_t)t * s.kv_heads + h) * s.dstride + d] = k[j];
         }
         sqk = wave_sum(sqk);
         if (lane == 0) a.qk[(size_t)t * s.kv_heads + h] = sqk;

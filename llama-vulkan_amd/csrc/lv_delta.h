@@ -41,7 +41,7 @@ struct DeltaStepArgs {
     float *o, *gate;               // [heads * vdim]
 };
 
-constexpr int kDeltaCols = 32;     // columns per workgroup of the one-token step
+constexpr int kDeltaCols = 32;     // columns per workgroup of the one-token step: 16 lanes to each
 constexpr uint32_t kDeltaMaxDim = 256;
 constexpr uint32_t kDeltaMaxRank = 4096;
 
@@ -52,29 +52,50 @@ __device__ __forceinline__ uint32_t delta_channel_at(const DeltaSpec &s, uint32_
     return c < nq ? s.q_off + c : c < 2 * nq ? s.k_off + (c - nq) : s.v_off + (c - 2 * nq);
 }
 
-// convolution and silu of channel c at position pos (slot = pos % taps).  y: the token's projection row; rows before it (in steps of ld floats)
-// belong to positions pos - 1, pos - 2, .. as far as `behind` of them, older inputs are in the ring.
+// Convolution and silu of channel c at position pos (slot = pos % taps).  y: the token's projection row; rows before it (in
+// steps of ld floats) belong to positions pos - 1, pos - 2, .. as far as `behind` of them, older inputs are in the ring.
+// fetch() requests the first four taps, which is usually all there are; value() does the rest.
+struct DeltaConv {
+    float x[4], w[4];
+    uint32_t at, c;
+
+    static __device__ __forceinline__ float input(const DeltaSpec &s, const float *y, size_t ld, uint32_t behind, uint32_t at, uint32_t c, uint32_t slot, uint32_t j)
+    {
+        return j <= behind ? y[at - (ptrdiff_t)(j * ld)] : s.ring[(size_t)(slot >= j ? slot - j : slot + s.taps - j) * s.channels() + c];
+    }
+    __device__ __forceinline__ void fetch(const DeltaSpec &s, const float *y, size_t ld, uint32_t behind, uint32_t c_, uint32_t pos, uint32_t slot)
+    {
+        c = c_;
+        at = delta_channel_at(s, c);
+        const float *wp = s.conv + (size_t)(s.taps - 1) * s.channels() + c;
+#pragma unroll
+        for (uint32_t j = 0; j < 4; j++) {
+            const bool ok = j < s.taps && j <= pos;
+            x[j] = ok ? input(s, y, ld, behind, at, c, slot, j) : 0.f;
+            w[j] = ok ? wp[-(ptrdiff_t)(j * (size_t)s.channels())] : 0.f;
+        }
+    }
+    __device__ __forceinline__ float value(const DeltaSpec &s, const float *y, size_t ld, uint32_t behind, uint32_t pos, uint32_t slot) const
+    {
+        float v = x[0] * w[0];
+#pragma unroll
+        for (int j = 1; j < 4; j++) v = fmaf(x[j], w[j], v);
+        for (uint32_t j = 4; j < s.taps && j <= pos; j++)
+            v = fmaf(input(s, y, ld, behind, at, c, slot, j), s.conv[(size_t)(s.taps - 1 - j) * s.channels() + c], v);
+        return silu_f(v);
+    }
+};
 __device__ __forceinline__ float delta_conv(const DeltaSpec &s, const float *y, size_t ld, uint32_t behind, uint32_t c, uint32_t pos, uint32_t slot)
 {
-    const uint32_t at = delta_channel_at(s, c), C = s.channels();
-    const float *w = s.conv + (size_t)(s.taps - 1) * C + c;
-    float v = w[0] * y[at];
-    for (uint32_t j0 = 1; j0 < s.taps && j0 <= pos; j0 += 3) {
-        float x[3], f[3];      // three inputs on their way at once
-#pragma unroll
-        for (uint32_t e = 0; e < 3; e++) {
-            const uint32_t j = j0 + e;
-            const bool ok = j < s.taps && j <= pos;
-            x[e] = !ok ? 0.f : j <= behind ? y[at - (ptrdiff_t)(j * ld)] : s.ring[(size_t)(slot >= j ? slot - j : slot + s.taps - j) * C + c];
-            f[e] = ok ? w[-(ptrdiff_t)(j * (size_t)C)] : 0.f;
-        }
-#pragma unroll
-        for (int e = 0; e < 3; e++) v = fmaf(f[e], x[e], v);
-    }
-    return silu_f(v);
+    DeltaConv v;
+    v.fetch(s, y, ld, behind, c, pos, slot);
+    return v.value(s, y, ld, behind, pos, slot);
 }
 
-// Rows row0 + 32 i (i < N) of a low-rank matrix against a vector in LDS, 8 consecutive lanes a row, every lane of the eight gets
+constexpr int kDeltaStepThreads = 512;
+constexpr int kLowRankRows = kDeltaStepThreads / 8;      // rows of a low-rank matrix a workgroup takes at a time
+
+// Rows row0 + kLowRankRows * i (i < N) of a low-rank matrix against a vector in LDS, 8 consecutive lanes a row, every lane of the eight gets
 // the sum.  fetch() requests the first 128 columns of all N rows, which is usually all there is; dot() does the rest.
 template <int N>
 struct LowRankRows {
@@ -86,13 +107,13 @@ struct LowRankRows {
     __device__ __forceinline__ void fetch(const uint16_t *m, uint32_t row0, uint32_t end, uint32_t kp_)
     {
         kp = kp_;
-        rows = row0 < end ? min((uint32_t)N, (end - row0 + 31) / 32) : 0;
+        rows = row0 < end ? min((uint32_t)N, (end - row0 + kLowRankRows - 1) / kLowRankRows) : 0;
         at = m + (size_t)row0 * kp + (threadIdx.x & 7) * 8;
 #pragma unroll
         for (int i = 0; i < N; i++)
 #pragma unroll
             for (int k = 0; k < 2; k++)
-                w[i][k] = i < (int)rows && k * 64 < (int)kp ? *reinterpret_cast<const uint4 *>(at + (size_t)i * 32 * kp + k * 64) : make_uint4(0, 0, 0, 0);
+                w[i][k] = i < (int)rows && k * 64 < (int)kp ? *reinterpret_cast<const uint4 *>(at + (size_t)i * kLowRankRows * kp + k * 64) : make_uint4(0, 0, 0, 0);
     }
     static __device__ __forceinline__ float dot8(const uint4 &v, const float *x)
     {
@@ -113,71 +134,71 @@ struct LowRankRows {
             float t = dot8(w[i][0], x);
             if (kp > 64) t += dot8(w[i][1], x + 64);
             if (i < (int)rows)
-                for (uint32_t k = 128; k < kp; k += 64) t += dot8(*reinterpret_cast<const uint4 *>(at + (size_t)i * 32 * kp + k), x + k);
+                for (uint32_t k = 128; k < kp; k += 64) t += dot8(*reinterpret_cast<const uint4 *>(at + (size_t)i * kLowRankRows * kp + k), x + k);
             out[i] = group8_sum(t);
         }
     }
 };
 
-__host__ __device__ constexpr uint32_t delta_step_lds_floats(uint32_t a_kp, uint32_t g_kp) { return 3 * kDeltaMaxDim + kDeltaCols + 16 + a_kp + g_kp; }
+__host__ __device__ constexpr uint32_t delta_step_lds_floats(uint32_t a_kp, uint32_t g_kp) { return 3 * kDeltaMaxDim + kDeltaCols + a_kp + g_kp; }
 
-// one token, one head, one block of kDeltaCols columns: 256 threads.  Everything the block reads is requested first.
+// One token, one head, one block of kDeltaCols columns: kDeltaStepThreads threads.  Everything the block reads is requested
+// first, the short-lived before the state (loads return in order).
 __device__ __forceinline__ void delta_step(const DeltaStepArgs &a, uint32_t idx, float *lds)
 {
     const DeltaSpec &s = a.s;
     const uint32_t head = idx / a.blocks, cb = idx % a.blocks, c_lo = cb * kDeltaCols, nc = min((uint32_t)kDeltaCols, s.vdim - c_lo);
     const uint32_t pos = *a.pos_ptr + a.pos_add, rep = s.heads / s.kv_heads, kvh = head / rep, nq = s.kv_heads * s.dim, C = s.channels();
-    float *q = lds, *k = q + kDeltaMaxDim, *g = k + kDeltaMaxDim, *v = g + kDeltaMaxDim, *scratch = v + kDeltaCols, *al = scratch + 16, *gl = al + s.a_kp;
-    const int l16 = threadIdx.x & 15, c_own = threadIdx.x >> 4, r8 = threadIdx.x >> 3;
-    const int J = s.dstride / 64;
+    float *q = lds, *k = q + kDeltaMaxDim, *g = k + kDeltaMaxDim, *v = g + kDeltaMaxDim, *al = v + kDeltaCols, *gl = al + s.a_kp;
+    const int lane = threadIdx.x & 63, l16 = threadIdx.x & 15, r8 = threadIdx.x >> 3, J = s.dstride / 64;
+    const uint32_t rslot = pos % s.taps;
 
-    float4 st[2][4];      // this thread's parts of columns c_own and c_own + 16
-    float4 *col[2];
-#pragma unroll
-    for (int h = 0; h < 2; h++) {
-        const uint32_t c = min((uint32_t)(c_own + 16 * h), nc - 1);
-        col[h] = reinterpret_cast<float4 *>(s.state + ((size_t)head * s.vdim + c_lo + c) * s.dstride) + l16;
-#pragma unroll
-        for (int j = 0; j < 4; j++) st[h][j] = pos && j < J ? col[h][j * 16] : make_float4(0.f, 0.f, 0.f, 0.f);
-    }
-    LowRankRows<4> ra;
+    // threads 0 .. 255: channel d of q, the others: of k; the first 32 also a column of v
+    const uint32_t d = threadIdx.x & 255, half = threadIdx.x >> 8, cq = half * nq + kvh * s.dim + d, cv = 2 * nq + head * s.vdim + c_lo + threadIdx.x;
+    DeltaConv qk_in{}, v_in{};
+    if (d < s.dim) qk_in.fetch(s, a.y, 0, 0, cq, pos, rslot);
+    if (threadIdx.x < nc) v_in.fetch(s, a.y, 0, 0, cv, pos, rslot);
+    const float beta_in = a.y[s.b_off + head], a_log = s.a_log[head];
+    for (uint32_t i = threadIdx.x; i < s.a_kp; i += kDeltaStepThreads) al[i] = i < s.a_rank ? a.y[s.a_off + i] : 0.f;
+    for (uint32_t i = threadIdx.x; i < s.g_kp; i += kDeltaStepThreads) gl[i] = i < s.g_rank ? a.y[s.g_off + i] : 0.f;
+    LowRankRows<2> ra;
     LowRankRows<1> rg;
     ra.fetch(s.a2, head * s.dim + r8, (head + 1) * s.dim, s.a_kp);
     rg.fetch(s.g2, head * s.vdim + c_lo + r8, head * s.vdim + c_lo + nc, s.g_kp);
-    for (uint32_t i = threadIdx.x; i < s.a_kp; i += 256) al[i] = i < s.a_rank ? a.y[s.a_off + i] : 0.f;
-    for (uint32_t i = threadIdx.x; i < s.g_kp; i += 256) gl[i] = i < s.g_rank ? a.y[s.g_off + i] : 0.f;
-    const float beta = sigmoid_f(a.y[s.b_off + head]), ea = __expf(s.a_log[head]);
+    const uint32_t c_own = threadIdx.x >> 4;      // this thread's column, 16 lanes to one
+    float4 *const col = reinterpret_cast<float4 *>(s.state + ((size_t)head * s.vdim + c_lo + min(c_own, nc - 1)) * s.dstride) + l16;
+    float4 st[4];
+#pragma unroll
+    for (int j = 0; j < 4; j++) st[j] = pos && j < J ? col[j * 16] : make_float4(0.f, 0.f, 0.f, 0.f);
 
-    float qv = 0.f, kv = 0.f;
-    const uint32_t d = threadIdx.x, rslot = pos % s.taps;
+    float x = 0.f;
     if (d < s.dim) {
-        const uint32_t cq = kvh * s.dim + d, ck = nq + cq;
-        qv = delta_conv(s, a.y, 0, 0, cq, pos, rslot);
-        kv = delta_conv(s, a.y, 0, 0, ck, pos, rslot);
-        if (cb == 0 && head % rep == 0) {
-            s.ring[(size_t)rslot * C + cq] = a.y[s.q_off + cq];
-            s.ring[(size_t)rslot * C + ck] = a.y[s.k_off + cq];
-        }
+        x = qk_in.value(s, a.y, 0, 0, pos, rslot);
+        if (cb == 0 && head % rep == 0) s.ring[(size_t)rslot * C + cq] = qk_in.x[0];
     }
+    (half ? k : q)[d] = x;
     if (threadIdx.x < nc) {
-        const uint32_t c = head * s.vdim + c_lo + threadIdx.x;
-        v[threadIdx.x] = delta_conv(s, a.y, 0, 0, 2 * nq + c, pos, rslot);
-        s.ring[(size_t)rslot * C + 2 * nq + c] = a.y[s.v_off + c];
+        v[threadIdx.x] = v_in.value(s, a.y, 0, 0, pos, rslot);
+        s.ring[(size_t)rslot * C + cv] = v_in.x[0];
     }
-    float sums[3] = {qv * qv, kv * kv, qv * kv};
-    block_sums_waves<3>(sums, scratch, 4);      // also publishes al, gl and v
-    const float fq = rsqrtf(sums[0] + 1e-6f) * rsqrtf((float)s.dim), fk = rsqrtf(sums[1] + 1e-6f), qk = sums[2] * fq * fk;
-    q[threadIdx.x] = qv * fq;
-    k[threadIdx.x] = kv * fk;
-    for (uint32_t r0 = 0; r0 < s.dstride; r0 += 128) {
+    __syncthreads();
+    // every wave sums over the head for itself; q and k stay as they are, their factors go into the products with them
+    float sq = 0.f, sk = 0.f, sqk = 0.f;
+    for (uint32_t e = lane; e < s.dstride; e += 64) {
+        sq = fmaf(q[e], q[e], sq);
+        sk = fmaf(k[e], k[e], sk);
+        sqk = fmaf(q[e], k[e], sqk);
+    }
+    const float fq = rsqrtf(wave_sum(sq) + 1e-6f) * rsqrtf((float)s.dim), fk = rsqrtf(wave_sum(sk) + 1e-6f), qk = wave_sum(sqk) * fq * fk;
+    const float beta = sigmoid_f(beta_in), ea = __expf(a_log);
+    for (uint32_t r0 = 0; r0 < s.dstride; r0 += 2 * kLowRankRows) {
         if (r0) ra.fetch(s.a2, head * s.dim + r0 + r8, (head + 1) * s.dim, s.a_kp);
-        float t[4];
+        float t[2];
         ra.dot(t, al);
 #pragma unroll
-        for (int i = 0; i < 4; i++) {
-            const uint32_t r = r0 + i * 32 + r8;
-            if ((threadIdx.x & 7) == i && r < s.dstride)      // four lanes of the eight share the exponentials
-                g[r] = r < s.dim ? decay_f(ea, t[i] + s.dt_bias[head * s.dim + r]) : 0.f;
+        for (int i = 0; i < 2; i++) {
+            const uint32_t r = r0 + i * kLowRankRows + r8;
+            if ((threadIdx.x & 7) == i && r < s.dstride) g[r] = r < s.dim ? decay_f(ea, t[i] + s.dt_bias[head * s.dim + r]) : 0.f;
         }
     }
     {
@@ -186,35 +207,31 @@ __device__ __forceinline__ void delta_step(const DeltaStepArgs &a, uint32_t idx,
         if (r8 < (int)nc && (threadIdx.x & 7) == 0) a.gate[head * s.vdim + c_lo + r8] = sigmoid_f(t[0]);
     }
     __syncthreads();
+    float pk = 0.f, pq = 0.f;
 #pragma unroll
-    for (int h = 0; h < 2; h++) {
-        const uint32_t c = c_own + 16 * h;
-        float pk = 0.f, pq = 0.f;
+    for (int j = 0; j < 4; j++)
+        if (j < J) {
+            const int at = j * 64 + l16 * 4;
+            float4 e = st[j];
+            const float4 gg = *reinterpret_cast<const float4 *>(g + at), kk = *reinterpret_cast<const float4 *>(k + at), qq = *reinterpret_cast<const float4 *>(q + at);
+            e.x *= gg.x; e.y *= gg.y; e.z *= gg.z; e.w *= gg.w;
+            pk = fmaf(e.x, kk.x, pk); pk = fmaf(e.y, kk.y, pk); pk = fmaf(e.z, kk.z, pk); pk = fmaf(e.w, kk.w, pk);
+            pq = fmaf(e.x, qq.x, pq); pq = fmaf(e.y, qq.y, pq); pq = fmaf(e.z, qq.z, pq); pq = fmaf(e.w, qq.w, pq);
+            st[j] = e;
+        }
+    pk = group16_sum(pk) * fk;
+    pq = group16_sum(pq) * fq;
+    if (c_own >= nc) return;
+    const float u = beta * (v[c_own] - pk), ku = fk * u;
 #pragma unroll
-        for (int j = 0; j < 4; j++)
-            if (j < J) {
-                const int at = j * 64 + l16 * 4;
-                float4 x = st[h][j];
-                const float4 gg = *reinterpret_cast<const float4 *>(g + at), kk = *reinterpret_cast<const float4 *>(k + at), qq = *reinterpret_cast<const float4 *>(q + at);
-                x.x *= gg.x; x.y *= gg.y; x.z *= gg.z; x.w *= gg.w;
-                pk = fmaf(x.x, kk.x, pk); pk = fmaf(x.y, kk.y, pk); pk = fmaf(x.z, kk.z, pk); pk = fmaf(x.w, kk.w, pk);
-                pq = fmaf(x.x, qq.x, pq); pq = fmaf(x.y, qq.y, pq); pq = fmaf(x.z, qq.z, pq); pq = fmaf(x.w, qq.w, pq);
-                st[h][j] = x;
-            }
-        pk = group16_sum(pk);
-        pq = group16_sum(pq);
-        if (c >= nc) continue;
-        const float u = beta * (v[c] - pk);
-#pragma unroll
-        for (int j = 0; j < 4; j++)
-            if (j < J) {
-                const float4 kk = *reinterpret_cast<const float4 *>(k + j * 64 + l16 * 4);
-                float4 x = st[h][j];
-                x.x = fmaf(kk.x, u, x.x); x.y = fmaf(kk.y, u, x.y); x.z = fmaf(kk.z, u, x.z); x.w = fmaf(kk.w, u, x.w);
-                col[h][j * 16] = x;
-            }
-        if (l16 == 0) a.o[head * s.vdim + c_lo + c] = fmaf(qk, u, pq);
-    }
+    for (int j = 0; j < 4; j++)
+        if (j < J) {
+            const float4 kk = *reinterpret_cast<const float4 *>(k + j * 64 + l16 * 4);
+            float4 e = st[j];
+            e.x = fmaf(kk.x, ku, e.x); e.y = fmaf(kk.y, ku, e.y); e.z = fmaf(kk.z, ku, e.z); e.w = fmaf(kk.w, ku, e.w);
+            col[j * 16] = e;
+        }
+    if (l16 == 0) a.o[head * s.vdim + c_lo + c_own] = fmaf(qk, u, pq);
 }
 
 // ---- batches -------------------------------------------------------------------------------------------------------------

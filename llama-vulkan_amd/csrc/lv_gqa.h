@@ -51,16 +51,20 @@ __host__ __device__ constexpr uint32_t gqa_split(uint32_t dp) { return dp == 256
 
 constexpr uint32_t kGqaMaxDim = 256;
 
-// (cos, sin) of a position's angles, one per rotated pair; readable after the caller's next barrier.  Angles are reduced in
-// double: positions far out lose nothing to the range reduction.
-__device__ __forceinline__ void rotation_table(float2 *turn, const GqaSpec &s, uint32_t pos)
+// (cos, sin) of a position's angle, freq in turns per position.  Reduced in double: positions far out lose nothing to the
+// range reduction.
+__device__ __forceinline__ float2 rotation(double freq, uint32_t pos)
 {
-    for (uint32_t i = threadIdx.x; i < s.rot_dims / 2; i += blockDim.x) {
-        const double a = (double)pos * s.freq[i];      // in turns
-        float sn, cs;
-        sincospif(2.f * (float)(a - rint(a)), &sn, &cs);
-        turn[i] = make_float2(cs, sn);
-    }
+    const double a = (double)pos * freq;
+    float sn, cs;
+    sincospif(2.f * (float)(a - rint(a)), &sn, &cs);
+    return make_float2(cs, sn);
+}
+__device__ __forceinline__ void turn_pair(float &u, float &v, float2 t)
+{
+    const float r = u * t.x - v * t.y;
+    v = v * t.x + u * t.y;
+    u = r;
 }
 
 template <int LPK> __device__ __forceinline__ float lanes_sum(float v)
@@ -71,89 +75,60 @@ template <int LPK> __device__ __forceinline__ float lanes_sum(float v)
     return v;
 }
 
-// Scores of the keys k_begin + 0 .. n - 1 against R queries in LDS, then weights and the weighted value sum.
-// key(j, f) / value(j, f): the 8 elements of key / value j (an index from 0) this lane holds (sub * 8 ..).
-template <int DP, int R>
+// A workgroup of NT threads works on keys a row at a time: DP / 8 lanes share a key, 8 elements each.
+template <int DP, int NT>
 struct GqaLanes {
     static constexpr int LPK = DP / 8;            // lanes per key
-    static constexpr int KPR = 256 / LPK;         // keys per round of the workgroup
+    static constexpr int KPR = NT / LPK;          // keys per round of the workgroup
 };
+constexpr int kGqaStepThreads = 512, kGqaRowThreads = 256;
 
-// LDS, in floats
-template <int DP, int R> constexpr int gqa_lds_floats() { return R * DP + 2 * DP + R * kGqaSplit + 4 * R * DP + 4 * R + 16 + DP; }
+// LDS, in floats: queries, own key and value, scores, sums of the waves, per-head scalars, scratch, rotation table
+template <int DP, int R, int NT> constexpr int gqa_lds_floats() { return R * DP + 2 * DP + R * kGqaSplit + NT / 64 * R * DP + 4 * R + 16 + DP; }
 
-// q [R][DP] and sc [R][kGqaSplit] in LDS
-template <int DP, int R, class Key>
-__device__ __forceinline__ void gqa_scores(const float *q, float *sc, uint32_t n, Key key)
-{
-    using L = GqaLanes<DP, R>;
-    const int sub = threadIdx.x % L::LPK, kg = threadIdx.x / L::LPK;
-    float qr[R][8];
-#pragma unroll
-    for (int r = 0; r < R; r++) load8(qr[r], q + r * DP + sub * 8);
-    for (uint32_t j0 = 0; j0 < n; j0 += L::KPR) {
-        const uint32_t j = j0 + kg;
-        float f[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-        if (j < n) key(j, sub * 8, f);
-#pragma unroll
-        for (int r = 0; r < R; r++) {
-            float s = 0.f;
-#pragma unroll
-            for (int e = 0; e < 8; e++) s = fmaf(qr[r][e], f[e], s);
-            s = lanes_sum<L::LPK>(s);
-            if (sub == 0 && j < n) sc[r * kGqaSplit + j] = s;
-        }
-    }
-}
-
-template <int DP, int R, class Value>
-__device__ __forceinline__ void gqa_values(float (&acc)[R][8], const float *sc, uint32_t n, Value value)
-{
-    using L = GqaLanes<DP, R>;
-    const int sub = threadIdx.x % L::LPK, kg = threadIdx.x / L::LPK;
-    for (uint32_t j = kg; j < n; j += L::KPR) {
-        float f[8];
-        value(j, sub * 8, f);
-#pragma unroll
-        for (int r = 0; r < R; r++) {
-            const float p = sc[r * kGqaSplit + j];
-#pragma unroll
-            for (int e = 0; e < 8; e++) acc[r][e] = fmaf(p, f[e], acc[r][e]);
-        }
-    }
-}
-
-// acc of all key groups -> red[0 .. R*DP) (summed over the workgroup)
-template <int DP, int R>
+// acc of all key groups -> red[0 .. R*DP), summed over the workgroup
+template <int DP, int R, int NT>
 __device__ __forceinline__ void gqa_reduce(float (&acc)[R][8], float *red)
 {
-    using L = GqaLanes<DP, R>;
+    constexpr int LPK = DP / 8, NW = NT / 64;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-#pragma unroll
-    for (int r = 0; r < R; r++)
-#pragma unroll
-        for (int e = 0; e < 8; e++) {
-#pragma unroll
-            for (int off = L::LPK; off < 64; off <<= 1) acc[r][e] += __shfl_xor(acc[r][e], off, 64);
-        }
-    if (lane < L::LPK) {
+    float *mine = red + wave * R * DP;
+    if constexpr (LPK == 8) {       // two keys in a 16-lane row: rotate by 8
 #pragma unroll
         for (int r = 0; r < R; r++)
 #pragma unroll
-            for (int e = 0; e < 8; e++) red[(wave * R + r) * DP + lane * 8 + e] = acc[r][e];
+            for (int e = 0; e < 8; e++) acc[r][e] += dpp_mov<0x128>(acc[r][e]);
+    }
+    if constexpr (LPK <= 16) {
+        // four values at a time over the wave's four 16-lane rows; row j ends up with the total of value quad_partial_of_lane
+        const int sub = lane % LPK, which = quad_partial_of_lane(lane);
+#pragma unroll
+        for (int r = 0; r < R; r++)
+#pragma unroll
+            for (int h = 0; h < 8; h += 4) {
+                auto s01 = __builtin_amdgcn_permlane32_swap(__float_as_uint(acc[r][h]), __float_as_uint(acc[r][h + 1]), false, false);
+                auto s23 = __builtin_amdgcn_permlane32_swap(__float_as_uint(acc[r][h + 2]), __float_as_uint(acc[r][h + 3]), false, false);
+                const float x = __uint_as_float(s01[0]) + __uint_as_float(s01[1]), y = __uint_as_float(s23[0]) + __uint_as_float(s23[1]);
+                auto t = __builtin_amdgcn_permlane16_swap(__float_as_uint(x), __float_as_uint(y), false, false);
+                if (LPK == 16 || (lane & 8) == 0) mine[r * DP + sub * 8 + h + which] = __uint_as_float(t[0]) + __uint_as_float(t[1]);
+            }
+    } else {
+#pragma unroll
+        for (int r = 0; r < R; r++)
+#pragma unroll
+            for (int h = 0; h < 8; h += 2) {
+                auto s01 = __builtin_amdgcn_permlane32_swap(__float_as_uint(acc[r][h]), __float_as_uint(acc[r][h + 1]), false, false);
+                mine[r * DP + (lane & 31) * 8 + h + (lane >> 5)] = __uint_as_float(s01[0]) + __uint_as_float(s01[1]);
+            }
     }
     __syncthreads();
-    for (int i = threadIdx.x; i < R * DP; i += 256) red[i] = (red[i] + red[R * DP + i]) + (red[2 * R * DP + i] + red[3 * R * DP + i]);
+    for (int i = threadIdx.x; i < R * DP; i += NT) {
+        float t = red[i];
+#pragma unroll
+        for (int w = 1; w < NW; w++) t += red[w * R * DP + i];
+        red[i] = t;
+    }
     __syncthreads();
-}
-
-// inverse root mean square of a projection (1 when it is not normalised)
-__device__ __forceinline__ float projection_inv(const float *y, uint32_t n, float eps, const float *w, float *scratch)
-{
-    if (!w) return 1.f;
-    float s = 0.f;
-    for (uint32_t i = threadIdx.x; i < n; i += blockDim.x) s = fmaf(y[i], y[i], s);
-    return rsqrtf(block_sum_waves(s, scratch, blockDim.x >> 6) / (float)n + eps);
 }
 
 // elements 2i, 2i+1 of one head, normalised and rotated
@@ -163,12 +138,7 @@ __device__ __forceinline__ void head_pair(float &u, float &v, const float *y, co
     const uint32_t d = 2 * i;
     u = d < dim ? y[base + d] * inv * (w ? w[base + d] : 1.f) : 0.f;
     v = d + 1 < dim ? y[base + d + 1] * inv * (w ? w[base + d + 1] : 1.f) : 0.f;
-    if (d < s.rot_dims) {
-        const float2 t = turn[i];
-        const float r = u * t.x - v * t.y;
-        v = v * t.x + u * t.y;
-        u = r;
-    }
+    if (d < s.rot_dims) turn_pair(u, v, turn[i]);
 }
 
 // eight elements as they lie in memory
@@ -196,14 +166,16 @@ template <> struct GqaRaw<float> {
     __device__ __forceinline__ void get(float (&f)[8]) const { f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w; f[4] = b.x; f[5] = b.y; f[6] = b.z; f[7] = b.w; }
 };
 
-// One token, one group of R heads that share a kv head, one split of its keys: 256 threads.  All cache rows of the split are
-// requested before anything else.  The splits of a group meet in the last of them to arrive (see attention_kernel for what the
-// hand-over relies on).  The split that holds the token's own position also appends its rows.
+// One token, one group of R heads that share a kv head, one split of its keys: kGqaStepThreads threads.  The projections are
+// requested first, then all cache rows of the split, so that norms and rotations go on while those are on their way (loads
+// return in order).  The splits of a group meet in the last of them to arrive (see attention_kernel for what the hand-over
+// relies on).  The split that holds the token's own position also appends its rows.
 template <class CT, int DP, int R>
 __device__ __forceinline__ void gqa_step(const GqaStepArgs &a, uint32_t idx, float *lds)
 {
-    using L = GqaLanes<DP, R>;
-    constexpr int SPLIT = gqa_split(DP), ROUNDS = SPLIT / L::KPR;
+    constexpr int NT = kGqaStepThreads, NW = NT / 64;
+    using L = GqaLanes<DP, NT>;
+    constexpr int SPLIT = gqa_split(DP), ROUNDS = SPLIT / L::KPR, PAIRS = (R * DP / 2 + NT - 1) / NT, SUMS = 8;
     const GqaSpec &s = a.s;
     const uint32_t split = idx % a.splits, grp = idx / a.splits, hg = grp % a.groups, kvh = grp / a.groups;
     const uint32_t pos = *a.pos_ptr + a.pos_add;
@@ -214,56 +186,82 @@ __device__ __forceinline__ void gqa_step(const GqaStepArgs &a, uint32_t idx, flo
     const bool own = split == active - 1;
     const uint32_t per_kv = s.heads / s.kv_heads, h0 = kvh * per_kv + hg * R, nh = min((uint32_t)R, per_kv - hg * R);
     const int sub = threadIdx.x % L::LPK, kg = threadIdx.x / L::LPK, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const float *yq = a.y + s.q_off, *yk = a.y + s.k_off, *yv = a.y + s.v_off;
+    const uint32_t nq = s.heads * s.dim, nk = s.kv_heads * s.dim;
+
+    float ys[SUMS], ks[2], pu[PAIRS], pv[PAIRS], wu[PAIRS], wv[PAIRS], ku = 0.f, kv = 0.f, kwu = 1.f, kwv = 1.f, vu = 0.f, vv = 0.f;
+    if (s.q_norm) {
+#pragma unroll
+        for (int i = 0; i < SUMS; i++) ys[i] = threadIdx.x + i * NT < nq ? yq[threadIdx.x + i * NT] : 0.f;
+#pragma unroll
+        for (int i = 0; i < 2; i++) ks[i] = threadIdx.x + i * NT < nk ? yk[threadIdx.x + i * NT] : 0.f;
+    }
+    // the pair p of head r, and of the own key and value, that this thread turns
+    const uint32_t own_d = 2 * threadIdx.x;
+#pragma unroll
+    for (int i = 0; i < PAIRS; i++) {
+        const uint32_t e = threadIdx.x + i * NT, r = e / (DP / 2), d = e % (DP / 2) * 2;
+        const uint32_t at = (h0 + r) * s.dim + d;
+        const bool u = r < nh && d < s.dim, v = r < nh && d + 1 < s.dim;
+        pu[i] = u ? yq[at] : 0.f;
+        pv[i] = v ? yq[at + 1] : 0.f;
+        wu[i] = u && s.q_norm ? s.q_norm[at] : 1.f;
+        wv[i] = v && s.q_norm ? s.q_norm[at + 1] : 1.f;
+    }
+    if (own && own_d < DP) {
+        const uint32_t at = kvh * s.dim + own_d, av = kvh * s.vdim + own_d;
+        if (own_d < s.dim) ku = yk[at];
+        if (own_d + 1 < s.dim) kv = yk[at + 1];
+        if (s.k_norm && own_d < s.dim) kwu = s.k_norm[at];
+        if (s.k_norm && own_d + 1 < s.dim) kwv = s.k_norm[at + 1];
+        if (own_d < s.vdim) vu = yv[av];
+        if (own_d + 1 < s.vdim) vv = yv[av + 1];
+    }
+    const double freq = threadIdx.x < s.rot_dims / 2 ? s.freq[threadIdx.x] : 0.0;
+
     CT *const kc = static_cast<CT *>(s.kc), *const vc = static_cast<CT *>(s.vc);
     GqaRaw<CT> kraw[ROUNDS], vraw[ROUNDS];
+    {
+        // row 0 of the split stands in for the rows it does not have
+        const size_t step = (size_t)L::KPR * s.kv_heads * DP;
+        const size_t at = ((size_t)(split * SPLIT) * s.kv_heads + kvh) * DP + sub * 8, mine = at + (size_t)kg * s.kv_heads * DP;
 #pragma unroll
-    for (int i = 0; i < ROUNDS; i++) {
-        const uint32_t row = split * SPLIT + min((uint32_t)(i * L::KPR + kg), n - 1);
-        kraw[i].load(kc + ((size_t)row * s.kv_heads + kvh) * DP + sub * 8);
-    }
+        for (int i = 0; i < ROUNDS; i++) kraw[i].load(kc + (i * L::KPR + kg < (int)n ? mine + i * step : at));
 #pragma unroll
-    for (int i = 0; i < ROUNDS; i++) {
-        const uint32_t row = split * SPLIT + min((uint32_t)(i * L::KPR + kg), n - 1);
-        vraw[i].load(vc + ((size_t)row * s.kv_heads + kvh) * DP + sub * 8);
+        for (int i = 0; i < ROUNDS; i++) vraw[i].load(vc + (i * L::KPR + kg < (int)n ? mine + i * step : at));
     }
-    float *q = lds, *krow = q + R * DP, *vrow = krow + DP, *sc = vrow + DP, *red = sc + R * kGqaSplit, *ml = red + 4 * R * DP, *scratch = ml + 4 * R;
+    float *q = lds, *krow = q + R * DP, *vrow = krow + DP, *sc = vrow + DP, *red = sc + R * kGqaSplit, *ml = red + NW * R * DP, *scratch = ml + 4 * R;
     float2 *turn = reinterpret_cast<float2 *>(scratch + 16);
 
-    const float *yq = a.y + s.q_off, *yk = a.y + s.k_off, *yv = a.y + s.v_off;
     float sq[2] = {0.f, 0.f};
     if (s.q_norm) {
-        const uint32_t nq = s.heads * s.dim, nk = s.kv_heads * s.dim;
-#pragma unroll 4
-        for (uint32_t i = threadIdx.x; i < nq; i += 256) sq[0] = fmaf(yq[i], yq[i], sq[0]);
-#pragma unroll 2
-        for (uint32_t i = threadIdx.x; i < nk; i += 256) sq[1] = fmaf(yk[i], yk[i], sq[1]);
+#pragma unroll
+        for (int i = 0; i < SUMS; i++) sq[0] = fmaf(ys[i], ys[i], sq[0]);
+        sq[1] = fmaf(ks[0], ks[0], ks[1] * ks[1]);
+        for (uint32_t i = threadIdx.x + SUMS * NT; i < nq; i += NT) sq[0] = fmaf(yq[i], yq[i], sq[0]);
+        for (uint32_t i = threadIdx.x + 2 * NT; i < nk; i += NT) sq[1] = fmaf(yk[i], yk[i], sq[1]);
     }
-    rotation_table(turn, s, pos);
-    block_sums_waves<2>(sq, scratch, 4);      // also publishes the rotation table
-    const float inv_q = s.q_norm ? rsqrtf(sq[0] / (float)(s.heads * s.dim) + s.eps) : 1.f;
-    const float inv_k = s.q_norm ? rsqrtf(sq[1] / (float)(s.kv_heads * s.dim) + s.eps) : 1.f;
-    for (uint32_t i = threadIdx.x; i < R * DP / 2; i += 256) {
-        const uint32_t r = i / (DP / 2), p = i % (DP / 2);
-        float u = 0.f, v = 0.f;
-        if (r < nh) head_pair(u, v, yq, s.q_norm, (h0 + r) * s.dim, p, s.dim, inv_q, s, turn);
-        q[r * DP + 2 * p] = u * s.scale;
-        q[r * DP + 2 * p + 1] = v * s.scale;
+    if (threadIdx.x < s.rot_dims / 2) turn[threadIdx.x] = rotation(freq, pos);
+    block_sums_waves<2>(sq, scratch, NW);      // also publishes the rotation table
+    const float inv_q = s.q_norm ? rsqrtf(sq[0] / (float)nq + s.eps) : 1.f;
+    const float inv_k = s.q_norm ? rsqrtf(sq[1] / (float)nk + s.eps) : 1.f;
+#pragma unroll
+    for (int i = 0; i < PAIRS; i++) {
+        const uint32_t e = threadIdx.x + i * NT, d = e % (DP / 2) * 2;
+        float u = pu[i] * inv_q * wu[i] * s.scale, v = pv[i] * inv_q * wv[i] * s.scale;
+        if (d < s.rot_dims) turn_pair(u, v, turn[d / 2]);
+        if (PAIRS * NT == R * DP / 2 || e < R * DP / 2) *reinterpret_cast<float2 *>(q + 2 * e) = make_float2(u, v);
     }
-    if (own) {
-        const size_t row = ((size_t)(pos - c0) * s.kv_heads + kvh) * DP;
-        for (uint32_t p = threadIdx.x; p < DP / 2; p += 256) {
-            float u, v;
-            head_pair(u, v, yk, s.k_norm, kvh * s.dim, p, s.dim, inv_k, s, turn);
-            const CT cu = float_to_elem<CT>(u), cv = float_to_elem<CT>(v);
-            krow[2 * p] = elem_to_float(cu);
-            krow[2 * p + 1] = elem_to_float(cv);
-            const CT v0 = float_to_elem<CT>(2 * p < s.vdim ? yv[kvh * s.vdim + 2 * p] : 0.f), v1 = float_to_elem<CT>(2 * p + 1 < s.vdim ? yv[kvh * s.vdim + 2 * p + 1] : 0.f);
-            vrow[2 * p] = elem_to_float(v0);
-            vrow[2 * p + 1] = elem_to_float(v1);
-            if (hg == 0) {
-                kc[row + 2 * p] = cu; kc[row + 2 * p + 1] = cv;
-                vc[row + 2 * p] = v0; vc[row + 2 * p + 1] = v1;
-            }
+    if (own && own_d < DP) {
+        const size_t row = ((size_t)(pos - c0) * s.kv_heads + kvh) * DP + own_d;
+        float u = ku * inv_k * kwu, v = kv * inv_k * kwv;
+        if (own_d < s.rot_dims) turn_pair(u, v, turn[threadIdx.x]);
+        const CT cu = float_to_elem<CT>(u), cv = float_to_elem<CT>(v), v0 = float_to_elem<CT>(vu), v1 = float_to_elem<CT>(vv);
+        *reinterpret_cast<float2 *>(krow + own_d) = make_float2(elem_to_float(cu), elem_to_float(cv));
+        *reinterpret_cast<float2 *>(vrow + own_d) = make_float2(elem_to_float(v0), elem_to_float(v1));
+        if (hg == 0) {
+            kc[row] = cu; kc[row + 1] = cv;
+            vc[row] = v0; vc[row + 1] = v1;
         }
     }
     __syncthreads();
@@ -288,7 +286,7 @@ __device__ __forceinline__ void gqa_step(const GqaStepArgs &a, uint32_t idx, flo
         }
     }
     __syncthreads();
-    for (int r = wave; r < R; r += 4) {
+    for (int r = wave; r < R; r += NW) {
         float m = -INFINITY, l = 0.f;
         for (int j = lane; j < SPLIT; j += 64) m = fmaxf(m, sc[r * kGqaSplit + j]);
 #pragma unroll
@@ -320,10 +318,10 @@ __device__ __forceinline__ void gqa_step(const GqaStepArgs &a, uint32_t idx, flo
             for (int e = 0; e < 8; e++) acc[r][e] = fmaf(p, f[e], acc[r][e]);
         }
     }
-    gqa_reduce<DP, R>(acc, red);
+    gqa_reduce<DP, R, NT>(acc, red);
 
     if (active == 1) {
-        for (uint32_t i = threadIdx.x; i < nh * s.vdim; i += 256) {
+        for (uint32_t i = threadIdx.x; i < nh * s.vdim; i += NT) {
             const uint32_t r = i / s.vdim, c = i % s.vdim;
             const float m = ml[2 * r], sk = s.sink ? s.sink[h0 + r] : -INFINITY, M = fmaxf(m, sk);
             a.out[(h0 + r) * s.vdim + c] = red[r * DP + c] * __expf(m - M) / (ml[2 * r + 1] * __expf(m - M) + __expf(sk - M));
@@ -332,7 +330,7 @@ __device__ __forceinline__ void gqa_step(const GqaStepArgs &a, uint32_t idx, flo
     }
     constexpr int PS = R * (DP + 2);
     uint32_t *part = reinterpret_cast<uint32_t *>(a.part + (size_t)grp * a.splits * PS);
-    for (uint32_t i = threadIdx.x; i < PS; i += 256) {
+    for (uint32_t i = threadIdx.x; i < PS; i += NT) {
         const uint32_t r = i / (DP + 2), c = i % (DP + 2);
         const float v = c < DP ? red[r * DP + c] : ml[2 * r + (c - DP)];
         __hip_atomic_store(part + (size_t)split * PS + i, __float_as_uint(v), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
@@ -345,13 +343,13 @@ __device__ __forceinline__ void gqa_step(const GqaStepArgs &a, uint32_t idx, flo
     if (*arrived != active - 1) return;
     auto get = [&](uint32_t sp, uint32_t i) { return __uint_as_float(__hip_atomic_load(part + (size_t)sp * PS + i, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT)); };
     // every thread sums its element over the splits, in split order, with a running maximum of its own: one pass of loads
-    for (uint32_t i = threadIdx.x; i < nh * s.vdim; i += 256) {
+    for (uint32_t i = threadIdx.x; i < nh * s.vdim; i += NT) {
         const uint32_t r = i / s.vdim, c = i % s.vdim;
         float M = s.sink ? s.sink[h0 + r] : -INFINITY, l = s.sink ? 1.f : 0.f, t = 0.f;
-        for (uint32_t s0 = 0; s0 < active; s0 += 8) {
-            float v[8], w[8], z[8];
+        for (uint32_t s0 = 0; s0 < active; s0 += 16) {
+            float v[16], w[16], z[16];
 #pragma unroll
-            for (int e = 0; e < 8; e++) {
+            for (int e = 0; e < 16; e++) {
                 const uint32_t sp = min(s0 + e, active - 1);
                 v[e] = get(sp, r * (DP + 2) + c);
                 w[e] = get(sp, r * (DP + 2) + DP);
@@ -359,13 +357,13 @@ __device__ __forceinline__ void gqa_step(const GqaStepArgs &a, uint32_t idx, flo
             }
             float top = M;
 #pragma unroll
-            for (int e = 0; e < 8; e++) top = fmaxf(top, w[e]);
+            for (int e = 0; e < 16; e++) top = fmaxf(top, w[e]);
             const float f = __expf(M - top);
             M = top;
             t *= f;
             l *= f;
 #pragma unroll
-            for (int e = 0; e < 8; e++) {
+            for (int e = 0; e < 16; e++) {
                 const float p = s0 + e < active ? __expf(w[e] - top) : 0.f;
                 t = fmaf(v[e], p, t);
                 l = fmaf(z[e], p, l);
@@ -391,11 +389,14 @@ struct GqaBatchArgs {
 template <class CT, int DP, int R>
 __global__ __launch_bounds__(256) void gqa_rows_kernel(GqaBatchArgs a)
 {
+    constexpr int NT = kGqaRowThreads;
+    using L = GqaLanes<DP, NT>;
     extern __shared__ float lds[];
     const GqaSpec &s = a.s;
     const uint32_t t = blockIdx.y, hg = blockIdx.x % a.groups, kvh = blockIdx.x / a.groups, pos = a.pos0 + t;
     const uint32_t per_kv = s.heads / s.kv_heads, h0 = kvh * per_kv + hg * R, nh = min((uint32_t)R, per_kv - hg * R);
-    float *q = lds, *sc = q + R * DP + 2 * DP, *red = sc + R * kGqaSplit, *ml = red + 4 * R * DP;
+    float *q = lds, *sc = q + R * DP + 2 * DP, *red = sc + R * kGqaSplit, *ml = red + NT / 64 * R * DP;
+    const int sub = threadIdx.x % L::LPK, kg = threadIdx.x / L::LPK;
     for (uint32_t i = threadIdx.x; i < R * DP; i += 256) {
         const uint32_t r = i / DP;
         q[i] = r < nh ? elem_to_float(static_cast<const CT *>(a.q)[((size_t)t * s.heads + h0 + r) * DP + i % DP]) : 0.f;
@@ -419,7 +420,20 @@ __global__ __launch_bounds__(256) void gqa_rows_kernel(GqaBatchArgs a)
             if (p >= a.pos0) load8(f, static_cast<const CT *>(mine) + ((size_t)(p - a.pos0) * s.kv_heads + kvh) * DP + d);
             else load8(f, static_cast<const CT *>(ring) + ((size_t)(p - c0) * s.kv_heads + kvh) * DP + d);
         };
-        gqa_scores<DP, R>(q, sc, n, [&](uint32_t j, int d, float (&f)[8]) { from(s.kc, a.k, j, d, f); });
+        for (uint32_t j0 = 0; j0 < n; j0 += L::KPR) {
+            const uint32_t j = j0 + kg;
+            float f[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+            if (j < n) from(s.kc, a.k, j, sub * 8, f);
+#pragma unroll
+            for (int r = 0; r < R; r++) {
+                float qr[8], t = 0.f;
+                load8(qr, q + r * DP + sub * 8);
+#pragma unroll
+                for (int e = 0; e < 8; e++) t = fmaf(qr[e], f[e], t);
+                t = lanes_sum<L::LPK>(t);
+                if (sub == 0 && j < n) sc[r * kGqaSplit + j] = t;
+            }
+        }
         __syncthreads();
         const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
         for (int r = wave; r < R; r += 4) {
@@ -449,10 +463,19 @@ __global__ __launch_bounds__(256) void gqa_rows_kernel(GqaBatchArgs a)
 #pragma unroll
             for (int e = 0; e < 8; e++) acc[r][e] *= f;
         }
-        gqa_values<DP, R>(acc, sc, n, [&](uint32_t j, int d, float (&f)[8]) { from(s.vc, a.v, j, d, f); });
+        for (uint32_t j = kg; j < n; j += L::KPR) {
+            float f[8];
+            from(s.vc, a.v, j, sub * 8, f);
+#pragma unroll
+            for (int r = 0; r < R; r++) {
+                const float p = sc[r * kGqaSplit + j];
+#pragma unroll
+                for (int e = 0; e < 8; e++) acc[r][e] = fmaf(p, f[e], acc[r][e]);
+            }
+        }
         __syncthreads();
     }
-    gqa_reduce<DP, R>(acc, red);
+    gqa_reduce<DP, R, NT>(acc, red);
     for (uint32_t i = threadIdx.x; i < nh * s.vdim; i += 256) {
         const uint32_t r = i / s.vdim, c = i % s.vdim;
         static_cast<CT *>(a.out)[(size_t)t * a.ldo + (h0 + r) * s.vdim + c] = float_to_elem<CT>(red[r * DP + c] / ml[4 * r + 1] * a.out_scale);
