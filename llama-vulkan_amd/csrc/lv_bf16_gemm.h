@@ -6,13 +6,15 @@
 // Both can be grouped (mixture of experts): a table of token tiles says which expert's rows a tile takes and which
 // positions of the expert-sorted token list it covers.
 //
-// Weights are row-major [rows][kp], kp a multiple of 64 (zero columns), rows padded with zero rows to a multiple of 128.
+// Weights are row-major [rows][kp], kp a multiple of 64 (zero columns), rows padded with zero rows to a multiple of 128 (a tile may read the rows behind those as well).
 // In the MFMA a weight tile is operand A (M = weight row) and the tokens are operand B (N = token): lane l of the result
 // holds token l % 16 and four consecutive weight rows 4 * (l / 16) .. + 3, i.e. one 16-byte store into the token's row.
 //
-// gemm_bf16_kernel: workgroup = 4 waves, tile 128 weight rows x 128 tokens, K step 64, each wave 64 x 64.  Both operand
-// tiles go to LDS by direct loads, two stages.  A row of a tile is 128 bytes; its eight 16-byte chunks are stored in the
-// order chunk ^ (row % 8), so that the 16 rows an MFMA operand reads at one k spread over all banks.
+// gemm_bf16_kernel<NW>: NW waves of 64 x 64 each, tile 32 NW weight rows x 128 tokens, K step 64.  Both operand tiles go to LDS
+// by direct loads: two stages and two workgroups a CU with four waves, three stages and one workgroup with eight (fewer bytes
+// into LDS per product, loads two steps ahead; for launches that fill the chip with it).  A row of a tile is 128 bytes; its
+// eight 16-byte chunks are stored in the order chunk ^ (row % 8), so that the 16 rows an MFMA operand reads at one k spread over
+// all banks.
 #pragma once
 
 #include "lv_device.h"
@@ -163,29 +165,32 @@ __device__ __forceinline__ bool bf_tile(const BfGemmArgs &a, uint32_t tile_token
 }
 inline uint32_t bf_grid(const BfGemmArgs &a) { return (a.row_tiles + 7) / 8 * 8 * a.token_tiles; }
 
-constexpr int kBfTile = 128;       // weight rows and tokens per workgroup, bf16
+constexpr int kBfTile = 128;       // tokens per workgroup, bf16
 constexpr int kBfStep = 64;
-constexpr int kBfStageBytes = 2 * kBfTile * kBfStep * 2;
+constexpr int bf_tile_rows(int nw) { return 32 * nw; }
+constexpr int bf_stages(int nw) { return nw == 4 ? 2 : 3; }
+constexpr int bf_stage_bytes(int nw) { return (bf_tile_rows(nw) + kBfTile) * kBfStep * 2; }
+constexpr int bf_lds_bytes(int nw) { return bf_stages(nw) * bf_stage_bytes(nw); }
 
-template <int EP, bool GROUPED>
-__global__ __launch_bounds__(256, 2) void gemm_bf16_kernel(BfGemmArgs a)
+template <int EP, bool GROUPED, int NW>
+__global__ __launch_bounds__(NW * 64, 2) void gemm_bf16_kernel(BfGemmArgs a)
 {
-    __shared__ __attribute__((aligned(128))) uint8_t lds[2 * kBfStageBytes];
+    constexpr int RM = bf_tile_rows(NW), NST = bf_stages(NW), STAGE = bf_stage_bytes(NW);
+    constexpr int LW = RM / NW / 8, LX = kBfTile / NW / 8, LPS = LW + LX;      // direct loads per wave and stage, 8 rows (1 KB) each
+    extern __shared__ __attribute__((aligned(128))) uint8_t bf_lds[];
     uint32_t rt, expert, first, count;
     if (!bf_tile<GROUPED>(a, kBfTile, rt, expert, first, count)) return;
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int l16 = lane & 15, g4 = lane >> 4;
     const uint32_t kp = a.kp;
 
-    // direct loads: a wave brings 32 rows of each tile, 8 rows (1 KB) per instruction
-    const uint16_t *gw[4], *gx[4];
+    const uint16_t *gw, *gx[LX];
     {
         const int r8 = lane >> 3, c = (lane & 7) ^ r8;
-        const uint16_t *wt = a.w + ((size_t)expert * a.expert_rows + (size_t)rt * kBfTile) * kp;
+        gw = a.w + ((size_t)expert * a.expert_rows + (size_t)rt * RM + wave * (RM / NW) + r8) * kp + c * 8;
 #pragma unroll
-        for (int i = 0; i < 4; i++) {
-            const int row = wave * 32 + i * 8 + r8;
-            gw[i] = wt + (size_t)row * kp + c * 8;
+        for (int i = 0; i < LX; i++) {
+            const int row = wave * (kBfTile / NW) + i * 8 + r8;
             size_t xr = (size_t)first + row;
             if constexpr (GROUPED) {
                 const uint32_t p = first + min((uint32_t)row, count - 1);
@@ -194,28 +199,35 @@ __global__ __launch_bounds__(256, 2) void gemm_bf16_kernel(BfGemmArgs a)
             gx[i] = static_cast<const uint16_t *>(a.x) + xr * a.ldx + c * 8;
         }
     }
-    auto issue = [&](int s, uint32_t k0) {
-        uint8_t *buf = lds + s * kBfStageBytes + wave * 32 * 128;
+    const uint32_t steps = kp / kBfStep;
+    // past the end a harmless repeat of the last step into a free buffer keeps the number of loads in flight the same
+    auto issue = [&](uint32_t s, uint32_t slot) {
+        uint8_t *buf = bf_lds + slot * STAGE;
+        const uint32_t k0 = min(s, steps - 1) * kBfStep;
 #pragma unroll
-        for (int i = 0; i < 4; i++) __builtin_amdgcn_global_load_lds((lv_glb_any *)(gw[i] + k0), (lv_lds_any *)(buf + i * 1024), 16, 0, 0);
+        for (int i = 0; i < LW; i++)
+            __builtin_amdgcn_global_load_lds((lv_glb_any *)(gw + (size_t)i * 8 * kp + k0), (lv_lds_any *)(buf + (wave * LW + i) * 1024), 16, 0, 0);
 #pragma unroll
-        for (int i = 0; i < 4; i++) __builtin_amdgcn_global_load_lds((lv_glb_any *)(gx[i] + k0), (lv_lds_any *)(buf + kBfStageBytes / 2 + i * 1024), 16, 0, 0);
+        for (int i = 0; i < LX; i++) __builtin_amdgcn_global_load_lds((lv_glb_any *)(gx[i] + k0), (lv_lds_any *)(buf + RM * 128 + (wave * LX + i) * 1024), 16, 0, 0);
     };
 
-    const int wm = wave & 1, wn = wave >> 1;
+    const int wm = wave % (NW / 2), wn = wave / (NW / 2);
     lv_f4 acc[4][4];
 #pragma unroll
     for (int i = 0; i < 4; i++)
 #pragma unroll
         for (int j = 0; j < 4; j++) acc[i][j] = lv_f4{0.f, 0.f, 0.f, 0.f};
 
-    const uint32_t steps = kp / kBfStep;
-    issue(0, 0);
-    for (uint32_t st = 0; st < steps; st++) {
-        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-        __syncthreads();      // the stage is in LDS for everyone, and everyone is done with the other one
-        if (st + 1 < steps) issue((st + 1) & 1, (st + 1) * kBfStep);
-        const uint8_t *bw = lds + (st & 1) * kBfStageBytes, *bx = bw + kBfStageBytes / 2;
+#pragma unroll
+    for (int s = 0; s < NST - 1; s++) issue(s, s);
+    uint32_t slot = 0, ahead = NST - 1;
+    for (uint32_t s = 0; s < steps; s++) {
+        // this wave's loads of stage s have landed; behind the barrier everyone's have, and everyone is done with stage s - 1
+        asm volatile("s_waitcnt vmcnt(%0)" ::"n"((NST - 2) * LPS) : "memory");
+        __builtin_amdgcn_s_barrier();
+        asm volatile("" ::: "memory");
+        issue(s + NST - 1, ahead);
+        const uint8_t *bw = bf_lds + slot * STAGE, *bx = bw + RM * 128;
 #pragma unroll
         for (int kk = 0; kk < 2; kk++) {
             lv_bf8 fa[4], fb[4];
@@ -229,7 +241,10 @@ __global__ __launch_bounds__(256, 2) void gemm_bf16_kernel(BfGemmArgs a)
 #pragma unroll
                 for (int j = 0; j < 4; j++) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa[i], fb[j], acc[i][j], 0, 0, 0);
         }
+        slot = slot + 1 == NST ? 0 : slot + 1;
+        ahead = ahead + 1 == NST ? 0 : ahead + 1;
     }
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");      // the repeats have landed before the workgroup gives up its LDS
 #pragma unroll
     for (int j = 0; j < 4; j++) {
         const uint32_t t = wn * 64 + j * 16 + l16;
@@ -239,13 +254,13 @@ __global__ __launch_bounds__(256, 2) void gemm_bf16_kernel(BfGemmArgs a)
             const float wt = a.weights[a.slots[p]];
 #pragma unroll
             for (int i = 0; i < 4; i += 2) {
-                const uint32_t row = rt * kBfTile + wm * 64 + i * 16;        // the pair's gate block
-                bf_store_glu<uint16_t>(a, p, row / 2 + g4 * 4, wt, acc[i][j], acc[i + 1][j]);
+                const uint32_t row = rt * RM + wm * 64 + i * 16;        // the pair's gate block
+                if (row < a.rows) bf_store_glu<uint16_t>(a, p, row / 2 + g4 * 4, wt, acc[i][j], acc[i + 1][j]);
             }
         } else {
             const uint32_t orow = EP == kEpScatter ? a.slots[p] : p;
 #pragma unroll
-            for (int i = 0; i < 4; i++) bf_store4<EP>(a, orow, rt * kBfTile + wm * 64 + i * 16 + g4 * 4, acc[i][j]);
+            for (int i = 0; i < 4; i++) bf_store4<EP>(a, orow, rt * RM + wm * 64 + i * 16 + g4 * 4, acc[i][j]);
         }
     }
 }

@@ -15,6 +15,14 @@
 
 namespace lv {
 
+// 16 bytes of weights: read once per step, so they are not to push anything out of the caches
+__device__ __forceinline__ uint4 load_once(const uint16_t *p)
+{
+    typedef uint32_t u4v __attribute__((ext_vector_type(4)));
+    const u4v v = __builtin_nontemporal_load(reinterpret_cast<const u4v *>(p));
+    return make_uint4(v.x, v.y, v.z, v.w);
+}
+
 enum BfInput { kInNorm = 0, kInPlain = 1, kInBranch = 2 };
 enum BfGemvMode { kGemvRows = 0, kGemvExperts = 1, kGemvDown = 2 };
 
@@ -234,7 +242,7 @@ __global__ __launch_bounds__(kBfGemvThreads) void bf16_gemv_kernel(BfGemvArgs a)
 #pragma unroll
         for (int r = 0; r < NR; r++) {
             const size_t off = MODE == kGemvExperts ? (size_t)(r % R + (r / R) * 16) * kp : (size_t)r * kp;
-            slot[r] = ok ? *reinterpret_cast<const uint4 *>(p + off) : make_uint4(0, 0, 0, 0);
+            slot[r] = ok ? load_once(p + off) : make_uint4(0, 0, 0, 0);
         }
         if (++fit == ksteps) {
             fit = 0;

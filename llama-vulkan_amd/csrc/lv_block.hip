@@ -374,6 +374,10 @@ int block_model_create(hipStream_t st, const void *base, uint64_t base_size, con
         delete m;
         return ld.error;
     }
+    // a GEMM tile of 256 rows may read up to 128 rows behind a matrix: of the next one, or of this margin
+    uint32_t widest = Dp;
+    for (const BlockLayer &l : m->layers) widest = std::max(widest, std::max(l.out.kp, std::max(l.down.kp, std::max(l.a2.kp, l.g2.kp))));
+    ld.bytes += 256ull * widest;
     hipError_t er = hipMalloc(reinterpret_cast<void **>(&m->arena), ld.bytes);
     if (er != hipSuccess) {
         (void)hipGetLastError();
@@ -595,20 +599,35 @@ template <int MODE, int INPUT> static int gemv(hipStream_t st, const BfGemvArgs 
     }
 }
 
+template <int EP, bool GROUPED, int NW> static int launch_bf_gemm(hipStream_t st, BfGemmArgs a)
+{
+    auto *k = &gemm_bf16_kernel<EP, GROUPED, NW>;
+    a.row_tiles = (a.rows + bf_tile_rows(NW) - 1) / bf_tile_rows(NW);
+    LV_TRY(allow_lds(k, bf_lds_bytes(NW)));
+    k<<<dim3(bf_grid(a)), dim3(NW * 64), bf_lds_bytes(NW), st>>>(a);
+    HIP_TRY(hipGetLastError());
+    return LV_OK;
+}
+
 template <int EP, bool GROUPED> static int gemm(hipStream_t st, bool f32, BfGemmArgs a, const BfMatrix &w, uint32_t n, uint32_t experts = 1)
 {
-    const uint32_t tile = f32 ? kF32Tile : kBfTile;
+    const uint32_t tile = f32 ? kF32Tile : kBfTile, token_tiles = (n + tile - 1) / tile;
     a.w = w.w;
     a.kp = w.kp;
     a.rows = w.rows;
     a.n = n;
-    a.row_tiles = (w.rows + tile - 1) / tile;
-    a.token_tiles = (n + tile - 1) / tile;
-    if (GROUPED) a.token_tiles = std::min(a.token_tiles + experts, n);
-    if (f32) gemm_f32_kernel<EP, GROUPED><<<dim3(bf_grid(a)), dim3(256), 0, st>>>(a);
-    else gemm_bf16_kernel<EP, GROUPED><<<dim3(bf_grid(a)), dim3(256), 0, st>>>(a);
-    HIP_TRY(hipGetLastError());
-    return LV_OK;
+    a.token_tiles = GROUPED ? std::min(token_tiles + experts, n) : token_tiles;
+    if (f32) {
+        a.row_tiles = (w.rows + tile - 1) / tile;
+        gemm_f32_kernel<EP, GROUPED><<<dim3(bf_grid(a)), dim3(256), 0, st>>>(a);
+        HIP_TRY(hipGetLastError());
+        return LV_OK;
+    }
+    if constexpr (EP != kEpDecay && EP != kEpSigmoid) {      // those two have a few K steps only
+        const uint64_t big_tiles = (uint64_t)((w.rows + 255) / 256) * std::max(token_tiles, GROUPED ? experts : 1u);
+        if (big_tiles >= 256) return launch_bf_gemm<EP, GROUPED, 8>(st, a);
+    }
+    return launch_bf_gemm<EP, GROUPED, 4>(st, a);
 }
 
 // calls fn(element, integral constant DP, integral constant R) for a layer's attention
@@ -960,7 +979,7 @@ static int step_batch(BlockSession *s, const uint32_t *tokens, uint32_t pos, uin
                 constexpr int J = decltype(j)::value;
                 const size_t lds = 2 * 4ull * scan_stage_floats<J>();
                 LV_TRY(allow_lds(&delta_scan_kernel<J>, lds));
-                delta_scan_kernel<J><<<dim3(d.heads, (d.vdim + 15) / 16), dim3(256), lds, st>>>(sc);
+                delta_scan_kernel<J><<<dim3(d.heads, (d.vdim + 15) / 16), dim3(kScanThreads), lds, st>>>(sc);
                 HIP_TRY(hipGetLastError());
                 return LV_OK;
             }));

@@ -8,7 +8,7 @@
 //   out      = o / rms(o) * norm * gate, gate = sigmoid of a low-rank projection, vdim values per head
 //
 // All of it is fp32.  With S' = g S the read-out is o = S'^T q + (k . q) u, so the two reductions of a step, S'^T k and S'^T q,
-// do not wait for each other.  Columns of S do not interact: 16 lanes share a column, each holding 4 J of its dim entries.
+// do not wait for each other.  Columns of S do not interact: 16 lanes (32 in a batch) share a column.
 //
 // State of a sequence and layer: S as [head][vdim][64 J] (a column contiguous, zero beyond dim) and a ring of the
 // convolution's last `taps` inputs, [position % taps][channel], channels in the order q, k, v.  Nothing has to be cleared for
@@ -249,41 +249,46 @@ struct DeltaScanArgs {
 constexpr int kScanTokens = 16;   // tokens staged in LDS at a time
 template <int J> constexpr int scan_stage_floats() { return kScanTokens * (3 * 64 * J + 16) + 64; }
 
-// All tokens of a batch for 16 columns of one head: a workgroup of 4 waves, 4 columns a wave.  grid (heads, vdim / 16 up).
+constexpr int kScanThreads = 512;
+
+// All tokens of a batch for 16 columns of one head: 8 waves, two columns a wave, 32 lanes a column with 2 J of its entries each.
+// grid (heads, vdim / 16 up).  The chain from token to token is what takes the time: the reductions of S'^T k and S'^T q share
+// their steps, and two waves per SIMD fill each other's gaps.
 template <int J>
-__global__ __launch_bounds__(256) void delta_scan_kernel(DeltaScanArgs a)
+__global__ __launch_bounds__(kScanThreads) void delta_scan_kernel(DeltaScanArgs a)
 {
     constexpr int W = 64 * J, SF = scan_stage_floats<J>();
+    constexpr int V = J % 2 ? 2 : 4, U = 2 * J / V;      // a lane's entries: U runs of V, the lanes' runs side by side
+    typedef float vec __attribute__((ext_vector_type(V)));
     extern __shared__ float lds[];       // two stages
     const DeltaSpec &s = a.s;
     const uint32_t head = blockIdx.x, kvh = head / (s.heads / s.kv_heads), HV = s.heads * s.vdim;
-    const int l16 = threadIdx.x & 15, ci = threadIdx.x >> 4;
+    const int l32 = threadIdx.x & 31, ci = threadIdx.x >> 5, lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const uint32_t col = blockIdx.y * 16 + ci;
     const bool live = col < s.vdim;
-    float4 *const colp = reinterpret_cast<float4 *>(s.state + ((size_t)head * s.vdim + (live ? col : 0)) * W);
-    float4 S[J];
+    vec *const colp = reinterpret_cast<vec *>(s.state + ((size_t)head * s.vdim + (live ? col : 0)) * W) + l32;
+    vec S[U];
 #pragma unroll
-    for (int j = 0; j < J; j++) S[j] = a.fresh || !live ? make_float4(0.f, 0.f, 0.f, 0.f) : colp[j * 16 + l16];
+    for (int u = 0; u < U; u++) S[u] = a.fresh || !live ? vec(0.f) : colp[u * 32];
 
     // One stage in LDS: k, q, g [16][W] each, v [16][16], beta [16], k.q [16].  Direct loads, lane after lane in LDS order; tokens
     // past the end and columns past vdim bring some other value that nothing uses.
-    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     auto issue = [&](uint32_t t0, int st) {
         float *b = lds + st * SF;
 #pragma unroll
-        for (int i = 0; i < J; i++) {
-            const int e = i * 256 + wave * 64;                   // first float4 of the wave
+        for (int i = 0; i < (J + 1) / 2; i++) {
+            const int e = i * kScanThreads + wave * 64;          // first float4 of the wave, of 256 J
+            if (e >= 256 * J) break;
             const uint32_t t = min(t0 + (e + lane) / (W / 4), a.n - 1), d = (e + lane) % (W / 4) * 4;
             const size_t kq = ((size_t)t * s.kv_heads + kvh) * W + d;
             __builtin_amdgcn_global_load_lds((lv_glb_any *)(a.k + kq), (lv_lds_any *)(b + e * 4), 16, 0, 0);
             __builtin_amdgcn_global_load_lds((lv_glb_any *)(a.q + kq), (lv_lds_any *)(b + kScanTokens * W + e * 4), 16, 0, 0);
             __builtin_amdgcn_global_load_lds((lv_glb_any *)(a.g + ((size_t)t * s.heads + head) * W + d), (lv_lds_any *)(b + 2 * kScanTokens * W + e * 4), 16, 0, 0);
         }
-        {
+        if (wave < 4) {
             const uint32_t t = min(t0 + wave * 4 + lane / 16, a.n - 1), c = min(blockIdx.y * 16 + lane % 16, s.vdim - 1);
             __builtin_amdgcn_global_load_lds((lv_glb_any *)(a.v + (size_t)t * HV + head * s.vdim + c), (lv_lds_any *)(b + 3 * kScanTokens * W + wave * 64), 4, 0, 0);
-        }
-        if (wave == 0) {
+        } else if (wave == 4) {
             const uint32_t t = min(t0 + (lane & 15), a.n - 1);
             const float *src = lane & 16 ? a.qk + (size_t)t * s.kv_heads + kvh : a.beta + (size_t)t * s.heads + head;
             __builtin_amdgcn_global_load_lds((lv_glb_any *)src, (lv_lds_any *)(b + 3 * kScanTokens * W + 256), 4, 0, 0);
@@ -294,30 +299,37 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaScanArgs a)
         asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
         __syncthreads();      // this stage is in LDS for everyone, and everyone is done with the other one
         if (t0 + kScanTokens < a.n) issue(t0 + kScanTokens, st ^ 1);
-        const float *b = lds + st * SF, *bk = b, *bq = b + kScanTokens * W, *bg = b + 2 * kScanTokens * W, *bv = b + 3 * kScanTokens * W;
+        const float *b = lds + st * SF, *bk = b + l32 * V, *bq = bk + kScanTokens * W, *bg = bq + kScanTokens * W, *bv = b + 3 * kScanTokens * W;
         uint32_t keep = 0;
         const int nt = (int)min((uint32_t)kScanTokens, a.n - t0);
         auto token = [&](int t) __attribute__((always_inline)) {
             float pk = 0.f, pq = 0.f;
-            float4 kk[J];
+            vec kk[U];
 #pragma unroll
-            for (int j = 0; j < J; j++) {
-                const int at = t * W + j * 64 + l16 * 4;
-                const float4 gg = *reinterpret_cast<const float4 *>(bg + at), qq = *reinterpret_cast<const float4 *>(bq + at);
-                kk[j] = *reinterpret_cast<const float4 *>(bk + at);
-                S[j].x *= gg.x; S[j].y *= gg.y; S[j].z *= gg.z; S[j].w *= gg.w;
-                pk = fmaf(S[j].x, kk[j].x, pk); pk = fmaf(S[j].y, kk[j].y, pk); pk = fmaf(S[j].z, kk[j].z, pk); pk = fmaf(S[j].w, kk[j].w, pk);
-                pq = fmaf(S[j].x, qq.x, pq); pq = fmaf(S[j].y, qq.y, pq); pq = fmaf(S[j].z, qq.z, pq); pq = fmaf(S[j].w, qq.w, pq);
-            }
-            pk = group16_sum(pk);
-            pq = group16_sum(pq);
-            const float u = bv[256 + t] * (bv[t * 16 + ci] - pk);
+            for (int u = 0; u < U; u++) {
+                const int at = t * W + u * 32 * V;
+                const vec gg = *reinterpret_cast<const vec *>(bg + at), qq = *reinterpret_cast<const vec *>(bq + at);
+                kk[u] = *reinterpret_cast<const vec *>(bk + at);
 #pragma unroll
-            for (int j = 0; j < J; j++) {
-                S[j].x = fmaf(kk[j].x, u, S[j].x); S[j].y = fmaf(kk[j].y, u, S[j].y); S[j].z = fmaf(kk[j].z, u, S[j].z); S[j].w = fmaf(kk[j].w, u, S[j].w);
+                for (int e = 0; e < V; e++) {
+                    S[u][e] *= gg[e];
+                    pk = fmaf(S[u][e], kk[u][e], pk);
+                    pq = fmaf(S[u][e], qq[e], pq);
+                }
             }
-            // lane t of the sixteen stores token t's read-out; picked by a mask, so that no branch parts the tokens
-            keep |= __float_as_uint(fmaf(bv[272 + t], u, pq)) & (uint32_t)((int)((l16 ^ t) - 1) >> 31);
+            // over the column's two 16-lane rows: the first row takes pk, the second pq, then both go on in one go and are
+            // handed to both rows again
+            auto x = __builtin_amdgcn_permlane16_swap(__float_as_uint(pk), __float_as_uint(pq), false, false);
+            const uint32_t both = __float_as_uint(group16_sum(__uint_as_float(x[0]) + __uint_as_float(x[1])));
+            auto y = __builtin_amdgcn_permlane16_swap(both, both, false, false);
+            const float sk = __uint_as_float(y[0]), sq = __uint_as_float(y[1]);
+            const float up = bv[256 + t] * (bv[t * 16 + ci] - sk);
+#pragma unroll
+            for (int u = 0; u < U; u++)
+#pragma unroll
+                for (int e = 0; e < V; e++) S[u][e] = fmaf(kk[u][e], up, S[u][e]);
+            // lane t of the column stores token t's read-out; picked by a mask, so that no branch parts the tokens
+            keep |= __float_as_uint(fmaf(bv[272 + t], up, sq)) & (uint32_t)((int)((l32 ^ t) - 1) >> 31);
         };
         if (nt == kScanTokens) {
 #pragma unroll
@@ -325,11 +337,11 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaScanArgs a)
         } else {
             for (int t = 0; t < nt; t++) token(t);
         }
-        if (live && l16 < nt) a.o[(size_t)(t0 + l16) * HV + head * s.vdim + col] = __uint_as_float(keep);
+        if (live && l32 < nt) a.o[(size_t)(t0 + l32) * HV + head * s.vdim + col] = __uint_as_float(keep);
     }
     if (live) {
 #pragma unroll
-        for (int j = 0; j < J; j++) colp[j * 16 + l16] = S[j];
+        for (int u = 0; u < U; u++) colp[u * 32] = S[u];
     }
 }
 
