@@ -13,6 +13,7 @@ import pytest
 
 import block_builder as bb
 import block_oracle as bo
+import server_client as sc
 
 pytestmark = pytest.mark.gpu
 F32, BF16 = 0, 30
@@ -124,7 +125,8 @@ def test_delta_rule_alone(lva, ctx, k, compute):
 
 
 @pytest.mark.parametrize("compute", [F32, BF16])
-@pytest.mark.parametrize("experts,top,ff,width", [(5, 2, 24, 40), (70, 6, 17, 33), (3, 3, 100, 130), (1, 1, 64, 64), (9, 1, 40, 70)])
+@pytest.mark.parametrize("experts,top,ff,width", [(5, 2, 24, 40), (70, 6, 17, 33), (3, 3, 100, 130), (1, 1, 64, 64), (9, 1, 40, 70),
+                                                   (256, 1, 20, 64), (257, 2, 136, 48)])      # many experts: tiles of 256 weight rows
 def test_mixture_alone(lva, ctx, experts, top, ff, width, compute):
     cfg = bb.config(width=width, layers=[bb.layer(experts=experts, top=top, ff=ff)])
     W = bb.weights(cfg, seed=30 + experts)
@@ -168,6 +170,19 @@ def test_portions_and_decoding_agree_in_bfloat16(lva, ctx):
         if l["mlp"]:
             l["mlp"]["router"]["top"] = l["mlp"]["router"]["experts"]
     check_model(lva, ctx, cfg, bb.weights(cfg, 42), 190, BF16, cuts=PORTIONS, tol=8e-2)
+
+
+def test_a_prompt_longer_than_a_batch(lva, ctx):
+    """2100 tokens at once: two batches inside one step, the wide forms of the matrix product and of the attention tiles, a chunk
+    that is open when the second batch starts"""
+    cfg = bb.config(vocab=4099, width=72, layers=[bb.layer(left=bb.attn(heads=16, kv_heads=2, dim=32, chunk=700), right=bb.delta(heads=2, kv_heads=1, dim=16, vdim=16), experts=0)])
+    W = bb.weights(cfg, 48)
+    toks = tokens_for(cfg, 2100, 4)
+    want = bo.forward(toks, bb.as_float(W), cfg)[0]
+    with Device(lva, ctx, cfg, W, BF16, backlog=2200) as d:
+        assert rel(d.run(toks, (2100,)), want) < TOL[BF16]
+        d.step(toks[:2090], 0)
+        assert rel(d.run(toks, (2050, 40, 1)), want) < TOL[BF16]
 
 
 @pytest.mark.parametrize("n", [1, 2, 3, 4, 15, 16, 17])
@@ -448,6 +463,34 @@ def test_command_line_generates_ids(lva, folder):
     assert [int(t) for t in out.stdout.split()[3:9]] == want
     bad = subprocess.run([exe, "-m", path, "--greedy", "-n", "6", "5 x"], capture_output=True, text=True, timeout=100)
     assert bad.returncode == 1 and "token ids" in bad.stderr
+
+
+def test_token_server(hostlib, folder):
+    path, cfg, W = folder
+    c = hostlib.LlavaContext()
+    assert c.load_model(path, compute=F32)
+    server = hostlib.LlavaServer(c)
+    a, b = sc.Client(server.port), sc.Client(server.port)
+    F = bb.as_float(W)
+    prompts = {}
+    for client, text in ((a, b"5 17 3 9"), (b, b"44, 2")):      # two sessions, ticks in turn
+        sid = client.new_session()
+        assert client.ack(sc.SET_OPTIONS, sid, sc.OPTION_GREEDY) == sc.RC_OK
+        assert client.ack(sc.ADD_TEXT, sid, text=text) == sc.RC_OK
+        prompts[client] = (sid, client.tokens(sid))
+    got = {client: [] for client in prompts}
+    for _ in range(8):
+        for client, (sid, _) in prompts.items():
+            got[client].append(client.tick(sid)[0])
+    for client, (sid, prompt) in prompts.items():
+        assert got[client] == bo.greedy(prompt, 8, F, cfg)
+        assert client.ack(sc.REWIND, sid, len(prompt) - 1) == sc.RC_OK
+        assert client.ack(sc.ADD_TOKEN, sid, prompt[-1]) == sc.RC_OK
+        assert [client.tick(sid)[0] for _ in range(3)] == got[client][:3]
+        assert client.ack(sc.ADD_TEXT, sid, text=b"x") == sc.RC_NOK
+        client.close()
+    server.stop()
+    c.close()
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
