@@ -79,6 +79,9 @@ struct BfGemmArgs {
     uint32_t row_tiles, token_tiles;
     float *out;
     uint32_t ldo;
+    // K cut in slices (kEpStore): grid z = slice, its sum goes to out + slice * slice_floats; the reader adds them up
+    uint32_t k_slice;        // columns per slice, a multiple of the K step; 0: one slice
+    uint64_t slice_floats;
     // decay epilogue
     const float *a_log, *bias;
     uint32_t head_dim, head_stride;
@@ -119,7 +122,7 @@ __device__ __forceinline__ void bf_store4(const BfGemmArgs &a, uint32_t orow, ui
 #pragma unroll
         for (int i = 0; i < 4; i++) r[i] = sigmoid_f(r[i]);
     }
-    float *o = a.out + (size_t)orow * a.ldo + row;
+    float *o = a.out + (EP == kEpStore && a.k_slice ? blockIdx.z * a.slice_floats : 0) + (size_t)orow * a.ldo + row;
     if (row + 3 < a.rows && (a.ldo & 3) == 0) {
         *reinterpret_cast<float4 *>(o) = make_float4(r[0], r[1], r[2], r[3]);
     } else {
@@ -199,11 +202,12 @@ __global__ __launch_bounds__(NW * 64, 2) void gemm_bf16_kernel(BfGemmArgs a)
             gx[i] = static_cast<const uint16_t *>(a.x) + xr * a.ldx + c * 8;
         }
     }
-    const uint32_t steps = kp / kBfStep;
+    const uint32_t k_lo = EP == kEpStore && a.k_slice ? blockIdx.z * a.k_slice : 0;
+    const uint32_t steps = (EP == kEpStore && a.k_slice ? min(a.k_slice, kp - k_lo) : kp) / kBfStep;
     // past the end a harmless repeat of the last step into a free buffer keeps the number of loads in flight the same
     auto issue = [&](uint32_t s, uint32_t slot) {
         uint8_t *buf = bf_lds + slot * STAGE;
-        const uint32_t k0 = min(s, steps - 1) * kBfStep;
+        const uint32_t k0 = k_lo + min(s, steps - 1) * kBfStep;
 #pragma unroll
         for (int i = 0; i < LW; i++)
             __builtin_amdgcn_global_load_lds((lv_glb_any *)(gw + (size_t)i * 8 * kp + k0), (lv_lds_any *)(buf + (wave * LW + i) * 1024), 16, 0, 0);

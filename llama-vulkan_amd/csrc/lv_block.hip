@@ -604,7 +604,7 @@ template <int EP, bool GROUPED, int NW> static int launch_bf_gemm(hipStream_t st
     auto *k = &gemm_bf16_kernel<EP, GROUPED, NW>;
     a.row_tiles = (a.rows + bf_tile_rows(NW) - 1) / bf_tile_rows(NW);
     LV_TRY(allow_lds(k, bf_lds_bytes(NW)));
-    k<<<dim3(bf_grid(a)), dim3(NW * 64), bf_lds_bytes(NW), st>>>(a);
+    k<<<dim3(bf_grid(a), 1, a.k_slice ? (a.kp + a.k_slice - 1) / a.k_slice : 1), dim3(NW * 64), bf_lds_bytes(NW), st>>>(a);
     HIP_TRY(hipGetLastError());
     return LV_OK;
 }
@@ -802,6 +802,9 @@ int block_step_token(BlockSession *s, const uint32_t *cfg, uint32_t idx, float *
     return LV_OK;
 }
 
+// router logits of a batch: K in at most so many slices, each a multiple of so many columns
+constexpr uint32_t kRouterParts = 8, kRouterSlice = 128;
+
 // ---- batches ---------------------------------------------------------------------------------------------------------------
 static int workspace_reserve(BlockSession *s, uint32_t n)
 {
@@ -837,7 +840,7 @@ static int workspace_reserve(BlockSession *s, uint32_t n)
     LV_TRY(dev_zeroed(st, &w.g1, T * E * mx([](const BlockLayer &l) { return l.g2.kp; })));
     LV_TRY(dev_zeroed(st, &w.cat, T * E * mx([](const BlockLayer &l) { return l.out.kp; })));
     const uint64_t experts = mx([](const BlockLayer &l) { return l.spec.moe.experts; }), top = mx([](const BlockLayer &l) { return l.spec.moe.top; });
-    LV_TRY(dev_zeroed(st, &w.z, T * 4 * up((uint32_t)experts, 4)));
+    LV_TRY(dev_zeroed(st, &w.z, T * 4 * up((uint32_t)experts, 4) * kRouterParts));
     LV_TRY(dev_zeroed(st, &w.scores, T * 4 * top));
     LV_TRY(dev_zeroed(st, &w.ids, T * 4 * top));
     LV_TRY(dev_zeroed(st, &w.slots, T * 4 * top));
@@ -1003,8 +1006,14 @@ static int step_batch(BlockSession *s, const uint32_t *tokens, uint32_t pos, uin
         LV_TRY(keep(i, LV_TRACE_POST_ATTN));
         BfGemmArgs rt{};
         rt.x = w.act; rt.ldx = Dp; rt.out = w.z; rt.ldo = ldz;
+        uint32_t z_parts = 1;
+        if (!f32 && Dp >= 2 * kRouterSlice) {       // few rows: slices of K fill the chip
+            rt.k_slice = up((Dp + kRouterParts - 1) / kRouterParts, kRouterSlice);
+            rt.slice_floats = (uint64_t)w.cap * ldz;
+            z_parts = (Dp + rt.k_slice - 1) / rt.k_slice;
+        }
         LV_TRY((gemm<kEpStore, false>(st, f32, rt, l.router, n)));
-        route_rows_kernel<<<dim3(n), dim3(64), e.experts * 4ull, st>>>(w.z, ldz, e.experts, e.top, w.ids, w.scores);
+        route_rows_kernel<<<dim3(n), dim3(64), e.experts * 4ull, st>>>(w.z, ldz, z_parts, rt.slice_floats, e.experts, e.top, w.ids, w.scores);
         HIP_TRY(hipGetLastError());
         sort_experts_kernel<<<dim3(1), dim3(1024), e.experts * 8ull, st>>>(w.ids, total, e.experts, f32 ? kF32Tile : kBfTile, w.slots, w.tiles);
         HIP_TRY(hipGetLastError());

@@ -231,13 +231,17 @@ __global__ __launch_bounds__(256) void gated_rows_kernel(T *__restrict__ act, ui
 }
 
 // ---- routing of a batch ----------------------------------------------------------------------------------------------------
-// one wave per token
-__global__ __launch_bounds__(64) void route_rows_kernel(const float *__restrict__ z, uint32_t ldz, uint32_t experts, uint32_t top, uint32_t *__restrict__ ids,
-                                                        float *__restrict__ scores)
+// one wave per token; z: the K slices of the router logits, added here
+__global__ __launch_bounds__(64) void route_rows_kernel(const float *__restrict__ z, uint32_t ldz, uint32_t parts, uint64_t part_floats, uint32_t experts, uint32_t top,
+                                                        uint32_t *__restrict__ ids, float *__restrict__ scores)
 {
     extern __shared__ float zs[];
     const size_t t = blockIdx.x;
-    for (uint32_t e = threadIdx.x; e < experts; e += 64) zs[e] = z[t * ldz + e];
+    for (uint32_t e = threadIdx.x; e < experts; e += 64) {
+        float v = z[t * ldz + e];
+        for (uint32_t p = 1; p < parts; p++) v += z[p * part_floats + t * ldz + e];
+        zs[e] = v;
+    }
     __syncthreads();
     top_experts(zs, experts, top, ids + t * top, scores + t * top);
 }
