@@ -57,8 +57,21 @@ __device__ __forceinline__ void load8(float (&f)[8], const float *p)
 // their code is fetched on the way
 __device__ __forceinline__ float sigmoid_f(float z) { return __builtin_amdgcn_rcpf(1.f + __expf(-z)); }
 __device__ __forceinline__ float silu_f(float z) { return z * sigmoid_f(z); }
-// log(1 + e^z) with an absolute error of about 1e-7, which is what its use in an exponent asks for
-__device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z : __logf(1.f + __expf(z)); }
+// log(1 + e^z) to a few units in the last place also where it is small (a slow decay multiplies over thousands of tokens):
+// max(z, 0) + log(1 + x) with x = e^-|z| <= 1, log(1 + x) = 2 artanh(t), t = x / (2 + x) <= 1/3, as its power series
+__device__ __forceinline__ float softplus_f(float z)
+{
+    const float x = __expf(-fabsf(z)), t = x * __builtin_amdgcn_rcpf(2.f + x), tt = t * t;
+    float p = 1.f / 15.f;
+    p = fmaf(p, tt, 1.f / 13.f);
+    p = fmaf(p, tt, 1.f / 11.f);
+    p = fmaf(p, tt, 1.f / 9.f);
+    p = fmaf(p, tt, 1.f / 7.f);
+    p = fmaf(p, tt, 1.f / 5.f);
+    p = fmaf(p, tt, 1.f / 3.f);
+    p = fmaf(p, tt, 1.f);
+    return fmaf(2.f * t, p, fmaxf(z, 0.f));
+}
 // decay of one key channel: exp(-exp(A_log) softplus(z)), ea = exp(A_log)
 __device__ __forceinline__ float decay_f(float ea, float z) { return __expf(-ea * softplus_f(z)); }
 

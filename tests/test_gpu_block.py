@@ -297,6 +297,21 @@ def test_the_recurrent_state_remembers(lva, ctx):
             assert rel(d.run(toks, cuts), want) < 1e-4, cuts
 
 
+def test_small_decays_add_up(lva, ctx):
+    """a rate of e^-9 times a large exp(A_log): what every token takes off the state has to be right, not only its absolute size"""
+    cfg = bb.config(vocab=40, width=40, layers=[bb.layer(experts=0, without=("left",), right=bb.delta(heads=2, kv_heads=1, dim=30, vdim=24, conv=4))])
+    W = bb.weights(cfg, 67)
+    W["l0.mix.right.dt_bias"] = bb.to_bf16(np.full(60, -9.0))
+    W["l0.mix.right.A_log"] = bb.to_bf16(np.full(2, 3.5))
+    W["l0.mix.right.a2"] = bb.to_bf16(bb.from_bf16(W["l0.mix.right.a2"]) * 0.2)
+    W["l0.mix.right.b"] = bb.to_bf16(bb.from_bf16(W["l0.mix.right.b"]) * 0.3)
+    toks = tokens_for(cfg, 400, 8)
+    want = bo.forward(toks, bb.as_float(W), cfg)[0]
+    with Device(lva, ctx, cfg, W, F32) as d:
+        for cuts in ((1000,), (150, 1)):
+            assert rel(d.run(toks, cuts), want) < 1e-5, cuts
+
+
 # ---- sessions --------------------------------------------------------------------------------------------------------------
 def test_a_session_used_again_and_sessions_side_by_side(lva, ctx):
     cfg = deep()
