@@ -4,7 +4,7 @@
 //   trace_run --model PATH [--dtype bfloat16|float32] --out DIR [--max-tokens N] [--device D]
 //
 // One JSON object a line:
-//   {"step": 0, "entries": [{"id": "a", "tokens": [5, 17, 3], "want": [0, 2]}], "end": []}
+//   {"step": 0, "entries": [{"id": "a", "tokens": [12, 7, 40, 9], "want": [1, 3]}], "end": []}
 // An entry's tokens continue the session of its id; `want` lists the places among them whose logits go to DIR/<step>.f32
 // (little-endian 32-bit floats, [wanted][vocab], entry by entry).  Sessions named in `end` are closed after the step.  A line
 // "done <step>" follows every step.
