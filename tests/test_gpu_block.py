@@ -410,7 +410,7 @@ def folder(tmp_path_factory):
 def test_greedy_generation_through_the_session_class(hostlib, folder):
     path, cfg, W = folder
     F = bb.as_float(W)
-    prompt = [5, 17, 3, 44, 60, 0, 9, 12, 12, 30, 31, 7, 8, 55, 2, 19, 40, 41, 6]
+    prompt = [12, 7, 40, 44, 60, 0, 9, 12, 12, 30, 31, 7, 8, 55, 2, 19, 40, 41, 6]
     want = bo.greedy(prompt, 24, F, cfg)
     c = hostlib.LlavaContext()
     assert c.load_model(path, compute=F32), c.error()
@@ -471,10 +471,10 @@ def test_snapshot_and_restore(hostlib, folder, tmp_path):
 def test_command_line_generates_ids(lva, folder):
     path, cfg, W = folder
     exe = os.path.join(lva.PKG_DIR, "bin", "llava")
-    out = subprocess.run([exe, "-m", path, "--dtype", "float32", "--greedy", "-n", "6", "5 17 3"], capture_output=True, text=True, timeout=100)
+    out = subprocess.run([exe, "-m", path, "--dtype", "float32", "--greedy", "-n", "6", "12 7 40"], capture_output=True, text=True, timeout=100)
     assert out.returncode == 0, out.stderr
-    assert [int(t) for t in out.stdout.split()[:3]] == [5, 17, 3]
-    want = bo.greedy([5, 17, 3], 6, bb.as_float(W), cfg)
+    assert [int(t) for t in out.stdout.split()[:3]] == [12, 7, 40]
+    want = bo.greedy([12, 7, 40], 6, bb.as_float(W), cfg)
     assert [int(t) for t in out.stdout.split()[3:9]] == want
     bad = subprocess.run([exe, "-m", path, "--greedy", "-n", "6", "5 x"], capture_output=True, text=True, timeout=100)
     assert bad.returncode == 1 and "token ids" in bad.stderr
@@ -488,7 +488,7 @@ def test_token_server(hostlib, folder):
     a, b = sc.Client(server.port), sc.Client(server.port)
     F = bb.as_float(W)
     prompts = {}
-    for client, text in ((a, b"5 17 3 9"), (b, b"44, 2")):      # two sessions, ticks in turn
+    for client, text in ((a, b"12 7 40 9"), (b, b"44, 2")):      # two sessions, ticks in turn
         sid = client.new_session()
         assert client.ack(sc.SET_OPTIONS, sid, sc.OPTION_GREEDY) == sc.RC_OK
         assert client.ack(sc.ADD_TEXT, sid, text=text) == sc.RC_OK
