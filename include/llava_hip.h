@@ -77,11 +77,17 @@ int lv_model_hparams(const lv_model *model, lv_hparams *out);
 int lv_model_arena_bytes(const lv_model *model, uint64_t *bytes);
 
 /* ---- block models: designs whose layers are put together from described mechanisms (no counterpart in the reference,
- *      which knows one design).  A layer is  x += post1(mixer(pre1(x)));  x += post2(ff(pre2(x)))  with RMS norms on both
- *      sides of each sublayer; the mixer is one or two branches reading the same input, summed with a scale each:
- *        attention  grouped-query softmax attention (csrc/lv_gqa.h)
- *        delta      gated delta rule with a decay per key channel (csrc/lv_delta.h)
- *      and the feed-forward a mixture of experts whose weights multiply the experts' inputs, or none.
+ *      which knows one design).  A layer is a mixer and, after it, a feed-forward or none.
+ *      Residual, lv_block_hparams.streams:
+ *        0     x += post(sublayer(pre(x))), RMS norms on both sides
+ *        s     hyper-connections over s copies x_1 .. x_s of the embedding: u = sum_t in[t] x_t, y = sublayer(pre(u)),
+ *              x_t = sum_f mix[f][t] x_f + out[t] y; the model's end reads the sum of the copies (csrc/lv_streams.h)
+ *      Mixer, one of
+ *        attention and / or delta   grouped-query softmax attention (csrc/lv_gqa.h) and a gated delta rule with a decay per key
+ *                                   channel (csrc/lv_delta.h), reading the same input, summed with a scale each
+ *        latent                     attention over a shared low-rank latent (csrc/lv_latent.h)
+ *        ssm                        state-space recurrence with a decay per head (csrc/lv_ssm.h)
+ *      Feed-forward: a mixture of experts whose weights multiply the experts' inputs, or a dense gated one, or none.
  *      Weights are bfloat16, [out][in].  Every lv_session_* / lv_step_* / lv_logits_* / lv_argmax call works on sessions of
  *      such a model; what differs is said at the call. ------------------------------------------------------------- */
 enum {
@@ -102,25 +108,60 @@ typedef struct {
     uint32_t conv;                         /* taps of the causal convolutions on q, k and v (the current token included) */
 } lv_delta_spec;
 typedef struct {
-    uint32_t experts, top, ff;             /* experts 0: the layer has no feed-forward */
-} lv_moe_spec;
+    uint32_t heads, dim, rot_dim, vdim;    /* heads 0: no such mixer; a query or key is dim unrotated and then rot_dim rotated dimensions */
+    uint32_t q_rank, kv_rank;              /* latent sizes; the rotated part of the key is one vector for all heads */
+    float scale;
+    uint32_t rot_dims;                     /* of the rotated part, the dimensions that turn (even), as in lv_attn_spec */
+    double rot_base;
+    uint32_t flags;                        /* LV_ATTN_SINK */
+} lv_latent_spec;
 typedef struct {
-    float attn_scale, delta_scale;         /* factors of the two branches */
+    uint32_t heads, groups, state, vdim;   /* heads 0: no such mixer; consecutive heads share a group's B and C of `state` entries */
+    uint32_t conv;                         /* taps of the causal convolution on x, B and C (the current token included) */
+    uint32_t norm_groups;                  /* equal parts of the gated read-out, each with an RMS norm of its own */
+} lv_ssm_spec;
+typedef struct {
+    uint32_t experts, top, ff;             /* experts 0: no mixture */
+} lv_moe_spec;
+enum { LV_ACT_SILU = 0, LV_ACT_RELU = 1 };
+typedef struct {
+    uint32_t ff;                           /* 0: no dense feed-forward */
+    uint32_t act;                          /* LV_ACT_*: down(act(gate h) * (up h)) */
+} lv_dense_spec;
+typedef struct {
+    float attn_scale, delta_scale;         /* factors of the attention and the delta branch */
     lv_attn_spec attn;
     lv_delta_spec delta;
     lv_moe_spec moe;
+    lv_latent_spec latent;
+    lv_ssm_spec ssm;
+    lv_dense_spec dense;
 } lv_block_spec;
+enum {
+    LV_NORM_RMS = 0,                       /* pre-norms and the final norm: x / rms(x) * w */
+    LV_NORM_TANH = 1                       /* tanh(alpha x) * w + b, alpha a scalar (models with streams) */
+};
 typedef struct {
-    uint32_t vocab, dim, layers;
+    uint32_t vocab, dim, layers;           /* layers: as listed; each pass of a loop counts as a layer of its own in lv_state_*, lv_trace_* */
     float eps;                             /* of every RMS norm */
+    uint32_t norm;                         /* LV_NORM_* */
+    uint32_t streams;
+    uint32_t tied_head;                    /* 1: the output matrix is the embedding table */
+    float embed_scale;                     /* factor of the embedding rows; 0: 1 */
+    uint32_t bigram_buckets;               /* 0: none; else row (previous token * prev + token * cur) mod buckets of a second table, row `buckets` for a sequence's first token */
+    uint32_t bigram_prev, bigram_cur;
+    uint32_t loop_start, loop_stop, loop_times;   /* listed layers start .. stop - 1 run `times` times in a row, with a state per pass; times 0: no loop */
 } lv_block_hparams;
 
-/* Uploads such a model.  Tensors are looked up by name in `table` (bf16; vectors may be f32): embed, final.norm, head, and
- * per layer i, prefix "l<i>.": norm1, norm1b, norm2, norm2b, mix.left.{q,k,v,o,q.norm,k.norm,sink} (attention),
- * mix.right.{q,k,v,b,a1,a2,g1,g2,o,q.conv,k.conv,v.conv,A_log,dt_bias,norm} (delta), mlp.router, mlp.e<j>.{gate,up,down}.
+/* Uploads such a model.  Tensors are looked up by name in `table` (bf16; vectors may be f32): embed, bigram, final.norm, head
+ * (unless tied), and per layer i, prefix "l<i>.": norm1, norm2 (where there is a feed-forward), with LV_NORM_TANH also
+ * <norm>.alpha and <norm>.b, without streams norm1b, norm2b, with streams hc1.{in,out,mix}, hc2.{in,out,mix};
+ * mix.left.{q,k,v,o,q.norm,k.norm,sink} (attention), mix.right.{q,k,v,b,a1,a2,g1,g2,o,q.conv,k.conv,v.conv,A_log,dt_bias,norm} (delta),
+ * mix.{dq,dq.norm,uq,dkv,dkv.norm,uk,uv,sink,o} (latent), mix.{in,conv,conv.b,dt_bias,A_log,D,norm,o} (ssm), mlp.router,
+ * mlp.e<j>.{gate,up,down} (mixture), mlp.{gate,up,down} (dense).
  * The ranks of a1 / a2 and g1 / g2 are taken from the tensors.  compute: LV_BF16 = matrix products of batches on bf16
  * activations with 32-bit accumulation and bf16 cache rows; LV_F32 = every operand in 32-bit.  Norms, scores, softmax,
- * router, the recurrence and the residual stream are fp32 in both. */
+ * router, the recurrences and the residual stream are fp32 in both. */
 int lv_block_model_upload(lv_ctx *ctx, const void *base, uint64_t base_size, const lv_block_hparams *hp, const lv_block_spec *blocks,
                           const lv_tensor_desc *table, uint32_t n_tensors, int compute, lv_model **out);
 

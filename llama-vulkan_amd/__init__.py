@@ -54,12 +54,28 @@ class MoeSpec(C.Structure):
     _fields_ = [("experts", C.c_uint32), ("top", C.c_uint32), ("ff", C.c_uint32)]
 
 
+class LatentSpec(C.Structure):
+    _fields_ = [("heads", C.c_uint32), ("dim", C.c_uint32), ("rot_dim", C.c_uint32), ("vdim", C.c_uint32), ("q_rank", C.c_uint32), ("kv_rank", C.c_uint32),
+                ("scale", C.c_float), ("rot_dims", C.c_uint32), ("rot_base", C.c_double), ("flags", C.c_uint32)]
+
+
+class SsmSpec(C.Structure):
+    _fields_ = [("heads", C.c_uint32), ("groups", C.c_uint32), ("state", C.c_uint32), ("vdim", C.c_uint32), ("conv", C.c_uint32), ("norm_groups", C.c_uint32)]
+
+
+class DenseSpec(C.Structure):
+    _fields_ = [("ff", C.c_uint32), ("act", C.c_uint32)]
+
+
 class BlockSpec(C.Structure):
-    _fields_ = [("attn_scale", C.c_float), ("delta_scale", C.c_float), ("attn", AttnSpec), ("delta", DeltaSpec), ("moe", MoeSpec)]
+    _fields_ = [("attn_scale", C.c_float), ("delta_scale", C.c_float), ("attn", AttnSpec), ("delta", DeltaSpec), ("moe", MoeSpec), ("latent", LatentSpec),
+                ("ssm", SsmSpec), ("dense", DenseSpec)]
 
 
 class BlockHParams(C.Structure):
-    _fields_ = [("vocab", C.c_uint32), ("dim", C.c_uint32), ("layers", C.c_uint32), ("eps", C.c_float)]
+    _fields_ = [("vocab", C.c_uint32), ("dim", C.c_uint32), ("layers", C.c_uint32), ("eps", C.c_float), ("norm", C.c_uint32), ("streams", C.c_uint32),
+                ("tied_head", C.c_uint32), ("embed_scale", C.c_float), ("bigram_buckets", C.c_uint32), ("bigram_prev", C.c_uint32), ("bigram_cur", C.c_uint32),
+                ("loop_start", C.c_uint32), ("loop_stop", C.c_uint32), ("loop_times", C.c_uint32)]
 
 
 class MkgConfig(C.Structure):
@@ -369,17 +385,18 @@ class Model:
 
 class BlockModel:
     """A block model uploaded through lv_block_model_upload.  blocks: list of BlockSpec; table: (name, type, offset, rows, cols,
-    size) per tensor with offsets into `base` (a uint8 array; tensors may share bytes)."""
+    size) per tensor with offsets into `base` (a uint8 array; tensors may share bytes); model_wide: further BlockHParams fields."""
 
-    def __init__(self, ctx, base, table, blocks, vocab, dim, eps, compute=LV_BF16):
+    def __init__(self, ctx, base, table, blocks, vocab, dim, eps, compute=LV_BF16, **model_wide):
         self.ctx = ctx
         self.lib = ctx.lib
-        self.header = dict(vocab=vocab, dim=dim, layers=len(blocks), ff=0, heads=0)
         descs = (TensorDesc * len(table))()
         names = [t[0].encode() for t in table]
         for d, t, nm in zip(descs, table, names):
             d.name, d.ftype, d.offset, d.rows, d.cols, d.size = nm, t[1], t[2], t[3], t[4], t[5]
-        hp = BlockHParams(vocab, dim, len(blocks), eps)
+        hp = BlockHParams(vocab, dim, len(blocks), eps, **model_wide)
+        passes = len(blocks) + max(0, hp.loop_times - 1) * (hp.loop_stop - hp.loop_start)
+        self.header = dict(vocab=vocab, dim=dim, layers=passes, ff=0, heads=0)
         self.h = C.c_void_p()
         check(self.lib.lv_block_model_upload(ctx.h, C.c_void_p(base.ctypes.data), base.nbytes, C.byref(hp), (BlockSpec * len(blocks))(*blocks), descs,
                                              len(table), compute, C.byref(self.h)))

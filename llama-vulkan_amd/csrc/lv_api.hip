@@ -1460,13 +1460,13 @@ extern "C" int lv_block_model_upload(lv_ctx *c, const void *base, uint64_t base_
     m->ctx = c;
     m->hp.vocab = hp->vocab;
     m->hp.dim = hp->dim;
-    m->hp.layers = hp->layers;
     const int rc = block_model_create(c->stream, base, base_size, hp, blocks, table, n_tensors, compute, &m->block);
     if (rc != LV_OK) {
         delete m;
         return rc;
     }
     m->arena_bytes = block_model_bytes(m->block);
+    m->hp.layers = block_model_passes(m->block);
     *out = m;
     return LV_OK;
 }

@@ -17,6 +17,7 @@
 // all banks.
 #pragma once
 
+#include "../../include/llava_hip.h"
 #include "lv_device.h"
 
 namespace lv {
@@ -72,6 +73,8 @@ __device__ __forceinline__ float softplus_f(float z)
     p = fmaf(p, tt, 1.f);
     return fmaf(2.f * t, p, fmaxf(z, 0.f));
 }
+// activation of a gated feed-forward, LV_ACT_*
+__device__ __forceinline__ float glu_f(uint32_t act, float z) { return act == LV_ACT_RELU ? fmaxf(z, 0.f) : silu_f(z); }
 // decay of one key channel: exp(-exp(A_log) softplus(z)), ea = exp(A_log)
 __device__ __forceinline__ float decay_f(float ea, float z) { return __expf(-ea * softplus_f(z)); }
 
@@ -81,6 +84,8 @@ enum BfEpilogue {
     kEpSigmoid = 2,  // out[token][row] = sigmoid(v)
     kEpGlu = 3,      // rows alternate 16 gate, 16 up: act[position][f] = silu(w g) * (w u), w = the expert's weight for the token
     kEpScatter = 4,  // grouped: out[slots[position]][row]
+    kEpDense = 5,    // rows as for kEpGlu, one expert: act[token][f] = activation(g) * u
+    kEpHeads = 6,    // activations instead of fp32, heads padded: act[token][head * head_stride + channel], row = head * head_dim + channel
 };
 
 struct BfGemmArgs {
@@ -95,7 +100,7 @@ struct BfGemmArgs {
     // K cut in slices (kEpStore): grid z = slice, its sum goes to out + slice * slice_floats; the reader adds them up
     uint32_t k_slice;        // columns per slice, a multiple of the K step; 0: one slice
     uint64_t slice_floats;
-    // decay epilogue
+    // decay and head epilogues
     const float *a_log, *bias;
     uint32_t head_dim, head_stride;
     // grouped
@@ -104,8 +109,9 @@ struct BfGemmArgs {
     const float *weights;    // [token * top + choice]
     uint32_t top, expert_rows;   // weight rows from one expert to the next
     bool gather;             // x rows are tokens (slots[position] / top), otherwise positions
-    void *act;               // kEpGlu output [position][lda]
+    void *act;               // kEpGlu, kEpDense, kEpHeads output [position][lda]
     uint32_t lda;
+    uint32_t activation;     // kEpDense: LV_ACT_*
 };
 
 // four results of one token: weight rows row .. row + 3
@@ -143,6 +149,39 @@ __device__ __forceinline__ void bf_store4(const BfGemmArgs &a, uint32_t orow, ui
         for (int i = 0; i < 4; i++)
             if (row + i < a.rows) o[i] = r[i];
     }
+}
+
+// four results of one token, rows row .. row + 3, into padded heads
+template <class T>
+__device__ __forceinline__ void bf_store_heads(const BfGemmArgs &a, uint32_t token, uint32_t row, const lv_f4 v)
+{
+    if (row >= a.rows) return;
+    T *o = static_cast<T *>(a.act) + (size_t)token * a.lda;
+    if (a.head_dim % 4 == 0) {
+        const uint32_t h = row / a.head_dim;
+        o += (size_t)h * a.head_stride + (row - h * a.head_dim);
+        if constexpr (sizeof(T) == 2)
+            *reinterpret_cast<uint2 *>(o) = make_uint2((uint32_t)float_to_bf16(v[0]) | ((uint32_t)float_to_bf16(v[1]) << 16),
+                                                       (uint32_t)float_to_bf16(v[2]) | ((uint32_t)float_to_bf16(v[3]) << 16));
+        else *reinterpret_cast<float4 *>(o) = make_float4(v[0], v[1], v[2], v[3]);
+        return;
+    }
+#pragma unroll
+    for (int i = 0; i < 4; i++)
+        if (row + i < a.rows) o[(size_t)((row + i) / a.head_dim) * a.head_stride + (row + i) % a.head_dim] = float_to_elem<T>(v[i]);
+}
+
+template <class T>
+__device__ __forceinline__ void bf_store_dense(const BfGemmArgs &a, uint32_t token, uint32_t f, const lv_f4 g, const lv_f4 u)
+{
+    T *o = static_cast<T *>(a.act) + (size_t)token * a.lda + f;
+    float v[4];
+#pragma unroll
+    for (int i = 0; i < 4; i++) v[i] = glu_f(a.activation, g[i]) * u[i];
+    if constexpr (sizeof(T) == 2)
+        *reinterpret_cast<uint2 *>(o) = make_uint2((uint32_t)float_to_bf16(v[0]) | ((uint32_t)float_to_bf16(v[1]) << 16),
+                                                   (uint32_t)float_to_bf16(v[2]) | ((uint32_t)float_to_bf16(v[3]) << 16));
+    else *reinterpret_cast<float4 *>(o) = make_float4(v[0], v[1], v[2], v[3]);
 }
 
 template <class T>
@@ -274,6 +313,15 @@ __global__ __launch_bounds__(NW * 64, 2) void gemm_bf16_kernel(BfGemmArgs a)
                 const uint32_t row = rt * RM + wm * 64 + i * 16;        // the pair's gate block
                 if (row < a.rows) bf_store_glu<uint16_t>(a, p, row / 2 + g4 * 4, wt, acc[i][j], acc[i + 1][j]);
             }
+        } else if constexpr (EP == kEpDense) {
+#pragma unroll
+            for (int i = 0; i < 4; i += 2) {
+                const uint32_t row = rt * RM + wm * 64 + i * 16;
+                if (row < a.rows) bf_store_dense<uint16_t>(a, p, row / 2 + g4 * 4, acc[i][j], acc[i + 1][j]);
+            }
+        } else if constexpr (EP == kEpHeads) {
+#pragma unroll
+            for (int i = 0; i < 4; i++) bf_store_heads<uint16_t>(a, p, rt * RM + wm * 64 + i * 16 + g4 * 4, acc[i][j]);
         } else {
             const uint32_t orow = EP == kEpScatter ? a.slots[p] : p;
 #pragma unroll
@@ -340,6 +388,11 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(BfGemmArgs a)
         const uint32_t p = first + t;
         if constexpr (EP == kEpGlu) {
             bf_store_glu<float>(a, p, (rt * kF32Tile + wm * 32) / 2 + g4 * 4, a.weights[a.slots[p]], acc[0][j], acc[1][j]);
+        } else if constexpr (EP == kEpDense) {
+            bf_store_dense<float>(a, p, (rt * kF32Tile + wm * 32) / 2 + g4 * 4, acc[0][j], acc[1][j]);
+        } else if constexpr (EP == kEpHeads) {
+#pragma unroll
+            for (int i = 0; i < 2; i++) bf_store_heads<float>(a, p, rt * kF32Tile + wm * 32 + i * 16 + g4 * 4, acc[i][j]);
         } else {
             const uint32_t orow = EP == kEpScatter ? a.slots[p] : p;
 #pragma unroll

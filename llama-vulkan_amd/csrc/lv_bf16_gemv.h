@@ -7,11 +7,14 @@
 //              residual and x in memory for later launches
 //   kInPlain   a vector in memory
 //   kInBranch  the concatenated outputs of two mixers: scaled attention heads, then gated and normalised recurrent heads
-// kGemvExperts multiplies the rows of several experts (gate and up interleaved, SwiGLU), chosen from the router logits in the
+//   kInGroups  a read-out times silu of its gate, normalised in equal parts
+//   kInStreams2 .. 8   the norm of a residual of up to 2, 4 or 8 streams (lv_streams.h)
+// kGemvGlu multiplies interleaved gate and up rows (act(gate) * up).  kGemvExperts multiplies the rows of several experts (gate and up interleaved, SwiGLU), chosen from the router logits in the
 // kernel's head; kGemvDown sums a row over the chosen experts' down projections.
 #pragma once
 
 #include "lv_bf16_gemm.h"
+#include "lv_streams.h"
 
 namespace lv {
 
@@ -23,8 +26,8 @@ __device__ __forceinline__ uint4 load_once(const uint16_t *p)
     return make_uint4(v.x, v.y, v.z, v.w);
 }
 
-enum BfInput { kInNorm = 0, kInPlain = 1, kInBranch = 2 };
-enum BfGemvMode { kGemvRows = 0, kGemvExperts = 1, kGemvDown = 2 };
+enum BfInput { kInNorm = 0, kInPlain = 1, kInBranch = 2, kInGroups = 3, kInStreams2 = 4, kInStreams4 = 5, kInStreams8 = 6 };
+enum BfGemvMode { kGemvRows = 0, kGemvExperts = 1, kGemvDown = 2, kGemvGlu = 3 };
 
 constexpr int kBfGemvThreads = 512;
 constexpr int kBfGemvWaves = kBfGemvThreads / 64;
@@ -47,6 +50,13 @@ struct BranchInput {
     float left_scale, right_scale, eps;
 };
 
+// o * silu(z) in `groups` equal parts, each divided by its own root mean square, times w
+struct GroupInput {
+    const float *o, *z, *w;
+    uint32_t n, groups;
+    float eps;
+};
+
 struct BfGemvArgs {
     const uint16_t *w;
     uint32_t rows, kp;
@@ -54,6 +64,9 @@ struct BfGemvArgs {
     NormInput norm;
     const float *x;              // kInPlain
     BranchInput branch;
+    GroupInput group;
+    StreamInput streams;
+    uint32_t act;                // kGemvGlu: LV_ACT_*
     // experts
     const float *z;              // router logits
     uint32_t experts, top, expert_rows;   // expert_rows: weight rows from one expert to the next
@@ -64,36 +77,6 @@ struct BfGemvArgs {
 // x lies in LDS in two planes, elements 8c .. 8c+3 and 8c+4 .. 8c+7, so that a lane's two 16-byte reads are consecutive over
 // the lanes
 __device__ __forceinline__ uint32_t bf_xs(uint32_t i, uint32_t kp) { return ((i >> 2) & 1) * (kp / 2) + (i >> 3) * 4 + (i & 3); }
-
-__device__ __forceinline__ float block_sum_waves(float v, float *scratch, int nw)
-{
-    v = wave_sum(v);
-    __syncthreads();
-    if ((threadIdx.x & 63) == 0) scratch[threadIdx.x >> 6] = v;
-    __syncthreads();
-    float t = 0.f;
-    for (int i = 0; i < nw; i++) t += scratch[i];
-    return t;
-}
-
-// the same for N values at once; scratch holds N * nw floats
-template <int N>
-__device__ __forceinline__ void block_sums_waves(float (&v)[N], float *scratch, int nw)
-{
-#pragma unroll
-    for (int i = 0; i < N; i++) v[i] = wave_sum(v[i]);
-    __syncthreads();
-    if ((threadIdx.x & 63) == 0) {
-#pragma unroll
-        for (int i = 0; i < N; i++) scratch[i * nw + (threadIdx.x >> 6)] = v[i];
-    }
-    __syncthreads();
-#pragma unroll
-    for (int i = 0; i < N; i++) {
-        v[i] = 0.f;
-        for (int w = 0; w < nw; w++) v[i] += scratch[i * nw + w];
-    }
-}
 
 // NormInput into xs; every thread keeps to its own elements between the passes
 __device__ __forceinline__ void norm_input(const NormInput &a, float *xs, float *scratch)
@@ -162,6 +145,35 @@ __device__ __forceinline__ void branch_input(const BranchInput &a, float *xs, ui
     }
 }
 
+// GroupInput: put(i, value).  Waves share a group where there are fewer groups than waves; `sums` holds group_sums() floats and
+// every thread keeps to its own elements between the passes.
+__host__ __device__ constexpr uint32_t group_parts(uint32_t groups, uint32_t waves) { return groups >= waves ? 1 : waves / groups; }
+__host__ __device__ constexpr uint32_t group_sums(uint32_t groups, uint32_t waves) { return groups * group_parts(groups, waves); }
+template <class Put, class Get>
+__device__ __forceinline__ void group_input(const GroupInput &a, float *sums, Put put, Get get)
+{
+    const uint32_t lane = threadIdx.x & 63, waves = blockDim.x >> 6, parts = group_parts(a.groups, waves), tasks = a.groups * parts, size = a.n / a.groups;
+    for (uint32_t k = threadIdx.x >> 6; k < tasks; k += waves) {
+        const uint32_t base = k / parts * size;
+        float s = 0.f;
+        for (uint32_t c = k % parts * 64 + lane; c < size; c += parts * 64) {
+            const float v = a.o[base + c] * silu_f(a.z[base + c]);
+            s = fmaf(v, v, s);
+            put(base + c, v);
+        }
+        s = wave_sum(s);
+        if (lane == 0) sums[k] = s;
+    }
+    __syncthreads();
+    for (uint32_t k = threadIdx.x >> 6; k < tasks; k += waves) {
+        const uint32_t g = k / parts, base = g * size;
+        float s = 0.f;
+        for (uint32_t p = 0; p < parts; p++) s += sums[g * parts + p];
+        const float inv = rsqrtf(s / (float)size + a.eps);
+        for (uint32_t c = k % parts * 64 + lane; c < size; c += parts * 64) put(base + c, get(base + c) * inv * a.w[base + c]);
+    }
+}
+
 // The `top` largest of n router logits, largest first, the lower index on equal values (one wave; zs is consumed).  Scores are
 // the sigmoids of the chosen logits, not renormalised.
 __device__ __forceinline__ void top_experts(float *zs, uint32_t n, uint32_t top, uint32_t *ids, float *scores)
@@ -196,7 +208,8 @@ __device__ __forceinline__ uint32_t kp_units(const BfGemvArgs &a) { return a.exp
 template <int MODE, int INPUT, int R, int DEPTH>
 __global__ __launch_bounds__(kBfGemvThreads) void bf16_gemv_kernel(BfGemvArgs a)
 {
-    constexpr int NR = MODE == kGemvExperts ? 2 * R : R;
+    constexpr bool PAIRS = MODE == kGemvExperts || MODE == kGemvGlu;      // gate and up rows
+    constexpr int NR = PAIRS ? 2 * R : R;
     extern __shared__ float xs[];          // kp floats (kGemvDown: top * kp), then kGemvExperts: router logits
     __shared__ float scratch[kBfGemvWaves];
     __shared__ uint32_t sel_id[kMaxTop];
@@ -205,7 +218,7 @@ __global__ __launch_bounds__(kBfGemvThreads) void bf16_gemv_kernel(BfGemvArgs a)
     const uint32_t kp = a.kp;
     const uint32_t segs = MODE == kGemvDown ? a.top : 1;
     const uint32_t ksteps = (kp + 511) / 512, iters = ksteps * segs;
-    const uint32_t units = MODE == kGemvExperts ? a.top * kp_units(a) : a.rows;
+    const uint32_t units = MODE == kGemvExperts ? a.top * kp_units(a) : MODE == kGemvGlu ? a.rows / 2 : a.rows;
     const uint32_t tasks = (units + R - 1) / R, nwaves = gridDim.x * kBfGemvWaves;
     const uint32_t first_task = blockIdx.x * kBfGemvWaves + wave;
 
@@ -235,13 +248,16 @@ __global__ __launch_bounds__(kBfGemvThreads) void bf16_gemv_kernel(BfGemvArgs a)
             const uint32_t u = ftask * R, per = kp_units(a);
             const uint32_t s = ok ? u / per : 0, f = ok ? u % per : 0;
             p += ((size_t)sel_id[s] * a.expert_rows + (f >> 4) * 32 + (f & 15)) * kp;
+        } else if constexpr (MODE == kGemvGlu) {
+            const uint32_t f = ftask * R;
+            p += ((size_t)(f >> 4) * 32 + (f & 15)) * kp;
         } else {
             p += (size_t)ftask * R * kp;
             if constexpr (MODE == kGemvDown) p += (size_t)sel_id[fseg] * a.expert_rows * kp;
         }
 #pragma unroll
         for (int r = 0; r < NR; r++) {
-            const size_t off = MODE == kGemvExperts ? (size_t)(r % R + (r / R) * 16) * kp : (size_t)r * kp;
+            const size_t off = PAIRS ? (size_t)(r % R + (r / R) * 16) * kp : (size_t)r * kp;
             slot[r] = ok ? load_once(p + off) : make_uint4(0, 0, 0, 0);
         }
         if (++fit == ksteps) {
@@ -259,6 +275,12 @@ __global__ __launch_bounds__(kBfGemvThreads) void bf16_gemv_kernel(BfGemvArgs a)
         norm_input(a.norm, xs, scratch);
     } else if constexpr (INPUT == kInBranch) {
         branch_input(a.branch, xs, kp);
+    } else if constexpr (INPUT == kInGroups) {
+        for (uint32_t i = a.group.n + threadIdx.x; i < kp; i += kBfGemvThreads) xs[bf_xs(i, kp)] = 0.f;
+        group_input(a.group, xs + kp, [&](uint32_t i, float v) { xs[bf_xs(i, kp)] = v; }, [&](uint32_t i) { return xs[bf_xs(i, kp)]; });
+    } else if constexpr (INPUT >= kInStreams2) {
+        stream_input<2 << (INPUT - kInStreams2)>(a.streams, blockIdx.x == 0, scratch, [&](uint32_t i, const float4 h) { *reinterpret_cast<float4 *>(xs + bf_xs(i, kp)) = h; },
+                                                 [&](uint32_t i) { return *reinterpret_cast<const float4 *>(xs + bf_xs(i, kp)); });
     } else {
         for (uint32_t i = threadIdx.x * 4; i < kp * segs; i += kBfGemvThreads * 4) {
             const uint32_t sg = i / kp, k = i % kp;
@@ -306,6 +328,8 @@ __global__ __launch_bounds__(kBfGemvThreads) void bf16_gemv_kernel(BfGemvArgs a)
                             if constexpr (MODE == kGemvExperts) {
                                 const float wt = sel_score[u / kp_units(a)];
                                 a.out[u] = silu_f(wt * v0) * (wt * v1);
+                            } else if constexpr (MODE == kGemvGlu) {
+                                a.out[u] = glu_f(a.act, v0) * v1;
                             } else {
                                 a.out[u] = v0;
                             }

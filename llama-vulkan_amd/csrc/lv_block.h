@@ -13,6 +13,8 @@ int block_model_create(hipStream_t st, const void *base, uint64_t base_size, con
                        const lv_tensor_desc *table, uint32_t n_tensors, int compute, BlockModel **out);
 void block_model_destroy(BlockModel *m);
 uint64_t block_model_bytes(const BlockModel *m);
+// layers as a sequence runs through them: each pass of a loop counts, and has a state of its own
+uint32_t block_model_passes(const BlockModel *m);
 
 int block_session_create(const BlockModel *m, hipStream_t st, BlockSession **out);
 void block_session_destroy(BlockSession *s);

@@ -4,15 +4,41 @@
 #pragma once
 
 #include "lv_delta.h"
-#include "lv_gqa.h"
+#include "lv_latent.h"
+#include "lv_ssm.h"
 
 namespace lv {
 
-// x[z][0 .. dp) = table[token[z]], fp32, zero beyond dim
-__global__ __launch_bounds__(256) void embed_bf16_kernel(float *__restrict__ x, const uint16_t *__restrict__ table, const uint32_t *tokens, uint32_t dim, uint32_t dp)
+// x[z][0 .. dp) = table[token] * scale (+ a row of the bigram table), fp32, zero beyond dim, in every stream
+struct EmbedArgs {
+    float *x;                    // [token][stream][dp]
+    const uint16_t *table;       // rows of `ld` elements
+    uint32_t ld, dim, dp, streams;
+    float scale;
+    const uint32_t *cfg;         // position of the step's first token, then the step's tokens
+    uint32_t idx;                // the launch's first token in the step
+    const uint16_t *bigram;      // [buckets + 1][dim]; null: none
+    uint32_t buckets, prev, cur;
+    uint32_t *last;              // a sequence's last token, at [position % 2]
+};
+static __global__ __launch_bounds__(256) void embed_bf16_kernel(EmbedArgs a)
 {
-    const uint32_t i = blockIdx.x * 256 + threadIdx.x, z = blockIdx.y;
-    if (i < dp) x[(size_t)z * dp + i] = i < dim ? bf16_to_float(table[(size_t)tokens[z] * dim + i]) : 0.f;
+    const uint32_t i = blockIdx.x * 256 + threadIdx.x, z = blockIdx.y, at = a.idx + z, pos = a.cfg[0] + at, token = a.cfg[1 + at];
+    const uint16_t *row = a.bigram;
+    if (a.bigram) {
+        uint32_t r = a.buckets;
+        if (pos) r = (uint32_t)(((uint64_t)(at ? a.cfg[at] : a.last[(pos - 1) & 1]) * a.prev + (uint64_t)token * a.cur) % a.buckets);
+        row += (size_t)r * a.dim;
+        // a launch of one token leaves it for the next; one of several is followed by a copy, since its first row may read the slot
+        if (gridDim.y == 1 && i == 0) a.last[pos & 1] = token;
+    }
+    if (i >= a.dp) return;
+    float v = 0.f;
+    if (i < a.dim) {
+        v = bf16_to_float(a.table[(size_t)token * a.ld + i]) * a.scale;
+        if (row) v += bf16_to_float(row[i]);
+    }
+    for (uint32_t t = 0; t < a.streams; t++) a.x[((size_t)z * a.streams + t) * a.dp + i] = v;
 }
 
 // NormInput for a batch: one workgroup per row; x in place, h as activations
@@ -163,7 +189,7 @@ __global__ __launch_bounds__(256) void prepare_kernel(PrepareArgs a, uint32_t n)
         const uint32_t c = (col - s.kv_heads) * 256 + threadIdx.x;
         if (c >= nv) return;
         for (uint32_t t = first; t < last; t++)
-            a.dv[(size_t)t * nv + c] = delta_conv(s, a.y + (size_t)t * a.ldy, a.ldy, t, 2 * nq + c, a.pos0 + t, (a.pos0 + t) % s.taps);
+            a.dv[(size_t)t * nv + c] = short_conv(s, a.y + (size_t)t * a.ldy, a.ldy, t, 2 * nq + c, a.pos0 + t, (a.pos0 + t) % s.taps);
         return;
     }
     const uint32_t lane = threadIdx.x & 63, h = col;
@@ -176,8 +202,8 @@ __global__ __launch_bounds__(256) void prepare_kernel(PrepareArgs a, uint32_t n)
             const uint32_t d = j * 64 + lane;
             q[j] = k[j] = 0.f;
             if (d < s.dim) {
-                q[j] = delta_conv(s, y, a.ldy, t, h * s.dim + d, pos, slot);
-                k[j] = delta_conv(s, y, a.ldy, t, nq + h * s.dim + d, pos, slot);
+                q[j] = short_conv(s, y, a.ldy, t, h * s.dim + d, pos, slot);
+                k[j] = short_conv(s, y, a.ldy, t, nq + h * s.dim + d, pos, slot);
             }
             sq = fmaf(q[j], q[j], sq);
             sk = fmaf(k[j], k[j], sk);
@@ -216,7 +242,7 @@ __global__ __launch_bounds__(256) void append_kernel(PrepareArgs a, uint32_t n)
     }
     if (a.delta.heads && blockIdx.x < a.delta.taps) {
         const uint32_t C = a.delta.channels();
-        for (uint32_t c = threadIdx.x; c < C; c += 256) a.delta.ring[(size_t)(pos % a.delta.taps) * C + c] = a.y[(size_t)t * a.ldy + delta_channel_at(a.delta, c)];
+        for (uint32_t c = threadIdx.x; c < C; c += 256) a.delta.ring[(size_t)(pos % a.delta.taps) * C + c] = a.y[(size_t)t * a.ldy + a.delta.channel_at(c)];
     }
 }
 

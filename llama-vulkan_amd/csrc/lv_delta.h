@@ -15,7 +15,7 @@
 // a new sequence: positions before 0 and the state at position 0 are never read.
 #pragma once
 
-#include "lv_bf16_gemv.h"
+#include "lv_conv.h"
 
 namespace lv {
 
@@ -30,6 +30,13 @@ struct DeltaSpec {
     float *state, *ring;
     uint32_t dstride;              // 64 J
     __host__ __device__ uint32_t channels() const { return 2 * kv_heads * dim + heads * vdim; }
+    // channel c (in q, k, v order) of the joint projection
+    __device__ __forceinline__ uint32_t channel_at(uint32_t c) const
+    {
+        const uint32_t nq = kv_heads * dim;
+        return c < nq ? q_off + c : c < 2 * nq ? k_off + (c - nq) : v_off + (c - 2 * nq);
+    }
+    __device__ __forceinline__ float conv_bias(uint32_t) const { return 0.f; }
 };
 
 struct DeltaStepArgs {
@@ -44,53 +51,6 @@ struct DeltaStepArgs {
 constexpr int kDeltaCols = 32;     // columns per workgroup of the one-token step: 16 lanes to each
 constexpr uint32_t kDeltaMaxDim = 256;
 constexpr uint32_t kDeltaMaxRank = 4096;
-
-// channel c (in q, k, v order) of the joint projection
-__device__ __forceinline__ uint32_t delta_channel_at(const DeltaSpec &s, uint32_t c)
-{
-    const uint32_t nq = s.kv_heads * s.dim;
-    return c < nq ? s.q_off + c : c < 2 * nq ? s.k_off + (c - nq) : s.v_off + (c - 2 * nq);
-}
-
-// Convolution and silu of channel c at position pos (slot = pos % taps).  y: the token's projection row; rows before it (in
-// steps of ld floats) belong to positions pos - 1, pos - 2, .. as far as `behind` of them, older inputs are in the ring.
-// fetch() requests the first four taps, which is usually all there are; value() does the rest.
-struct DeltaConv {
-    float x[4], w[4];
-    uint32_t at, c;
-
-    static __device__ __forceinline__ float input(const DeltaSpec &s, const float *y, size_t ld, uint32_t behind, uint32_t at, uint32_t c, uint32_t slot, uint32_t j)
-    {
-        return j <= behind ? y[at - (ptrdiff_t)(j * ld)] : s.ring[(size_t)(slot >= j ? slot - j : slot + s.taps - j) * s.channels() + c];
-    }
-    __device__ __forceinline__ void fetch(const DeltaSpec &s, const float *y, size_t ld, uint32_t behind, uint32_t c_, uint32_t pos, uint32_t slot)
-    {
-        c = c_;
-        at = delta_channel_at(s, c);
-        const float *wp = s.conv + (size_t)(s.taps - 1) * s.channels() + c;
-#pragma unroll
-        for (uint32_t j = 0; j < 4; j++) {
-            const bool ok = j < s.taps && j <= pos;
-            x[j] = ok ? input(s, y, ld, behind, at, c, slot, j) : 0.f;
-            w[j] = ok ? wp[-(ptrdiff_t)(j * (size_t)s.channels())] : 0.f;
-        }
-    }
-    __device__ __forceinline__ float value(const DeltaSpec &s, const float *y, size_t ld, uint32_t behind, uint32_t pos, uint32_t slot) const
-    {
-        float v = x[0] * w[0];
-#pragma unroll
-        for (int j = 1; j < 4; j++) v = fmaf(x[j], w[j], v);
-        for (uint32_t j = 4; j < s.taps && j <= pos; j++)
-            v = fmaf(input(s, y, ld, behind, at, c, slot, j), s.conv[(size_t)(s.taps - 1 - j) * s.channels() + c], v);
-        return silu_f(v);
-    }
-};
-__device__ __forceinline__ float delta_conv(const DeltaSpec &s, const float *y, size_t ld, uint32_t behind, uint32_t c, uint32_t pos, uint32_t slot)
-{
-    DeltaConv v;
-    v.fetch(s, y, ld, behind, c, pos, slot);
-    return v.value(s, y, ld, behind, pos, slot);
-}
 
 constexpr int kDeltaStepThreads = 512;
 constexpr int kLowRankRows = kDeltaStepThreads / 8;      // rows of a low-rank matrix a workgroup takes at a time
@@ -155,7 +115,7 @@ __device__ __forceinline__ void delta_step(const DeltaStepArgs &a, uint32_t idx,
 
     // threads 0 .. 255: channel d of q, the others: of k; the first 32 also a column of v
     const uint32_t d = threadIdx.x & 255, half = threadIdx.x >> 8, cq = half * nq + kvh * s.dim + d, cv = 2 * nq + head * s.vdim + c_lo + threadIdx.x;
-    DeltaConv qk_in{}, v_in{};
+    ShortConv qk_in{}, v_in{};
     if (d < s.dim) qk_in.fetch(s, a.y, 0, 0, cq, pos, rslot);
     if (threadIdx.x < nc) v_in.fetch(s, a.y, 0, 0, cv, pos, rslot);
     const float beta_in = a.y[s.b_off + head], a_log = s.a_log[head];

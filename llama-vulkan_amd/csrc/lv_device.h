@@ -115,6 +115,37 @@ __device__ __forceinline__ float block_max_256(float v, float *lds /* >= 4 float
     return fmaxf(fmaxf(lds[0], lds[1]), fmaxf(lds[2], lds[3]));
 }
 
+// ---- sums over a workgroup of nw waves ---------------------------------------------------------------------
+__device__ __forceinline__ float block_sum_waves(float v, float *scratch, int nw)
+{
+    v = wave_sum(v);
+    __syncthreads();
+    if ((threadIdx.x & 63) == 0) scratch[threadIdx.x >> 6] = v;
+    __syncthreads();
+    float t = 0.f;
+    for (int i = 0; i < nw; i++) t += scratch[i];
+    return t;
+}
+
+// the same for N values at once; scratch holds N * nw floats
+template <int N>
+__device__ __forceinline__ void block_sums_waves(float (&v)[N], float *scratch, int nw)
+{
+#pragma unroll
+    for (int i = 0; i < N; i++) v[i] = wave_sum(v[i]);
+    __syncthreads();
+    if ((threadIdx.x & 63) == 0) {
+#pragma unroll
+        for (int i = 0; i < N; i++) scratch[i * nw + (threadIdx.x >> 6)] = v[i];
+    }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < N; i++) {
+        v[i] = 0.f;
+        for (int w = 0; w < nw; w++) v[i] += scratch[i * nw + w];
+    }
+}
+
 // ---- fp16 ------------------------------------------------------------------------------------------------
 __device__ __forceinline__ float half_bits_to_float(uint16_t h)
 {

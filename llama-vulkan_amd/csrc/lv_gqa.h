@@ -12,7 +12,7 @@
 // batch's first position on come from there, older ones from the ring); those of its last chunk are appended afterwards, so
 // that a batch may run over any number of chunk borders.
 //
-// Everything but the MFMA path (attention_tile_kernel: bf16 operands, weights as two bf16 pieces) is fp32 arithmetic on
+// Everything but the MFMA path (gqa_tile_kernel: bf16 operands, weights as two bf16 pieces) is fp32 arithmetic on
 // cache rows of either element type.
 #pragma once
 
@@ -379,7 +379,8 @@ struct GqaBatchArgs {
     GqaSpec s;
     uint32_t pos0, n;            // the batch's first position and its tokens
     const void *q;               // [n][heads][DP], normalised, rotated, scaled
-    const void *k, *v;           // [n][kv head][DP]: the batch's own rows
+    const void *k, *v;           // [positions from own0][kv head][DP]: rows that are not in the ring, the batch's own among them
+    uint32_t own0;
     void *out;                   // [n][ldo] activations, heads * vdim columns
     uint32_t ldo, groups;
     float out_scale;
@@ -417,7 +418,7 @@ __global__ __launch_bounds__(256) void gqa_rows_kernel(GqaBatchArgs a)
         const uint32_t n = min((uint32_t)kGqaSplit, pos + 1 - k_begin);
         auto from = [&](const void *ring, const void *mine, uint32_t j, int d, float (&f)[8]) {
             const uint32_t p = k_begin + j;
-            if (p >= a.pos0) load8(f, static_cast<const CT *>(mine) + ((size_t)(p - a.pos0) * s.kv_heads + kvh) * DP + d);
+            if (p >= a.own0) load8(f, static_cast<const CT *>(mine) + ((size_t)(p - a.own0) * s.kv_heads + kvh) * DP + d);
             else load8(f, static_cast<const CT *>(ring) + ((size_t)(p - c0) * s.kv_heads + kvh) * DP + d);
         };
         for (uint32_t j0 = 0; j0 < n; j0 += L::KPR) {

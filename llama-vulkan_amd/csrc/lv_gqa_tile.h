@@ -22,11 +22,11 @@ struct GqaTileArgs {
 
 constexpr int kTileKeys = 64;
 
-// row of position p: the batch's own or the ring's
+// row of position p: the batch's (from own0 on) or the ring's
 __device__ __forceinline__ const uint16_t *gqa_row(const GqaTileArgs &a, const void *mine, const void *ring, uint32_t p, uint32_t kvh, uint32_t dp)
 {
     const GqaSpec &s = a.b.s;
-    return p >= a.b.pos0 ? static_cast<const uint16_t *>(mine) + ((size_t)(p - a.b.pos0) * s.kv_heads + kvh) * dp
+    return p >= a.b.own0 ? static_cast<const uint16_t *>(mine) + ((size_t)(p - a.b.own0) * s.kv_heads + kvh) * dp
                          : static_cast<const uint16_t *>(ring) + ((size_t)(p - a.base) * s.kv_heads + kvh) * dp;
 }
 
@@ -61,13 +61,13 @@ __global__ __launch_bounds__(256) void gqa_values_kernel(GqaTileArgs a)
     }
 }
 
-template <int DP> constexpr int gqa_tile_lds() { return 2 * 2 * kTileKeys * DP * 2; }
+template <int DK, int DV> constexpr int gqa_tile_lds() { return 2 * kTileKeys * (DK + DV) * 2; }
 
-// QT = tiles of 16 queries per wave; a workgroup takes 64 * QT queries.  grid (heads, query tiles)
-template <int DP, int QT>
+// DK, DV = padded sizes of queries and keys, and of values.  QT = tiles of 16 queries per wave; a workgroup takes 64 * QT queries.  grid (heads, query tiles)
+template <int DK, int DV, int QT>
 __global__ __launch_bounds__(256) void gqa_tile_kernel(GqaTileArgs a)
 {
-    constexpr int KS = DP / 32, DT = DP / 16, ROW = DP * 2, STAGE = 2 * kTileKeys * ROW, CH = DP / 8;
+    constexpr int KS = DK / 32, DT = DV / 16, ROW = DK * 2, STAGE = kTileKeys * (DK + DV) * 2, CH = DK / 8;
     extern __shared__ __attribute__((aligned(128))) uint8_t tile[];
     const GqaSpec &s = a.b.s;
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), l16 = lane & 15, g4 = lane >> 4;
@@ -84,7 +84,7 @@ __global__ __launch_bounds__(256) void gqa_tile_kernel(GqaTileArgs a)
         const uint32_t t = min(t0 + (wave * QT + i) * 16 + l16, a.b.n - 1);
         hi[i] = a.b.pos0 + t;
         lo[i] = chunk_start(hi[i]);
-        const uint16_t *qr = static_cast<const uint16_t *>(a.b.q) + ((size_t)t * s.heads + head) * DP + g4 * 8;
+        const uint16_t *qr = static_cast<const uint16_t *>(a.b.q) + ((size_t)t * s.heads + head) * DK + g4 * 8;
 #pragma unroll
         for (int k = 0; k < KS; k++) q[i][k] = *reinterpret_cast<const lv_bf8 *>(qr + k * 32);
     }
@@ -95,17 +95,17 @@ __global__ __launch_bounds__(256) void gqa_tile_kernel(GqaTileArgs a)
     const uint32_t p_max = a.base + a.keys - 1;
     auto issue = [&](int st, uint32_t k0) {
         uint8_t *kb = tile + st * STAGE, *vb = kb + kTileKeys * ROW;
-        // 64 rows of DP keys elements, then DP rows of 64 values: 1 KB (64 chunks of 16 bytes) per wave and instruction
+        // 64 rows of DK key elements, then DV rows of 64 values: 1 KB (64 chunks of 16 bytes) per wave and instruction
 #pragma unroll
         for (int i = 0; i < kTileKeys * CH / 256; i++) {
             const int c = (i * 4 + wave) * 64 + lane, row = c / CH, ch = c % CH;
-            const uint16_t *src = gqa_row(a, a.b.k, s.kc, min(a.base + k0 + row, p_max), kvh, DP) + (ch ^ (row & 7)) * 8;
+            const uint16_t *src = gqa_row(a, a.b.k, s.kc, min(a.base + k0 + row, p_max), kvh, DK) + (ch ^ (row & 7)) * 8;
             __builtin_amdgcn_global_load_lds((lv_glb_any *)src, (lv_lds_any *)(kb + (i * 4 + wave) * 1024), 16, 0, 0);
         }
 #pragma unroll
-        for (int i = 0; i < DP * 8 / 256; i++) {
+        for (int i = 0; i < DV * 8 / 256; i++) {
             const int c = (i * 4 + wave) * 64 + lane, row = c / 8, ch = c % 8;
-            const uint16_t *src = a.vt + ((size_t)kvh * DP + row) * a.vt_ld + k0 + (ch ^ (row & 7)) * 8;
+            const uint16_t *src = a.vt + ((size_t)kvh * DV + row) * a.vt_ld + k0 + (ch ^ (row & 7)) * 8;
             __builtin_amdgcn_global_load_lds((lv_glb_any *)src, (lv_lds_any *)(vb + (i * 4 + wave) * 1024), 16, 0, 0);
         }
     };

@@ -62,10 +62,10 @@ int block_model_file::upload(lv_ctx *ctx, int compute, lv_model **out) const
 {
     std::vector<lv_tensor_desc> table;
     for (const safetensors_entry &e : weights->entries()) {
-        // a matrix is [rows][cols]; a vector has one column; other ranks and types belong to no tensor the device library reads
+        // a matrix is [rows][cols]; a vector has one column, a scalar one row; other ranks and types belong to no tensor the device library reads
         const u32 type = e.dtype == "BF16" ? u32{LV_BF16} : e.dtype == "F32" ? u32{LV_F32} : ~0u;
-        if (type == ~0u || e.shape.empty() || e.shape.size() > 2 || e.shape[0] > 0xffffffffu || (e.shape.size() == 2 && e.shape[1] > 0xffffffffu)) continue;
-        table.push_back({e.name.c_str(), type, e.offset, static_cast<u32>(e.shape[0]), e.shape.size() == 2 ? static_cast<u32>(e.shape[1]) : 1u, e.size});
+        if (type == ~0u || e.shape.size() > 2 || (e.shape.size() >= 1 && e.shape[0] > 0xffffffffu) || (e.shape.size() == 2 && e.shape[1] > 0xffffffffu)) continue;
+        table.push_back({e.name.c_str(), type, e.offset, e.shape.empty() ? 1u : static_cast<u32>(e.shape[0]), e.shape.size() == 2 ? static_cast<u32>(e.shape[1]) : 1u, e.size});
     }
     return lv_block_model_upload(ctx, weights->data(), weights->data_size(), &description.hparams, description.layers.data(), table.data(),
                                  static_cast<u32>(table.size()), compute, out);

@@ -14,6 +14,8 @@
 struct block_description {
     lv_block_hparams hparams{};
     std::vector<lv_block_spec> layers;
+    // layers as a sequence runs through them
+    [[nodiscard]] u32 passes() const { return hparams.layers + (hparams.loop_times ? (hparams.loop_times - 1) * (hparams.loop_stop - hparams.loop_start) : 0); }
 };
 
 struct block_design {
@@ -30,7 +32,7 @@ public:
     [[nodiscard]] const std::string &error() const override { return problem; }
     void print_info() const override;
     [[nodiscard]] u32 vocab_size() const override { return description.hparams.vocab; }
-    [[nodiscard]] u32 layer_count() const override { return description.hparams.layers; }
+    [[nodiscard]] u32 layer_count() const override { return description.passes(); }
     [[nodiscard]] u32 width() const override { return description.hparams.dim; }
     [[nodiscard]] u32 max_context() const override { return 1u << 20; }
     [[nodiscard]] u32 end_token() const override { return ~0u; }
