@@ -21,6 +21,8 @@ ROOT_DIR = os.path.dirname(PKG_DIR)
 
 LV_F32, LV_F16, LV_Q4_0, LV_Q8_0, LV_BF16 = 0, 1, 2, 8, 30
 ATTN_NORM_FULL, ATTN_KEYS_AS_VALUES, ATTN_SINK = 1, 2, 4
+ACT_SILU, ACT_RELU = 0, 1
+NORM_RMS, NORM_TANH = 0, 1
 PATH_AUTO, PATH_KERNELS, PATH_GRAPH, PATH_PERSISTENT = range(4)
 TRACE_NORM_IN, TRACE_POST_ATTN, TRACE_POST_ATTN_NORM, TRACE_FF, TRACE_OUT, TRACE_ATTN = range(6)
 

@@ -136,12 +136,12 @@ def specs(cfg, W):
     return out
 
 
-def upload(ctx, cfg, W, compute):
+def upload(ctx, cfg, W, compute, blocks=None, **model_wide):
     """BlockModel straight through the C-ABI"""
     lva = importlib.import_module("llama-vulkan_amd")
     base = np.concatenate([v.reshape(-1) for v in W.values()]).view(np.uint8)
     table, off = [], 0
     for k, v in W.items():
-        table.append((k, lva.LV_BF16, off, v.shape[0], v.shape[1] if v.ndim == 2 else 1, v.nbytes))
+        table.append((k, lva.LV_BF16, off, v.shape[0] if v.ndim else 1, v.shape[1] if v.ndim == 2 else 1, v.nbytes))
         off += v.nbytes
-    return lva.BlockModel(ctx, base, table, specs(cfg, W), cfg["vocab"], cfg["width"], cfg["norm"]["eps"], compute)
+    return lva.BlockModel(ctx, base, table, blocks or specs(cfg, W), cfg["vocab"], cfg["width"], cfg["norm"]["eps"], compute, **model_wide)

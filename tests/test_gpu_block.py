@@ -12,8 +12,10 @@ import numpy as np
 import pytest
 
 import block_builder as bb
+import block_device
 import block_oracle as bo
 import server_client as sc
+from block_device import rel, tokens_for
 
 pytestmark = pytest.mark.gpu
 F32, BF16 = 0, 30
@@ -25,47 +27,8 @@ def hostlib():
     return importlib.import_module("llama-vulkan_amd.hostlib")
 
 
-class Device:
-    """a model and one session of it"""
-
-    def __init__(self, lva, ctx, cfg, W, compute, backlog=512):
-        self.model = bb.upload(ctx, cfg, W, compute)
-        self.sess = lva.Session(self.model, backlog)
-        self.sess.keep_all_logits(True)
-
-    def close(self):
-        self.sess.close()
-        self.model.close()
-
-    def __enter__(self):
-        return self
-
-    def __exit__(self, *a):
-        self.close()
-
-    def step(self, tokens, pos):
-        self.sess.begin(tokens, pos)
-        return self.sess.logits_rows(0, len(tokens))
-
-    def run(self, tokens, cuts):
-        """tokens in portions of the given sizes (the last size repeats)"""
-        out, pos, i = [], 0, 0
-        while pos < len(tokens):
-            n = min(cuts[min(i, len(cuts) - 1)], len(tokens) - pos)
-            out.append(self.step(tokens[pos:pos + n], pos))
-            pos += n
-            i += 1
-        return np.concatenate(out)
-
-
-def rel(got, want):
-    """root mean square of the difference, row by row, against the rows' own"""
-    d = np.sqrt(np.mean((got - want) ** 2, axis=-1))
-    return float(np.max(d / np.sqrt(np.mean(np.asarray(want) ** 2))))
-
-
-def tokens_for(cfg, n, seed):
-    return np.random.default_rng(seed).integers(0, cfg["vocab"], n).astype(np.uint32)
+def Device(lva, ctx, cfg, W, compute, backlog=512):
+    return block_device.Device(lva, bb.upload(ctx, cfg, W, compute), backlog)
 
 
 def check_model(lva, ctx, cfg, W, n, compute=F32, cuts=((1000,), (1,)), seed=0, tol=None):

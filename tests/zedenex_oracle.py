@@ -4,7 +4,7 @@ simple; shares nothing with the product.
 Weights come as a dict name -> float array (scalars 0-D, vectors 1-D, matrices [out, in]); `cfg` is the configuration."""
 import numpy as np
 
-from block_oracle import rms_norm, rotate, silu, sink_softmax, softplus
+from block_oracle import attention, delta_rule, mixture, rms_norm, rotate, silu, sink_softmax, softplus
 
 
 def dynamic_tanh(x, alpha, w, b):
@@ -57,7 +57,7 @@ def latent_attention(h, W, p, c, eps, mask=None, with_sink=True):
     out = np.zeros((n, H, vd))
     for head in range(H):
         s = (q[:, head, :d] @ k[:, head].T + q_rot[:, head] @ kr_rot.T) * c["scale"]
-        out[:, head] = sink_softmax(s, m, W[p + "sink"][head] if with_sink else None) @ v[:, head]
+        out[:, head] = sink_softmax(s, m, W[p + "sink"][head] if with_sink and p + "sink" in W else None) @ v[:, head]
     return out.reshape(n, H * vd) @ W[p + "o"].T
 
 
@@ -98,32 +98,50 @@ def mamba2(h, W, p, c, eps):
     return grouped_rms_norm(y.reshape(n, inner) * silu(z), c["norm_groups"], W[p + "norm"], eps) @ W[p + "o"].T
 
 
-def dense(h, W, p):
-    return (np.maximum(h @ W[p + "gate"].T, 0.0) * (h @ W[p + "up"].T)) @ W[p + "down"].T
+def dense(h, W, p, act="relu"):
+    g = h @ W[p + "gate"].T
+    return ((np.maximum(g, 0.0) if act == "relu" else silu(g)) * (h @ W[p + "up"].T)) @ W[p + "down"].T
+
+
+def sublayers(layer, p, W, eps, **attention_options):
+    """what a layer does, one function per sublayer: the mixer, and the feed-forward if it has one"""
+    m = layer["mixer"]
+    if layer["type"] == "latent_attention":
+        yield lambda h: latent_attention(h, W, p + "mix.", m, eps, **attention_options)
+    elif layer["type"] == "mamba2":
+        yield lambda h: mamba2(h, W, p + "mix.", m, eps)
+    else:
+        yield lambda h: m["left_scale"] * attention(h, W, p + "mix.left.", m["left"], eps) + m["right_scale"] * delta_rule(h, W, p + "mix.right.", m["right"], eps)
+    mlp = layer["mlp"]
+    if mlp and mlp["kind"] == "moe":
+        yield lambda h: mixture(h, W, p + "mlp.", mlp["router"]["top"])
+    elif mlp:
+        yield lambda h: dense(h, W, p + "mlp.", mlp.get("act", "relu"))
+
+
+def norm(x, W, name, eps):
+    """by what the weights hold: a tanh norm or an RMS norm"""
+    return dynamic_tanh(x, W[name + ".alpha"], W[name], W[name + ".b"]) if name + ".alpha" in W else rms_norm(x, W[name], eps)
 
 
 def forward(tokens, W, cfg, **attention_options):
-    """logits [n, vocab]; the sum of the streams behind every mixer and behind every layer, pass by pass"""
+    """logits [n, vocab]; the sum of the streams behind every mixer and behind every layer, pass by pass.  Without streams: one
+    residual, and a norm on each sublayer's output."""
     eps = cfg["norm"]["eps"]
-    x = np.stack([embedding(tokens, W, cfg["embedding"])] * cfg["streams"])
-    behind_mixer, behind_layer = [], []
-
-    def sublayer(x, p, q, f):
-        hc, n = f"{p}hc{q}.", f"{p}norm{q}"
-        h = dynamic_tanh(gather_streams(x, W[hc + "in"]), W[n + ".alpha"], W[n], W[n + ".b"])
-        return spread_streams(x, W[hc + "mix"], W[hc + "out"], f(h))
+    x = np.stack([embedding(tokens, W, cfg["embedding"])] * max(1, cfg["streams"]))
+    behind = [[], []]
     for i in run_order(cfg):
-        layer, p = cfg["layers"][i], f"l{i}."
-        if layer["type"] == "latent_attention":
-            x = sublayer(x, p, 1, lambda h: latent_attention(h, W, p + "mix.", layer["mixer"], eps, **attention_options))
-        else:
-            x = sublayer(x, p, 1, lambda h: mamba2(h, W, p + "mix.", layer["mixer"], eps))
-        behind_mixer.append(x.sum(0))
-        if layer["mlp"]:
-            x = sublayer(x, p, 2, lambda h: dense(h, W, p + "mlp."))
-        behind_layer.append(x.sum(0))
-    h = dynamic_tanh(x.sum(0), W["final.norm.alpha"], W["final.norm"], W["final.norm.b"])
-    return h @ W["embed"].T, behind_mixer, behind_layer
+        p = f"l{i}."
+        for q, f in enumerate(sublayers(cfg["layers"][i], p, W, eps, **attention_options), 1):
+            hc, n = f"{p}hc{q}.", f"{p}norm{q}"
+            if cfg["streams"]:
+                x = spread_streams(x, W[hc + "mix"], W[hc + "out"], f(norm(gather_streams(x, W[hc + "in"]), W, n, eps)))
+            else:
+                x = x + rms_norm(f(norm(x[0], W, n, eps)), W[n + "b"], eps)
+            if q == 1:
+                behind[0].append(x.sum(0))
+        behind[1].append(x.sum(0))
+    return norm(x.sum(0), W, "final.norm", eps) @ W["head" if "head" in W else "embed"].T, *behind
 
 
 def greedy(tokens, count, W, cfg):
