@@ -167,14 +167,16 @@ def main():
     ap.add_argument("--warmup", type=int, default=8)
     ap.add_argument("--cpu-steps", type=int, default=64, help="decode steps the CPU checker is timed on, the last ones of the timed region (0 = skip)")
     ap.add_argument("--no-cases", action="store_true", help="skip the other configurations (the \"cases\" key)")
-    ap.add_argument("--block", action="store_true", help="instead of the default workload: prefill and decode of Somesun-shaped block models beside LLaMA layers of the same width")
+    ap.add_argument("--block", nargs="?", const="Somesun", choices=["Somesun", "Zedenex"],
+                    help="instead of the default workload: prefill and decode of block models of real layer sizes, Somesun beside LLaMA layers of the same width or Zedenex beside Somesun")
     args = ap.parse_args()
     if args.block:
         lva = importlib.import_module("llama-vulkan_amd")
         measure = importlib.import_module("llama-vulkan_amd.measure")
         ctx = lva.Context(0)
+        cases = measure.zedenex_cases if args.block == "Zedenex" else measure.block_cases
         print(json.dumps({"metric": "block models: prefill and decode tok/s", "dtype": "bf16", "data": "synthetic", "device": ctx.info()[0],
-                          "cases": measure.block_cases(ctx, report=measure.quiet)}), flush=True)
+                          "cases": cases(ctx, report=measure.quiet)}), flush=True)
         ctx.close()
         return
     if args.gpus != 1:

@@ -145,20 +145,29 @@ __device__ __forceinline__ void branch_input(const BranchInput &a, float *xs, ui
     }
 }
 
-// GroupInput: put(i, value).  Waves share a group where there are fewer groups than waves; `sums` holds group_sums() floats and
-// every thread keeps to its own elements between the passes.
+// GroupInput: put(i, value) for one element or, where parts are multiples of four, a float4 of them; get(i, value) the other way.
+// Waves share a group where there are fewer groups than waves; `sums` holds group_sums() floats and every thread keeps to its own
+// elements between the passes.
 __host__ __device__ constexpr uint32_t group_parts(uint32_t groups, uint32_t waves) { return groups >= waves ? 1 : waves / groups; }
 __host__ __device__ constexpr uint32_t group_sums(uint32_t groups, uint32_t waves) { return groups * group_parts(groups, waves); }
-template <class Put, class Get>
-__device__ __forceinline__ void group_input(const GroupInput &a, float *sums, Put put, Get get)
+template <class V, class Put, class Get>
+__device__ __forceinline__ void group_passes(const GroupInput &a, float *sums, Put put, Get get)
 {
+    constexpr uint32_t N = sizeof(V) / 4;
     const uint32_t lane = threadIdx.x & 63, waves = blockDim.x >> 6, parts = group_parts(a.groups, waves), tasks = a.groups * parts, size = a.n / a.groups;
     for (uint32_t k = threadIdx.x >> 6; k < tasks; k += waves) {
         const uint32_t base = k / parts * size;
         float s = 0.f;
-        for (uint32_t c = k % parts * 64 + lane; c < size; c += parts * 64) {
-            const float v = a.o[base + c] * silu_f(a.z[base + c]);
-            s = fmaf(v, v, s);
+        for (uint32_t c = (k % parts * 64 + lane) * N; c < size; c += parts * 64 * N) {
+            V v = *reinterpret_cast<const V *>(a.o + base + c);
+            const V z = *reinterpret_cast<const V *>(a.z + base + c);
+            float *f = reinterpret_cast<float *>(&v);
+            const float *g = reinterpret_cast<const float *>(&z);
+#pragma unroll
+            for (uint32_t e = 0; e < N; e++) {
+                f[e] *= silu_f(g[e]);
+                s = fmaf(f[e], f[e], s);
+            }
             put(base + c, v);
         }
         s = wave_sum(s);
@@ -170,8 +179,23 @@ __device__ __forceinline__ void group_input(const GroupInput &a, float *sums, Pu
         float s = 0.f;
         for (uint32_t p = 0; p < parts; p++) s += sums[g * parts + p];
         const float inv = rsqrtf(s / (float)size + a.eps);
-        for (uint32_t c = k % parts * 64 + lane; c < size; c += parts * 64) put(base + c, get(base + c) * inv * a.w[base + c]);
+        for (uint32_t c = (k % parts * 64 + lane) * N; c < size; c += parts * 64 * N) {
+            V v;
+            get(base + c, v);
+            const V w = *reinterpret_cast<const V *>(a.w + base + c);
+            float *f = reinterpret_cast<float *>(&v);
+            const float *h = reinterpret_cast<const float *>(&w);
+#pragma unroll
+            for (uint32_t e = 0; e < N; e++) f[e] *= inv * h[e];
+            put(base + c, v);
+        }
     }
+}
+template <class Put, class Get>
+__device__ __forceinline__ void group_input(const GroupInput &a, float *sums, Put put, Get get)
+{
+    if (a.n / a.groups % 4 == 0) group_passes<float4>(a, sums, put, get);
+    else group_passes<float>(a, sums, put, get);
 }
 
 // The `top` largest of n router logits, largest first, the lower index on equal values (one wave; zs is consumed).  Scores are
@@ -277,7 +301,8 @@ __global__ __launch_bounds__(kBfGemvThreads) void bf16_gemv_kernel(BfGemvArgs a)
         branch_input(a.branch, xs, kp);
     } else if constexpr (INPUT == kInGroups) {
         for (uint32_t i = a.group.n + threadIdx.x; i < kp; i += kBfGemvThreads) xs[bf_xs(i, kp)] = 0.f;
-        group_input(a.group, xs + kp, [&](uint32_t i, float v) { xs[bf_xs(i, kp)] = v; }, [&](uint32_t i) { return xs[bf_xs(i, kp)]; });
+        group_input(a.group, xs + kp, [&](uint32_t i, auto v) { *reinterpret_cast<decltype(v) *>(xs + bf_xs(i, kp)) = v; },
+                    [&](uint32_t i, auto &v) { v = *reinterpret_cast<std::decay_t<decltype(v)> *>(xs + bf_xs(i, kp)); });
     } else if constexpr (INPUT >= kInStreams2) {
         stream_input<2 << (INPUT - kInStreams2)>(a.streams, blockIdx.x == 0, scratch, [&](uint32_t i, const float4 h) { *reinterpret_cast<float4 *>(xs + bf_xs(i, kp)) = h; },
                                                  [&](uint32_t i) { return *reinterpret_cast<const float4 *>(xs + bf_xs(i, kp)); });

@@ -51,6 +51,7 @@ struct BlockLayer {
     NormSite site[2];                  // mixer, feed-forward
     const float *q_norm = nullptr, *k_norm = nullptr, *sink = nullptr;
     const double *freq = nullptr;
+    uint32_t freq_at = 0;              // latent attention: where its frequencies start in the model's
     const float *conv = nullptr, *conv_bias = nullptr, *a_log = nullptr, *dt_bias = nullptr, *skip = nullptr, *onorm = nullptr;
     const uint16_t *uk_t = nullptr;    // W_uk transposed head by head
     bool ff() const { return moe || dense; }
@@ -79,6 +80,8 @@ struct BlockModel {
     BfMatrix head;
     std::vector<BlockLayer> layers;
     std::vector<uint32_t> order;       // layer of every pass
+    const double *freq = nullptr;      // frequencies of all layers of latent attention, layer after layer
+    uint32_t n_freq = 0;
     uint32_t elem() const { return f32 ? 4 : 2; }
     const BlockLayer &pass(size_t i) const { return layers[order[i]]; }
 };
@@ -93,9 +96,9 @@ struct LayerState {
 struct Workspace {                     // of batches; sized for `cap` tokens
     uint32_t cap = 0;
     float *x = nullptr, *y1 = nullptr, *y = nullptr, *dq = nullptr, *dk = nullptr, *dv = nullptr, *dg = nullptr, *beta = nullptr, *qk = nullptr, *o = nullptr,
-          *gate = nullptr, *z = nullptr, *scores = nullptr, *y2 = nullptr, *sx = nullptr, *sb = nullptr, *sc = nullptr, *sdt = nullptr, *sdecay = nullptr;
+          *gate = nullptr, *z = nullptr, *scores = nullptr, *y2 = nullptr, *sdt = nullptr, *sdecay = nullptr;
     void *act = nullptr, *q = nullptr, *k = nullptr, *v = nullptr, *vt = nullptr, *a1 = nullptr, *g1 = nullptr, *cat = nullptr, *ff = nullptr, *cq = nullptr,
-         *ek = nullptr, *ev = nullptr;
+         *ek = nullptr, *ev = nullptr, *sx = nullptr, *sb = nullptr, *sc = nullptr, *sbt = nullptr;
     uint32_t *ids = nullptr, *slots = nullptr, *tiles = nullptr;
     uint64_t vt_elems = 0, ek_elems = 0, ev_elems = 0;
 };
@@ -108,7 +111,9 @@ struct BlockSession {
     std::vector<LayerState> layers;
     // one token
     float *xa = nullptr, *xb = nullptr, *y1 = nullptr, *left = nullptr, *o = nullptr, *gate = nullptr, *yo = nullptr, *h2 = nullptr, *z = nullptr, *act = nullptr,
-          *yd = nullptr, *scores = nullptr, *part = nullptr, *y2 = nullptr, *ql = nullptr;
+          *yd = nullptr, *scores = nullptr, *part = nullptr, *y2 = nullptr;
+    void *ql = nullptr;                // latent attention: queries (latent_put)
+    float2 *turn = nullptr;            // the model's frequencies as (cos, sin) at the token's position
     uint32_t *ids = nullptr, *counters = nullptr, *last = nullptr;      // last: the sequence's last token, at [position % 2]
     Workspace ws;
 };
@@ -214,6 +219,9 @@ private:
     uint64_t size_;
     std::unordered_map<std::string, const lv_tensor_desc *> by_name_;
 };
+
+// of pair k, in full turns per position
+double frequency(double base, uint32_t dims, uint32_t k) { return std::pow(base, -2.0 * k / dims) / 6.283185307179586476925; }
 
 uint32_t latent_kc(const lv_latent_spec &l) { return up(l.kv_rank, 16); }
 uint32_t latent_width(const lv_latent_spec &l) { return up(latent_kc(l) + l.rot_dim, 64); }
@@ -353,6 +361,7 @@ int block_model_create(hipStream_t st, const void *base, uint64_t base_size, con
     site(&m->final, "final.norm", "");
     if (!hp->tied_head)
         if (const lv_tensor_desc *d = tensor("head", V, D)) matrix(&m->head, {{d, 0, 0}}, V, Dp);
+    std::vector<double> freqs;
     for (uint32_t i = 0; i < hp->layers && ld.error == LV_OK; i++) {
         BlockLayer &l = m->layers[i];
         l.spec = blocks[i];
@@ -373,15 +382,6 @@ int block_model_create(hipStream_t st, const void *base, uint64_t base_size, con
         if (l.ff()) site(&l.site[1], p + "norm2", p + "hc2.");
         std::vector<Part> in, outp;
         uint32_t row = 0;
-        auto frequencies = [&](uint32_t dims, double rb) {
-            if (!dims) return;
-            at(&l.freq, ld.place((uint64_t)dims / 2 * 8, [=](uint8_t *dst) {
-                for (uint32_t k = 0; k < dims / 2; k++) {
-                    const double f = std::pow(rb, -2.0 * k / dims) / 6.283185307179586476925;      // in full turns
-                    std::memcpy(dst + 8 * (size_t)k, &f, 8);
-                }
-            }));
-        };
         // convolution weights, [channel][tap] in the file, as [tap][channel]
         auto convolution = [&](std::vector<const lv_tensor_desc *> parts, uint32_t taps) {
             struct Src { const uint8_t *data; uint32_t rows, type; };
@@ -421,7 +421,16 @@ int block_model_create(hipStream_t st, const void *base, uint64_t base_size, con
                 vec(&l.k_norm, pa + "k.norm", a.kv_heads * a.dim, 1, a.kv_heads * a.dim);
             }
             if (a.flags & LV_ATTN_SINK) vec(&l.sink, pa + "sink", a.heads, 1, a.heads);
-            frequencies(a.rot_dims, a.rot_base);
+            if (a.rot_dims) {
+                const uint32_t dims = a.rot_dims;
+                const double rb = a.rot_base;
+                at(&l.freq, ld.place((uint64_t)dims / 2 * 8, [=](uint8_t *dst) {
+                    for (uint32_t k = 0; k < dims / 2; k++) {
+                        const double f = frequency(rb, dims, k);
+                        std::memcpy(dst + 8 * (size_t)k, &f, 8);
+                    }
+                }));
+            }
             l.left_kp = up(a.heads * a.vdim, 64);
             if (const lv_tensor_desc *d = tensor(pa + "o", D, a.heads * a.vdim)) outp.push_back({d, 0, 0});
             l.dp = 64;
@@ -456,7 +465,8 @@ int block_model_create(hipStream_t st, const void *base, uint64_t base_size, con
             vec(&l.q_norm, px + "dq.norm", lt.q_rank, 1, up(lt.q_rank, 64));
             vec(&l.k_norm, px + "dkv.norm", lt.kv_rank, 1, kv_p);
             if (lt.flags & LV_ATTN_SINK) vec(&l.sink, px + "sink", lt.heads, 1, lt.heads);
-            frequencies(lt.rot_dims, lt.rot_base);
+            l.freq_at = (uint32_t)freqs.size();
+            for (uint32_t k = 0; k < lt.rot_dims / 2; k++) freqs.push_back(frequency(lt.rot_base, lt.rot_dims, k));
             if (const lv_tensor_desc *d = tensor(px + "uq", lt.heads * size, lt.q_rank)) matrix(&l.uq, {{d, 0, 0}}, d->rows, up(lt.q_rank, 64));
             if (const lv_tensor_desc *d = tensor(px + "uk", lt.heads * lt.dim, lt.kv_rank)) {
                 matrix(&l.uk, {{d, 0, 0}}, d->rows, kv_p);
@@ -547,6 +557,8 @@ int block_model_create(hipStream_t st, const void *base, uint64_t base_size, con
         delete m;
         return ld.error;
     }
+    m->n_freq = (uint32_t)freqs.size();
+    at(&m->freq, ld.place(freqs.size() * 8 + 8, [freqs](uint8_t *dst) { std::memcpy(dst, freqs.data(), freqs.size() * 8); }));
     // a GEMM tile of 256 rows may read up to 128 rows behind a matrix: of the next one, or of this margin
     uint32_t widest = Dp;
     for (const BlockLayer &l : m->layers) widest = std::max(widest, std::max({l.out.kp, l.down.kp, l.a2.kp, l.g2.kp, l.uq.kp, l.uk.kp}));
@@ -632,13 +644,14 @@ int block_session_create(const BlockModel *m, hipStream_t st, BlockSession **out
         LV_TRY(dev_zeroed(st, &s->xa, m->copies * Dp * 4ull));
         LV_TRY(dev_zeroed(st, &s->xb, m->copies * Dp * 4ull));
         LV_TRY(dev_zeroed(st, &s->last, 8));
+        LV_TRY(dev_zeroed(st, &s->turn, 8ull * m->n_freq));
         LV_TRY(dev_zeroed(st, &s->yo, Dp * 4ull));
         LV_TRY(dev_zeroed(st, &s->yd, Dp * 4ull));
         LV_TRY(dev_zeroed(st, &s->h2, Dp * 4ull));
         LV_TRY(dev_zeroed(st, &s->y1, 4ull * layer_max(m, [](const BlockLayer &l) { return l.in.rows; })));
         LV_TRY(dev_zeroed(st, &s->left, 4ull * layer_max(m, [](const BlockLayer &l) { return l.left_kp; })));
         LV_TRY(dev_zeroed(st, &s->y2, 4ull * layer_max(m, [](const BlockLayer &l) { return l.uq.rows; })));
-        LV_TRY(dev_zeroed(st, &s->ql, 4ull * layer_max(m, [](const BlockLayer &l) { return l.spec.latent.heads * l.width; })));
+        LV_TRY(dev_zeroed(st, &s->ql, (m->f32 ? 4ull : 6ull) * layer_max(m, [](const BlockLayer &l) { return l.spec.latent.heads * l.width; })));
         const uint64_t hv = 4ull * layer_max(m, [](const BlockLayer &l) { return std::max(l.spec.delta.heads * l.spec.delta.vdim, l.ssm_inner()); });
         LV_TRY(dev_zeroed(st, &s->o, hv));
         LV_TRY(dev_zeroed(st, &s->gate, hv));
@@ -667,8 +680,8 @@ int block_session_create(const BlockModel *m, hipStream_t st, BlockSession **out
 
 static void workspace_free(Workspace &w)
 {
-    for (float **p : {&w.x, &w.y1, &w.y, &w.dq, &w.dk, &w.dv, &w.dg, &w.beta, &w.qk, &w.o, &w.gate, &w.z, &w.scores, &w.y2, &w.sx, &w.sb, &w.sc, &w.sdt, &w.sdecay}) drop(*p);
-    for (void **p : {&w.act, &w.q, &w.k, &w.v, &w.vt, &w.a1, &w.g1, &w.cat, &w.ff, &w.cq, &w.ek, &w.ev}) drop(*p);
+    for (float **p : {&w.x, &w.y1, &w.y, &w.dq, &w.dk, &w.dv, &w.dg, &w.beta, &w.qk, &w.o, &w.gate, &w.z, &w.scores, &w.y2, &w.sdt, &w.sdecay}) drop(*p);
+    for (void **p : {&w.act, &w.q, &w.k, &w.v, &w.vt, &w.a1, &w.g1, &w.cat, &w.ff, &w.cq, &w.ek, &w.ev, &w.sx, &w.sb, &w.sc, &w.sbt}) drop(*p);
     for (uint32_t **p : {&w.ids, &w.slots, &w.tiles}) drop(*p);
     w.cap = 0;
     w.vt_elems = w.ek_elems = w.ev_elems = 0;
@@ -683,9 +696,11 @@ void block_session_destroy(BlockSession *s)
         drop(l.state);
         drop(l.conv);
     }
-    for (float **p : {&s->xa, &s->xb, &s->y1, &s->left, &s->o, &s->gate, &s->yo, &s->h2, &s->z, &s->act, &s->yd, &s->scores, &s->part, &s->y2, &s->ql}) drop(*p);
+    for (float **p : {&s->xa, &s->xb, &s->y1, &s->left, &s->o, &s->gate, &s->yo, &s->h2, &s->z, &s->act, &s->yd, &s->scores, &s->part, &s->y2}) drop(*p);
+    drop(s->ql);
     drop(s->ids);
     drop(s->last);
+    drop(s->turn);
     drop(s->counters);
     workspace_free(s->ws);
     delete s;
@@ -767,21 +782,29 @@ template <int MODE, int INPUT, int R, int DEPTH> static int launch_gemv(hipStrea
     return LV_OK;
 }
 
-// rows a wave walks together: as many as still give every wave of the chip work
+// Rows a wave walks together: as many as still give every wave of the chip work, fewer where the last round of waves would then be
+// far from full.
+static uint32_t gemv_rows_together(uint32_t units, uint32_t most)
+{
+    constexpr uint32_t kWaves = 512 * kBfGemvWaves;
+    auto rows_in_turn = [&](uint32_t r) { return ((units + r - 1) / r + kWaves - 1) / kWaves * r; };      // of the busiest wave
+    uint32_t best = most;
+    for (uint32_t r = most / 2; r; r /= 2)
+        if (rows_in_turn(r) < rows_in_turn(best)) best = r;
+    return best;
+}
+
 template <int MODE, int INPUT> static int gemv(hipStream_t st, const BfGemvArgs &a)
 {
     const size_t lds = (size_t)a.kp * (MODE == kGemvDown ? a.top : 1) * 4 + (MODE == kGemvExperts ? a.experts * 4ull : 0) +
                        (INPUT == kInGroups ? group_sums(a.group.groups, kBfGemvWaves) * 4ull : 0);
-    if constexpr (MODE == kGemvExperts) {
-        const uint32_t units = a.top * (a.expert_rows / 2);
-        return units >= 8192 ? launch_gemv<MODE, INPUT, 2, 2>(st, a, units, lds) : launch_gemv<MODE, INPUT, 1, 4>(st, a, units, lds);
-    } else if constexpr (MODE == kGemvGlu) {
-        const uint32_t units = a.rows / 2;
-        return units >= 8192 ? launch_gemv<MODE, INPUT, 2, 2>(st, a, units, lds) : launch_gemv<MODE, INPUT, 1, 4>(st, a, units, lds);
+    if constexpr (MODE == kGemvExperts || MODE == kGemvGlu) {
+        const uint32_t units = MODE == kGemvExperts ? a.top * (a.expert_rows / 2) : a.rows / 2, r = gemv_rows_together(units, units >= 8192 ? 2 : 1);
+        return r == 2 ? launch_gemv<MODE, INPUT, 2, 2>(st, a, units, lds) : launch_gemv<MODE, INPUT, 1, 4>(st, a, units, lds);
     } else {
-        if (a.rows >= 16384) return launch_gemv<MODE, INPUT, 4, 2>(st, a, a.rows, lds);
-        if (a.rows >= 8192) return launch_gemv<MODE, INPUT, 2, 4>(st, a, a.rows, lds);
-        return launch_gemv<MODE, INPUT, 1, 8>(st, a, a.rows, lds);
+        const uint32_t r = gemv_rows_together(a.rows, a.rows >= 16384 ? 4 : a.rows >= 8192 ? 2 : 1);
+        return r == 4 ? launch_gemv<MODE, INPUT, 4, 2>(st, a, a.rows, lds) : r == 2 ? launch_gemv<MODE, INPUT, 2, 4>(st, a, a.rows, lds)
+                                                                                    : launch_gemv<MODE, INPUT, 1, 8>(st, a, a.rows, lds);
     }
 }
 
@@ -883,7 +906,7 @@ static LatentSpec latent_spec(const BlockSession *s, size_t i)
     LatentSpec g{};
     g.heads = a.heads; g.dim = a.dim; g.rot_dim = a.rot_dim; g.rot_dims = a.rot_dims; g.vdim = a.vdim; g.q_rank = a.q_rank; g.kv_rank = a.kv_rank;
     g.q_off = l.q_off; g.kv_off = l.k_off; g.kc = l.kc; g.width = l.width; g.dim_p = up(a.dim, 64); g.kv_p = l.uv.kp;
-    g.q_norm = l.q_norm; g.kv_norm = l.k_norm; g.sink = l.sink; g.freq = l.freq;
+    g.q_norm = l.q_norm; g.kv_norm = l.k_norm; g.sink = l.sink; g.freq = s->m->freq + l.freq_at; g.turn = s->turn + l.freq_at;
     g.uk_t = l.uk_t; g.uv = l.uv.w; g.scale = a.scale; g.eps = s->m->hp.eps; g.cache = s->layers[i].kc;
     return g;
 }
@@ -972,7 +995,12 @@ static int embed(BlockSession *s, float *x, const uint32_t *cfg, uint32_t idx, u
     EmbedArgs e{};
     e.x = x; e.table = m->embed; e.ld = m->embed_ld; e.dim = m->hp.dim; e.dp = m->dp; e.streams = m->copies; e.scale = m->hp.embed_scale ? m->hp.embed_scale : 1.f;
     e.cfg = cfg; e.idx = idx; e.bigram = m->bigram; e.buckets = m->hp.bigram_buckets; e.prev = m->hp.bigram_prev; e.cur = m->hp.bigram_cur; e.last = s->last;
-    embed_bf16_kernel<<<dim3((m->dp + 255) / 256, n), dim3(256), 0, s->st>>>(e);
+    if (n == 1) {
+        e.freq = m->freq;
+        e.turn = s->turn;
+        e.n_freq = m->n_freq;
+    }
+    embed_bf16_kernel<<<dim3((std::max(m->dp / 4, e.n_freq) + 255) / 256, n), dim3(256), 0, s->st>>>(e);
     HIP_TRY(hipGetLastError());
     return LV_OK;
 }
@@ -1056,11 +1084,20 @@ template <class CT> static int token_latent(BlockSession *s, size_t i, const uin
     HIP_TRY(hipGetLastError());
     LatentStepArgs a{};
     a.s = sp; a.q = s->ql; a.pos_ptr = cfg; a.pos_add = idx; a.splits = latent_splits(sp.heads, s->positions); a.part = s->part; a.out = s->left;
-    auto *k = &latent_attn_kernel<CT>;
-    const size_t lds = latent_attn_lds<CT>(sp.width);
-    LV_TRY(allow_lds(k, lds));
-    k<<<dim3(latent_groups(sp.heads), a.splits), dim3(kLatentStepThreads), lds, s->st>>>(a);
-    HIP_TRY(hipGetLastError());
+    auto attend = [&](auto nq, auto nb) -> int {
+        auto *k = &latent_attn_kernel<CT, decltype(nq)::value, decltype(nb)::value>;
+        const size_t lds = latent_attn_lds<CT>(sp.width);
+        LV_TRY(allow_lds(k, lds));
+        k<<<dim3(latent_groups(sp.heads), a.splits), dim3(kLatentStepThreads), lds, s->st>>>(a);
+        HIP_TRY(hipGetLastError());
+        return LV_OK;
+    };
+    static_assert(kLatentMaxWidth <= 6 * 128, "pieces of a cache row");
+    using std::integral_constant;
+    using One = integral_constant<int, 1>;
+    LV_TRY(sp.width <= 256                   ? attend(integral_constant<int, 2>{}, One{})
+           : sp.width <= 640 && sp.kc <= 512 ? attend(integral_constant<int, 5>{}, One{})
+                                             : attend(integral_constant<int, 6>{}, integral_constant<int, 2>{}));
     latent_value_kernel<<<dim3(sp.heads, (sp.vdim + kLatentValueRows - 1) / kLatentValueRows), dim3(kLatentStepThreads), 0, s->st>>>(a);
     HIP_TRY(hipGetLastError());
     o.x = s->left;
@@ -1185,12 +1222,13 @@ static int workspace_reserve(BlockSession *s, uint32_t n)
     LV_TRY(dev_zeroed(st, &w.o, T * 4 * std::max<uint64_t>(hv, mx([](const BlockLayer &l) { return l.ssm_inner(); }))));
     LV_TRY(dev_zeroed(st, &w.y2, T * 4 * mx([](const BlockLayer &l) { return l.uq.rows; })));
     LV_TRY(dev_zeroed(st, &w.cq, T * E * mx([](const BlockLayer &l) { return l.uq.kp; })));
-    LV_TRY(dev_zeroed(st, &w.sx, T * 4 * mx([](const BlockLayer &l) { return l.ssm_inner(); })));
+    LV_TRY(dev_zeroed(st, &w.sx, T * E * mx([](const BlockLayer &l) { return l.ssm_inner(); })));
     const uint64_t bc = mx([](const BlockLayer &l) { return l.spec.ssm.groups * l.sstride(); }), sh = mx([](const BlockLayer &l) { return l.spec.ssm.heads; });
-    LV_TRY(dev_zeroed(st, &w.sb, T * 4 * bc));
-    LV_TRY(dev_zeroed(st, &w.sc, T * 4 * bc));
+    LV_TRY(dev_zeroed(st, &w.sb, T * E * bc));
+    LV_TRY(dev_zeroed(st, &w.sc, T * E * bc));
+    LV_TRY(dev_zeroed(st, &w.sbt, m->f32 ? 0 : T * E * bc));
     LV_TRY(dev_zeroed(st, &w.sdt, T * 4 * sh));
-    LV_TRY(dev_zeroed(st, &w.sdecay, T * 4 * sh));
+    LV_TRY(dev_zeroed(st, &w.sdecay, m->f32 ? T * 4 * sh : 0));
     LV_TRY(dev_zeroed(st, &w.gate, T * 4 * hv));
     const uint64_t heads = mx([](const BlockLayer &l) { return l.spec.delta.heads; });
     LV_TRY(dev_zeroed(st, &w.beta, T * 4 * heads));
@@ -1365,23 +1403,39 @@ template <class T> static int batch_ssm(BlockSession *s, size_t i, uint32_t pos,
     const BlockLayer &l = s->m->pass(i);
     Workspace &w = s->ws;
     hipStream_t st = s->st;
+    const SsmSpec sp = ssm_spec(s, i);
     SsmBatchArgs a{};
-    a.s = ssm_spec(s, i); a.y = w.y1; a.ldy = l.in.rows; a.pos0 = pos; a.n = n;
-    a.x = w.sx; a.b = w.sb; a.c = w.sc; a.dt = w.sdt; a.decay = w.sdecay; a.o = w.o;
-    ssm_prepare_kernel<<<dim3(ssm_prepare_columns(a.s), (n + kSsmPrepareTokens - 1) / kSsmPrepareTokens), dim3(256), 0, st>>>(a);
-    HIP_TRY(hipGetLastError());
-    ssm_append_kernel<<<dim3(std::min(n, a.s.taps)), dim3(256), 0, st>>>(a);
-    HIP_TRY(hipGetLastError());
-    LV_TRY(with_j(l.sstride() / 64, [&](auto j) -> int {
-        constexpr int J = decltype(j)::value;
-        const size_t lds = 2 * 4ull * ssm_stage_floats<J>();
-        LV_TRY(allow_lds(&ssm_scan_kernel<J>, lds));
-        ssm_scan_kernel<J><<<dim3(a.s.heads, (a.s.vdim + 15) / 16), dim3(kSsmScanThreads), lds, st>>>(a);
+    a.s = sp; a.y = w.y1; a.ldy = l.in.rows; a.pos0 = pos; a.n = n; a.o = w.o;
+    if constexpr (sizeof(T) == 4) {
+        a.x = static_cast<float *>(w.sx); a.b = static_cast<float *>(w.sb); a.c = static_cast<float *>(w.sc); a.dt = w.sdt; a.decay = w.sdecay;
+        ssm_prepare_kernel<<<dim3(ssm_prepare_columns(sp), (n + kSsmPrepareTokens - 1) / kSsmPrepareTokens), dim3(256), 0, st>>>(a);
         HIP_TRY(hipGetLastError());
-        return LV_OK;
-    }));
-    const GroupInput g = group_in(a.s, w.o, w.y1);
-    const size_t lds = 4ull * (g.n + group_sums(g.groups, 4));
+        LV_TRY(with_j(l.sstride() / 64, [&](auto j) -> int {
+            constexpr int J = decltype(j)::value;
+            const size_t lds = 2 * 4ull * ssm_stage_floats<J>();
+            LV_TRY(allow_lds(&ssm_scan_kernel<J>, lds));
+            ssm_scan_kernel<J><<<dim3(sp.heads, (sp.vdim + 15) / 16), dim3(kSsmScanThreads), lds, st>>>(a);
+            HIP_TRY(hipGetLastError());
+            return LV_OK;
+        }));
+    } else {
+        SsmChunkArgs c{};
+        c.s = sp; c.y = w.y1; c.ldy = l.in.rows; c.pos0 = pos; c.n = n; c.ldt = up(n, kSsmChunk); c.o = w.o; c.dt = w.sdt;
+        c.xt = static_cast<uint16_t *>(w.sx); c.b = static_cast<uint16_t *>(w.sb); c.c = static_cast<uint16_t *>(w.sc); c.bt = static_cast<uint16_t *>(w.sbt);
+        ssm_operands_kernel<<<dim3(ssm_prepare_columns(sp), c.ldt / 8), dim3(256), 0, st>>>(c);
+        HIP_TRY(hipGetLastError());
+        LV_TRY(with_j(l.sstride() / 64, [&](auto j) -> int {
+            constexpr int J = decltype(j)::value;
+            LV_TRY(allow_lds(&ssm_chunk_kernel<J>, ssm_chunk_lds<J>()));
+            ssm_chunk_kernel<J><<<dim3(sp.heads, (sp.vdim + 63) / 64), dim3(kSsmChunkThreads), ssm_chunk_lds<J>(), st>>>(c);
+            HIP_TRY(hipGetLastError());
+            return LV_OK;
+        }));
+    }
+    ssm_append_kernel<<<dim3(std::min(n, sp.taps)), dim3(256), 0, st>>>(a);
+    HIP_TRY(hipGetLastError());
+    const GroupInput g = group_in(sp, w.o, w.y1);
+    const size_t lds = 4ull * (g.n + group_sums(g.groups, 4) + 4);
     LV_TRY(allow_lds(&ssm_gate_kernel<T>, lds));
     ssm_gate_kernel<T><<<dim3(n), dim3(256), lds, st>>>(g, l.in.rows, static_cast<T *>(w.cat), l.out.kp);
     HIP_TRY(hipGetLastError());

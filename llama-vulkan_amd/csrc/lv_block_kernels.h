@@ -20,7 +20,17 @@ struct EmbedArgs {
     const uint16_t *bigram;      // [buckets + 1][dim]; null: none
     uint32_t buckets, prev, cur;
     uint32_t *last;              // a sequence's last token, at [position % 2]
+    const double *freq;          // one token: the model's rotation frequencies, to `turn` as (cos, sin) at its position
+    float2 *turn;
+    uint32_t n_freq;
 };
+__device__ __forceinline__ void quad(float (&f)[4], const uint16_t *p)
+{
+    const uint2 u = *reinterpret_cast<const uint2 *>(p);
+    f[0] = __uint_as_float(u.x << 16); f[1] = __uint_as_float(u.x & 0xffff0000u);
+    f[2] = __uint_as_float(u.y << 16); f[3] = __uint_as_float(u.y & 0xffff0000u);
+}
+// a thread takes four elements
 static __global__ __launch_bounds__(256) void embed_bf16_kernel(EmbedArgs a)
 {
     const uint32_t i = blockIdx.x * 256 + threadIdx.x, z = blockIdx.y, at = a.idx + z, pos = a.cfg[0] + at, token = a.cfg[1 + at];
@@ -32,13 +42,28 @@ static __global__ __launch_bounds__(256) void embed_bf16_kernel(EmbedArgs a)
         // a launch of one token leaves it for the next; one of several is followed by a copy, since its first row may read the slot
         if (gridDim.y == 1 && i == 0) a.last[pos & 1] = token;
     }
-    if (i >= a.dp) return;
-    float v = 0.f;
-    if (i < a.dim) {
-        v = bf16_to_float(a.table[(size_t)token * a.ld + i]) * a.scale;
-        if (row) v += bf16_to_float(row[i]);
+    if (i < a.n_freq) a.turn[i] = rotation(a.freq[i], pos);
+    const uint32_t d = i * 4;
+    if (d >= a.dp) return;
+    const uint16_t *table = a.table + (size_t)token * a.ld;
+    float v[4] = {0.f, 0.f, 0.f, 0.f};
+    if (a.dim % 4 == 0 && a.ld % 4 == 0) {
+        if (d < a.dim) {
+            quad(v, table + d);
+            float w[4] = {0.f, 0.f, 0.f, 0.f};
+            if (row) quad(w, row + d);
+#pragma unroll
+            for (uint32_t e = 0; e < 4; e++) v[e] = row ? v[e] * a.scale + w[e] : v[e] * a.scale;
+        }
+    } else {
+#pragma unroll
+        for (uint32_t e = 0; e < 4; e++)
+            if (d + e < a.dim) {
+                v[e] = bf16_to_float(table[d + e]) * a.scale;
+                if (row) v[e] += bf16_to_float(row[d + e]);
+            }
     }
-    for (uint32_t t = 0; t < a.streams; t++) a.x[((size_t)z * a.streams + t) * a.dp + i] = v;
+    for (uint32_t t = 0; t < a.streams; t++) *reinterpret_cast<float4 *>(a.x + ((size_t)z * a.streams + t) * a.dp + d) = make_float4(v[0], v[1], v[2], v[3]);
 }
 
 // NormInput for a batch: one workgroup per row; x in place, h as activations

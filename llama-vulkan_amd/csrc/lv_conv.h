@@ -54,4 +54,43 @@ __device__ __forceinline__ float short_conv(const Spec &s, const float *y, size_
     return v.value(s, y, ld, behind, pos, slot);
 }
 
+// Eight consecutive tokens t0 .. t0 + 7 (t0 a multiple of 8) of a batch of n, whose first row is y and first position pos0; 0 for
+// tokens past the end.  Up to four taps every input is read once.
+template <class Spec>
+__device__ __forceinline__ void short_conv8(float (&out)[8], const Spec &s, const float *y, size_t ld, uint32_t c, uint32_t pos0, uint32_t t0, uint32_t n)
+{
+    if (s.taps > 4) {
+#pragma unroll 1
+        for (uint32_t i = 0; i < 8; i++) {
+            const uint32_t t = t0 + i;
+            const float v = t < n ? short_conv(s, y + t * ld, ld, t, c, pos0 + t, (pos0 + t) % s.taps) : 0.f;
+#pragma unroll
+            for (uint32_t e = 0; e < 8; e++) out[e] = e == i ? v : out[e];
+        }
+        return;
+    }
+    const uint32_t at = s.channel_at(c);
+    const float b = s.conv_bias(c);
+    float in[11], w[4];      // in[i]: token t0 + i - 3
+#pragma unroll
+    for (uint32_t j = 0; j < 4; j++) w[j] = j < s.taps ? s.conv[(size_t)(s.taps - 1 - j) * s.channels() + c] : 0.f;
+#pragma unroll
+    for (uint32_t i = 0; i < 11; i++) {
+        const uint32_t back = i < 3 ? 3 - i : 0, t = t0 + i - 3;
+        in[i] = 0.f;
+        if (t0 || !back) {
+            if (t < n) in[i] = y[(size_t)t * ld + at];
+        } else if (back < s.taps && back <= pos0) {
+            in[i] = s.ring[(size_t)((pos0 - back) % s.taps) * s.channels() + c];
+        }
+    }
+#pragma unroll
+    for (uint32_t i = 0; i < 8; i++) {
+        float v = fmaf(in[i + 3], w[0], b);
+#pragma unroll
+        for (uint32_t j = 1; j < 4; j++) v = fmaf(in[i + 3 - j], w[j], v);
+        out[i] = t0 + i < n ? silu_f(v) : 0.f;
+    }
+}
+
 }  // namespace lv

@@ -43,6 +43,34 @@ __device__ __forceinline__ float group16_sum(float v)
     v += dpp_mov<0x140>(v);  // row_mirror: lane i <- lane 15-i of its row
     return v;
 }
+// running sum over the wavefront: lane l gets the sum of lanes 0 .. l
+__device__ __forceinline__ float wave_running_sum(float v)
+{
+    v += dpp_mov<0x111>(v);      // row_shr 1, 2, 4, 8: 0 comes in at a row's start
+    v += dpp_mov<0x112>(v);
+    v += dpp_mov<0x114>(v);
+    v += dpp_mov<0x118>(v);
+    // the last lane of a row to the row behind it (rows 1 and 3), then lane 31 to rows 2 and 3
+    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x142, 0xa, 0xf, false));
+    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x143, 0xc, 0xf, false));
+    return v;
+}
+// the 32 lanes of each half of a wavefront; every lane gets the result
+__device__ __forceinline__ float half_wave_sum(float v)
+{
+    v = group16_sum(v);
+    auto r = __builtin_amdgcn_permlane16_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+    return __uint_as_float(r[0]) + __uint_as_float(r[1]);
+}
+__device__ __forceinline__ float half_wave_max(float v)
+{
+    v = fmaxf(v, dpp_mov<0xB1>(v));
+    v = fmaxf(v, dpp_mov<0x4E>(v));
+    v = fmaxf(v, dpp_mov<0x141>(v));
+    v = fmaxf(v, dpp_mov<0x140>(v));
+    auto r = __builtin_amdgcn_permlane16_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+    return fmaxf(__uint_as_float(r[0]), __uint_as_float(r[1]));
+}
 // whole wavefront; every lane gets the total
 __device__ __forceinline__ float wave_sum(float v)
 {

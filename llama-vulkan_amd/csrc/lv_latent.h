@@ -12,7 +12,7 @@
 // in LDS), and W_uv is applied to the summed latent (latent_value_kernel).  A batch expands keys and values of every position it
 // can see with one product each and goes through the tile kernels of grouped-query attention.
 //
-// Queries of one token enter the products with bf16 rows as three bf16 pieces (24 bits) and with fp32 rows as they are; weights
+// Queries of one token enter the products with bf16 rows as three bf16 pieces (24 bits), with fp32 rows as they are; weights
 // of the softmax and their sums are fp32.
 #pragma once
 
@@ -28,6 +28,7 @@ struct LatentSpec {
     const float *q_norm, *kv_norm;
     const float *sink;                  // null: none
     const double *freq;                 // rot_dims / 2 angles per position, in full turns
+    const float2 *turn;                 // the same as (cos, sin) at the position of a one-token step
     const uint16_t *uk_t;               // [head][kv_p][dim_p]: W_uk transposed head by head
     const uint16_t *uv;                 // [heads * vdim][kv_p]
     float scale, eps;
@@ -50,30 +51,50 @@ inline uint32_t latent_splits(uint32_t heads, uint32_t positions)
 }
 __host__ __device__ constexpr uint32_t latent_part_stride(uint32_t kc) { return kc + 4; }     // sums, then maximum and sum of weights
 
-// element i of a rotated part of n entries, turned; pairs behind rot_dims pass
-__device__ __forceinline__ float2 latent_turn(const float *v, uint32_t pair, uint32_t n, const LatentSpec &s, uint32_t pos)
+// pair of a rotated part of rot_dim entries, turned by turn(pair); pairs behind rot_dims pass, and there are zeros behind rot_dim
+template <class Turn>
+__device__ __forceinline__ float2 latent_turn(const float *v, uint32_t pair, const LatentSpec &s, Turn turn)
 {
-    float a = v[2 * pair], b = 2 * pair + 1 < n ? v[2 * pair + 1] : 0.f;
-    if (2 * pair < s.rot_dims) turn_pair(a, b, rotation(s.freq[pair], pos));
+    float a = 0.f, b = 0.f;
+    if (2 * pair < s.rot_dim) {
+        a = v[2 * pair];
+        b = v[2 * pair + 1];
+        if (2 * pair < s.rot_dims) turn_pair(a, b, turn(pair));
+    }
     return make_float2(a, b);
 }
 
 // latent, rotated key part -> cache row; `scratch` a float per wave
-template <class CT>
-__device__ __forceinline__ void latent_append(const LatentSpec &s, const float *y, uint32_t pos, float *scratch)
+template <class CT, class Turn>
+__device__ __forceinline__ void latent_append(const LatentSpec &s, const float *y, uint32_t pos, float *scratch, Turn turn)
 {
     const float *c = y + s.kv_off;
     CT *row = static_cast<CT *>(s.cache) + (size_t)pos * s.width;
     float sum = 0.f;
     for (uint32_t i = threadIdx.x; i < s.kv_rank; i += blockDim.x) sum = fmaf(c[i], c[i], sum);
     const float inv = rsqrtf(block_sum_waves(sum, scratch, blockDim.x >> 6) / (float)s.kv_rank + s.eps);
+#pragma unroll 1
     for (uint32_t i = threadIdx.x; i < s.kc; i += blockDim.x) row[i] = float_to_elem<CT>(i < s.kv_rank ? c[i] * inv * s.kv_norm[i] : 0.f);
+#pragma unroll 1
     for (uint32_t i = threadIdx.x; i < (s.width - s.kc) / 2; i += blockDim.x) {
-        const float2 t = 2 * i < s.rot_dim ? latent_turn(c + s.kv_rank, i, s.rot_dim, s, pos) : make_float2(0.f, 0.f);
+        const float2 t = latent_turn(c + s.kv_rank, i, s, turn);
         row[s.kc + 2 * i] = float_to_elem<CT>(t.x);
         row[s.kc + 2 * i + 1] = float_to_elem<CT>(t.y);
     }
 }
+
+// A query as the attention kernel wants it: with bf16 rows three planes of bf16 pieces (largest first, 24 bits together), else fp32.
+// `plane` = elements of a plane
+__device__ __forceinline__ void latent_put(uint16_t *q, size_t plane, size_t i, float v)
+{
+#pragma unroll
+    for (int p = 0; p < 3; p++) {
+        const uint16_t h = float_to_bf16(v);
+        q[p * plane + i] = h;
+        v -= bf16_to_float(h);
+    }
+}
+__device__ __forceinline__ void latent_put(float *q, size_t, size_t i, float v) { q[i] = v; }
 
 // ---- one token -------------------------------------------------------------------------------------------------------------
 struct LatentAbsorbArgs {
@@ -82,7 +103,7 @@ struct LatentAbsorbArgs {
     const float *q;                     // [heads][dim + rot_dim]
     const uint32_t *pos_ptr;
     uint32_t pos_add;
-    float *out;                         // [heads][width], scaled
+    void *out;                          // [heads][width], scaled (latent_put)
 };
 constexpr int kAbsorbRows = 64;         // latent dimensions per workgroup
 
@@ -94,7 +115,7 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(LatentAbsorbArgs a)
     __shared__ float scratch[4];
     const LatentSpec &s = a.s;
     const uint32_t pos = *a.pos_ptr + a.pos_add, blocks = s.kv_p / kAbsorbRows, head = blockIdx.x / blocks, r0 = blockIdx.x % blocks * kAbsorbRows;
-    if (head >= s.heads) return latent_append<CT>(s, a.y, pos, scratch);
+    if (head >= s.heads) return latent_append<CT>(s, a.y, pos, scratch, [&](uint32_t i) { return s.turn[i]; });
     const int sub = threadIdx.x & 7, r8 = threadIdx.x >> 3;
     const uint16_t *w = s.uk_t + ((size_t)head * s.kv_p + r0 + r8) * s.dim_p + sub * 8;
     uint4 v[2][4];
@@ -105,11 +126,14 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(LatentAbsorbArgs a)
             v[i][k] = k * 64 < (int)s.dim_p ? load_once(w + (size_t)i * 32 * s.dim_p + k * 64) : make_uint4(0, 0, 0, 0);
     const float *mine = a.q + (size_t)head * (s.dim + s.rot_dim);
     for (uint32_t i = threadIdx.x; i < s.dim_p; i += 256) q[i] = i < s.dim ? mine[i] * s.scale : 0.f;
-    float *out = a.out + (size_t)head * s.width;
+    CT *out = static_cast<CT *>(a.out);
+    const size_t plane = (size_t)s.heads * s.width, at = (size_t)head * s.width;
     if (r0 == 0)
+#pragma unroll 1
         for (uint32_t i = threadIdx.x; i < (s.width - s.kc) / 2; i += 256) {
-            const float2 t = 2 * i < s.rot_dim ? latent_turn(mine + s.dim, i, s.rot_dim, s, pos) : make_float2(0.f, 0.f);
-            *reinterpret_cast<float2 *>(out + s.kc + 2 * i) = make_float2(t.x * s.scale, t.y * s.scale);
+            const float2 t = latent_turn(mine + s.dim, i, s, [&](uint32_t k) { return s.turn[k]; });
+            latent_put(out, plane, at + s.kc + 2 * i, t.x * s.scale);
+            latent_put(out, plane, at + s.kc + 2 * i + 1, t.y * s.scale);
         }
     __syncthreads();
 #pragma unroll
@@ -128,13 +152,13 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(LatentAbsorbArgs a)
         }
         t = group8_sum(t);
         const uint32_t r = r0 + i * 32 + r8;
-        if (sub == 0 && r < s.kc) out[r] = t;
+        if (sub == 0 && r < s.kc) latent_put(out, plane, at + r, t);
     }
 }
 
 struct LatentStepArgs {
     LatentSpec s;
-    const float *q;                     // [heads][width]
+    const void *q;                      // [heads][width] (latent_put)
     const uint32_t *pos_ptr;
     uint32_t pos_add;
     uint32_t splits;                    // key ranges the grid provides
@@ -153,44 +177,85 @@ __device__ __forceinline__ void latent_ranges(const LatentStepArgs &a, uint32_t 
 template <class CT> constexpr uint32_t latent_key_stride(uint32_t width) { return width + 16 / sizeof(CT); }
 template <class CT> inline size_t latent_attn_lds(uint32_t width)
 {
-    return (size_t)kLatentKeys * latent_key_stride<CT>(width) * sizeof(CT) + 4ull * (kLatentTile * (width + 4) + 4 * kLatentKeys * 17 + kLatentTile * 36 + 3 * kLatentTile);
+    return (size_t)kLatentKeys * latent_key_stride<CT>(width) * sizeof(CT) + 4ull * (4 * kLatentKeys * 17 + kLatentTile * 36 + 3 * kLatentTile);
 }
 
-// grid (tiles of 16 heads, splits), 8 waves.  A block of 32 cache rows lies in LDS (the next one is on its way to registers).
-// Scores: two key tiles x four quarters of the row, S^T = K Q^T, one wave each.  Sums: P [16 heads][4 keys] x rows [4 keys][16
-// latent dimensions] in fp32; a wave takes 64 latent dimensions, of which a lane's four neighbours belong to four products.
-template <class CT>
-__global__ __launch_bounds__(kLatentStepThreads) void latent_attn_kernel(LatentStepArgs a)
+// One head's query as a lane's part of an operand: eight columns
+template <class CT> struct LatentQuery;
+template <> struct LatentQuery<uint16_t> {
+    lv_bf8 p[3];
+    __device__ __forceinline__ void load(const uint16_t *q, size_t plane, bool there)
+    {
+#pragma unroll
+        for (int i = 0; i < 3; i++) p[i] = there ? *reinterpret_cast<const lv_bf8 *>(q + i * plane) : lv_bf8(0.f);
+    }
+    __device__ __forceinline__ lv_f4 times(const GqaRaw<uint16_t> &k, lv_f4 acc) const
+    {
+        const lv_bf8 f = __builtin_bit_cast(lv_bf8, k.v);
+#pragma unroll
+        for (int i = 2; i >= 0; i--) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(f, p[i], acc, 0, 0, 0);
+        return acc;
+    }
+};
+template <> struct LatentQuery<float> {
+    float q[8];
+    __device__ __forceinline__ void load(const float *p, size_t, bool there)
+    {
+#pragma unroll
+        for (int e = 0; e < 8; e++) q[e] = 0.f;
+        if (there) load8(q, p);
+    }
+    __device__ __forceinline__ lv_f4 times(const GqaRaw<float> &k, lv_f4 acc) const
+    {
+        float f[8];
+        k.get(f);
+#pragma unroll
+        for (int e = 0; e < 8; e++) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(f[e], q[e], acc, 0, 0, 0);
+        return acc;
+    }
+};
+__device__ __forceinline__ void raw_to(uint16_t *p, const GqaRaw<uint16_t> &r) { *reinterpret_cast<uint4 *>(p) = r.v; }
+__device__ __forceinline__ void raw_to(float *p, const GqaRaw<float> &r)
 {
-    constexpr int NT = kLatentStepThreads, EPC = 16 / sizeof(CT);           // elements of a 16-byte chunk
-    constexpr int LOADS = kLatentMaxWidth * sizeof(CT) / 256;               // chunks a thread brings of a block, at most
-    constexpr int NB = (kLatentMaxWidth + 511) / 512;                       // 64-wide pieces of the latent a wave takes, at most
+    reinterpret_cast<float4 *>(p)[0] = r.a;
+    reinterpret_cast<float4 *>(p)[1] = r.b;
+}
+
+// grid (tiles of 16 heads, splits), 8 waves.  A wave brings its part of a block of 32 cache rows (16 rows, a quarter of their
+// columns) straight into the registers of a matrix operand, multiplies it by the queries it holds, S^T = K Q^T, and leaves it in
+// LDS for the sums; the next block is on its way meanwhile.  Sums: P [16 heads][4 keys] x rows [4 keys][16 latent dimensions] in
+// fp32; a wave takes 64 latent dimensions, of which a lane's four neighbours belong to four products.
+// NQ = 128-wide pieces of a row, NB = 512-wide pieces of the latent.  Code is kept short: every line of it is fetched on the way.
+template <class CT, int NQ, int NB>
+__global__ __launch_bounds__(kLatentStepThreads, 2) void latent_attn_kernel(LatentStepArgs a)
+{
     extern __shared__ __attribute__((aligned(16))) uint8_t lat_lds[];
     const LatentSpec &s = a.s;
-    const uint32_t W = s.width, KS = latent_key_stride<CT>(W), QS = W + 4;
+    const uint32_t W = s.width, KS = latent_key_stride<CT>(W);
     CT *kb = reinterpret_cast<CT *>(lat_lds);
-    float *qb = reinterpret_cast<float *>(lat_lds + (size_t)kLatentKeys * KS * sizeof(CT)), *ps = qb + kLatentTile * QS, *p = ps + 4 * kLatentKeys * 17, *ml = p + kLatentTile * 36;
+    float *ps = reinterpret_cast<float *>(lat_lds + (size_t)kLatentKeys * KS * sizeof(CT)), *p = ps + 4 * kLatentKeys * 17, *ml = p + kLatentTile * 36;
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), l16 = lane & 15, g4 = lane >> 4;
+    const uint32_t h0 = blockIdx.x * kLatentTile;
+    const int kt = wave & 1, kq = wave >> 1;
+    // columns (j * 4 + kq) * 32 + g4 * 8 .. + 7; columns past the row meet zero queries
+    LatentQuery<CT> q[NQ];
+#pragma unroll
+    for (int j = 0; j < NQ; j++) {
+        const uint32_t k = (j * 4 + kq) * 32;
+        q[j].load(static_cast<const CT *>(a.q) + (size_t)(h0 + l16) * W + k + g4 * 8, (size_t)s.heads * W, k < W && h0 + l16 < s.heads);
+    }
     const uint32_t pos = *a.pos_ptr + a.pos_add;
     uint32_t blocks, per, active;
     latent_ranges(a, pos, blocks, per, active);
     if (blockIdx.y >= active) return;
-    const uint32_t b0 = blockIdx.y * per, b1 = min(b0 + per, blocks), h0 = blockIdx.x * kLatentTile;
-    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), l16 = lane & 15, g4 = lane >> 4;
-    const uint32_t cpr = W / EPC, chunks = kLatentKeys * cpr;               // chunks per row and block
-
-    uint4 next[LOADS];
+    const uint32_t b0 = blockIdx.y * per, b1 = min(b0 + per, blocks);
+    GqaRaw<CT> next[NQ];
     auto request = [&](uint32_t b) {
+        const CT *row = static_cast<const CT *>(s.cache) + (size_t)min(b * kLatentKeys + kt * 16 + l16, pos) * W + g4 * 8;
 #pragma unroll
-        for (int i = 0; i < LOADS; i++) {
-            const uint32_t c = i * NT + threadIdx.x;
-            if (c < chunks) next[i] = *reinterpret_cast<const uint4 *>(static_cast<const CT *>(s.cache) + (size_t)min(b * kLatentKeys + c / cpr, pos) * W + c % cpr * EPC);
-        }
+        for (int j = 0; j < NQ; j++) next[j].load(row + min((j * 4 + kq) * 32u, W - 32));
     };
     request(b0);
-    for (uint32_t i = threadIdx.x; i < kLatentTile * W / 4; i += NT) {
-        const uint32_t h = i / (W / 4), d = i % (W / 4) * 4;
-        *reinterpret_cast<float4 *>(qb + h * QS + d) = h0 + h < s.heads ? *reinterpret_cast<const float4 *>(a.q + (size_t)(h0 + h) * W + d) : make_float4(0.f, 0.f, 0.f, 0.f);
-    }
     if (threadIdx.x < kLatentTile) {
         ml[threadIdx.x] = -INFINITY;
         ml[kLatentTile + threadIdx.x] = 0.f;
@@ -202,45 +267,17 @@ __global__ __launch_bounds__(kLatentStepThreads) void latent_attn_kernel(LatentS
         for (int e = 0; e < 4; e++) acc[n][e] = lv_f4{0.f, 0.f, 0.f, 0.f};
 
     for (uint32_t b = b0; b < b1; b++) {
-        __syncthreads();      // the block before has been read
+        if (b != b0) __syncthreads();      // the block before has been read
+        lv_f4 sc = lv_f4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int i = 0; i < LOADS; i++) {
-            const uint32_t c = i * NT + threadIdx.x;
-            if (c < chunks) *reinterpret_cast<uint4 *>(kb + (size_t)(c / cpr) * KS + c % cpr * EPC) = next[i];
+        for (int j = 0; j < NQ; j++) {
+            const uint32_t k = (j * 4 + kq) * 32;
+            if (k < W) raw_to(kb + (size_t)(kt * 16 + l16) * KS + k + g4 * 8, next[j]);
+            sc = q[j].times(next[j], sc);
         }
-        __syncthreads();
+#pragma unroll
+        for (int r = 0; r < 4; r++) ps[(kq * kLatentKeys + kt * 16 + g4 * 4 + r) * 17 + l16] = sc[r];
         if (b + 1 < b1) request(b + 1);
-        {
-            const int kt = wave & 1, kq = wave >> 1;
-            const CT *kr = kb + (size_t)(kt * 16 + l16) * KS + g4 * 8;
-            const float *qr = qb + l16 * QS + g4 * 8;
-            lv_f4 sc = lv_f4{0.f, 0.f, 0.f, 0.f};
-            for (uint32_t k = kq * 32; k < W; k += 128) {
-                float q[8];
-                load8(q, qr + k);
-                if constexpr (sizeof(CT) == 2) {
-                    const lv_bf8 fk = *reinterpret_cast<const lv_bf8 *>(kr + k);
-                    lv_bf8 q1, q2, q3;
-#pragma unroll
-                    for (int e = 0; e < 8; e++) {
-                        q1[e] = (__bf16)q[e];
-                        const float r = q[e] - (float)q1[e];
-                        q2[e] = (__bf16)r;
-                        q3[e] = (__bf16)(r - (float)q2[e]);
-                    }
-                    sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fk, q3, sc, 0, 0, 0);
-                    sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fk, q2, sc, 0, 0, 0);
-                    sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fk, q1, sc, 0, 0, 0);
-                } else {
-                    float f[8];
-                    load8(f, kr + k);
-#pragma unroll
-                    for (int e = 0; e < 8; e++) sc = __builtin_amdgcn_mfma_f32_16x16x4f32(f[e], q[e], sc, 0, 0, 0);
-                }
-            }
-#pragma unroll
-            for (int r = 0; r < 4; r++) ps[(kq * kLatentKeys + kt * 16 + g4 * 4 + r) * 17 + l16] = sc[r];
-        }
         __syncthreads();
         {
             const uint32_t key = threadIdx.x & 31, h = threadIdx.x >> 5;
@@ -249,12 +286,7 @@ __global__ __launch_bounds__(kLatentStepThreads) void latent_attn_kernel(LatentS
             for (int k = 0; k < 4; k++) v += ps[(k * kLatentKeys + key) * 17 + h];
             if (b * kLatentKeys + key > pos) v = -INFINITY;
             const float old = ml[h];
-            float m = fmaxf(v, old);
-#pragma unroll
-            for (int off = 1; off < 32; off <<= 1) m = fmaxf(m, __shfl_xor(m, off, 64));
-            const float w = __expf(v - m);
-            float l = group16_sum(w);
-            l += __shfl_xor(l, 16, 64);
+            const float m = fmaxf(half_wave_max(v), old), w = __expf(v - m), l = half_wave_sum(w);
             p[h * 36 + key] = w;
             if (key == 0) {
                 const float f = __expf(old - m);
@@ -310,48 +342,55 @@ __global__ __launch_bounds__(kLatentStepThreads) void latent_attn_kernel(LatentS
 }
 
 constexpr int kLatentValueRows = 64;
-// grid (heads, vdim / 64 up): the ranges' sums of one head, then up to 64 rows of W_uv
-static __global__ __launch_bounds__(kLatentStepThreads) void latent_value_kernel(LatentStepArgs a)
+// grid (heads, vdim / 64 up): the ranges' sums of one head, then up to 64 rows of W_uv.  Four groups of 128 threads take up to 16
+// ranges each, four columns a thread; everything is requested before anything is used.
+static __global__ __launch_bounds__(kLatentStepThreads, 2) void latent_value_kernel(LatentStepArgs a)
 {
-    constexpr int AHEAD = 8;
-    __shared__ __attribute__((aligned(16))) float o[kLatentMaxWidth];
+    constexpr int AHEAD = 8, COLS = 512, RANGES = kLatentMaxSplits / 4;
+    __shared__ __attribute__((aligned(16))) float o[kLatentMaxWidth], sums[4][COLS];
     __shared__ float weight[kLatentMaxSplits];
     const LatentSpec &s = a.s;
     const uint32_t head = blockIdx.x, row = blockIdx.y * kLatentValueRows + (threadIdx.x >> 3), sub = threadIdx.x & 7, steps = s.kv_p / 64;
     const uint16_t *w = s.uv + ((size_t)head * s.vdim + min(row, s.vdim - 1)) * s.kv_p + sub * 8;
     uint4 v[AHEAD];
 #pragma unroll
-    for (int i = 0; i < AHEAD; i++)
-        if (i < (int)steps) v[i] = load_once(w + i * 64);
+    for (int i = 0; i < AHEAD; i++) v[i] = load_once(w + min((uint32_t)i, steps - 1) * 64);
     const uint32_t pos = *a.pos_ptr + a.pos_add, PS = latent_part_stride(s.kc);
     uint32_t blocks, per, active;
     latent_ranges(a, pos, blocks, per, active);
     const float *part = a.part + (size_t)head * PS;
     const size_t next = (size_t)s.heads * PS;
-    if (threadIdx.x < 64) {
-        const uint32_t i = threadIdx.x;
-        const float sink = s.sink ? s.sink[head] : -INFINITY, m = i < active ? part[i * next + s.kc] : -INFINITY, l = i < active ? part[i * next + s.kc + 1] : 0.f;
-        float top = fmaxf(m, sink);
+    const uint32_t grp = __builtin_amdgcn_readfirstlane(threadIdx.x >> 7), c4 = (threadIdx.x & 127) * 4;
+#pragma unroll 1
+    for (uint32_t c0 = 0; c0 < s.kv_p; c0 += COLS) {
+        const uint32_t c = min(c0 + c4, s.kc - 4);
+        float4 z[RANGES];
 #pragma unroll
-        for (int off = 1; off < 64; off <<= 1) top = fmaxf(top, __shfl_xor(top, off, 64));
-        const float e = __expf(m - top), sum = wave_sum(e * l) + __expf(sink - top);
-        weight[i] = e / sum;
-    }
-    __syncthreads();
-    for (uint32_t c = threadIdx.x; c < s.kv_p; c += kLatentStepThreads) {
-        float t = 0.f;
-        if (c < s.kc) {
-            for (uint32_t i = 0; i < active; i += 8) {
-                float z[8];
-#pragma unroll
-                for (int e = 0; e < 8; e++) z[e] = part[min(i + e, active - 1) * next + c];
-#pragma unroll
-                for (int e = 0; e < 8; e++) t = fmaf(z[e], i + e < active ? weight[i + e] : 0.f, t);
+        for (int i = 0; i < RANGES; i++) z[i] = *reinterpret_cast<const float4 *>(part + min(grp * RANGES + i, active - 1) * next + c);
+        if (c0 == 0) {
+            if (threadIdx.x < 64) {
+                const uint32_t i = threadIdx.x;
+                const float sink = s.sink ? s.sink[head] : -INFINITY, m = i < active ? part[i * next + s.kc] : -INFINITY, l = i < active ? part[i * next + s.kc + 1] : 0.f;
+                const float half = half_wave_max(m), top = fmaxf(fmaxf(half, __shfl_xor(half, 32, 64)), sink);
+                const float e = __expf(m - top), sum = wave_sum(e * l) + __expf(sink - top);
+                weight[i] = e / sum;
             }
+            __syncthreads();
         }
-        o[c] = t;
+        float4 t = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+        for (int i = 0; i < RANGES; i++) {
+            const float f = weight[grp * RANGES + i];          // 0 for a range without keys
+            t.x = fmaf(z[i].x, f, t.x); t.y = fmaf(z[i].y, f, t.y); t.z = fmaf(z[i].z, f, t.z); t.w = fmaf(z[i].w, f, t.w);
+        }
+        *reinterpret_cast<float4 *>(&sums[grp][c4]) = t;
+        __syncthreads();
+        if (c0 + threadIdx.x < s.kv_p) {
+            const uint32_t i = threadIdx.x;
+            o[c0 + i] = c0 + i < s.kc ? (sums[0][i] + sums[1][i]) + (sums[2][i] + sums[3][i]) : 0.f;
+        }
+        __syncthreads();
     }
-    __syncthreads();
     auto dot8 = [&](const uint4 &q, const float *x) {
         const uint32_t u[4] = {q.x, q.y, q.z, q.w};
         float t = 0.f;
@@ -366,6 +405,7 @@ static __global__ __launch_bounds__(kLatentStepThreads) void latent_value_kernel
 #pragma unroll
     for (int i = 0; i < AHEAD; i++)
         if (i < (int)steps) t += dot8(v[i], o + i * 64 + sub * 8);
+#pragma unroll 1
     for (uint32_t i = AHEAD; i < steps; i++) t += dot8(*reinterpret_cast<const uint4 *>(w + i * 64), o + i * 64 + sub * 8);
     t = group8_sum(t);
     if (sub == 0 && row < s.vdim) a.out[(size_t)head * s.vdim + row] = t;
@@ -383,7 +423,7 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(LatentSpec s, const
     for (uint32_t i = threadIdx.x; i < s.q_rank; i += 256) sum = fmaf(q[i], q[i], sum);
     const float inv = rsqrtf(block_sum_waves(sum, scratch, 4) / (float)s.q_rank + s.eps);
     for (uint32_t i = threadIdx.x; i < ldq; i += 256) cq[(size_t)t * ldq + i] = float_to_elem<T>(i < s.q_rank ? q[i] * inv * s.q_norm[i] : 0.f);
-    latent_append<T>(s, row, pos0 + t, scratch);
+    latent_append<T>(s, row, pos0 + t, scratch, [&](uint32_t i) { return rotation(s.freq[i], pos0 + t); });
 }
 
 // one workgroup per token: [heads][dim + rot_dim] -> rotated, scaled, heads padded to dk elements

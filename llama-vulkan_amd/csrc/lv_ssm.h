@@ -5,8 +5,11 @@
 //   S    <- a S + dt B x^T   (B and C shared by the consecutive heads of a group);  y = S^T C + D x
 //   out  = RMS norm of y silu(z) in equal parts, times weights (GroupInput)
 //
-// All of it is fp32.  Columns of S do not interact and nothing is fed back from a read-out: from token to token a state entry goes
+// State, step sizes, decays and their products are fp32.  Columns of S do not interact and nothing is fed back from a read-out: from token to token a state entry goes
 // through one multiply-add, and the sums of the read-outs are off that chain.
+//
+// Token by token (one-token steps, and batches of 32-bit models) a step is taken as it stands.  Batches with bf16 activations go
+// in chunks of tokens on the matrix cores (ssm_chunk_kernel).
 //
 // State of a sequence and pass: S as [head][vdim][64 J] (a column contiguous, zero beyond the state size) and a ring of the
 // convolution's last `taps` inputs.  Nothing has to be cleared for a new sequence: positions before 0 and the state at position 0
@@ -123,7 +126,11 @@ static __global__ __launch_bounds__(256) void ssm_prepare_kernel(SsmBatchArgs a)
             pad = d >= s.n;
             channel = inner + (which * s.groups + g) * s.n + d;
         }
-        for (uint32_t t = first; t < last; t++) out[t * ld] = pad ? 0.f : short_conv(s, a.y + (size_t)t * a.ldy, a.ldy, t, channel, a.pos0 + t, (a.pos0 + t) % s.taps);
+        float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+        if (!pad) short_conv8(v, s, a.y, a.ldy, channel, a.pos0, first, a.n);
+#pragma unroll
+        for (uint32_t i = 0; i < kSsmPrepareTokens; i++)
+            if (first + i < last) out[(first + i) * ld] = v[i];
         return;
     }
     c -= inner + 2 * gn;
@@ -219,17 +226,282 @@ __global__ __launch_bounds__(kSsmScanThreads) void ssm_scan_kernel(SsmBatchArgs 
     }
 }
 
-// gated, normed read-outs of a batch as activations; LDS: inner + group_sums floats.  z: [row][ldz]
+// ---- batches in chunks -------------------------------------------------------------------------------------------------------
+// With l_t the running sum of -exp(A) dt inside a chunk of Q tokens, l its last one and S the state in front of it:
+//   y_t = exp(l_t) S^T C_t + sum_{s <= t} (C_t . B_s) exp(l_t - l_s) dt_s x_s + D x_t
+//   S  <- exp(l) S + sum_s B_s (exp(l - l_s) dt_s x_s)^T
+// all products of matrices over the chunk; every exponent is a sum of decays of tokens in a row, so none of them overflows.  x, B
+// and C are bf16 as a convolution's output; the state enters a product as three bf16 pieces (24 bits), weights and weighted x as
+// two; sums are fp32.
+struct SsmChunkArgs {
+    SsmSpec s;
+    const float *y;                      // [n][ldy]: the projections
+    uint32_t ldy, pos0, n;
+    uint32_t ldt;                        // n rounded up to kSsmChunk: tokens the operands below have, zeros past the end
+    uint16_t *xt;                        // [ldt / 8][inner][8 tokens]
+    uint16_t *b, *c;                     // [ldt][groups][nstride], zero beyond the state size, entries in ssm_place order
+    uint16_t *bt;                        // [ldt / 8][groups][nstride][8 tokens]
+    float *dt;                           // [heads][ldt]
+    float *o;                            // [n][inner]
+};
+constexpr uint32_t kSsmChunk = 64;
+// Where entry d of B or C lies in its row: the order in which a lane's state registers make up a matrix operand (place 8 g + 4 t + r
+// of 32 holds entry 16 t + 4 g + r)
+__host__ __device__ constexpr uint32_t ssm_place(uint32_t d) { return (d & ~31u) | ((d >> 2) & 3) << 3 | ((d >> 4) & 1) << 2 | (d & 3); }
+
+// grid (ssm_prepare_columns, ldt / 8): a thread per channel (B and C padded) or head, eight tokens
+static __global__ __launch_bounds__(256) void ssm_operands_kernel(SsmChunkArgs a)
+{
+    const SsmSpec &s = a.s;
+    const uint32_t inner = s.inner(), gn = s.groups * s.nstride, t8 = blockIdx.y, t0 = t8 * 8;
+    uint32_t c = blockIdx.x * 256 + threadIdx.x;
+    if (c >= inner + 2 * gn) {
+        c -= inner + 2 * gn;
+        if (c >= s.heads) return;
+        const float bias = s.dt_bias[c];
+        float dt[8];
+#pragma unroll
+        for (uint32_t i = 0; i < 8; i++) dt[i] = t0 + i < a.n ? softplus_f(a.y[(size_t)(t0 + i) * a.ldy + s.dt_off + c] + bias) : 0.f;
+        float4 *out = reinterpret_cast<float4 *>(a.dt + (size_t)c * a.ldt + t0);
+        out[0] = make_float4(dt[0], dt[1], dt[2], dt[3]);
+        out[1] = make_float4(dt[4], dt[5], dt[6], dt[7]);
+        return;
+    }
+    uint32_t channel = c, place = 0, e = 0;
+    bool pad = false;
+    if (c >= inner) {
+        e = c - inner;                   // of B, then of C
+        const uint32_t d = e % s.nstride;
+        pad = d >= s.n;
+        channel = inner + e / s.nstride * s.n + d;
+        place = e - d + ssm_place(d);
+    }
+    float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    if (!pad) short_conv8(v, s, a.y, a.ldy, channel, a.pos0, t0, a.n);
+    uint16_t h[8];
+#pragma unroll
+    for (uint32_t i = 0; i < 8; i++) h[i] = float_to_bf16(v[i]);
+    const uint4 eight = make_uint4(h[0] | (uint32_t)h[1] << 16, h[2] | (uint32_t)h[3] << 16, h[4] | (uint32_t)h[5] << 16, h[6] | (uint32_t)h[7] << 16);
+    if (c < inner) {
+        reinterpret_cast<uint4 *>(a.xt)[(size_t)t8 * inner + c] = eight;
+        return;
+    }
+    uint16_t *rows = e < gn ? a.b + place : a.c + (place - gn);
+#pragma unroll
+    for (uint32_t i = 0; i < 8; i++) rows[(size_t)(t0 + i) * gn] = h[i];
+    if (e < gn) reinterpret_cast<uint4 *>(a.bt)[(size_t)t8 * gn + e] = eight;
+}
+
+constexpr int kSsmChunkThreads = 256;
+template <int J> constexpr int ssm_chunk_stages() { return J <= 2 ? 2 : 1; }
+template <int J> constexpr int ssm_chunk_stage_bytes() { return 3 * kSsmChunk * 64 * J * 2; }      // C and B rows, B by 8 tokens
+constexpr int kSsmWeightLd = kSsmChunk + 8;
+template <int J> constexpr int ssm_chunk_lds() { return ssm_chunk_stages<J>() * ssm_chunk_stage_bytes<J>() + 2 * kSsmChunk * kSsmWeightLd * 2 + 4 * 4 * kSsmChunk * 4; }
+
+// All chunks of a batch, one after the other, for 64 columns of one head: 4 waves, 16 columns and all of their state each.  grid
+// (heads, vdim / 64 up).  The weights (C_t . B_s) exp(l_t - l_s) dt_s of a chunk are shared out, 16 tokens a wave, and meet in LDS.
+template <int J>
+__global__ __launch_bounds__(kSsmChunkThreads) void ssm_chunk_kernel(SsmChunkArgs a)
+{
+    constexpr int W = 64 * J, ROW = W * 2, NST = ssm_chunk_stages<J>(), STAGE = ssm_chunk_stage_bytes<J>(), TILE = kSsmChunk * ROW;
+    extern __shared__ __attribute__((aligned(128))) uint8_t chunk_lds[];
+    const SsmSpec &s = a.s;
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), l16 = lane & 15, g4 = lane >> 4;
+    uint16_t *const mh = reinterpret_cast<uint16_t *>(chunk_lds + NST * STAGE), *const ml = mh + kSsmChunk * kSsmWeightLd;
+    // of this wave's own: l_t, dt_t, exp(l_t), exp(l - l_t) dt_t
+    float *const lt = reinterpret_cast<float *>(ml + kSsmChunk * kSsmWeightLd) + wave * 4 * kSsmChunk, *const dts = lt + kSsmChunk, *const el = dts + kSsmChunk, *const wt = el + kSsmChunk;
+    const uint32_t head = blockIdx.x, grp = head / (s.heads / s.groups), inner = s.inner(), p = blockIdx.y * 64 + wave * 16 + l16;
+    const bool live = p < s.vdim;
+    const uint32_t channel = head * s.vdim + min(p, s.vdim - 1);
+    float4 *const state = reinterpret_cast<float4 *>(s.state + (size_t)channel * W);
+    const float rate = -__expf(s.a_log[head]), skip = s.skip[head];
+
+    auto issue = [&](uint32_t t0, int st) {
+        uint8_t *b = chunk_lds + st * STAGE;
+#pragma unroll
+        for (int i = 0; i < 2 * J; i++) {
+            const uint32_t first = (i * 4 + wave) * 64, e = first + lane, row = e / (8 * J), ch = e % (8 * J);
+            const size_t at = ((size_t)(t0 + row) * s.groups + grp) * W + (ch ^ (row & 7)) * 8;
+            __builtin_amdgcn_global_load_lds((lv_glb_any *)(a.c + at), (lv_lds_any *)(b + first * 16), 16, 0, 0);
+            __builtin_amdgcn_global_load_lds((lv_glb_any *)(a.b + at), (lv_lds_any *)(b + TILE + first * 16), 16, 0, 0);
+            const size_t by8 = (((size_t)(t0 / 8 + e / W) * s.groups + grp) * W + e % W) * 8;
+            __builtin_amdgcn_global_load_lds((lv_glb_any *)(a.bt + by8), (lv_lds_any *)(b + 2 * TILE + first * 16), 16, 0, 0);
+        }
+    };
+    uint4 xn[2];
+    float dtn;
+    auto request = [&](uint32_t t0) {
+#pragma unroll
+        for (int k = 0; k < 2; k++) xn[k] = reinterpret_cast<const uint4 *>(a.xt)[(size_t)(t0 / 8 + k * 4 + g4) * inner + channel];
+        dtn = a.dt[(size_t)head * a.ldt + t0 + lane];
+    };
+    issue(0, 0);
+    request(0);
+    lv_f4 S[4 * J];
+#pragma unroll
+    for (int i = 0; i < 4 * J; i++) {
+        const float4 v = a.pos0 == 0 || !live ? make_float4(0.f, 0.f, 0.f, 0.f) : state[i * 4 + g4];
+        S[i] = lv_f4{v.x, v.y, v.z, v.w};
+    }
+
+    for (uint32_t t0 = 0, st = 0; t0 < a.n; t0 += kSsmChunk, st = NST == 2 ? st ^ 1 : 0) {
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        __syncthreads();      // this stage is in LDS for everyone, and everyone is done with the other one and with the weights
+        const uint4 x[2] = {xn[0], xn[1]};
+        const float dt = dtn;
+        const bool more = t0 + kSsmChunk < a.n;
+        if (more) {
+            if (NST == 2) issue(t0 + kSsmChunk, st ^ 1);
+            request(t0 + kSsmChunk);
+        }
+        const uint8_t *bc = chunk_lds + st * STAGE, *bb = bc + TILE, *bt = bb + TILE;
+        auto frag = [&](const uint8_t *tile, int row, int k) { return *reinterpret_cast<const lv_bf8 *>(tile + row * ROW + ((k * 4 + g4) ^ (row & 7)) * 16); };
+
+        const float l = wave_running_sum(rate * dt), end = __shfl(l, 63, 64);
+        lt[lane] = l;
+        dts[lane] = dt;
+        el[lane] = __expf(l);
+        wt[lane] = __expf(end - l) * dt;
+        __builtin_amdgcn_fence(__ATOMIC_SEQ_CST, "wavefront");
+        __builtin_amdgcn_wave_barrier();
+
+        {
+            const int t = wave * 16 + l16;
+            const float mine = lt[t];
+            lv_bf8 fc[2 * J];
+#pragma unroll
+            for (int k = 0; k < 2 * J; k++) fc[k] = frag(bc, t, k);
+#pragma unroll 1
+            for (int j = 0; j <= (wave | 1); j++) {
+                float m[4] = {0.f, 0.f, 0.f, 0.f};
+                if (j <= wave) {
+                    lv_f4 g = lv_f4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                    for (int k = 0; k < 2 * J; k++) g = __builtin_amdgcn_mfma_f32_16x16x32_bf16(frag(bb, j * 16 + l16, k), fc[k], g, 0, 0, 0);
+                    const float4 ls = *reinterpret_cast<const float4 *>(lt + j * 16 + g4 * 4), ds = *reinterpret_cast<const float4 *>(dts + j * 16 + g4 * 4);
+                    const float lsv[4] = {ls.x, ls.y, ls.z, ls.w}, dsv[4] = {ds.x, ds.y, ds.z, ds.w};
+#pragma unroll
+                    for (int r = 0; r < 4; r++) {
+                        const int u = j * 16 + g4 * 4 + r;
+                        const float w = g[r] * dsv[r] * __expf(mine - lsv[r]);
+                        m[r] = u < t ? w : u == t ? w + skip : 0.f;
+                    }
+                }
+                uint16_t h[4], q[4];
+#pragma unroll
+                for (int r = 0; r < 4; r++) {
+                    h[r] = float_to_bf16(m[r]);
+                    q[r] = float_to_bf16(m[r] - bf16_to_float(h[r]));
+                }
+                const int at = t * kSsmWeightLd + j * 16 + g4 * 4;
+                *reinterpret_cast<uint2 *>(mh + at) = make_uint2(h[0] | (uint32_t)h[1] << 16, h[2] | (uint32_t)h[3] << 16);
+                *reinterpret_cast<uint2 *>(ml + at) = make_uint2(q[0] | (uint32_t)q[1] << 16, q[2] | (uint32_t)q[3] << 16);
+            }
+        }
+        // read-outs: the state's part needs no weights and runs up to the barrier
+        lv_f4 y[4];
+#pragma unroll
+        for (int i = 0; i < 4; i++) y[i] = lv_f4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int k = 0; k < 2 * J; k++) {
+            lv_bf8 q[3];
+#pragma unroll
+            for (int e = 0; e < 8; e++) {
+                float v = S[2 * k + e / 4][e % 4];
+#pragma unroll
+                for (int c = 0; c < 3; c++) {
+                    q[c][e] = (__bf16)v;
+                    v -= (float)q[c][e];
+                }
+            }
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const lv_bf8 f = frag(bc, i * 16 + l16, k);
+#pragma unroll
+                for (int c = 2; c >= 0; c--) y[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(f, q[c], y[i], 0, 0, 0);
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            const float4 e = *reinterpret_cast<const float4 *>(el + i * 16 + g4 * 4);
+            y[i][0] *= e.x; y[i][1] *= e.y; y[i][2] *= e.z; y[i][3] *= e.w;
+        }
+        const lv_bf8 fx[2] = {__builtin_bit_cast(lv_bf8, x[0]), __builtin_bit_cast(lv_bf8, x[1])};
+        __syncthreads();      // the weights are there
+#pragma unroll
+        for (int i = 0; i < 4; i++)
+#pragma unroll
+            for (int k = 0; k <= i / 2; k++) {
+                const int at = (i * 16 + l16) * kSsmWeightLd + k * 32 + g4 * 8;
+                y[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const lv_bf8 *>(ml + at), fx[k], y[i], 0, 0, 0);
+                y[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const lv_bf8 *>(mh + at), fx[k], y[i], 0, 0, 0);
+            }
+        // the state behind the chunk
+        const float all = __expf(end);
+#pragma unroll
+        for (int i = 0; i < 4 * J; i++)
+#pragma unroll
+            for (int r = 0; r < 4; r++) S[i][r] *= all;
+#pragma unroll
+        for (int k = 0; k < 2; k++) {
+            float w[8];
+            load8(w, wt + k * 32 + g4 * 8);
+            lv_bf8 xh, xl;
+#pragma unroll
+            for (int e = 0; e < 8; e++) {
+                const float v = (float)fx[k][e] * w[e];
+                xh[e] = (__bf16)v;
+                xl[e] = (__bf16)(v - (float)xh[e]);
+            }
+#pragma unroll
+            for (int i = 0; i < 4 * J; i++) {
+                const lv_bf8 f = *reinterpret_cast<const lv_bf8 *>(bt + ((k * 4 + g4) * W + i * 16 + l16) * 16);
+                S[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(f, xl, S[i], 0, 0, 0);
+                S[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(f, xh, S[i], 0, 0, 0);
+            }
+        }
+        if (live) {
+#pragma unroll
+            for (int i = 0; i < 4; i++)
+#pragma unroll
+                for (int r = 0; r < 4; r++) {
+                    const uint32_t t = t0 + i * 16 + g4 * 4 + r;
+                    if (t < a.n) a.o[(size_t)t * inner + channel] = y[i][r];
+                }
+        }
+        if (NST == 1 && more) {
+            __syncthreads();
+            issue(t0 + kSsmChunk, 0);
+        }
+    }
+    if (live) {
+#pragma unroll
+        for (int i = 0; i < 4 * J; i++) state[i * 4 + g4] = make_float4(S[i][0], S[i][1], S[i][2], S[i][3]);
+    }
+}
+
+// gated, normed read-outs of a batch as activations; LDS: inner + group_sums + 4 floats.  z: [row][ldz]
 template <class T>
 __global__ __launch_bounds__(256) void ssm_gate_kernel(GroupInput g, uint32_t ldz, T *__restrict__ act, uint32_t ld)
 {
-    extern __shared__ float gs[];
+    extern __shared__ __attribute__((aligned(16))) float gs[];
     const size_t row = blockIdx.x;
     g.o += row * g.n;
     g.z += row * ldz;
-    group_input(g, gs + g.n, [&](uint32_t i, float v) { gs[i] = v; }, [&](uint32_t i) { return gs[i]; });
+    group_input(g, gs + g.n, [&](uint32_t i, auto v) { *reinterpret_cast<decltype(v) *>(gs + i) = v; },
+                [&](uint32_t i, auto &v) { v = *reinterpret_cast<std::decay_t<decltype(v)> *>(gs + i); });
     __syncthreads();
-    for (uint32_t i = threadIdx.x; i < ld; i += 256) act[row * ld + i] = float_to_elem<T>(i < g.n ? gs[i] : 0.f);
+    T *out = act + row * ld;          // ld is a multiple of 64; gs is readable to the next multiple of four
+    for (uint32_t i = threadIdx.x * 4; i < ld; i += 1024) {
+        const float4 v = *reinterpret_cast<const float4 *>(gs + min(i, g.n & ~3u));
+        float f[4] = {v.x, v.y, v.z, v.w};
+#pragma unroll
+        for (uint32_t e = 0; e < 4; e++) f[e] = i + e < g.n ? f[e] : 0.f;
+        if constexpr (sizeof(T) == 2)
+            *reinterpret_cast<uint2 *>(out + i) = make_uint2((uint32_t)float_to_bf16(f[0]) | ((uint32_t)float_to_bf16(f[1]) << 16),
+                                                             (uint32_t)float_to_bf16(f[2]) | ((uint32_t)float_to_bf16(f[3]) << 16));
+        else *reinterpret_cast<float4 *>(out + i) = make_float4(f[0], f[1], f[2], f[3]);
+    }
 }
 
 }  // namespace lv

@@ -30,61 +30,84 @@ struct StreamInput {
     float eps;
 };
 
-// Elements i .. i + 3: takes in the pending output and returns u.  NS: streams there is room for.
+// elements i .. i + 3 of the streams and of the pending output.  NS: streams there is room for
 template <int NS>
-__device__ __forceinline__ float4 stream_gather(const StreamInput &a, uint32_t i, bool store)
-{
-    float4 x[NS], u = make_float4(0.f, 0.f, 0.f, 0.f);
+struct StreamQuad {
+    float4 x[NS], y;
+
+    __device__ __forceinline__ void load(const StreamInput &a, uint32_t i)
+    {
 #pragma unroll
-    for (int t = 0; t < NS; t++)
-        if (t < (int)a.streams) x[t] = *reinterpret_cast<const float4 *>(a.x + (size_t)t * a.dp + i);
-    float4 y = u;
-    if (a.y) y = *reinterpret_cast<const float4 *>(a.y + i);
-#pragma unroll
-    for (int t = 0; t < NS; t++) {
-        if (t >= (int)a.streams) break;
-        float4 v = x[t];
-        if (a.y) {
-            const float o = a.spread->out[t];
-            v = make_float4(o * y.x, o * y.y, o * y.z, o * y.w);
-#pragma unroll
-            for (int f = 0; f < NS; f++) {
-                if (f >= (int)a.streams) break;
-                const float c = a.spread->mix[f * kMaxStreams + t];
-                v.x = fmaf(c, x[f].x, v.x); v.y = fmaf(c, x[f].y, v.y); v.z = fmaf(c, x[f].z, v.z); v.w = fmaf(c, x[f].w, v.w);
-            }
-            if (store && a.x_out) *reinterpret_cast<float4 *>(a.x_out + (size_t)t * a.dp + i) = v;
-        }
-        const float g = a.gather->in[t];
-        u.x = fmaf(g, v.x, u.x); u.y = fmaf(g, v.y, u.y); u.z = fmaf(g, v.z, u.z); u.w = fmaf(g, v.w, u.w);
+        for (int t = 0; t < NS; t++)
+            if (t < (int)a.streams) x[t] = *reinterpret_cast<const float4 *>(a.x + (size_t)t * a.dp + i);
+        y = a.y ? *reinterpret_cast<const float4 *>(a.y + i) : make_float4(0.f, 0.f, 0.f, 0.f);
     }
-    return u;
+    // takes in the pending output and returns u
+    __device__ __forceinline__ float4 gather(const StreamInput &a, uint32_t i, bool store) const
+    {
+        float4 u = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+        for (int t = 0; t < NS; t++) {
+            if (t >= (int)a.streams) break;
+            float4 v = x[t];
+            if (a.y) {
+                const float o = a.spread->out[t];
+                v = make_float4(o * y.x, o * y.y, o * y.z, o * y.w);
+#pragma unroll
+                for (int f = 0; f < NS; f++) {
+                    if (f >= (int)a.streams) break;
+                    const float c = a.spread->mix[f * kMaxStreams + t];
+                    v.x = fmaf(c, x[f].x, v.x); v.y = fmaf(c, x[f].y, v.y); v.z = fmaf(c, x[f].z, v.z); v.w = fmaf(c, x[f].w, v.w);
+                }
+                if (store && a.x_out) *reinterpret_cast<float4 *>(a.x_out + (size_t)t * a.dp + i) = v;
+            }
+            const float g = a.gather->in[t];
+            u.x = fmaf(g, v.x, u.x); u.y = fmaf(g, v.y, u.y); u.z = fmaf(g, v.z, u.z); u.w = fmaf(g, v.w, u.w);
+        }
+        return u;
+    }
+};
+
+// u of all elements, four at a time: use(i, u).  The next four are on their way meanwhile.
+template <int NS, class Use>
+__device__ __forceinline__ void stream_each(const StreamInput &a, bool store, Use use)
+{
+    const uint32_t step = blockDim.x * 4;
+    uint32_t i = threadIdx.x * 4;
+    if (i >= a.dp) return;
+    StreamQuad<NS> next;
+    next.load(a, i);
+#pragma unroll 1
+    do {
+        const StreamQuad<NS> q = next;
+        const uint32_t at = i;
+        i += step;
+        if (i < a.dp) next.load(a, i);
+        use(at, q.gather(a, at, store));
+    } while (i < a.dp);
 }
 
 // The whole input: put(i, h) gets four elements at a time, get(i) returns what put left there.  scratch: a float per wave.
 template <int NS, class Put, class Get>
 __device__ __forceinline__ void stream_input(const StreamInput &a, bool lead, float *scratch, Put put, Get get)
 {
-    const uint32_t step = blockDim.x * 4;
     if (a.alpha) {
         const float al = *a.alpha;
-        for (uint32_t i = threadIdx.x * 4; i < a.dp; i += step) {
-            const float4 u = stream_gather<NS>(a, i, lead);
+        stream_each<NS>(a, lead, [&](uint32_t i, const float4 u) {
             const float4 w = *reinterpret_cast<const float4 *>(a.w + i), b = *reinterpret_cast<const float4 *>(a.b + i);
-            const float4 h = make_float4(fmaf(tanhf(al * u.x), w.x, b.x), fmaf(tanhf(al * u.y), w.y, b.y), fmaf(tanhf(al * u.z), w.z, b.z), fmaf(tanhf(al * u.w), w.w, b.w));
+            const float4 h = make_float4(fmaf(tanh_f(al * u.x), w.x, b.x), fmaf(tanh_f(al * u.y), w.y, b.y), fmaf(tanh_f(al * u.z), w.z, b.z), fmaf(tanh_f(al * u.w), w.w, b.w));
             put(i, h);
             if (lead && a.h_out) *reinterpret_cast<float4 *>(a.h_out + i) = h;
-        }
+        });
         return;
     }
     float s = 0.f;
-    for (uint32_t i = threadIdx.x * 4; i < a.dp; i += step) {
-        const float4 u = stream_gather<NS>(a, i, lead);
+    stream_each<NS>(a, lead, [&](uint32_t i, const float4 u) {
         s = fmaf(u.x, u.x, s); s = fmaf(u.y, u.y, s); s = fmaf(u.z, u.z, s); s = fmaf(u.w, u.w, s);
         put(i, u);
-    }
+    });
     const float inv = rsqrtf(block_sum_waves(s, scratch, blockDim.x >> 6) / (float)a.dim + a.eps);
-    for (uint32_t i = threadIdx.x * 4; i < a.dp; i += step) {
+    for (uint32_t i = threadIdx.x * 4; i < a.dp; i += blockDim.x * 4) {
         const float4 u = get(i), w = *reinterpret_cast<const float4 *>(a.w + i);
         const float4 h = make_float4(u.x * inv * w.x, u.y * inv * w.y, u.z * inv * w.z, u.w * inv * w.w);
         put(i, h);
@@ -124,7 +147,7 @@ __global__ __launch_bounds__(256) void stream_rows_kernel(StreamRowsArgs a)
         }
     }
     if (!a.act) {
-        for (uint32_t i = threadIdx.x * 4; i < in.dp; i += 1024) (void)stream_gather<NS>(in, i, true);
+        stream_each<NS>(in, true, [](uint32_t, const float4) {});
         return;
     }
     T *act = static_cast<T *>(a.act) + row * in.dp;

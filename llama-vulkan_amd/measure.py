@@ -16,7 +16,8 @@
     python llama-vulkan_amd/measure.py copy          1 GiB device-to-device copy: achievable bandwidth, counter calibration
     python llama-vulkan_amd/measure.py read-stream   4 GiB read by a kernel that only reads: the bandwidth a weight stream can reach
     python llama-vulkan_amd/measure.py block [SIZE]  block models beside LLaMA layers of the same width (bench.py --block)
-    python llama-vulkan_amd/measure.py block-only SIZE   prompts and decode steps of a block model alone (for kernel traces)
+    python llama-vulkan_amd/measure.py zedenex [SIZE]    Zedenex beside Somesun of the same width (bench.py --block Zedenex)
+    python llama-vulkan_amd/measure.py block-only SIZE   prompts and decode steps of Somesun alone (for kernel traces); zedenex-only SIZE: of Zedenex
     python llama-vulkan_amd/measure.py all
 
 Every figure is algorithmic bytes (weights as stored in the GGML file, 18 B / 34 B per 32 weights, plus vectors and the
@@ -368,43 +369,123 @@ def block_step_cost(c, pos):
     return L * (2 * w + state) + 2 * V * D, 2.0 * L * w
 
 
-def block_cases(ctx, report=emit, sizes=None, prompts=(512, 2048), steps=64):
+# Zedenex at layer sizes of real models: latent attention with a dense feed-forward behind it, and state-space layers without one;
+# compared with Somesun of the same width above
+ZEDENEX_SIZES = {
+    "4096": dict(vocab=32000, width=4096, streams=4, latent=(32, 128, 64, 128, 1536, 512), ssm=(128, 8, 128, 64, 4), ff=11008, layers="LMLM"),
+    "2048": dict(vocab=32000, width=2048, streams=2, latent=(16, 128, 64, 128, 768, 512), ssm=(64, 1, 128, 64, 4), ff=5504, layers="LMLMLM"),
+}
+
+
+def zedenex_model(ctx, size, compute=None):
+    """random weights, as block_model has them: matrices share random bytes on the host; a layer "L" is latent attention with its
+    feed-forward, "M" a state-space layer"""
+    import numpy as np
+    c = ZEDENEX_SIZES[size]
+    D, V, S, ff = c["width"], c["vocab"], c["streams"], c["ff"]
+    H, d, r, vd, qr, kr = c["latent"]
+    mh, g, n, mv, taps = c["ssm"]
+    inner, chan = mh * mv, mh * mv + 2 * g * n
+    blob = max(V * D, ff * D, (inner + chan + mh) * D, H * (d + r) * qr)
+    rng = np.random.default_rng(7)
+    x = np.tile((rng.standard_normal(1 << 22) * 0.02).astype(np.float32), (blob + (1 << 22) - 1) >> 22)[:blob]
+    ones = max(D, inner, qr, kr)
+    base = np.concatenate([(x.view(np.uint32) >> 16).astype(np.uint16), np.full(ones, 0x3F80, np.uint16)])
+    table, blocks = [], []
+
+    def t(name, rows, cols=1, one=False):
+        table.append((name, lva.LV_BF16, blob * 2 if one else 0, rows, cols, rows * cols * 2))
+
+    def site(norm, hc):
+        t(norm, D, one=True); t(norm + ".b", D); t(norm + ".alpha", 1, one=True)
+        if hc:
+            t(hc + "in", S, one=True); t(hc + "out", S, one=True); t(hc + "mix", S, S)
+    t("embed", V, D); t("bigram", 4098, D); site("final.norm", None)
+    for i, kind in enumerate(c["layers"]):
+        p, m, b = f"l{i}.", f"l{i}.mix.", lva.BlockSpec()
+        site(p + "norm1", p + "hc1.")
+        if kind == "L":
+            site(p + "norm2", p + "hc2.")
+            t(m + "dq", qr, D); t(m + "dq.norm", qr, one=True); t(m + "uq", H * (d + r), qr); t(m + "dkv", kr + r, D); t(m + "dkv.norm", kr, one=True)
+            t(m + "uk", H * d, kr); t(m + "uv", H * vd, kr); t(m + "sink", H); t(m + "o", D, H * vd)
+            t(p + "mlp.gate", ff, D); t(p + "mlp.up", ff, D); t(p + "mlp.down", D, ff)
+            b.latent = lva.LatentSpec(H, d, r, vd, qr, kr, (d + r) ** -0.5, r, 10000.0, lva.ATTN_SINK)
+            b.dense = lva.DenseSpec(ff, lva.ACT_RELU)
+        else:
+            t(m + "in", inner + chan + mh, D); t(m + "conv", chan, taps); t(m + "conv.b", chan); t(m + "dt_bias", mh); t(m + "A_log", mh); t(m + "D", mh)
+            t(m + "norm", inner, one=True); t(m + "o", D, inner)
+            b.ssm = lva.SsmSpec(mh, g, n, mv, taps, g)
+        blocks.append(b)
+    return lva.BlockModel(ctx, base.view(np.uint8), table, blocks, V, D, 1e-5, lva.LV_BF16 if compute is None else compute, norm=lva.NORM_TANH, streams=S,
+                          tied_head=1, embed_scale=8.0, bigram_buckets=4097, bigram_prev=31, bigram_cur=17)
+
+
+def zedenex_step_cost(c, pos):
+    """as block_step_cost: a decode step reads the weights of every product once (W_uk as its transpose), the cache rows and the
+    recurrent state; a prompt's token goes through every weight once"""
+    D, V, ff = c["width"], c["vocab"], c["ff"]
+    H, d, r, vd, qr, kr = c["latent"]
+    mh, g, n, mv, _ = c["ssm"]
+    inner, chan = mh * mv, mh * mv + 2 * g * n
+    wl = D * (qr + kr + r) + H * (d + r) * qr + H * (d + vd) * kr + D * H * vd + 3 * D * ff
+    wm = D * (inner + chan + mh) + D * inner
+    nl, nm = c["layers"].count("L"), c["layers"].count("M")
+    return nl * (2 * wl + 2 * (kr + r) * (pos + 1)) + nm * (2 * wm + 8 * inner * n) + 2 * V * D, 2.0 * (nl * wl + nm * wm)
+
+
+def prompt_and_decode(s, vocab, label, cost, flops_per_token, report, prompts=(512, 2048), steps=64, **kw):
+    """one model's prompts (each third run timed, with HIP events) and decode steps (wall clock, greedy pick included)"""
+    out, n_max = [], max(prompts)
+    for n in prompts:
+        toks = lva.synth_tokens(n, 3, vocab, seed=n)
+        for _ in range(2):
+            s.begin(toks, 0)
+            s.wait()
+        s.timer_start()
+        s.begin(toks, 0)
+        ms = s.timer_stop()
+        tf = flops_per_token * n / ms / 1e9
+        out.append(report(case=label + " prompt", tokens=n, ms=round(ms, 3), tok_s=round(n / ms * 1e3, 1), TFLOPs=round(tf, 1),
+                          frac_of_mfma_peak=round(tf / MFMA_PEAK_TFLOPS, 4), **kw))
+    s.begin(lva.synth_tokens(n_max, 3, vocab, seed=1), 0)
+    tok, pos, total = s.argmax(), n_max, 0
+    for i in range(8 + steps):
+        if i == 8:
+            t0 = time.perf_counter()
+        s.begin([tok], pos)
+        tok = s.argmax()
+        total += cost(pos) if i >= 8 else 0
+        pos += 1
+    dt = time.perf_counter() - t0
+    out.append(report(case=label + " decode", positions=[n_max + 8, pos - 1], tok_s=round(steps / dt, 1), ms=round(dt / steps * 1e3, 4),
+                      GBps=round(total / dt / 1e9, 1), frac_of_hbm_peak=round(total / dt / 1e9 / HBM_PEAK_GBS, 4), **kw))
+    return out
+
+
+def zedenex_cases(ctx, report=emit, sizes=None):
+    """prefill and decode of Zedenex and of Somesun at the same width, same machine, same clock"""
+    out = []
+    for size in sizes or ZEDENEX_SIZES:
+        for label, sizes_of, make, cost in ((f"Zedenex width {size}", ZEDENEX_SIZES, zedenex_model, zedenex_step_cost), (f"Somesun width {size}", BLOCK_SIZES, block_model, block_step_cost)):
+            c = sizes_of[size]
+            m = make(ctx, size)
+            s = lva.Session(m, 2048 + 64 + 16)
+            out += prompt_and_decode(s, c["vocab"], label, lambda pos: cost(c, pos)[0], cost(c, 0)[1], report, layers=len(c["layers"]) if isinstance(c["layers"], str) else c["layers"])
+            s.close()
+            m.close()
+    return out
+
+
+def block_cases(ctx, report=emit, sizes=None):
     """prefill and decode of a block model and of its LLaMA counterpart (q8_0, on the persistent kernel where it has one and on the
     graph of single kernels), same machine, same clock"""
     out_cases = []
-
-    def timed(s, vocab, label, cost, flops_per_token, **kw):
-        n_max = max(prompts)
-        for n in prompts:
-            toks = lva.synth_tokens(n, 3, vocab, seed=n)
-            for _ in range(2):
-                s.begin(toks, 0)
-                s.wait()
-            s.timer_start()
-            s.begin(toks, 0)
-            ms = s.timer_stop()
-            tf = flops_per_token * n / ms / 1e9
-            out_cases.append(report(case=label + " prompt", tokens=n, ms=round(ms, 3), tok_s=round(n / ms * 1e3, 1), TFLOPs=round(tf, 1),
-                                    frac_of_mfma_peak=round(tf / MFMA_PEAK_TFLOPS, 4), **kw))
-        s.begin(lva.synth_tokens(n_max, 3, vocab, seed=1), 0)
-        tok, pos, total = s.argmax(), n_max, 0
-        for i in range(8 + steps):
-            if i == 8:
-                t0 = time.perf_counter()
-            s.begin([tok], pos)
-            tok = s.argmax()
-            total += cost(pos) if i >= 8 else 0
-            pos += 1
-        dt = time.perf_counter() - t0
-        out_cases.append(report(case=label + " decode", positions=[n_max + 8, pos - 1], tok_s=round(steps / dt, 1), ms=round(dt / steps * 1e3, 4),
-                                GBps=round(total / dt / 1e9, 1), frac_of_hbm_peak=round(total / dt / 1e9 / HBM_PEAK_GBS, 4), **kw))
-
     for size in sizes or BLOCK_SIZES:
         c = BLOCK_SIZES[size]
         m = block_model(ctx, size)
-        s = lva.Session(m, max(prompts) + steps + 16)
+        s = lva.Session(m, 2048 + 64 + 16)
         _, fl = block_step_cost(c, 0)
-        timed(s, c["vocab"], f"Somesun width {size}", lambda pos: block_step_cost(c, pos)[0], fl, layers=c["layers"])
+        out_cases += prompt_and_decode(s, c["vocab"], f"Somesun width {size}", lambda pos: block_step_cost(c, pos)[0], fl, report, layers=c["layers"])
         s.close()
         m.close()
         L = c["llama"]
@@ -414,12 +495,12 @@ def block_cases(ctx, report=emit, sizes=None, prompts=(512, 2048), steps=64):
             lva.write_model(path + ".tmp", wtype=lva.LV_Q8_0, seed=5, **L)
             os.replace(path + ".tmp", path)
         lm = lva.Model(ctx, path)
-        s = lva.Session(lm, max(prompts) + steps + 16)
+        s = lva.Session(lm, 2048 + 64 + 16)
         kinds = [lva.PATH_PERSISTENT, lva.PATH_GRAPH] if s.path() == lva.PATH_PERSISTENT else [lva.PATH_GRAPH]
         for k in kinds:
             s.set_path(k)
-            timed(s, L["vocab"], f"LLaMA width {size} q8_0, {'persistent' if k == lva.PATH_PERSISTENT else 'graph'}", lambda pos: step_bytes(L, lva.LV_Q8_0, pos),
-                  2.0 * L["layers"] * (4 * L["dim"] ** 2 + 3 * L["dim"] * L["ff"]), layers=L["layers"])
+            out_cases += prompt_and_decode(s, L["vocab"], f"LLaMA width {size} q8_0, {'persistent' if k == lva.PATH_PERSISTENT else 'graph'}",
+                                           lambda pos: step_bytes(L, lva.LV_Q8_0, pos), 2.0 * L["layers"] * (4 * L["dim"] ** 2 + 3 * L["dim"] * L["ff"]), report, layers=L["layers"])
         s.close()
         lm.close()
     return out_cases
@@ -446,9 +527,11 @@ def main():
         gemm_cases(ctx)
     if which == "block":
         block_cases(ctx, sizes=sys.argv[2:3] or None)
-    if which == "block-only":     # without the LLaMA side, for kernel traces: prompts of 2048, then decode
-        c = BLOCK_SIZES[sys.argv[2]]
-        m = block_model(ctx, sys.argv[2])
+    if which == "zedenex":
+        zedenex_cases(ctx, sizes=sys.argv[2:3] or None)
+    if which in ("block-only", "zedenex-only"):     # one model by itself, for kernel traces: prompts of 2048, then decode
+        c = (BLOCK_SIZES if which == "block-only" else ZEDENEX_SIZES)[sys.argv[2]]
+        m = (block_model if which == "block-only" else zedenex_model)(ctx, sys.argv[2])
         s = lva.Session(m, 2200)
         toks = lva.synth_tokens(2048, 3, c["vocab"], seed=1)
         for _ in range(3):
