@@ -57,7 +57,7 @@ struct BlockLayer {
     bool ff() const { return moe || dense; }
     uint32_t dstride() const { return up(spec.delta.dim, 64); }
     uint32_t channels() const { return 2 * spec.delta.kv_heads * spec.delta.dim + spec.delta.heads * spec.delta.vdim; }
-    uint32_t sstride() const { return up(spec.ssm.state, 64); }
+    uint32_t sstride() const { return spec.ssm.state <= 64 ? 64 : spec.ssm.state <= 128 ? 128 : 256; }
     uint32_t ssm_inner() const { return spec.ssm.heads * spec.ssm.vdim; }
     uint32_t ssm_channels() const { return ssm_inner() + 2 * spec.ssm.groups * spec.ssm.state; }
     uint32_t latent_size() const { return spec.latent.dim + spec.latent.rot_dim; }
@@ -731,7 +731,7 @@ int block_session_reserve(BlockSession *s, uint32_t positions)
             const uint64_t splits = (ring + gqa_split(l.dp) - 1) / gqa_split(l.dp);
             part = std::max<uint64_t>(part, l.spec.attn.kv_heads * l.groups * splits * l.r * (l.dp + 2));
         } else {
-            part = std::max<uint64_t>(part, (uint64_t)latent_splits(l.spec.latent.heads, positions) * l.spec.latent.heads * latent_part_stride(l.kc));
+            part = std::max<uint64_t>(part, ((uint64_t)l.spec.latent.heads * latent_part_stride(l.kc)) << latent_split_bits(l.spec.latent.heads, positions));
         }
         if (ring == ls.ring) continue;
         // A ring that grows has not wrapped yet (it held every position so far), and one that shrinks keeps the rows that
@@ -866,6 +866,16 @@ template <class Fn> static int with_j(uint32_t j, Fn &&fn)
     case 1: return fn(std::integral_constant<int, 1>{});
     case 2: return fn(std::integral_constant<int, 2>{});
     case 3: return fn(std::integral_constant<int, 3>{});
+    default: return fn(std::integral_constant<int, 4>{});
+    }
+}
+
+// the same for a state-space recurrence's entries
+template <class Fn> static int with_state(uint32_t j, Fn &&fn)
+{
+    switch (j) {
+    case 1: return fn(std::integral_constant<int, 1>{});
+    case 2: return fn(std::integral_constant<int, 2>{});
     default: return fn(std::integral_constant<int, 4>{});
     }
 }
@@ -1083,12 +1093,12 @@ template <class CT> static int token_latent(BlockSession *s, size_t i, const uin
     latent_absorb_kernel<CT><<<dim3(sp.heads * (sp.kv_p / kAbsorbRows) + 1), dim3(256), 0, s->st>>>(LatentAbsorbArgs{sp, s->y1, s->y2, cfg, idx, s->ql});
     HIP_TRY(hipGetLastError());
     LatentStepArgs a{};
-    a.s = sp; a.q = s->ql; a.pos_ptr = cfg; a.pos_add = idx; a.splits = latent_splits(sp.heads, s->positions); a.part = s->part; a.out = s->left;
+    a.s = sp; a.q = s->ql; a.pos_ptr = cfg; a.pos_add = idx; a.split_bits = latent_split_bits(sp.heads, s->positions); a.part = s->part; a.out = s->left;
     auto attend = [&](auto nq, auto nb) -> int {
         auto *k = &latent_attn_kernel<CT, decltype(nq)::value, decltype(nb)::value>;
         const size_t lds = latent_attn_lds<CT>(sp.width);
         LV_TRY(allow_lds(k, lds));
-        k<<<dim3(latent_groups(sp.heads), a.splits), dim3(kLatentStepThreads), lds, s->st>>>(a);
+        k<<<dim3(latent_groups(sp.heads), 1u << a.split_bits), dim3(kLatentStepThreads), lds, s->st>>>(a);
         HIP_TRY(hipGetLastError());
         return LV_OK;
     };
@@ -1410,7 +1420,7 @@ template <class T> static int batch_ssm(BlockSession *s, size_t i, uint32_t pos,
         a.x = static_cast<float *>(w.sx); a.b = static_cast<float *>(w.sb); a.c = static_cast<float *>(w.sc); a.dt = w.sdt; a.decay = w.sdecay;
         ssm_prepare_kernel<<<dim3(ssm_prepare_columns(sp), (n + kSsmPrepareTokens - 1) / kSsmPrepareTokens), dim3(256), 0, st>>>(a);
         HIP_TRY(hipGetLastError());
-        LV_TRY(with_j(l.sstride() / 64, [&](auto j) -> int {
+        LV_TRY(with_state(l.sstride() / 64, [&](auto j) -> int {
             constexpr int J = decltype(j)::value;
             const size_t lds = 2 * 4ull * ssm_stage_floats<J>();
             LV_TRY(allow_lds(&ssm_scan_kernel<J>, lds));
@@ -1424,7 +1434,7 @@ template <class T> static int batch_ssm(BlockSession *s, size_t i, uint32_t pos,
         c.xt = static_cast<uint16_t *>(w.sx); c.b = static_cast<uint16_t *>(w.sb); c.c = static_cast<uint16_t *>(w.sc); c.bt = static_cast<uint16_t *>(w.sbt);
         ssm_operands_kernel<<<dim3(ssm_prepare_columns(sp), c.ldt / 8), dim3(256), 0, st>>>(c);
         HIP_TRY(hipGetLastError());
-        LV_TRY(with_j(l.sstride() / 64, [&](auto j) -> int {
+        LV_TRY(with_state(l.sstride() / 64, [&](auto j) -> int {
             constexpr int J = decltype(j)::value;
             LV_TRY(allow_lds(&ssm_chunk_kernel<J>, ssm_chunk_lds<J>()));
             ssm_chunk_kernel<J><<<dim3(sp.heads, (sp.vdim + 63) / 64), dim3(kSsmChunkThreads), ssm_chunk_lds<J>(), st>>>(c);
@@ -1432,7 +1442,7 @@ template <class T> static int batch_ssm(BlockSession *s, size_t i, uint32_t pos,
             return LV_OK;
         }));
     }
-    ssm_append_kernel<<<dim3(std::min(n, sp.taps)), dim3(256), 0, st>>>(a);
+    ssm_append_kernel<<<dim3(std::min(n, sp.taps), (sp.channels() + 255) / 256), dim3(256), 0, st>>>(a);
     HIP_TRY(hipGetLastError());
     const GroupInput g = group_in(sp, w.o, w.y1);
     const size_t lds = 4ull * (g.n + group_sums(g.groups, 4) + 4);

@@ -39,15 +39,17 @@ constexpr uint32_t kLatentMaxWidth = 768;
 constexpr uint32_t kLatentMaxHeads = 512;
 constexpr int kLatentKeys = 32;         // keys of a block
 constexpr int kLatentTile = 16;         // heads of a workgroup
-constexpr uint32_t kLatentMaxSplits = 64;
+constexpr uint32_t kLatentMaxSplits = 128;
 constexpr int kLatentStepThreads = 512;
 inline uint32_t latent_groups(uint32_t heads) { return (heads + kLatentTile - 1) / kLatentTile; }
-// key ranges the grid of a one-token step provides, for a cache of `positions` rows
-inline uint32_t latent_splits(uint32_t heads, uint32_t positions)
+// key ranges the grid of a one-token step provides, for a cache of `positions` rows: 2^this
+inline uint32_t latent_split_bits(uint32_t heads, uint32_t positions)
 {
     const uint32_t blocks = (positions + kLatentKeys - 1) / kLatentKeys, want = 256 / latent_groups(heads);
     const uint32_t most = want < 8 ? 8 : want > kLatentMaxSplits ? kLatentMaxSplits : want;
-    return blocks < most ? blocks : most;
+    uint32_t bits = 0;
+    while (1u << bits < blocks && 2u << bits <= most) bits++;
+    return bits;
 }
 __host__ __device__ constexpr uint32_t latent_part_stride(uint32_t kc) { return kc + 4; }     // sums, then maximum and sum of weights
 
@@ -161,17 +163,16 @@ struct LatentStepArgs {
     const void *q;                      // [heads][width] (latent_put)
     const uint32_t *pos_ptr;
     uint32_t pos_add;
-    uint32_t splits;                    // key ranges the grid provides
+    uint32_t split_bits;                // the grid provides 2^this key ranges
     float *part;                        // [split][head][latent_part_stride(kc)]
     float *out;                         // latent_value_kernel: [heads * vdim]
 };
 
-// key blocks of a range, and ranges that have keys, at position pos
-__device__ __forceinline__ void latent_ranges(const LatentStepArgs &a, uint32_t pos, uint32_t &blocks, uint32_t &per, uint32_t &active)
+// key blocks a query at pos sees, and how many of them a range takes; range i has keys if i * per < blocks
+__device__ __forceinline__ void latent_ranges(const LatentStepArgs &a, uint32_t pos, uint32_t &blocks, uint32_t &per)
 {
     blocks = pos / kLatentKeys + 1;
-    per = (blocks + a.splits - 1) / a.splits;
-    active = (blocks + per - 1) / per;
+    per = (blocks + (1u << a.split_bits) - 1) >> a.split_bits;
 }
 
 template <class CT> constexpr uint32_t latent_key_stride(uint32_t width) { return width + 16 / sizeof(CT); }
@@ -245,10 +246,10 @@ __global__ __launch_bounds__(kLatentStepThreads, 2) void latent_attn_kernel(Late
         q[j].load(static_cast<const CT *>(a.q) + (size_t)(h0 + l16) * W + k + g4 * 8, (size_t)s.heads * W, k < W && h0 + l16 < s.heads);
     }
     const uint32_t pos = *a.pos_ptr + a.pos_add;
-    uint32_t blocks, per, active;
-    latent_ranges(a, pos, blocks, per, active);
-    if (blockIdx.y >= active) return;
+    uint32_t blocks, per;
+    latent_ranges(a, pos, blocks, per);
     const uint32_t b0 = blockIdx.y * per, b1 = min(b0 + per, blocks);
+    if (b0 >= blocks) return;
     GqaRaw<CT> next[NQ];
     auto request = [&](uint32_t b) {
         const CT *row = static_cast<const CT *>(s.cache) + (size_t)min(b * kLatentKeys + kt * 16 + l16, pos) * W + g4 * 8;
@@ -342,11 +343,11 @@ __global__ __launch_bounds__(kLatentStepThreads, 2) void latent_attn_kernel(Late
 }
 
 constexpr int kLatentValueRows = 64;
-// grid (heads, vdim / 64 up): the ranges' sums of one head, then up to 64 rows of W_uv.  Four groups of 128 threads take up to 16
-// ranges each, four columns a thread; everything is requested before anything is used.
+// grid (heads, vdim / 64 up): the ranges' sums of one head, then up to 64 rows of W_uv.  Four groups of 128 threads take 16 ranges
+// each at a time, four columns a thread; weights and the first 64 ranges are requested before anything is used.
 static __global__ __launch_bounds__(kLatentStepThreads, 2) void latent_value_kernel(LatentStepArgs a)
 {
-    constexpr int AHEAD = 8, COLS = 512, RANGES = kLatentMaxSplits / 4;
+    constexpr int AHEAD = 8, COLS = 512, RANGES = 16;
     __shared__ __attribute__((aligned(16))) float o[kLatentMaxWidth], sums[4][COLS];
     __shared__ float weight[kLatentMaxSplits];
     const LatentSpec &s = a.s;
@@ -356,32 +357,44 @@ static __global__ __launch_bounds__(kLatentStepThreads, 2) void latent_value_ker
 #pragma unroll
     for (int i = 0; i < AHEAD; i++) v[i] = load_once(w + min((uint32_t)i, steps - 1) * 64);
     const uint32_t pos = *a.pos_ptr + a.pos_add, PS = latent_part_stride(s.kc);
-    uint32_t blocks, per, active;
-    latent_ranges(a, pos, blocks, per, active);
+    uint32_t blocks, per;
+    latent_ranges(a, pos, blocks, per);
     const float *part = a.part + (size_t)head * PS;
     const size_t next = (size_t)s.heads * PS;
     const uint32_t grp = __builtin_amdgcn_readfirstlane(threadIdx.x >> 7), c4 = (threadIdx.x & 127) * 4;
 #pragma unroll 1
     for (uint32_t c0 = 0; c0 < s.kv_p; c0 += COLS) {
         const uint32_t c = min(c0 + c4, s.kc - 4);
-        float4 z[RANGES];
-#pragma unroll
-        for (int i = 0; i < RANGES; i++) z[i] = *reinterpret_cast<const float4 *>(part + min(grp * RANGES + i, active - 1) * next + c);
-        if (c0 == 0) {
-            if (threadIdx.x < 64) {
-                const uint32_t i = threadIdx.x;
-                const float sink = s.sink ? s.sink[head] : -INFINITY, m = i < active ? part[i * next + s.kc] : -INFINITY, l = i < active ? part[i * next + s.kc + 1] : 0.f;
-                const float half = half_wave_max(m), top = fmaxf(fmaxf(half, __shfl_xor(half, 32, 64)), sink);
-                const float e = __expf(m - top), sum = wave_sum(e * l) + __expf(sink - top);
-                weight[i] = e / sum;
-            }
-            __syncthreads();
-        }
         float4 t = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll 1
+        for (uint32_t g0 = grp * RANGES; g0 < kLatentMaxSplits; g0 += 4 * RANGES) {
+            float4 z[RANGES];
 #pragma unroll
-        for (int i = 0; i < RANGES; i++) {
-            const float f = weight[grp * RANGES + i];          // 0 for a range without keys
-            t.x = fmaf(z[i].x, f, t.x); t.y = fmaf(z[i].y, f, t.y); t.z = fmaf(z[i].z, f, t.z); t.w = fmaf(z[i].w, f, t.w);
+            for (int i = 0; i < RANGES; i++) z[i] = *reinterpret_cast<const float4 *>(part + ((g0 + i) * per < blocks ? g0 + i : 0) * next + c);      // range 0 stands in for one without keys
+            if (c0 == 0 && g0 < 4 * RANGES) {
+                if (threadIdx.x < 64) {
+                    const float sink = s.sink ? s.sink[head] : -INFINITY;
+                    float m[2], l[2];
+#pragma unroll
+                    for (uint32_t k = 0; k < 2; k++) {
+                        const uint32_t i = threadIdx.x + k * 64;
+                        const bool has = i * per < blocks;
+                        m[k] = has ? part[i * next + s.kc] : -INFINITY;
+                        l[k] = has ? part[i * next + s.kc + 1] : 0.f;
+                    }
+                    const float half = half_wave_max(fmaxf(m[0], m[1])), top = fmaxf(fmaxf(half, __shfl_xor(half, 32, 64)), sink);
+                    const float e0 = __expf(m[0] - top), e1 = __expf(m[1] - top), inv = 1.f / (wave_sum(fmaf(e0, l[0], e1 * l[1])) + __expf(sink - top));
+                    weight[threadIdx.x] = e0 * inv;
+                    weight[threadIdx.x + 64] = e1 * inv;
+                }
+                __syncthreads();
+            }
+#pragma unroll
+            for (int i = 0; i < RANGES; i++) {
+                const float f = weight[g0 + i];          // 0 for a range without keys
+                t.x = fmaf(z[i].x, f, t.x); t.y = fmaf(z[i].y, f, t.y); t.z = fmaf(z[i].z, f, t.z); t.w = fmaf(z[i].w, f, t.w);
+            }
+            if ((g0 + 4 * RANGES) * per >= blocks) break;
         }
         *reinterpret_cast<float4 *>(&sums[grp][c4]) = t;
         __syncthreads();

@@ -27,7 +27,7 @@ struct SsmSpec {
     const float *a_log, *dt_bias, *skip, *norm;
     float eps;
     float *state, *ring;
-    uint32_t nstride;                    // 64 J
+    uint32_t nstride;                    // 64 J, J = 1, 2 or 4
     __host__ __device__ uint32_t inner() const { return heads * vdim; }
     __host__ __device__ uint32_t channels() const { return heads * vdim + 2 * groups * n; }
     __device__ __forceinline__ uint32_t channel_at(uint32_t c) const { return x_off + c; }
@@ -143,12 +143,12 @@ static __global__ __launch_bounds__(256) void ssm_prepare_kernel(SsmBatchArgs a)
     }
 }
 
-// the batch's last convolution inputs into the ring; blockIdx.x = token counted from the end
+// the batch's last convolution inputs into the ring; blockIdx.x = token counted from the end, blockIdx.y = 256 channels
 static __global__ __launch_bounds__(256) void ssm_append_kernel(SsmBatchArgs a)
 {
     const SsmSpec &s = a.s;
-    const uint32_t t = a.n - 1 - blockIdx.x, C = s.channels();
-    for (uint32_t c = threadIdx.x; c < C; c += 256) s.ring[(size_t)((a.pos0 + t) % s.taps) * C + c] = a.y[(size_t)t * a.ldy + s.channel_at(c)];
+    const uint32_t t = a.n - 1 - blockIdx.x, C = s.channels(), c = blockIdx.y * 256 + threadIdx.x;
+    if (c < C) s.ring[(size_t)((a.pos0 + t) % s.taps) * C + c] = a.y[(size_t)t * a.ldy + s.channel_at(c)];
 }
 
 constexpr int kSsmScanTokens = 16, kSsmScanThreads = 256;
@@ -292,6 +292,23 @@ static __global__ __launch_bounds__(256) void ssm_operands_kernel(SsmChunkArgs a
     if (e < gn) reinterpret_cast<uint4 *>(a.bt)[(size_t)t8 * gn + e] = eight;
 }
 
+// the upper halves of two words, the first one's below
+__device__ __forceinline__ uint32_t upper_halves(uint32_t a, uint32_t b) { return __builtin_amdgcn_perm(b, a, 0x07060302u); }
+// The leading bf16 pieces of eight values, cut off them (not rounded: three in a row are all 24 bits); v keeps the rest
+__device__ __forceinline__ lv_bf8 next_piece(float (&v)[8])
+{
+    uint4 p;
+    uint32_t *w = reinterpret_cast<uint32_t *>(&p);
+#pragma unroll
+    for (int e = 0; e < 8; e += 2) {
+        const uint32_t a = __float_as_uint(v[e]), b = __float_as_uint(v[e + 1]);
+        w[e / 2] = upper_halves(a, b);
+        v[e] -= __uint_as_float(a & 0xffff0000u);
+        v[e + 1] -= __uint_as_float(b & 0xffff0000u);
+    }
+    return __builtin_bit_cast(lv_bf8, p);
+}
+
 constexpr int kSsmChunkThreads = 256;
 template <int J> constexpr int ssm_chunk_stages() { return J <= 2 ? 2 : 1; }
 template <int J> constexpr int ssm_chunk_stage_bytes() { return 3 * kSsmChunk * 64 * J * 2; }      // C and B rows, B by 8 tokens
@@ -316,17 +333,22 @@ __global__ __launch_bounds__(kSsmChunkThreads) void ssm_chunk_kernel(SsmChunkArg
     float4 *const state = reinterpret_cast<float4 *>(s.state + (size_t)channel * W);
     const float rate = -__expf(s.a_log[head]), skip = s.skip[head];
 
-    auto issue = [&](uint32_t t0, int st) {
-        uint8_t *b = chunk_lds + st * STAGE;
+    // a stage: 256 threads bring 32 / J rows of C and of B at a time, and as many entries of B by 8 tokens
+    const uint32_t gw = s.groups * W, row0 = threadIdx.x / (8 * J), ch0 = threadIdx.x % (8 * J);
+    const size_t rows_at = ((size_t)row0 * s.groups + grp) * W + (ch0 ^ (row0 & 7)) * 8, by8_at = (((size_t)(threadIdx.x / W) * s.groups + grp) * W + threadIdx.x % W) * 8;
+    const uint16_t *gc = a.c + rows_at, *gb = a.b + rows_at, *gt = a.bt + by8_at;      // of the next stage
+    auto issue = [&](int st) {
+        uint8_t *b = chunk_lds + st * STAGE + wave * 1024;
 #pragma unroll
         for (int i = 0; i < 2 * J; i++) {
-            const uint32_t first = (i * 4 + wave) * 64, e = first + lane, row = e / (8 * J), ch = e % (8 * J);
-            const size_t at = ((size_t)(t0 + row) * s.groups + grp) * W + (ch ^ (row & 7)) * 8;
-            __builtin_amdgcn_global_load_lds((lv_glb_any *)(a.c + at), (lv_lds_any *)(b + first * 16), 16, 0, 0);
-            __builtin_amdgcn_global_load_lds((lv_glb_any *)(a.b + at), (lv_lds_any *)(b + TILE + first * 16), 16, 0, 0);
-            const size_t by8 = (((size_t)(t0 / 8 + e / W) * s.groups + grp) * W + e % W) * 8;
-            __builtin_amdgcn_global_load_lds((lv_glb_any *)(a.bt + by8), (lv_lds_any *)(b + 2 * TILE + first * 16), 16, 0, 0);
+            const uint32_t on = i * (32 / J) * gw;       // both in steps of 256 threads' worth
+            __builtin_amdgcn_global_load_lds((lv_glb_any *)(gc + on), (lv_lds_any *)(b + i * 4096), 16, 0, 0);
+            __builtin_amdgcn_global_load_lds((lv_glb_any *)(gb + on), (lv_lds_any *)(b + TILE + i * 4096), 16, 0, 0);
+            __builtin_amdgcn_global_load_lds((lv_glb_any *)(gt + on), (lv_lds_any *)(b + 2 * TILE + i * 4096), 16, 0, 0);
         }
+        gc += kSsmChunk * gw;
+        gb += kSsmChunk * gw;
+        gt += kSsmChunk * gw;
     };
     uint4 xn[2];
     float dtn;
@@ -335,7 +357,7 @@ __global__ __launch_bounds__(kSsmChunkThreads) void ssm_chunk_kernel(SsmChunkArg
         for (int k = 0; k < 2; k++) xn[k] = reinterpret_cast<const uint4 *>(a.xt)[(size_t)(t0 / 8 + k * 4 + g4) * inner + channel];
         dtn = a.dt[(size_t)head * a.ldt + t0 + lane];
     };
-    issue(0, 0);
+    issue(0);
     request(0);
     lv_f4 S[4 * J];
 #pragma unroll
@@ -351,7 +373,7 @@ __global__ __launch_bounds__(kSsmChunkThreads) void ssm_chunk_kernel(SsmChunkArg
         const float dt = dtn;
         const bool more = t0 + kSsmChunk < a.n;
         if (more) {
-            if (NST == 2) issue(t0 + kSsmChunk, st ^ 1);
+            if (NST == 2) issue(st ^ 1);
             request(t0 + kSsmChunk);
         }
         const uint8_t *bc = chunk_lds + st * STAGE, *bb = bc + TILE, *bt = bb + TILE;
@@ -365,38 +387,27 @@ __global__ __launch_bounds__(kSsmChunkThreads) void ssm_chunk_kernel(SsmChunkArg
         __builtin_amdgcn_fence(__ATOMIC_SEQ_CST, "wavefront");
         __builtin_amdgcn_wave_barrier();
 
-        {
-            const int t = wave * 16 + l16;
-            const float mine = lt[t];
-            lv_bf8 fc[2 * J];
+        // weights: three tiles of 16 x 16 a wave, as (token tile, source tile); (0, 1) and (2, 3) are zeros
+        const uint32_t mine = wave == 0 ? 0x302000u : wave == 1 ? 0x311110u : wave == 2 ? 0x232221u : 0x013332u;
 #pragma unroll
-            for (int k = 0; k < 2 * J; k++) fc[k] = frag(bc, t, k);
-#pragma unroll 1
-            for (int j = 0; j <= (wave | 1); j++) {
-                float m[4] = {0.f, 0.f, 0.f, 0.f};
-                if (j <= wave) {
-                    lv_f4 g = lv_f4{0.f, 0.f, 0.f, 0.f};
+        for (int q = 0; q < 3; q++) {
+            const int ti = mine >> (8 * q + 4) & 15, si = mine >> (8 * q) & 15, t = ti * 16 + l16;
+            lv_f4 g = lv_f4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-                    for (int k = 0; k < 2 * J; k++) g = __builtin_amdgcn_mfma_f32_16x16x32_bf16(frag(bb, j * 16 + l16, k), fc[k], g, 0, 0, 0);
-                    const float4 ls = *reinterpret_cast<const float4 *>(lt + j * 16 + g4 * 4), ds = *reinterpret_cast<const float4 *>(dts + j * 16 + g4 * 4);
-                    const float lsv[4] = {ls.x, ls.y, ls.z, ls.w}, dsv[4] = {ds.x, ds.y, ds.z, ds.w};
+            for (int k = 0; k < 2 * J; k++) g = __builtin_amdgcn_mfma_f32_16x16x32_bf16(frag(bb, si * 16 + l16, k), frag(bc, t, k), g, 0, 0, 0);
+            const float4 ls = *reinterpret_cast<const float4 *>(lt + si * 16 + g4 * 4), ds = *reinterpret_cast<const float4 *>(dts + si * 16 + g4 * 4);
+            const float lsv[4] = {ls.x, ls.y, ls.z, ls.w}, dsv[4] = {ds.x, ds.y, ds.z, ds.w}, to = lt[t];
+            uint32_t m[4], r[4];
 #pragma unroll
-                    for (int r = 0; r < 4; r++) {
-                        const int u = j * 16 + g4 * 4 + r;
-                        const float w = g[r] * dsv[r] * __expf(mine - lsv[r]);
-                        m[r] = u < t ? w : u == t ? w + skip : 0.f;
-                    }
-                }
-                uint16_t h[4], q[4];
-#pragma unroll
-                for (int r = 0; r < 4; r++) {
-                    h[r] = float_to_bf16(m[r]);
-                    q[r] = float_to_bf16(m[r] - bf16_to_float(h[r]));
-                }
-                const int at = t * kSsmWeightLd + j * 16 + g4 * 4;
-                *reinterpret_cast<uint2 *>(mh + at) = make_uint2(h[0] | (uint32_t)h[1] << 16, h[2] | (uint32_t)h[3] << 16);
-                *reinterpret_cast<uint2 *>(ml + at) = make_uint2(q[0] | (uint32_t)q[1] << 16, q[2] | (uint32_t)q[3] << 16);
+            for (int e = 0; e < 4; e++) {
+                const int u = si * 16 + g4 * 4 + e;
+                const float w = g[e] * dsv[e] * __expf(to - lsv[e]), v = u < t ? w : u == t ? w + skip : 0.f;
+                m[e] = __float_as_uint(v);
+                r[e] = __float_as_uint(v - __uint_as_float(m[e] & 0xffff0000u));
             }
+            const int at = t * kSsmWeightLd + si * 16 + g4 * 4;
+            *reinterpret_cast<uint2 *>(mh + at) = make_uint2(upper_halves(m[0], m[1]), upper_halves(m[2], m[3]));
+            *reinterpret_cast<uint2 *>(ml + at) = make_uint2(upper_halves(r[0], r[1]), upper_halves(r[2], r[3]));
         }
         // read-outs: the state's part needs no weights and runs up to the barrier
         lv_f4 y[4];
@@ -405,14 +416,12 @@ __global__ __launch_bounds__(kSsmChunkThreads) void ssm_chunk_kernel(SsmChunkArg
 #pragma unroll
         for (int k = 0; k < 2 * J; k++) {
             lv_bf8 q[3];
+            {
+                float v[8];
 #pragma unroll
-            for (int e = 0; e < 8; e++) {
-                float v = S[2 * k + e / 4][e % 4];
+                for (int e = 0; e < 8; e++) v[e] = S[2 * k + e / 4][e % 4];
 #pragma unroll
-                for (int c = 0; c < 3; c++) {
-                    q[c][e] = (__bf16)v;
-                    v -= (float)q[c][e];
-                }
+                for (int c = 0; c < 3; c++) q[c] = next_piece(v);
             }
 #pragma unroll
             for (int i = 0; i < 4; i++) {
@@ -446,13 +455,9 @@ __global__ __launch_bounds__(kSsmChunkThreads) void ssm_chunk_kernel(SsmChunkArg
         for (int k = 0; k < 2; k++) {
             float w[8];
             load8(w, wt + k * 32 + g4 * 8);
-            lv_bf8 xh, xl;
 #pragma unroll
-            for (int e = 0; e < 8; e++) {
-                const float v = (float)fx[k][e] * w[e];
-                xh[e] = (__bf16)v;
-                xl[e] = (__bf16)(v - (float)xh[e]);
-            }
+            for (int e = 0; e < 8; e++) w[e] *= (float)fx[k][e];
+            const lv_bf8 xh = next_piece(w), xl = next_piece(w);
 #pragma unroll
             for (int i = 0; i < 4 * J; i++) {
                 const lv_bf8 f = *reinterpret_cast<const lv_bf8 *>(bt + ((k * 4 + g4) * W + i * 16 + l16) * 16);
@@ -461,17 +466,24 @@ __global__ __launch_bounds__(kSsmChunkThreads) void ssm_chunk_kernel(SsmChunkArg
             }
         }
         if (live) {
+            float *out = a.o + (size_t)(t0 + g4 * 4) * inner + channel;
+            const uint32_t left = a.n - t0;
+            if (left >= kSsmChunk) {
 #pragma unroll
-            for (int i = 0; i < 4; i++)
+                for (int i = 0; i < 4; i++)
 #pragma unroll
-                for (int r = 0; r < 4; r++) {
-                    const uint32_t t = t0 + i * 16 + g4 * 4 + r;
-                    if (t < a.n) a.o[(size_t)t * inner + channel] = y[i][r];
-                }
+                    for (int r = 0; r < 4; r++) out[(i * 16 + r) * inner] = y[i][r];
+            } else {
+#pragma unroll
+                for (int i = 0; i < 4; i++)
+#pragma unroll
+                    for (int r = 0; r < 4; r++)
+                        if ((uint32_t)(i * 16 + g4 * 4 + r) < left) out[(i * 16 + r) * inner] = y[i][r];
+            }
         }
         if (NST == 1 && more) {
             __syncthreads();
-            issue(t0 + kSsmChunk, 0);
+            issue(0);
         }
     }
     if (live) {

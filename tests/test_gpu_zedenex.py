@@ -243,6 +243,18 @@ def test_a_prompt_longer_than_a_batch(lva, ctx):
             assert rel(d.run(toks, (2049, 81, 1)), want) < TOL[compute]
 
 
+@pytest.mark.parametrize("compute", [F32, BF16])
+def test_more_key_blocks_than_ranges(lva, ctx, compute):
+    """many heads leave few key ranges a head: several blocks each, the last range with fewer or none"""
+    cfg = zb.config(width=40, streams=1, layers=[zb.layer(zb.latent(heads=250, dim=4, rot_dim=2, vdim=3, q_rank=16, kv_rank=12), 0)])
+    W = zb.weights(cfg, 49)
+    toks = tokens_for(cfg, 1060, 4)
+    want = zo.forward(toks, bb.as_float(W), cfg)[0]
+    with device(lva, ctx, cfg, W, compute, backlog=1100) as d:
+        for first in (500, 700, 1020):
+            assert rel(d.run(toks[:first + 40], (first, 1)), want[:first + 40]) < TOL[compute], first
+
+
 def test_long_decoding_follows_the_prompt_form(lva, ctx):
     """420 tokens decoded one by one through graph replays, the cache growing under them"""
     cfg = deep()
